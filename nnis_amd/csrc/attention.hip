@@ -64,6 +64,23 @@ constexpr int HDR = NNIS_REG_DIM;
 #if NNIS_POOLED_BLOCKS && !NNIS_SCORE_EXTRAS
 #error "pooled blocks come with the scores' extras"
 #endif
+// 1: scores fall with the logarithm of the distance (NnisHeadTerms: r1, r2); compiled in, into all of the kernels' loops
+#ifndef NNIS_DISTANCE_LOG
+#define NNIS_DISTANCE_LOG 0
+#endif
+// 1: the matrix-core kernels multiply a head's output by a gate on its way out (NnisHeadTerms: gate)
+#ifndef NNIS_HEAD_GATES
+#define NNIS_HEAD_GATES 0
+#endif
+
+// What an attention may take head by head beyond the plain formula, each off when null.  The entry points that end in
+// `_terms` take a pointer to this structure (host memory, read during the call).
+struct NnisHeadTerms {
+  const float* r1;   // [heads], with r2: a key n positions back loses r1 * ln(1 + r2 * n) of its scaled score
+  const float* r2;   // [heads], not negative
+  const void* gate;  // [tokens][gate_stride]: head h's output is multiplied by sigmoid(gate[token][h])
+  int gate_dtype, gate_stride;
+};
 
 struct AttnArgs {
   const void* q;  // [tokens, heads, HD]
@@ -94,7 +111,12 @@ struct AttnArgs {
   const int* pool_table;  // [slots][pool_max_pages]
   int pool_max_pages;
   int pool;
+  NnisHeadTerms terms;
 };
+
+__device__ __forceinline__ float head_gate(const NnisHeadTerms& terms, size_t token, int head) {
+  return 1.0f / (1.0f + expf(-load_as_f32(terms.gate, terms.gate_dtype, token * terms.gate_stride + head)));
+}
 
 // One wave per (token, query head); lanes take keys lo+lane, lo+lane+64, ...,
 // each keeps its own running maximum, sum and output, merged at the end.
@@ -133,6 +155,7 @@ __global__ __launch_bounds__(256) void attention_rows_kernel(AttnArgs a) {
 #pragma unroll
   for (int d = 0; d < HDV; ++d) o[d] = 0.0f;
   const float* bias_row = a.bias ? a.bias + (size_t)head * (a.reach + 1) : nullptr;
+  const float r1 = a.terms.r1 ? a.terms.r1[head] : 0.0f, r2 = a.terms.r1 ? a.terms.r2[head] : 0.0f;
 
   auto take = [&](const CacheT* kp, const CacheT* vp, const int* pages, int j, bool near) {
     const int page = pages[j / kPageTokens];
@@ -144,6 +167,7 @@ __global__ __launch_bounds__(256) void attention_rows_kernel(AttnArgs a) {
     float s = dot * a.scale;
     if (a.softcap > 0.0f) s = a.softcap * tanhf(s / a.softcap);
     if (bias_row && near) s += bias_row[min(pos - j, a.reach)];
+    if (a.terms.r1 && near) s -= r1 * log1pf(r2 * (float)(pos - j));
     const float m_new = fmaxf(m, s);
     const float alpha = expf(m - m_new);  // exp(-inf) = 0 on the first key
     const float p = expf(s - m_new);
@@ -168,7 +192,7 @@ __global__ __launch_bounds__(256) void attention_rows_kernel(AttnArgs a) {
   m_all = fmaxf(m_all, sink);
   const float factor = (m == -INFINITY) ? 0.0f : expf(m - m_all);
   const float l_all = wave_sum(l * factor) + (a.sink ? expf(sink - m_all) : 0.0f);
-  const float inv = 1.0f / l_all;
+  const float inv = (a.terms.gate ? head_gate(a.terms, token, head) : 1.0f) / l_all;
   float mine[(HDV + kWave - 1) / kWave];
 #pragma unroll
   for (int d = 0; d < HDV; ++d) {
@@ -316,11 +340,38 @@ __device__ __forceinline__ void load_block(BlockFrags& f, const bf16_t* k_page, 
   for (int t = 0; t < kTilesD; ++t) f.values[t] = *(const bf16x8*)(v_page + nnis_v_offset(16 * t + r, 32 * h + 8 * g));
 }
 
+// What a wave needs beyond lo and hi where the module takes the extras: the row of the bias table of each
+// column's head (null without a bias; a column's query sits at hi[c], so a key's distance is hi[c] - key), how
+// far the table reaches, and how many first keys stay visible below a window's lower end.  Where scores fall with the
+// logarithm of the distance: the two numbers of each column's head, r1 in the units of raw scores and base-2 logarithms.
+template <int C>
+struct More {
+#if NNIS_SCORE_EXTRAS
+  const float* bias_row[C];
+  float far_bias[C];  // the table's last row in the softmax's base-2 units: what every key `reach` and more back gets
+  int reach;
+  int keep;
+#endif
+#if NNIS_DISTANCE_LOG
+  float r1[C], r2[C];
+#endif
+};
+
+// Raw scores s of four keys one behind the other, the first of them n positions back from the column's query, each less
+// its r1 * log2(1 + r2 * distance): three instructions a score.  (A key beyond the query has a negative distance and
+// leaves whatever it leaves: it is masked behind this.)
+__device__ __forceinline__ void recede(f32x4& s, float r1, float r2, int n) {
+  const float first = fmaf(r2, (float)n, 1.0f);
+#pragma unroll
+  for (int e = 0; e < 4; ++e) s[e] = fmaf(-r1, __builtin_amdgcn_logf(fmaf(-(float)e, r2, first)), s[e]);
+}
+
 // Scores, softmax update and output update of one loaded block for C column tiles.
 //   lo[c], hi[c]: the column of this lane reads keys lo <= key <= hi
 template <int C>
 __device__ __forceinline__ void attend_block(AttnState<C>& st, const QFrag (&q)[C], const BlockFrags& f, int key0,
-                                             const int (&lo)[C], const int (&hi)[C], float scale_log2, const ScoreCap& cap, int g) {
+                                             const int (&lo)[C], const int (&hi)[C], float scale_log2, const ScoreCap& cap,
+                                             const More<C>& more, int g) {
 #pragma unroll
   for (int c = 0; c < C; ++c) {
     f32x4 s[2];
@@ -329,6 +380,9 @@ __device__ __forceinline__ void attend_block(AttnState<C>& st, const QFrag (&q)[
     for (int t = 0; t < 2; ++t) {
       s[t] = score_tile(f.keys[t], q[c]);
       bend(s[t], cap);
+#if NNIS_DISTANCE_LOG
+      recede(s[t], more.r1[c], more.r2[c], hi[c] - (key0 + 8 * g + 4 * t));
+#endif
     }
     // most blocks lie wholly inside what every lane's column reads: then no key needs a look at its index
     if (!__all(key0 >= lo[c] && key0 + 31 <= hi[c])) {
@@ -377,19 +431,6 @@ __device__ __forceinline__ void attend_block(AttnState<C>& st, const QFrag (&q)[
   }
 }
 
-// What a wave needs beyond lo and hi where the module takes the extras: the row of the bias table of each
-// column's head (null without a bias; a column's query sits at hi[c], so a key's distance is hi[c] - key), how
-// far the table reaches, and how many first keys stay visible below a window's lower end.
-template <int C>
-struct More {
-#if NNIS_SCORE_EXTRAS
-  const float* bias_row[C];
-  float far_bias[C];  // the table's last row in the softmax's base-2 units: what every key `reach` and more back gets
-  int reach;
-  int keep;
-#endif
-};
-
 #if NNIS_SCORE_EXTRAS
 // attend_block with the extras: a key counts if it is at or below the column's position and inside the window or
 // among the kept first keys; the bias by distance joins the scaled score (both in base-2 units) before the maximum.
@@ -408,6 +449,9 @@ __device__ __forceinline__ void attend_block_more(AttnState<C>& st, const QFrag 
     for (int t = 0; t < 2; ++t) {
       s[t] = score_tile(f.keys[t], q[c]);
       bend(s[t], cap);
+#if NNIS_DISTANCE_LOG
+      recede(s[t], more.r1[c], more.r2[c], hi[c] - (key0 + 8 * g + 4 * t));
+#endif
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         const int key = key0 + 8 * g + 4 * t + e;
@@ -472,10 +516,15 @@ __device__ __forceinline__ float sink_term(const float* sink, int head, float re
 // instructions, a few vector instructions, and so on.
 template <int C, bool AHEAD, int c>
 __device__ __forceinline__ void attend_unit_ahead(AttnState<C>& st, const QFrag (&q)[C], const BlockFrags& f, const BlockFrags& next,
-                                                  f32x4 (&s)[2], bf16x8& before, float scale_log2, float (&rise)[C], const ScoreCap& cap) {
+                                                  f32x4 (&s)[2], bf16x8& before, float scale_log2, float (&rise)[C], const ScoreCap& cap,
+                                                  const More<C>& more, const int (&back)[C]) {
   constexpr int kScores = 2 * (kFullD + (kTailD ? 1 : 0));
   bend(s[0], cap);  // (the scores come in as the matrix unit left them)
   bend(s[1], cap);
+#if NNIS_DISTANCE_LOG
+  recede(s[0], more.r1[c], more.r2[c], back[c]);
+  recede(s[1], more.r1[c], more.r2[c], back[c] - 4);
+#endif
   // rise[c]: the raw score (before the scale) above which column c's reference moves, (st.m[c] + kLazyRise) / scale:
   // the test of every unit is then the scores' maximum against a register
   float block_max = -INFINITY;
@@ -548,14 +597,16 @@ __device__ __forceinline__ void attend_unit_ahead(AttnState<C>& st, const QFrag 
     s[0] = ahead[0];
     s[1] = ahead[1];
   }
-  if constexpr (c + 1 < C) attend_unit_ahead<C, AHEAD, c + 1>(st, q, f, next, s, before, scale_log2, rise, cap);
+  if constexpr (c + 1 < C) attend_unit_ahead<C, AHEAD, c + 1>(st, q, f, next, s, before, scale_log2, rise, cap, more, back);
 }
 
+// back[c] (where scores fall with the distance): how far column c's query is behind the first of this lane's keys
 template <int C, bool AHEAD>
 __device__ __forceinline__ void attend_block_ahead(AttnState<C>& st, const QFrag (&q)[C], const BlockFrags& f, const BlockFrags& next,
-                                                   f32x4 (&s)[2], float scale_log2, float (&rise)[C], const ScoreCap& cap) {
+                                                   f32x4 (&s)[2], float scale_log2, float (&rise)[C], const ScoreCap& cap,
+                                                   const More<C>& more, const int (&back)[C]) {
   bf16x8 before;  // the probabilities of the column before, whose outputs are still to be multiplied
-  attend_unit_ahead<C, AHEAD, 0>(st, q, f, next, s, before, scale_log2, rise, cap);
+  attend_unit_ahead<C, AHEAD, 0>(st, q, f, next, s, before, scale_log2, rise, cap, more, back);
 }
 
 // The pages of a run of key blocks, 64 at a time in the lanes of the wave: a
@@ -607,7 +658,31 @@ struct MfmaArgs {
   const int* pool_table;  // [slots][pool_max_pages]
   int pool_max_pages;
   int pool;
+  NnisHeadTerms terms;    // with NNIS_DISTANCE_LOG and NNIS_HEAD_GATES
 };
+
+// the two numbers of column c's head into `more` (off: nothing is taken off any score)
+template <int C>
+__device__ __forceinline__ void take_decay(More<C>& more, const MfmaArgs& a, int c, int head) {
+#if NNIS_DISTANCE_LOG
+  more.r1[c] = a.terms.r1 ? a.terms.r1[head] / a.scale_log2 : 0.0f;
+  more.r2[c] = a.terms.r1 ? a.terms.r2[head] : 0.0f;
+#endif
+}
+
+// the factor of a head's output, asked for early (1 without gates)
+__device__ __forceinline__ float ask_gate(const NnisHeadTerms& terms, size_t token, int head) {
+#if NNIS_HEAD_GATES
+  if (terms.gate) return load_as_f32(terms.gate, terms.gate_dtype, token * terms.gate_stride + head);
+#endif
+  return 0.0f;
+}
+__device__ __forceinline__ float gate_factor(const NnisHeadTerms& terms, float logit) {
+#if NNIS_HEAD_GATES
+  if (terms.gate) return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-kLog2e * logit));
+#endif
+  return 1.0f;
+}
 
 __device__ __forceinline__ const bf16_t* k_page_ptr(const MfmaArgs& a, int page, int kv_head) {
   return a.k_pages + ((size_t)page * a.kv_heads + kv_head) * nnis_k_page_elems(HD);
@@ -736,7 +811,7 @@ __device__ __forceinline__ void attend_run(AttnState<C>& st, const QFrag (&q)[C]
 #if NNIS_SCORE_EXTRAS
     attend_block_more<C>(st, q, f, (first + (b >> 1) * stride) * kPageTokens + (b & 1) * 32, lo, hi, a.scale_log2, a.cap, more, g);
 #else
-    attend_block<C>(st, q, f, (first + (b >> 1) * stride) * kPageTokens + (b & 1) * 32, lo, hi, a.scale_log2, a.cap, g);
+    attend_block<C>(st, q, f, (first + (b >> 1) * stride) * kPageTokens + (b & 1) * 32, lo, hi, a.scale_log2, a.cap, more, g);
 #endif
   };
   int b0 = 0;
@@ -808,7 +883,13 @@ __device__ __forceinline__ void attend_run(AttnState<C>& st, const QFrag (&q)[C]
 #pragma unroll
           for (int t = 0; t < 2; ++t) s[t] = score_tile(ring[i].keys[t], q[0]);
         }
-        attend_block_ahead<C, kAhead>(st, q, ring[i], ring[(i + 1) % RING], s, a.scale_log2, rise, a.cap);
+        int back[C];
+#if NNIS_DISTANCE_LOG
+        const int b = b0 + i, lane_key = (first + (b >> 1) * stride) * kPageTokens + (b & 1) * 32 + 8 * g;
+#pragma unroll
+        for (int c = 0; c < C; ++c) back[c] = hi[c] - lane_key;
+#endif
+        attend_block_ahead<C, kAhead>(st, q, ring[i], ring[(i + 1) % RING], s, a.scale_log2, rise, a.cap, more, back);
         ask(ring[i], b0 + i + RING);
       }
     }
@@ -858,6 +939,10 @@ __device__ __forceinline__ void attend_pooled(AttnState<C>& st, const QFrag (&q)
   for (int c = 0; c < C; ++c) {
     none.bias_row[c] = nullptr;
     none.far_bias[c] = 0.0f;
+#if NNIS_DISTANCE_LOG
+    none.r1[c] = 0.0f;
+    none.r2[c] = 0.0f;
+#endif
   }
   const int page_count = last / kPageTokens + 1;
   const int mine = page_count > index ? (page_count - index + size - 1) / size : 0;
@@ -917,6 +1002,7 @@ __global__ __launch_bounds__(64 * kBlockWaves) void attention_prefill_kernel(Mfm
     QFrag q[C];
     int lo[C], hi[C];
     bool live[C];
+    float gates[C];
     int last = -1;
 #pragma unroll
     for (int qt = 0; qt < QT; ++qt)
@@ -929,6 +1015,7 @@ __global__ __launch_bounds__(64 * kBlockWaves) void attention_prefill_kernel(Mfm
         const int safe_row = row < rows ? row : rows - 1;
         const int safe_head = head < a.heads ? head : a.heads - 1;
         q[c] = load_row_operand(a.q + ((size_t)(start + safe_row) * a.heads + safe_head) * HD, g);
+        gates[c] = ask_gate(a.terms, start + safe_row, safe_head);
         hi[c] = live[c] ? pos0 + row : -1;
         lo[c] = (a.window > 0 && hi[c] + 1 > a.window) ? hi[c] + 1 - a.window : 0;
         last = hi[c] > last ? hi[c] : last;
@@ -954,6 +1041,10 @@ __global__ __launch_bounds__(64 * kBlockWaves) void attention_prefill_kernel(Mfm
       more.bias_row[c] = a.bias ? a.bias + (size_t)head * (a.reach + 1) : nullptr;
       more.far_bias[c] = a.bias ? more.bias_row[c][a.reach] * kLog2e : 0.0f;
     }
+#endif
+#if NNIS_DISTANCE_LOG
+#pragma unroll
+    for (int c = 0; c < C; ++c) take_decay(more, a, c, min(head0 + c % GH, a.heads - 1));
 #endif
     if (last >= 0) {
       const int first_page = first / kPageTokens, page_count = last / kPageTokens + 1 - first_page;
@@ -984,7 +1075,7 @@ __global__ __launch_bounds__(64 * kBlockWaves) void attention_prefill_kernel(Mfm
 #if NNIS_SCORE_EXTRAS
         total += sink_term(a.sink, head0 + gh, st.m[c]);
 #endif
-        const float inv = 1.0f / total;
+        const float inv = gate_factor(a.terms, gates[c]) / total;
         bf16_t* dst = a.out + ((size_t)(start + row0 + 16 * qt + r) * a.heads + head0 + gh) * HDV;
 #pragma unroll
         for (int t = 0; t < kTilesD; ++t) {
@@ -1032,7 +1123,8 @@ __global__ __launch_bounds__(64 * kBlockWaves) void attention_prefill_kernel(Mfm
 // (one split) or leaves its state in `partial` for the combine kernel.
 template <int C>
 __device__ __forceinline__ void finish_decode(AttnState<C>& st, const bool (&live)[C], const MfmaArgs& a, float* merge,
-                                              int token, int kv_head, int split, int wave, int waves, int lane) {
+                                              const float (&gates)[C], int token, int kv_head, int split, int wave, int waves,
+                                              int lane) {
   const int r = lane % 16, g = lane / 16;
   const int group = a.heads / a.kv_heads;
   if (!merge_waves<C>(st, merge, wave, waves, lane)) return;  // one wave is left
@@ -1051,7 +1143,7 @@ __device__ __forceinline__ void finish_decode(AttnState<C>& st, const bool (&liv
 #pragma unroll
     for (int c = 0; c < C; ++c) {
       if (!live[c]) continue;
-      const float inv = 1.0f / total[c];
+      const float inv = gate_factor(a.terms, gates[c]) / total[c];
       bf16_t* dst = a.out + ((size_t)token * a.heads + kv_head * group + 16 * c + r) * HDV;
 #pragma unroll
       for (int t = 0; t < kTilesD; ++t) {
@@ -1100,12 +1192,16 @@ __global__ __launch_bounds__(64 * kBlockWaves) void attention_decode_kernel(Mfma
   QFrag q[C];
   int lo[C], hi[C];
   bool live[C];
+  float gates[C];
+  More<C> more;
 #pragma unroll
   for (int c = 0; c < C; ++c) {
     const int member = 16 * c + r;
     live[c] = member < group;
     const int head = kv_head * group + (live[c] ? member : 0);
     q[c] = load_row_operand(a.q + ((size_t)token * a.heads + head) * HD, g);
+    gates[c] = ask_gate(a.terms, token, head);
+    take_decay(more, a, c, head);
     lo[c] = first_key;
     hi[c] = live[c] ? pos : -1;
   }
@@ -1116,7 +1212,6 @@ __global__ __launch_bounds__(64 * kBlockWaves) void attention_decode_kernel(Mfma
   const int end = min(begin + per_split, page_first + page_count);
   AttnState<C> st;
   init_state(st);
-  More<C> more;
 #if NNIS_SCORE_EXTRAS
   more.reach = a.reach;
   more.keep = a.window > 0 ? a.keep_first : 0;
@@ -1142,7 +1237,7 @@ __global__ __launch_bounds__(64 * kBlockWaves) void attention_decode_kernel(Mfma
     if (pool_slot >= 0) attend_pooled<C, (kDecodeRing / C >= 2 ? kDecodeRing / C : 2)>(st, q, a, pool_slot, kv_head, wave, waves, lo, hi, lane);
   }
 #endif
-  finish_decode<C>(st, live, a, merge, token, kv_head, split, wave, waves, lane);
+  finish_decode<C>(st, live, a, merge, gates, token, kv_head, split, wave, waves, lane);
 }
 
 // ---- decode with keys on lanes, for groups of up to 4 query heads ------------------------------------
@@ -1193,6 +1288,10 @@ __global__ __launch_bounds__(64 * kKeysWaves) void attention_decode_keys_kernel(
   const int first_key = (a.window > 0 && pos + 1 > a.window) ? pos + 1 - a.window : 0;
   const int* pages = a.block_table + (size_t)(a.rows_by_token ? token : slot) * a.max_pages;
 
+  // the end's columns are the heads r of the group; the scores' are the heads j
+  float gates[1] = {ask_gate(a.terms, token, kv_head * group + (r < group ? r : 0))};
+  More<1> more;
+  take_decay(more, a, 0, kv_head * group + (j < group ? j : 0));
   // the query of head j, all channels (heads beyond the group: zeros, their columns are never written)
   bf16x8 q[HD / 8];
   {
@@ -1245,6 +1344,9 @@ __global__ __launch_bounds__(64 * kKeysWaves) void attention_decode_keys_kernel(
       }
       f32x4 s = s0 + s1;
       bend(s, a.cap);
+#if NNIS_DISTANCE_LOG
+      recede(s, more.r1[0], more.r2[0], pos - (key0 + 4 * blk));
+#endif
       const bool inside = key0 >= first_key && key0 + kPageTokens - 1 <= pos;  // every key of the page is read
       float top = -INFINITY;
 #pragma unroll
@@ -1330,7 +1432,7 @@ __global__ __launch_bounds__(64 * kKeysWaves) void attention_decode_keys_kernel(
     st.m[0] = -INFINITY;
     st.l[0] = 0.0f;
   }
-  finish_decode<1>(st, live, a, merge, token, kv_head, split, wave, waves, lane);
+  finish_decode<1>(st, live, a, merge, gates, token, kv_head, split, wave, waves, lane);
 }
 #endif  // NNIS_REG_DIM <= 128
 
@@ -1338,8 +1440,9 @@ __global__ __launch_bounds__(64 * kKeysWaves) void attention_decode_keys_kernel(
 // A kernel of its own: letting the last block of a (token, kv head) do it needs a device-wide fence in
 // every block, which was measured several times dearer than this launch.
 __global__ void attention_combine_kernel(const float* __restrict__ partial, bf16_t* __restrict__ out,
-                                         const int* __restrict__ tok_slot, int heads, int splits) {
+                                         const int* __restrict__ tok_slot, int heads, int splits, NnisHeadTerms terms) {
   const int token = blockIdx.x, head = blockIdx.y;
+  const float gate = ask_gate(terms, token, head);
   const float* base = partial + ((size_t)token * heads + head) * splits * kPartial;
   constexpr int kAtOnce = 8;  // runs whose references, sums and outputs a thread asks for together: one round trip
   if (splits <= kAtOnce) {
@@ -1367,7 +1470,7 @@ __global__ void attention_combine_kernel(const float* __restrict__ partial, bf16
           den += l[s] * w;
         }
       }
-      if (slot >= 0) out[((size_t)token * heads + head) * HDV + d] = (bf16_t)(num / den);
+      if (slot >= 0) out[((size_t)token * heads + head) * HDV + d] = (bf16_t)(num / den * gate_factor(terms, gate));
     }
     return;
   }
@@ -1383,7 +1486,7 @@ __global__ void attention_combine_kernel(const float* __restrict__ partial, bf16
       num += p[d] * w;
       den += p[HDV + 1] * w;
     }
-    out[((size_t)token * heads + head) * HDV + d] = (bf16_t)(num / den);
+    out[((size_t)token * heads + head) * HDV + d] = (bf16_t)(num / den * gate_factor(terms, gate));
   }
 }
 
@@ -1391,13 +1494,27 @@ __global__ void attention_combine_kernel(const float* __restrict__ partial, bf16
 
 }  // namespace
 
-extern "C" int nnis_attention_rows_pooled(const void* q, int q_dtype, void* out, int out_dtype, const void* k_pages,
+static NnisHeadTerms no_terms() {
+  NnisHeadTerms terms;
+  terms.r1 = terms.r2 = nullptr; terms.gate = nullptr; terms.gate_dtype = terms.gate_stride = 0;
+  return terms;
+}
+
+static int fill_terms(NnisHeadTerms& into, const NnisHeadTerms* terms, int heads) {
+  into = terms ? *terms : no_terms();
+  NNIS_REQUIRE((into.r1 == nullptr) == (into.r2 == nullptr), "attention: the two numbers of a bias by distance come together");
+  NNIS_REQUIRE(into.gate == nullptr || (nnis_dtype_ok(into.gate_dtype) && into.gate_stride >= heads),
+               "attention: gates of type %d in rows of %d for %d heads", into.gate_dtype, into.gate_stride, heads);
+  return 0;
+}
+
+extern "C" int nnis_attention_rows_terms(const void* q, int q_dtype, void* out, int out_dtype, const void* k_pages,
                                           const void* v_pages, int cache_dtype, const int* block_table, int max_pages,
                                           const int* tok_slot, const int* tok_pos, int tokens, int heads, int kv_heads,
                                           int head_dim, int window, float scale, int value_dim, float softcap, int keep_first,
                                           const float* bias, int reach, const float* sink, const void* pool_k,
                                           const void* pool_v, const int* pool_table, int pool_max_pages, int pool,
-                                          void* stream) {
+                                          const NnisHeadTerms* terms, void* stream) {
   NNIS_REQUIRE(pool >= 0 && (pool == 0 || (window > 0 && pool_k && pool_v && pool_table && pool_max_pages > 0)),
                "attention: pooled blocks (%d tokens each) need a window and pages of their own", pool);
   NNIS_REQUIRE(head_dim == HD, "attention: this module is compiled for head_dim %d, got %d", HD, head_dim);
@@ -1417,6 +1534,7 @@ extern "C" int nnis_attention_rows_pooled(const void* q, int q_dtype, void* out,
   a.tokens = tokens; a.heads = heads; a.kv_heads = kv_heads; a.window = window; a.scale = scale; a.softcap = softcap;
   a.keep_first = window > 0 ? keep_first : 0; a.bias = bias; a.reach = reach; a.sink = sink;
   a.pool_k = pool_k; a.pool_v = pool_v; a.pool_table = pool_table; a.pool_max_pages = pool_max_pages; a.pool = pool;
+  if (fill_terms(a.terms, terms, heads)) return 1;
   const long long items = (long long)tokens * heads;
   const unsigned blocks = (unsigned)((items + 3) / 4);
   if (cache_dtype == NNIS_F32) {
@@ -1428,6 +1546,17 @@ extern "C" int nnis_attention_rows_pooled(const void* q, int q_dtype, void* out,
   return 0;
 }
 
+extern "C" int nnis_attention_rows_pooled(const void* q, int q_dtype, void* out, int out_dtype, const void* k_pages,
+                                          const void* v_pages, int cache_dtype, const int* block_table, int max_pages,
+                                          const int* tok_slot, const int* tok_pos, int tokens, int heads, int kv_heads,
+                                          int head_dim, int window, float scale, int value_dim, float softcap, int keep_first,
+                                          const float* bias, int reach, const float* sink, const void* pool_k,
+                                          const void* pool_v, const int* pool_table, int pool_max_pages, int pool,
+                                          void* stream) {
+  return nnis_attention_rows_terms(q, q_dtype, out, out_dtype, k_pages, v_pages, cache_dtype, block_table, max_pages, tok_slot,
+                                   tok_pos, tokens, heads, kv_heads, head_dim, window, scale, value_dim, softcap, keep_first,
+                                   bias, reach, sink, pool_k, pool_v, pool_table, pool_max_pages, pool, nullptr, stream);
+}
 
 extern "C" int nnis_attention_rows_more(const void* q, int q_dtype, void* out, int out_dtype, const void* k_pages,
                                         const void* v_pages, int cache_dtype, const int* block_table, int max_pages,
@@ -1481,7 +1610,15 @@ int fill_extras(MfmaArgs& a, int keep_first, const float* bias, int reach, const
                "attention: this module is compiled without kept first keys, a bias by distance and a sink");
   NNIS_REQUIRE(keep_first >= 0 && (bias == nullptr || reach >= 0), "attention: bad keep_first %d or reach %d", keep_first, reach);
   a.keep_first = a.window > 0 ? keep_first : 0; a.bias = bias; a.reach = reach; a.sink = sink;
+  a.terms = no_terms();
   a.pool_k = nullptr; a.pool_v = nullptr; a.pool_table = nullptr; a.pool_max_pages = 0; a.pool = 0;
+  return 0;
+}
+
+int fill_matrix_terms(MfmaArgs& a, const NnisHeadTerms* terms) {
+  if (fill_terms(a.terms, terms, a.heads)) return 1;
+  NNIS_REQUIRE(NNIS_DISTANCE_LOG || a.terms.r1 == nullptr, "attention: this module is compiled without scores that fall with the distance");
+  NNIS_REQUIRE(NNIS_HEAD_GATES || a.terms.gate == nullptr, "attention: this module is compiled without gates of the heads");
   return 0;
 }
 
@@ -1541,18 +1678,19 @@ extern "C" int nnis_attention_prefill_max_waves(int heads, int kv_heads, int col
   return waves;
 }
 
-extern "C" int nnis_attention_prefill_bf16_pooled(const void* q, void* out, const void* k_pages, const void* v_pages,
+extern "C" int nnis_attention_prefill_bf16_terms(const void* q, void* out, const void* k_pages, const void* v_pages,
                                                   const int* block_table, int max_pages, const int* tile_seq,
                                                   const int* tile_row0, int tiles, const int* seq_slot, const int* seq_start,
                                                   const int* seq_pos0, int heads, int kv_heads, int head_dim, int window,
                                                   float scale, int waves, int columns, float softcap, int keep_first,
                                                   const float* bias, int reach, const float* sink, const void* pool_k,
                                                   const void* pool_v, const int* pool_table, int pool_max_pages, int pool,
-                                                  void* stream) {
+                                                  const NnisHeadTerms* terms, void* stream) {
   MfmaArgs a;
   if (fill_common(a, q, out, k_pages, v_pages, block_table, max_pages, heads, kv_heads, head_dim, window, scale, softcap)) return 1;
   if (fill_extras(a, keep_first, bias, reach, sink)) return 1;
   if (fill_pooled(a, pool_k, pool_v, pool_table, pool_max_pages, pool)) return 1;
+  if (fill_matrix_terms(a, terms)) return 1;
   if (tiles <= 0) return 0;
   a.tile_seq = tile_seq; a.tile_row0 = tile_row0; a.seq_slot = seq_slot; a.seq_start = seq_start; a.seq_pos0 = seq_pos0;
   const int group = heads / kv_heads;
@@ -1627,17 +1765,18 @@ extern "C" int nnis_attention_decode_max_waves(int heads, int kv_heads) {
 // for columns or keys on lanes and fail where that kernel does not take the sizes.  combine: 0 leaves the
 // runs in `partial` ([tokens, heads, splits, head_dim + 4]: outputs, reference, sum) and writes no output: the
 // projection that follows, or nnis_attention_combine, adds them up.
-extern "C" int nnis_attention_decode_bf16_pooled(const void* q, void* out, const void* k_pages, const void* v_pages,
+extern "C" int nnis_attention_decode_bf16_terms(const void* q, void* out, const void* k_pages, const void* v_pages,
                                                  const int* block_table, int max_pages, const int* tok_slot, const int* tok_pos,
                                                  int tokens, int heads, int kv_heads, int head_dim, int window, float scale,
                                                  int splits, int waves, float* partial, int kind, int combine, int rows_by_token,
                                                  float softcap, int keep_first, const float* bias, int reach, const float* sink,
                                                  const void* pool_k, const void* pool_v, const int* pool_table, int pool_max_pages,
-                                                 int pool, void* stream) {
+                                                 int pool, const NnisHeadTerms* terms, void* stream) {
   MfmaArgs a;
   if (fill_common(a, q, out, k_pages, v_pages, block_table, max_pages, heads, kv_heads, head_dim, window, scale, softcap)) return 1;
   if (fill_extras(a, keep_first, bias, reach, sink)) return 1;
   if (fill_pooled(a, pool_k, pool_v, pool_table, pool_max_pages, pool)) return 1;
+  if (fill_matrix_terms(a, terms)) return 1;
   a.rows_by_token = rows_by_token ? 1 : 0;
   NNIS_REQUIRE(splits >= 1 && splits <= 65535, "attention: bad number of splits %d", splits);
   NNIS_REQUIRE(splits == 1 || partial != nullptr, "attention: splits need scratch memory");
@@ -1674,7 +1813,7 @@ extern "C" int nnis_attention_decode_bf16_pooled(const void* q, void* out, const
       NNIS_LAUNCH_CHECK("attention_decode");
       if (splits > 1 && combine) {
         hipLaunchKernelGGL(attention_combine_kernel, dim3(tokens, heads), dim3(HDV < 64 ? 64 : (HDV > 256 ? 256 : HDV)), 0, s,
-                           partial, (bf16_t*)out, tok_slot, heads, splits);
+                           partial, (bf16_t*)out, tok_slot, heads, splits, a.terms);
         NNIS_LAUNCH_CHECK("attention_combine");
       }
       return 0;
@@ -1687,10 +1826,24 @@ extern "C" int nnis_attention_decode_bf16_pooled(const void* q, void* out, const
   NNIS_LAUNCH_CHECK("attention_decode");
   if (splits > 1 && combine) {
     hipLaunchKernelGGL(attention_combine_kernel, dim3(tokens, heads), dim3(HDV < 64 ? 64 : (HDV > 256 ? 256 : HDV)), 0, s, partial,
-                       (bf16_t*)out, tok_slot, heads, splits);
+                       (bf16_t*)out, tok_slot, heads, splits, a.terms);
     NNIS_LAUNCH_CHECK("attention_combine");
   }
   return 0;
+}
+
+extern "C" int nnis_attention_decode_bf16_pooled(const void* q, void* out, const void* k_pages, const void* v_pages,
+                                                 const int* block_table, int max_pages, const int* tok_slot, const int* tok_pos,
+                                                 int tokens, int heads, int kv_heads, int head_dim, int window, float scale,
+                                                 int splits, int waves, float* partial, int kind, int combine, int rows_by_token,
+                                                 float softcap, int keep_first, const float* bias, int reach, const float* sink,
+                                                 const void* pool_k, const void* pool_v, const int* pool_table, int pool_max_pages,
+                                                 int pool, void* stream) {
+  return nnis_attention_decode_bf16_terms(
+         q, out, k_pages, v_pages, block_table, max_pages, tok_slot, tok_pos, tokens,
+         heads, kv_heads, head_dim, window, scale, splits, waves, partial,
+         kind, combine, rows_by_token, softcap, keep_first, bias, reach, sink,
+         pool_k, pool_v, pool_table, pool_max_pages, pool, nullptr, stream);
 }
 
 extern "C" int nnis_attention_decode_bf16_more(const void* q, void* out, const void* k_pages, const void* v_pages,
@@ -1702,6 +1855,21 @@ extern "C" int nnis_attention_decode_bf16_more(const void* q, void* out, const v
   return nnis_attention_decode_bf16_pooled(q, out, k_pages, v_pages, block_table, max_pages, tok_slot, tok_pos, tokens, heads, kv_heads,
                                            head_dim, window, scale, splits, waves, partial, kind, combine, rows_by_token, softcap,
                                            keep_first, bias, reach, sink, nullptr, nullptr, nullptr, 0, 0, stream);
+}
+
+extern "C" int nnis_attention_prefill_bf16_pooled(const void* q, void* out, const void* k_pages, const void* v_pages,
+                                                  const int* block_table, int max_pages, const int* tile_seq,
+                                                  const int* tile_row0, int tiles, const int* seq_slot, const int* seq_start,
+                                                  const int* seq_pos0, int heads, int kv_heads, int head_dim, int window,
+                                                  float scale, int waves, int columns, float softcap, int keep_first,
+                                                  const float* bias, int reach, const float* sink, const void* pool_k,
+                                                  const void* pool_v, const int* pool_table, int pool_max_pages, int pool,
+                                                  void* stream) {
+  return nnis_attention_prefill_bf16_terms(
+         q, out, k_pages, v_pages, block_table, max_pages, tile_seq, tile_row0, tiles,
+         seq_slot, seq_start, seq_pos0, heads, kv_heads, head_dim, window,
+         scale, waves, columns, softcap, keep_first, bias, reach, sink,
+         pool_k, pool_v, pool_table, pool_max_pages, pool, nullptr, stream);
 }
 
 extern "C" int nnis_attention_prefill_bf16_more(const void* q, void* out, const void* k_pages, const void* v_pages,
@@ -1743,12 +1911,24 @@ extern "C" int nnis_attention_combine(const float* partial, void* out, const int
   NNIS_REQUIRE(partial && out && tok_slot && splits >= 1 && heads > 0, "attention_combine: missing operand");
   if (tokens <= 0) return 0;
   hipLaunchKernelGGL(attention_combine_kernel, dim3(tokens, heads), dim3(HDV < 64 ? 64 : (HDV > 256 ? 256 : HDV)), 0,
-                     (hipStream_t)stream, partial, (bf16_t*)out, tok_slot, heads, splits);
+                     (hipStream_t)stream, partial, (bf16_t*)out, tok_slot, heads, splits, no_terms());
   NNIS_LAUNCH_CHECK("attention_combine");
   return 0;
 }
 #else
 extern "C" int nnis_attention_prefill_tile_rows(int, int, int) { return 0; }
+extern "C" int nnis_attention_prefill_bf16_terms(const void*, void*, const void*, const void*, const int*, int, const int*, const int*,
+                                                 int, const int*, const int*, const int*, int, int, int, int, float, int, int, float, int,
+                                                 const float*, int, const float*, const void*, const void*, const int*, int, int,
+                                                 const NnisHeadTerms*, void*) {
+  return nnis_fail("attention: the matrix-core kernels need keys and values in steps of 16 channels; this module has %d and %d", NNIS_HEAD_DIM, NNIS_VALUE_DIM);
+}
+extern "C" int nnis_attention_decode_bf16_terms(const void*, void*, const void*, const void*, const int*, int, const int*, const int*,
+                                                int, int, int, int, int, float, int, int, float*, int, int, int, float, int, const float*,
+                                                int, const float*, const void*, const void*, const int*, int, int,
+                                                const NnisHeadTerms*, void*) {
+  return nnis_fail("attention: the matrix-core kernels need keys and values in steps of 16 channels; this module has %d and %d", NNIS_HEAD_DIM, NNIS_VALUE_DIM);
+}
 extern "C" int nnis_attention_prefill_max_waves(int, int, int) { return 1; }
 extern "C" int nnis_attention_prefill_bf16(const void*, void*, const void*, const void*, const int*, int, const int*, const int*,
                                            int, const int*, const int*, const int*, int, int, int, int, float, int, int, float, void*) {

@@ -77,6 +77,70 @@ extern "C" int nnis_embed_packed(const int* ids, const void* packed, float* out,
   return 0;
 }
 
+// The row copy with an RMS norm behind it: out[t, :] = e / sqrt(mean(e^2) + eps) * weight, e = table[ids[t], :] * scale.
+// A block a token; the row is read twice, the second time from the caches.  Eight channels a thread and access where the
+// table is packed (its pieces of a row), one otherwise.
+__global__ __launch_bounds__(256) void embed_norm_kernel(const int* __restrict__ ids, const void* __restrict__ table, int table_dtype,
+                                                         int packed, const void* __restrict__ weight, int weight_dtype, float eps,
+                                                         float* __restrict__ out, int width, int vocab, float scale) {
+  __shared__ float scratch[16];
+  const int token = blockIdx.x;
+  const int id = ids[token];
+  float* dst = out + (size_t)token * width;
+  if (id < 0 || id >= vocab) {  // (the whole block: a padding row)
+    for (int c = threadIdx.x; c < width; c += blockDim.x) dst[c] = 0.0f;
+    return;
+  }
+  if (packed) {
+    const bf16_t* strip = (const bf16_t*)table + (size_t)(id >> 4) * nnis_packed_strip_elems(width) + (size_t)(id & 15) * 8;
+    auto piece = [&](int k) {
+      return *(const uint4*)(strip + (size_t)(k / 64) * kPackedChunkElems + (size_t)((k % 16) / 8) * kPackedHalfElems + (size_t)((k % 64) / 16) * 128);
+    };
+    float ss = 0.0f;
+    for (int k = threadIdx.x * 8; k < width; k += blockDim.x * 8) {
+      const uint4 p = piece(k);
+      const uint32_t words[4] = {p.x, p.y, p.z, p.w};
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const float lo = __uint_as_float(words[i] << 16) * scale, hi = __uint_as_float(words[i] & 0xffff0000u) * scale;
+        ss = fmaf(lo, lo, fmaf(hi, hi, ss));
+      }
+    }
+    const float inv = scale / sqrtf(block_sum(ss, scratch) / (float)width + eps);
+    for (int k = threadIdx.x * 8; k < width; k += blockDim.x * 8) {
+      const uint4 p = piece(k);
+      const uint32_t words[4] = {p.x, p.y, p.z, p.w};
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        dst[k + 2 * i] = __uint_as_float(words[i] << 16) * inv * load_as_f32(weight, weight_dtype, k + 2 * i);
+        dst[k + 2 * i + 1] = __uint_as_float(words[i] & 0xffff0000u) * inv * load_as_f32(weight, weight_dtype, k + 2 * i + 1);
+      }
+    }
+    return;
+  }
+  const size_t base = (size_t)id * width;
+  float ss = 0.0f;
+  for (int c = threadIdx.x; c < width; c += blockDim.x) {
+    const float v = load_as_f32(table, table_dtype, base + c) * scale;
+    ss = fmaf(v, v, ss);
+  }
+  const float inv = scale / sqrtf(block_sum(ss, scratch) / (float)width + eps);
+  for (int c = threadIdx.x; c < width; c += blockDim.x)
+    dst[c] = load_as_f32(table, table_dtype, base + c) * inv * load_as_f32(weight, weight_dtype, c);
+}
+
+extern "C" int nnis_embed_norm(const int* ids, const void* table, int table_dtype, int packed, const void* weight, int weight_dtype, float eps,
+                               float* out, int tokens, int width, int vocab, float scale, void* stream) {
+  NNIS_REQUIRE(nnis_dtype_ok(table_dtype) && nnis_dtype_ok(weight_dtype) && weight, "embed_norm: unknown types or no weight");
+  NNIS_REQUIRE(tokens >= 0 && width > 0 && vocab > 0, "embed_norm: bad sizes tokens=%d width=%d vocab=%d", tokens, width, vocab);
+  NNIS_REQUIRE(!packed || (width % 8 == 0 && table_dtype == NNIS_BF16), "embed_norm: a packed table is bfloat16 with a width that is a multiple of 8");
+  if (tokens == 0) return 0;
+  hipLaunchKernelGGL(embed_norm_kernel, dim3(tokens), dim3(256), 0, (hipStream_t)stream, ids, table, table_dtype, packed ? 1 : 0, weight,
+                     weight_dtype, eps, out, width, vocab, scale);
+  NNIS_LAUNCH_CHECK("embed_norm");
+  return 0;
+}
+
 // -----------------------------------------------------------------------------
 // The step's tables: what every layer's kernels would otherwise look up again through each token's slot and
 // position, gathered once per step by token: its rows of the rotation tables, the cache page that takes its

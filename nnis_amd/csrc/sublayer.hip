@@ -6,7 +6,7 @@
 //   poly_norm          a N(z) + b N(z^2) + c N(z^3) + e, N a division by the root mean square of a row
 //   router_logits      a router's logits as 32-bit dot products
 //   route_top          softmax of router logits, the `top` largest of score + correction, dense weights out
-//   routed_act         weight[row, expert] * relu(z)^2 on the experts' fused up projection
+//   routed_act         weight[row, expert] * activation on the experts' fused up (and gate) projection
 //   rows_axpy          y[row] += c[row] * h[row]
 //   sigmoid_gate       o *= sigmoid(g)
 //   head_norm_write    per-head RMS norm of queries and keys, rotation (neighbouring channels or halves), queries out,
@@ -336,15 +336,25 @@ constexpr int kRouteMost = 16;  // outputs a lane holds: n <= 64 * kRouteMost
 // one row by one wave; `logits`: the row's n logits (global memory or LDS)
 // group_count > 1: the outputs form that many equal groups of neighbours; a group's mark is its largest corrected
 // score, and only outputs of the group_keep groups with the largest marks (the lower group on a tie) can be chosen.
-__device__ __forceinline__ void route_row(const float* logits, const float* __restrict__ correction, int row, int n, int experts, int top,
-                                          float* __restrict__ gates, float* __restrict__ keep, int lane, int group_count = 1,
-                                          int group_keep = 1) {
+// bias: joins the logits before anything else (null: none).  chosen_softmax: outputs are chosen by logit (+ correction)
+// and the weights are the softmax over the chosen logits alone.
+struct RouteRule {
+  const float* bias;
+  const float* correction;
+  int chosen_softmax, group_count, group_keep;
+};
+
+__device__ __forceinline__ void route_row(const float* logits, const RouteRule& rule, int row, int n, int experts, int top,
+                                          float* __restrict__ gates, float* __restrict__ keep, int lane) {
+  const float* __restrict__ correction = rule.correction;
+  const int group_count = rule.group_count, group_keep = rule.group_keep;
   float s[kRouteMost], choice[kRouteMost];
   float top_logit = -INFINITY;
 #pragma unroll
   for (int i = 0; i < kRouteMost; ++i) {
     const int e = i * kWave + lane;
-    s[i] = e < n ? logits[e] : -INFINITY;
+    s[i] = e < n ? logits[e] + (rule.bias ? rule.bias[e] : 0.0f) : -INFINITY;
+    choice[i] = s[i];  // (stays where outputs are chosen by logit)
     top_logit = fmaxf(top_logit, s[i]);
   }
   top_logit = wave_max(top_logit);
@@ -354,13 +364,13 @@ __device__ __forceinline__ void route_row(const float* logits, const float* __re
     s[i] = (i * kWave + lane) < n ? expf(s[i] - top_logit) : 0.0f;
     sum += s[i];
   }
-  const float inv = 1.0f / wave_sum(sum);
+  const float inv = rule.chosen_softmax ? 1.0f : 1.0f / wave_sum(sum);
   unsigned chosen = 0;
 #pragma unroll
   for (int i = 0; i < kRouteMost; ++i) {
     const int e = i * kWave + lane;
     s[i] *= inv;
-    choice[i] = e < n ? s[i] + (correction ? correction[e] : 0.0f) : -INFINITY;
+    choice[i] = e < n ? (rule.chosen_softmax ? choice[i] : s[i]) + (correction ? correction[e] : 0.0f) : -INFINITY;
   }
   if (group_count > 1 && group_keep < group_count) {
     // lane g holds group g's mark (up to 64 groups); the kept groups are found one at a time
@@ -399,6 +409,7 @@ __device__ __forceinline__ void route_row(const float* logits, const float* __re
     }
   }
   float kept = 0.0f;
+  float weight = 0.0f;  // of this lane's chosen outputs together
   for (int round = 0; round < top; ++round) {
     float best = -INFINITY;
     int best_e = 0x7fffffff;
@@ -425,24 +436,27 @@ __device__ __forceinline__ void route_row(const float* logits, const float* __re
       chosen |= 1u << i;
 #pragma unroll
       for (int k = 0; k < kRouteMost; ++k)
-        if (k == i && best_e >= experts) kept += s[k];
+        if (k == i) {
+          weight += s[k];
+          if (best_e >= experts) kept += s[k];
+        }
     }
   }
+  const float share = rule.chosen_softmax ? 1.0f / wave_sum(weight) : 1.0f;
 #pragma unroll
   for (int i = 0; i < kRouteMost; ++i) {
     const int e = i * kWave + lane;
-    if (e < experts) gates[(size_t)row * experts + e] = (chosen >> i & 1u) ? s[i] : 0.0f;
+    if (e < experts) gates[(size_t)row * experts + e] = (chosen >> i & 1u) ? s[i] * share : 0.0f;
   }
-  kept = wave_sum(kept);
+  kept = wave_sum(kept) * share;
   if (lane == 0) keep[row] = kept;
 }
 
-__global__ __launch_bounds__(256) void route_top_kernel(const float* __restrict__ logits, const float* __restrict__ correction, int rows,
-                                                        int n, int experts, int top, float* __restrict__ gates,
-                                                        float* __restrict__ keep, int group_count, int group_keep) {
+__global__ __launch_bounds__(256) void route_top_kernel(const float* __restrict__ logits, RouteRule rule, int rows, int n, int experts,
+                                                        int top, float* __restrict__ gates, float* __restrict__ keep) {
   const int row = blockIdx.x * 4 + threadIdx.x / kWave;
   if (row >= rows) return;
-  route_row(logits + (size_t)row * n, correction, row, n, experts, top, gates, keep, threadIdx.x % kWave, group_count, group_keep);
+  route_row(logits + (size_t)row * n, rule, row, n, experts, top, gates, keep, threadIdx.x % kWave);
 }
 
 // the dot products of R rows with every output's weights, into `out` [R][n] (LDS or global memory with a row stride
@@ -485,9 +499,8 @@ __device__ __forceinline__ void router_dots(const float* xs, const float* __rest
 // LDS, then wave r routes row r.
 template <int R>
 __global__ __launch_bounds__(R == 1 ? 1024 : 256) void route_kernel(const void* __restrict__ x, int x_dtype, const float* __restrict__ w,
-                                                    const float* __restrict__ correction, int rows, int n, int width, int experts,
-                                                    int top, float* __restrict__ gates, float* __restrict__ keep, int group_count,
-                                                    int group_keep) {
+                                                    RouteRule rule, int rows, int n, int width, int experts, int top,
+                                                    float* __restrict__ gates, float* __restrict__ keep) {
   extern __shared__ __attribute__((aligned(16))) float lds[];  // [R][width] rows, then [R][n] logits
   float* xs = lds;
   float* lg = lds + (size_t)R * width;
@@ -501,7 +514,7 @@ __global__ __launch_bounds__(R == 1 ? 1024 : 256) void route_kernel(const void* 
   __syncthreads();
   const int wave = threadIdx.x / kWave;
   if (wave < R && row0 + wave < rows)
-    route_row(lg + wave * n, correction, row0 + wave, n, experts, top, gates, keep, threadIdx.x % kWave, group_count, group_keep);
+    route_row(lg + wave * n, rule, row0 + wave, n, experts, top, gates, keep, threadIdx.x % kWave);
 }
 
 // the logits alone, to global memory [rows, n]
@@ -535,79 +548,78 @@ __global__ __launch_bounds__(256) void router_logits_kernel(const void* __restri
   }
 }
 
-// out[row, e * ff + c] = gates[row, e] * relu(z[row, e * ff + c])^2
-__global__ void routed_act_kernel(const void* __restrict__ z, int z_dtype, const float* __restrict__ gates, void* __restrict__ out,
-                                  int out_dtype, int experts, int ff, size_t total) {
-  const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
-  if (i >= total) return;
-  const size_t per_row = (size_t)experts * ff;
-  const size_t row = i / per_row;
-  const int e = (int)((i % per_row) / ff);
-  const float g = gates[row * experts + e];
-  const float v = fmaxf(load_as_f32(z, z_dtype, i), 0.0f);
-  store_from_f32(out, out_dtype, i, g == 0.0f ? 0.0f : g * v * v);
+// What the experts do between their projections, weighed with the scores: out[row, e * ff + c] = gates[row, e] *
+//   form 0: relu(z[row, e * ff + c])^2
+//   form 1: silu(a) * u            a = z[row, e * 2 ff + c], u = z[row, e * 2 ff + ff + c] (an expert's gate columns,
+//   form 2: clamped_swiglu(a, u)   then its up columns)
+// Without gates every weight is one.
+struct RoutedActArgs {
+  const void* z;
+  int z_dtype;
+  size_t z_stride;  // elements from a row to the next
+  const float* gates;
+  void* out;
+  int out_dtype;
+  size_t out_stride;
+  int experts, ff;
+  float limit;
+};
+
+// a held at most at `limit`, u within plus or minus it (0: not held): a sigmoid(1.702 a) (u + 1)
+__device__ __forceinline__ float clamped_swiglu(float a, float u, float limit) {
+  if (limit > 0.0f) {
+    a = fminf(a, limit);
+    u = fminf(fmaxf(u, -limit), limit);
+  }
+  return a * sigmoid_f(1.702f * a) * (u + 1.0f);
 }
 
-// The gated form: z [rows, experts * 2 * ff], an expert's gate columns then its up columns;
-// out[row, e * ff + c] = gates[row, e] * silu(z[row, e * 2 ff + c]) * z[row, e * 2 ff + ff + c]
-__global__ void routed_gated_kernel(const void* __restrict__ z, int z_dtype, const float* __restrict__ gates, void* __restrict__ out,
-                                    int out_dtype, int experts, int ff, size_t total) {
+template <int FORM>
+__device__ __forceinline__ float routed_value(float a, float u, float limit) {
+  if (FORM == 0) {
+    const float v = fmaxf(a, 0.0f);
+    return v * v;
+  }
+  return FORM == 1 ? a * sigmoid_f(a) * u : clamped_swiglu(a, u, limit);
+}
+
+template <int FORM>
+__global__ void routed_act_kernel(RoutedActArgs a, size_t total) {
   const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= total) return;
-  const size_t per_row = (size_t)experts * ff;
+  const size_t per_row = (size_t)a.experts * a.ff;
   const size_t row = i / per_row;
-  const int e = (int)((i % per_row) / ff), c = (int)(i % ff);
-  const float g = gates[row * experts + e];
+  const int at = (int)(i % per_row), e = at / a.ff, c = at % a.ff;
+  const float g = a.gates ? a.gates[row * a.experts + e] : 1.0f;
   float v = 0.0f;
   if (g != 0.0f) {
-    const size_t at = (row * experts + e) * 2 * (size_t)ff + c;
-    const float a = load_as_f32(z, z_dtype, at), u = load_as_f32(z, z_dtype, at + ff);
-    v = g * (a * sigmoid_f(a) * u);
+    const size_t from = row * a.z_stride + (FORM == 0 ? (size_t)at : (size_t)e * 2 * a.ff + c);
+    const float u = FORM == 0 ? 0.0f : load_as_f32(a.z, a.z_dtype, from + a.ff);
+    v = g * routed_value<FORM>(load_as_f32(a.z, a.z_dtype, from), u, a.limit);
   }
-  store_from_f32(out, out_dtype, i, v);
+  store_from_f32(a.out, a.out_dtype, row * a.out_stride + at, v);
 }
 
-// the gated form, eight bfloat16 values a thread (ff a multiple of 8); the gating itself rounds to bfloat16 before the score weighs it
-__global__ void routed_gated_bf16x8_kernel(const bf16_t* __restrict__ z, const float* __restrict__ gates, bf16_t* __restrict__ out,
-                                           int experts, int ff8, size_t total8) {
+// the same, eight bfloat16 values a thread (ff and the strides multiples of 8)
+template <int FORM>
+__global__ void routed_act_bf16x8_kernel(RoutedActArgs a, size_t total8) {
   const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= total8) return;
-  const size_t per_row = (size_t)experts * ff8;
+  const int ff8 = a.ff / 8;
+  const size_t per_row = (size_t)a.experts * ff8;
   const size_t row = i / per_row;
-  const int e = (int)((i % per_row) / ff8), c8 = (int)(i % ff8);
-  const float g = gates[row * experts + e];
+  const int at = (int)(i % per_row), e = at / ff8, c8 = at % ff8;
+  const float g = a.gates ? a.gates[row * a.experts + e] : 1.0f;
   typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 bf16x8_t;
   bf16x8_t o = {};
   if (g != 0.0f) {
-    const bf16_t* at = z + ((row * experts + e) * 2 * (size_t)ff8 + c8) * 8;
-    const bf16x8_t a = *(const bf16x8_t*)at, u = *(const bf16x8_t*)(at + (size_t)ff8 * 8);
+    const bf16_t* from = (const bf16_t*)a.z + row * a.z_stride + (FORM == 0 ? (size_t)at : (size_t)e * 2 * ff8 + c8) * 8;
+    const bf16x8_t av = *(const bf16x8_t*)from;
+    const bf16x8_t uv = FORM == 0 ? av : *(const bf16x8_t*)(from + a.ff);
 #pragma unroll
-    for (int k = 0; k < 8; ++k) {
-      const float av = (float)a[k];
-      o[k] = (__bf16)(g * (av * sigmoid_f(av) * (float)u[k]));
-    }
+    for (int k = 0; k < 8; ++k) o[k] = (__bf16)(g * routed_value<FORM>((float)av[k], (float)uv[k], a.limit));
   }
-  *(bf16x8_t*)(out + i * 8) = o;
-}
-
-// the same, eight bfloat16 values a thread (ff a multiple of 8)
-__global__ void routed_act_bf16x8_kernel(const bf16_t* __restrict__ z, const float* __restrict__ gates, bf16_t* __restrict__ out,
-                                         int experts, int ff8, size_t total8) {
-  const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
-  if (i >= total8) return;
-  const size_t per_row = (size_t)experts * ff8;
-  const size_t row = i / per_row;
-  const int e = (int)((i % per_row) / ff8);
-  const float g = gates[row * experts + e];
-  typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 bf16x8_t;
-  bf16x8_t v = g == 0.0f ? bf16x8_t{} : *(const bf16x8_t*)(z + i * 8);
-  bf16x8_t o;
-#pragma unroll
-  for (int k = 0; k < 8; ++k) {
-    const float a = fmaxf((float)v[k], 0.0f);
-    o[k] = (__bf16)(g == 0.0f ? 0.0f : g * a * a);
-  }
-  *(bf16x8_t*)(out + i * 8) = o;
+  *(bf16x8_t*)((bf16_t*)a.out + row * a.out_stride + (size_t)at * 8) = o;
 }
 
 // y[row, c] += keep[row] * h[row, c]
@@ -659,6 +671,8 @@ struct HeadWriteArgs {
   const int* block_table;
   int max_pages;
   int heads, kv_heads, head_dim, value_dim;
+  int unit;               // 1: the norm without a weight
+  const float* q_factor;  // [heads] or null: a query head's own factor behind the norm
 };
 
 __global__ __launch_bounds__(64) void head_norm_write_kernel(HeadWriteArgs a) {
@@ -684,6 +698,10 @@ __global__ __launch_bounds__(64) void head_norm_write_kernel(HeadWriteArgs a) {
   if (weight) {
     const float inv = 1.0f / sqrtf(ss / (float)hd + a.eps);
     for (int d = lane; d < hd; d += kWave) row[d] = row[d] * inv * load_as_f32(weight, a.w_dtype, d);
+    __syncthreads();
+  } else if (a.unit || (a.q_factor && !is_key)) {
+    const float inv = (a.unit ? 1.0f / sqrtf(ss / (float)hd + a.eps) : 1.0f) * (a.q_factor && !is_key ? a.q_factor[head] : 1.0f);
+    for (int d = lane; d < hd; d += kWave) row[d] = row[d] * inv;
     __syncthreads();
   }
   const bool rotate = a.cos_table != nullptr && pos < a.table_positions;
@@ -950,8 +968,8 @@ extern "C" int nnis_router_logits(const void* x, int x_dtype, const float* w, fl
   return 0;
 }
 
-extern "C" int nnis_route(const void* x, int x_dtype, const float* w, const float* correction, int rows, int n, int width, int experts, int top,
-                          float* gates, float* keep, int group_count, int group_keep, void* stream) {
+extern "C" int nnis_route(const void* x, int x_dtype, const float* w, const float* bias, const float* correction, int rows, int n, int width,
+                          int experts, int top, int chosen_softmax, float* gates, float* keep, int group_count, int group_keep, void* stream) {
   NNIS_REQUIRE(x && w && gates && keep && n > 0 && width > 0, "route: missing operand");
   NNIS_REQUIRE(group_count >= 1 && group_count <= kWave && n % group_count == 0 && group_keep >= 1 && group_keep <= group_count,
                "route: %d outputs in %d groups (up to %d, equal ones) of which %d are kept", n, group_count, kWave, group_keep);
@@ -965,64 +983,58 @@ extern "C" int nnis_route(const void* x, int x_dtype, const float* w, const floa
   const size_t lds = (size_t)together * (width + n) * sizeof(float);
   const dim3 grid((rows + together - 1) / together);
   hipStream_t s = (hipStream_t)stream;
+  const RouteRule rule = {bias, correction, chosen_softmax ? 1 : 0, group_count, group_keep};
   if (together == 4) {
-    hipLaunchKernelGGL((route_kernel<4>), grid, dim3(256), lds, s, x, x_dtype, w, correction, rows, n, width, experts, top, gates, keep,
-                       group_count, group_keep);
+    hipLaunchKernelGGL((route_kernel<4>), grid, dim3(256), lds, s, x, x_dtype, w, rule, rows, n, width, experts, top, gates, keep);
   } else if (together == 2) {
-    hipLaunchKernelGGL((route_kernel<2>), grid, dim3(256), lds, s, x, x_dtype, w, correction, rows, n, width, experts, top, gates, keep,
-                       group_count, group_keep);
+    hipLaunchKernelGGL((route_kernel<2>), grid, dim3(256), lds, s, x, x_dtype, w, rule, rows, n, width, experts, top, gates, keep);
   } else {
     // a row a block: a wave an output where the outputs are many, so that every weight row is asked for at once
     const int threads = n > 8 ? 1024 : (n > 4 ? 512 : 256);
-    hipLaunchKernelGGL((route_kernel<1>), grid, dim3(threads), lds, s, x, x_dtype, w, correction, rows, n, width, experts, top, gates, keep,
-                       group_count, group_keep);
+    hipLaunchKernelGGL((route_kernel<1>), grid, dim3(threads), lds, s, x, x_dtype, w, rule, rows, n, width, experts, top, gates, keep);
   }
   NNIS_LAUNCH_CHECK("route");
   return 0;
 }
 
-extern "C" int nnis_route_top(const float* logits, const float* correction, int rows, int n, int experts, int top, float* gates,
-                              float* keep, int group_count, int group_keep, void* stream) {
+extern "C" int nnis_route_top(const float* logits, const float* bias, const float* correction, int rows, int n, int experts, int top,
+                              int chosen_softmax, float* gates, float* keep, int group_count, int group_keep, void* stream) {
   NNIS_REQUIRE(logits && gates && keep, "route_top: missing operand");
   NNIS_REQUIRE(group_count >= 1 && group_count <= kWave && n % group_count == 0 && group_keep >= 1 && group_keep <= group_count,
                "route_top: %d outputs in %d groups (up to %d, equal ones) of which %d are kept", n, group_count, kWave, group_keep);
   NNIS_REQUIRE(n > 0 && n <= kWave * kRouteMost, "route_top: 1 to %d router outputs, got %d", kWave * kRouteMost, n);
   NNIS_REQUIRE(experts >= 0 && experts <= n && top > 0 && top <= n, "route_top: %d experts and the %d largest of %d outputs", experts, top, n);
   if (rows <= 0) return 0;
-  hipLaunchKernelGGL(route_top_kernel, dim3((rows + 3) / 4), dim3(256), 0, (hipStream_t)stream, logits, correction, rows, n, experts, top,
-                     gates, keep, group_count, group_keep);
+  const RouteRule rule = {bias, correction, chosen_softmax ? 1 : 0, group_count, group_keep};
+  hipLaunchKernelGGL(route_top_kernel, dim3((rows + 3) / 4), dim3(256), 0, (hipStream_t)stream, logits, rule, rows, n, experts, top, gates,
+                     keep);
   NNIS_LAUNCH_CHECK("route_top");
   return 0;
 }
 
-// form 0: z [rows, experts * ff], out = score * relu(z)^2; form 1: z [rows, experts * 2 * ff] (gate columns, then up
-// columns, expert by expert), out = score * silu(gate) * up
-extern "C" int nnis_routed_act(const void* z, int z_dtype, const float* gates, void* out, int out_dtype, int rows, int experts, int ff,
-                               int form, void* stream) {
-  NNIS_REQUIRE(z && gates && out && experts > 0 && ff > 0, "routed_act: missing operand");
+// see RoutedActArgs; z_stride, out_stride: elements from a row to the next
+extern "C" int nnis_routed_act(const void* z, int z_dtype, int z_stride, const float* gates, void* out, int out_dtype, int out_stride, int rows,
+                               int experts, int ff, int form, float limit, void* stream) {
+  NNIS_REQUIRE(z && out && experts > 0 && ff > 0, "routed_act: missing operand");
   NNIS_REQUIRE(nnis_dtype_ok(z_dtype) && nnis_dtype_ok(out_dtype), "routed_act: unknown dtype");
-  NNIS_REQUIRE(form == 0 || form == 1, "routed_act: unknown form %d", form);
+  NNIS_REQUIRE(form >= 0 && form <= 2, "routed_act: unknown form %d", form);
+  NNIS_REQUIRE(z_stride >= experts * ff * (form == 0 ? 1 : 2) && out_stride >= experts * ff, "routed_act: rows of %d and %d for %d experts of %d",
+               z_stride, out_stride, experts, ff);
   if (rows <= 0) return 0;
   const size_t total = (size_t)rows * experts * ff;
-  if (form == 1) {
-    if (z_dtype == NNIS_BF16 && out_dtype == NNIS_BF16 && ff % 8 == 0 && (uintptr_t)z % 16 == 0 && (uintptr_t)out % 16 == 0) {
-      hipLaunchKernelGGL(routed_gated_bf16x8_kernel, dim3(blocks_for(total / 8, 256)), dim3(256), 0, (hipStream_t)stream, (const bf16_t*)z,
-                         gates, (bf16_t*)out, experts, ff / 8, total / 8);
-    } else {
-      hipLaunchKernelGGL(routed_gated_kernel, dim3(blocks_for(total, 256)), dim3(256), 0, (hipStream_t)stream, z, z_dtype, gates, out,
-                         out_dtype, experts, ff, total);
-    }
-    NNIS_LAUNCH_CHECK("routed_act");
-    return 0;
-  }
-  if (z_dtype == NNIS_BF16 && out_dtype == NNIS_BF16 && ff % 8 == 0 && (uintptr_t)z % 16 == 0 && (uintptr_t)out % 16 == 0) {
-    hipLaunchKernelGGL(routed_act_bf16x8_kernel, dim3(blocks_for(total / 8, 256)), dim3(256), 0, (hipStream_t)stream, (const bf16_t*)z, gates,
-                       (bf16_t*)out, experts, ff / 8, total / 8);
-    NNIS_LAUNCH_CHECK("routed_act");
-    return 0;
-  }
-  hipLaunchKernelGGL(routed_act_kernel, dim3(blocks_for(total, 256)), dim3(256), 0, (hipStream_t)stream, z, z_dtype, gates, out, out_dtype,
-                     experts, ff, total);
+  const RoutedActArgs a = {z, z_dtype, (size_t)z_stride, gates, out, out_dtype, (size_t)out_stride, experts, ff, limit};
+  const bool eights = z_dtype == NNIS_BF16 && out_dtype == NNIS_BF16 && ff % 8 == 0 && z_stride % 8 == 0 && out_stride % 8 == 0 &&
+                      (uintptr_t)z % 16 == 0 && (uintptr_t)out % 16 == 0;
+  hipStream_t s = (hipStream_t)stream;
+#define NNIS_ROUTED_ACT(FORM_)                                                                                                    \
+  do {                                                                                                                            \
+    if (eights) hipLaunchKernelGGL(routed_act_bf16x8_kernel<FORM_>, dim3(blocks_for(total / 8, 256)), dim3(256), 0, s, a, total / 8); \
+    else hipLaunchKernelGGL(routed_act_kernel<FORM_>, dim3(blocks_for(total, 256)), dim3(256), 0, s, a, total);                    \
+  } while (0)
+  if (form == 0) NNIS_ROUTED_ACT(0);
+  else if (form == 1) NNIS_ROUTED_ACT(1);
+  else NNIS_ROUTED_ACT(2);
+#undef NNIS_ROUTED_ACT
   NNIS_LAUNCH_CHECK("routed_act");
   return 0;
 }
@@ -1053,7 +1065,8 @@ extern "C" int nnis_head_norm_write(const void* rows, int dtype, int stride, int
                                     const void* q_weight, const void* k_weight, int w_dtype, float eps, const float* cos_table,
                                     const float* sin_table, int table_positions, int rot_dim, int neighbours, const int* tok_slot,
                                     const int* tok_pos, void* k_pages, void* v_pages, int cache_dtype, const int* block_table,
-                                    int max_pages, int tokens, int heads, int kv_heads, int head_dim, int value_dim, void* stream) {
+                                    int max_pages, int tokens, int heads, int kv_heads, int head_dim, int value_dim, int unit,
+                                    const float* q_factor, void* stream) {
   NNIS_REQUIRE(rows && q_out && tok_slot && tok_pos, "head_norm_write: missing operand");
   NNIS_REQUIRE(nnis_dtype_ok(dtype) && nnis_dtype_ok(q_dtype), "head_norm_write: unknown dtype");
   NNIS_REQUIRE(heads > 0 && kv_heads >= 0 && head_dim > 0 && head_dim <= kHeadMost, "head_norm_write: heads of 1 to %d channels, got %d",
@@ -1062,6 +1075,7 @@ extern "C" int nnis_head_norm_write(const void* rows, int dtype, int stride, int
                rot_dim, head_dim);
   NNIS_REQUIRE((cos_table == nullptr) == (sin_table == nullptr), "head_norm_write: cos and sin tables must come together");
   NNIS_REQUIRE((q_weight == nullptr && k_weight == nullptr) || nnis_dtype_ok(w_dtype), "head_norm_write: unknown weight dtype");
+  NNIS_REQUIRE((q_weight == nullptr && k_weight == nullptr) || (!unit && q_factor == nullptr), "head_norm_write: a norm with a weight has no factors beside it");
   if (kv_heads > 0) {
     NNIS_REQUIRE(k_col >= 0 && v_col >= 0 && k_pages && v_pages && block_table && max_pages > 0 && nnis_dtype_ok(cache_dtype) && value_dim > 0,
                  "head_norm_write: keys without pages to go to");
@@ -1074,6 +1088,7 @@ extern "C" int nnis_head_norm_write(const void* rows, int dtype, int stride, int
   a.neighbours = neighbours; a.tok_slot = tok_slot; a.tok_pos = tok_pos; a.k_pages = k_pages; a.v_pages = v_pages;
   a.cache_dtype = cache_dtype; a.block_table = block_table; a.max_pages = max_pages;
   a.heads = heads; a.kv_heads = kv_heads; a.head_dim = head_dim; a.value_dim = value_dim;
+  a.unit = unit ? 1 : 0; a.q_factor = q_factor;
   hipLaunchKernelGGL(head_norm_write_kernel, dim3(tokens, heads + kv_heads), dim3(64), 0, (hipStream_t)stream, a);
   NNIS_LAUNCH_CHECK("head_norm_write");
   return 0;

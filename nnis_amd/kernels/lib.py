@@ -113,7 +113,8 @@ def register_module_family(prefix: str, recipe: Callable[[str], ModuleRecipe], r
 
 def _attention_recipe(rest: str) -> ModuleRecipe:
     """``attn_hd<N>``: keys and values of N channels; ``attn_hd<N>v<M>``: values of M; a ``c`` behind either: with a
-    cap of the scores compiled in; an ``x`` at the very end: with the extras of the scores (first keys kept visible
+    cap of the scores compiled in; an ``l`` behind that: with scores that fall with the logarithm of the distance; a
+    ``g``: with gated heads; an ``x`` at the very end: with the extras of the scores (first keys kept visible
     beside a window, a bias by distance, a sink in the denominator) compiled into the matrix-core kernels; ``xp``:
     with pooled blocks beside a window as well."""
     name = rest
@@ -122,6 +123,12 @@ def _attention_recipe(rest: str) -> ModuleRecipe:
         rest = rest[:-1]
     extras = rest.endswith("x")
     if extras:
+        rest = rest[:-1]
+    gated = rest.endswith("g")
+    if gated:
+        rest = rest[:-1]
+    fading = rest.endswith("l")
+    if fading:
         rest = rest[:-1]
     capped = rest.endswith("c")
     try:
@@ -135,6 +142,10 @@ def _attention_recipe(rest: str) -> ModuleRecipe:
         defines.append(("NNIS_VALUE_DIM", str(sizes[1])))
     if capped:
         defines.append(("NNIS_SCORE_CAP", "1"))
+    if fading:
+        defines.append(("NNIS_DISTANCE_LOG", "1"))
+    if gated:
+        defines.append(("NNIS_HEAD_GATES", "1"))
     if extras:
         defines.append(("NNIS_SCORE_EXTRAS", "1"))
     if pooled:

@@ -26,6 +26,7 @@ _I64 = ctypes.c_longlong
 _CORE_SIGNATURES = {
     "nnis_embed": [_VOID, _VOID, _INT, _VOID, _INT, _INT, _INT, _FLT, _VOID],
     "nnis_embed_packed": [_VOID, _VOID, _VOID, _INT, _INT, _INT, _FLT, _VOID],
+    "nnis_embed_norm": [_VOID, _VOID, _INT, _INT, _VOID, _INT, _FLT, _VOID, _INT, _INT, _INT, _FLT, _VOID],
     "nnis_step_tables": [_VOID, _VOID, _INT, _VOID, _VOID, _INT, _INT, _VOID, _INT, _VOID, _VOID, _VOID, _VOID, _VOID],
     "nnis_rmsnorm": [_VOID, _INT, _VOID, _INT, _VOID, _INT, _VOID, _INT, _VOID, _INT, _INT, _FLT, _VOID],
     "nnis_rope_kv_write": [_VOID, _INT, _VOID, _INT, _VOID, _VOID, _INT, _INT, _VOID, _VOID, _VOID, _VOID, _INT,
@@ -80,6 +81,14 @@ _ATTN_SIGNATURES = {
     "nnis_attention_decode_bf16_pooled": [_VOID, _VOID, _VOID, _VOID, _VOID, _INT, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _FLT,
                                           _INT, _INT, _VOID, _INT, _INT, _INT, _FLT, _INT, _VOID, _INT, _VOID,
                                           _VOID, _VOID, _VOID, _INT, _INT, _VOID],
+    "nnis_attention_rows_terms": [_VOID, _INT, _VOID, _INT, _VOID, _VOID, _INT, _VOID, _INT, _VOID, _VOID, _INT, _INT, _INT,
+                                  _INT, _INT, _FLT, _INT, _FLT, _INT, _VOID, _INT, _VOID, _VOID, _VOID, _VOID, _INT, _INT, _VOID, _VOID],
+    "nnis_attention_prefill_bf16_terms": [_VOID, _VOID, _VOID, _VOID, _VOID, _INT, _VOID, _VOID, _INT, _VOID, _VOID, _VOID, _INT,
+                                          _INT, _INT, _INT, _FLT, _INT, _INT, _FLT, _INT, _VOID, _INT, _VOID,
+                                          _VOID, _VOID, _VOID, _INT, _INT, _VOID, _VOID],
+    "nnis_attention_decode_bf16_terms": [_VOID, _VOID, _VOID, _VOID, _VOID, _INT, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _FLT,
+                                         _INT, _INT, _VOID, _INT, _INT, _INT, _FLT, _INT, _VOID, _INT, _VOID,
+                                         _VOID, _VOID, _VOID, _INT, _INT, _VOID, _VOID],
     "nnis_attention_prefill_tile_rows": [_INT, _INT, _INT],
     "nnis_attention_prefill_bf16": [_VOID, _VOID, _VOID, _VOID, _VOID, _INT, _VOID, _VOID, _INT, _VOID, _VOID, _VOID, _INT,
                                     _INT, _INT, _INT, _FLT, _INT, _INT, _FLT, _VOID],
@@ -114,15 +123,15 @@ _SUBLAYER_SIGNATURES = {
     "nnis_cast_rows": [_VOID, _INT, _VOID, _INT, _VOID, _INT, _INT, _VOID],
     "nnis_rms_post_step": [_VOID, _VOID, _INT, _VOID, _INT, _FLT, _FLT, _VOID, _INT, _INT, _INT, _VOID, _VOID, _INT, _VOID],
     "nnis_rms_between": [_VOID, _VOID, _INT, _VOID, _VOID, _INT, _FLT, _VOID, _INT, _INT, _INT, _VOID, _VOID, _INT, _VOID],
-    "nnis_route": [_VOID, _INT, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _VOID, _VOID, _INT, _INT, _VOID],
+    "nnis_route": [_VOID, _INT, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _VOID, _VOID, _INT, _INT, _VOID],
     "nnis_poly_norm": [_VOID, _INT, _VOID, _FLT, _VOID, _INT, _INT, _INT, _VOID],
     "nnis_router_logits": [_VOID, _INT, _VOID, _VOID, _INT, _INT, _INT, _VOID],
-    "nnis_route_top": [_VOID, _VOID, _INT, _INT, _INT, _INT, _VOID, _VOID, _INT, _INT, _VOID],
-    "nnis_routed_act": [_VOID, _INT, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _VOID],
+    "nnis_route_top": [_VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _VOID, _VOID, _INT, _INT, _VOID],
+    "nnis_routed_act": [_VOID, _INT, _INT, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _FLT, _VOID],
     "nnis_rows_axpy": [_VOID, _INT, _VOID, _INT, _VOID, _INT, _INT, _VOID],
     "nnis_sigmoid_gate": [_VOID, _INT, _VOID, _INT, _INT, _INT, _INT, _VOID],
     "nnis_head_norm_write": [_VOID, _INT, _INT, _INT, _INT, _INT, _VOID, _INT, _VOID, _VOID, _INT, _FLT, _VOID, _VOID, _INT, _INT, _INT,
-                             _VOID, _VOID, _VOID, _VOID, _INT, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _VOID],
+                             _VOID, _VOID, _VOID, _VOID, _INT, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _INT, _VOID, _VOID],
     "nnis_pool_blocks": [_VOID, _VOID, _INT, _VOID, _INT, _VOID, _VOID, _VOID, _INT, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT,
                          _VOID],
 }
@@ -244,17 +253,18 @@ def attention_check(head_dim: int, value_dim: Optional[int] = None, most: int = 
         _wide_heads.add((head_dim, value_dim or head_dim))
 
 
-def attention_module_name(head_dim: int, value_dim: Optional[int] = None, softcap: float = 0.0, extras=None, pooled=None) -> str:
+def attention_module_name(head_dim: int, value_dim: Optional[int] = None, softcap: float = 0.0, extras=None, pooled=None, terms=None) -> str:
     """The module compiled for keys of ``head_dim`` channels and values of ``value_dim`` (None: as the keys), with a
-    cap of the scores (``softcap`` > 0) or without, with the scores' extras (``ScoreExtras``) or without, and, with the
-    extras, with pooled blocks beside a window (``PooledBlocks``) or without."""
+    cap of the scores (``softcap`` > 0) or without, with what ``terms`` (``HeadTerms``) has or without, with the
+    scores' extras (``ScoreExtras``) or without, and, with the extras, with pooled blocks beside a window
+    (``PooledBlocks``) or without."""
     wide = value_dim is not None and value_dim != head_dim
     return ((f"attn_hd{head_dim}v{value_dim}" if wide else f"attn_hd{head_dim}") + ("c" if softcap else "")
-            + ("xp" if pooled is not None else ("x" if extras else "")))
+            + (terms.letters if terms is not None else "") + ("xp" if pooled is not None else ("x" if extras else "")))
 
 
-def attention_module(head_dim: int, value_dim: Optional[int] = None, softcap: float = 0.0, extras=None, pooled=None):
-    name = attention_module_name(head_dim, value_dim, softcap, extras, pooled)
+def attention_module(head_dim: int, value_dim: Optional[int] = None, softcap: float = 0.0, extras=None, pooled=None, terms=None):
+    name = attention_module_name(head_dim, value_dim, softcap, extras, pooled, terms)
     if name not in _attn:
         accepted = (head_dim, value_dim or head_dim) in _wide_heads
         attention_check(head_dim, value_dim, ATTENTION_ROWS_MOST_CHANNELS if accepted else ATTENTION_MOST_CHANNELS)
@@ -327,6 +337,21 @@ def embed(ids: torch.Tensor, table, out: torch.Tensor, scale: float = 1.0) -> to
     lib = core()
     _check(lib, lib.nnis_embed(ids.data_ptr(), table.data_ptr(), _code(table), out.data_ptr(), tokens, width,
                                table.shape[0], float(scale), _stream()))
+    return out
+
+
+def embed_norm(ids: torch.Tensor, table, weight: torch.Tensor, eps: float, out: torch.Tensor, scale: float = 1.0) -> torch.Tensor:
+    """``embed`` with an RMS norm of every row behind it (weight [width], eps inside the root), in one kernel."""
+    _dev(ids, "ids"), _dev(table, "embedding table"), _dev(weight, "norm weight"), _dev(out, "out")
+    tokens, width = out.shape
+    packed = isinstance(table, PackedWeight)
+    if ids.dtype != torch.int32 or ids.numel() < tokens:
+        raise KernelError(f"embed_norm: ids must be int32 with at least {tokens} entries")
+    if table.shape[1] != width or out.dtype != torch.float32 or weight.numel() != width:
+        raise KernelError(f"embed_norm: table {tuple(table.shape)} / weight {tuple(weight.shape)} / out {tuple(out.shape)} {out.dtype} do not fit")
+    lib = core()
+    _check(lib, lib.nnis_embed_norm(ids.data_ptr(), table.data_ptr(), _DTYPE_CODE[table.dtype], 1 if packed else 0, weight.data_ptr(),
+                                    _code(weight), float(eps), out.data_ptr(), tokens, width, table.shape[0], float(scale), _stream()))
     return out
 
 
@@ -549,6 +574,60 @@ class ScoreExtras:
             raise KernelError(f"attention: keep_first must not be negative, got {self.keep_first}")
 
 
+class _HeadTermsStruct(ctypes.Structure):
+    _fields_ = [("r1", _VOID), ("r2", _VOID), ("gate", _VOID), ("gate_dtype", _INT), ("gate_stride", _INT)]
+
+
+class HeadTerms:
+    """What an attention may take head by head beyond the plain formula, each
+    off when None.  ``decay``: (r1, r2), float32 [heads] each, r2 not
+    negative: the scaled score of a key ``n`` positions back loses r1 * ln(1 +
+    r2 * n).  ``gated``: a head's output is multiplied by sigmoid(gate[token,
+    head]); the logits of a step come with ``with_gate``: a tensor or a view
+    [tokens, heads] with adjacent columns, in either type."""
+
+    def __init__(self, decay=None, gated: bool = False):
+        self.decay, self.gated, self.gate = decay, bool(gated), None
+        self.letters = ("l" if decay is not None else "") + ("g" if gated else "")
+
+    def __bool__(self) -> bool:
+        return bool(self.letters)
+
+    def with_gate(self, gate: Optional[torch.Tensor]) -> "HeadTerms":
+        out = HeadTerms(self.decay, self.gated)
+        out.gate = gate
+        return out
+
+    def struct(self, tokens: int, heads: int) -> _HeadTermsStruct:
+        """The kernels' structure, its operands checked; keep it until the call it is handed to has returned."""
+        out = _HeadTermsStruct()
+        if self.decay is not None:
+            for t in self.decay:
+                _dev(t, "attention decay")
+                if t.dtype != torch.float32 or tuple(t.shape) != (heads,):
+                    raise KernelError(f"attention: a decay's numbers are float32, one a head ({heads}); got {tuple(t.shape)} {t.dtype}")
+            out.r1, out.r2 = self.decay[0].data_ptr(), self.decay[1].data_ptr()
+        if self.gated != (self.gate is not None):
+            raise KernelError("attention: gated heads and a step's gates come together")
+        if self.gate is not None:
+            if not self.gate.is_cuda or self.gate.dim() != 2 or tuple(self.gate.shape) != (tokens, heads) or (heads > 1 and self.gate.stride(1) != 1):
+                raise KernelError(f"attention: gates {tuple(self.gate.shape)} for {tokens} tokens of {heads} heads, columns adjacent")
+            out.gate, out.gate_dtype = self.gate.data_ptr(), _code(self.gate)
+            out.gate_stride = self.gate.stride(0) if tokens > 1 else heads
+        return out
+
+
+def _more_arguments(heads: int, k_pages, v_pages, kv_heads: int, head_dim: int, value_dim: int, window: int, extras, pooled):
+    """The arguments of the kernels' longest form that stand for the extras and the pooled blocks, checked."""
+    extras = extras or ScoreExtras()
+    extras.check(heads)
+    out = [extras.keep_first, _ptr(extras.bias), extras.reach, _ptr(extras.sink)]
+    if pooled is None:
+        return out + [None, None, None, 0, 0]
+    pooled.check(k_pages, v_pages, kv_heads, head_dim, value_dim, window)
+    return out + [pooled.k_pages.data_ptr(), pooled.v_pages.data_ptr(), pooled.block_table.data_ptr(), pooled.block_table.shape[1], pooled.pool]
+
+
 class PooledBlocks:
     """Beside a window of ``window`` tokens: pages whose entry b holds one key
     and one value for the tokens b * pool .. b * pool + pool - 1 of a
@@ -573,7 +652,8 @@ class PooledBlocks:
 def attention_rows(q: torch.Tensor, out: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor,
                    block_table: torch.Tensor, tok_slot: torch.Tensor, tok_pos: torch.Tensor, heads: int, kv_heads: int,
                    head_dim: int, scale: float, window: int = 0, value_dim: Optional[int] = None,
-                   softcap: float = 0.0, extras: Optional[ScoreExtras] = None, pooled: Optional["PooledBlocks"] = None) -> torch.Tensor:
+                   softcap: float = 0.0, extras: Optional[ScoreExtras] = None, pooled: Optional["PooledBlocks"] = None,
+                   terms: Optional[HeadTerms] = None) -> torch.Tensor:
     """Causal attention of each token over the cached keys of its slot up to
     its own position (32-bit arithmetic, any storage type).  ``value_dim``:
     channels of a value head and of a head's output (None: as the keys).
@@ -592,7 +672,15 @@ def attention_rows(q: torch.Tensor, out: torch.Tensor, k_pages: torch.Tensor, v_
         raise KernelError("attention: key and value pages differ in type")
     if tok_slot.dtype != torch.int32 or tok_pos.dtype != torch.int32 or block_table.dtype != torch.int32:
         raise KernelError("attention: tok_slot, tok_pos and block_table must be int32")
-    lib = attention_module(head_dim, value_dim, softcap, extras, pooled)
+    lib = attention_module(head_dim, value_dim, softcap, extras, pooled, terms)
+    if terms:
+        held = terms.struct(tokens, heads)
+        _check(lib, lib.nnis_attention_rows_terms(
+            q.data_ptr(), _code(q), out.data_ptr(), _code(out), k_pages.data_ptr(), v_pages.data_ptr(), _code(k_pages), block_table.data_ptr(),
+            block_table.shape[1], tok_slot.data_ptr(), tok_pos.data_ptr(), tokens, heads, kv_heads, head_dim, int(window), float(scale),
+            int(value_dim), float(softcap), *_more_arguments(heads, k_pages, v_pages, kv_heads, head_dim, value_dim, window, extras, pooled),
+            ctypes.addressof(held), _stream()))
+        return out
     if pooled is not None:
         extras = extras or ScoreExtras()
         extras.check(heads)
@@ -998,20 +1086,21 @@ def _check_pages(q, out, k_pages, v_pages, block_table, heads, kv_heads, head_di
             raise KernelError(f"attention: the matrix-core kernels take bfloat16, {what} is {t.dtype}")
 
 
-def prefill_tile_rows(heads: int, kv_heads: int, head_dim: int, columns: int = 0, value_dim=None, softcap=0.0, extras=None, pooled=None) -> int:
+def prefill_tile_rows(heads: int, kv_heads: int, head_dim: int, columns: int = 0, value_dim=None, softcap=0.0, extras=None, pooled=None, terms=None) -> int:
     """Query rows per work item of ``attention_prefill_bf16`` for these sizes.
     ``columns``: the most 16-column tiles (query tiles x heads of a group) a
     wave carries; 0 for as many as the head size allows."""
-    return attention_module(head_dim, value_dim, softcap, extras, pooled).nnis_attention_prefill_tile_rows(heads, kv_heads, columns)
+    return attention_module(head_dim, value_dim, softcap, extras, pooled, terms).nnis_attention_prefill_tile_rows(heads, kv_heads, columns)
 
 
-def prefill_max_waves(heads: int, kv_heads: int, head_dim: int, columns: int = 0, value_dim=None, softcap=0.0, extras=None, pooled=None) -> int:
-    return attention_module(head_dim, value_dim, softcap, extras, pooled).nnis_attention_prefill_max_waves(heads, kv_heads, columns)
+def prefill_max_waves(heads: int, kv_heads: int, head_dim: int, columns: int = 0, value_dim=None, softcap=0.0, extras=None, pooled=None, terms=None) -> int:
+    return attention_module(head_dim, value_dim, softcap, extras, pooled, terms).nnis_attention_prefill_max_waves(heads, kv_heads, columns)
 
 
 def attention_prefill_bf16(q, out, k_pages, v_pages, block_table, tile_seq, tile_row0, seq_slot, seq_start, seq_pos0,
                            heads, kv_heads, head_dim, scale, window=0, waves=1, columns=0, value_dim=None, softcap=0.0,
-                           extras: Optional[ScoreExtras] = None, pooled: Optional[PooledBlocks] = None):
+                           extras: Optional[ScoreExtras] = None, pooled: Optional[PooledBlocks] = None,
+                           terms: Optional[HeadTerms] = None):
     """Causal attention of whole runs of new tokens over the cache, on the
     matrix cores.  ``tile_seq``/``tile_row0`` (int32) name, per work item, a
     sequence of the step and the first of ``prefill_tile_rows`` rows of its
@@ -1024,7 +1113,16 @@ def attention_prefill_bf16(q, out, k_pages, v_pages, block_table, tile_seq, tile
     tiles = tile_seq.numel()
     if tile_row0.numel() != tiles or seq_start.numel() != seq_slot.numel() + 1 or seq_pos0.numel() != seq_slot.numel():
         raise KernelError("attention: step metadata arrays do not fit each other")
-    lib = attention_module(head_dim, value_dim, softcap, extras, pooled)
+    lib = attention_module(head_dim, value_dim, softcap, extras, pooled, terms)
+    if terms:
+        held = terms.struct(q.shape[0], heads)
+        _check(lib, lib.nnis_attention_prefill_bf16_terms(
+            q.data_ptr(), out.data_ptr(), k_pages.data_ptr(), v_pages.data_ptr(), block_table.data_ptr(), block_table.shape[1],
+            tile_seq.data_ptr(), tile_row0.data_ptr(), tiles, seq_slot.data_ptr(), seq_start.data_ptr(), seq_pos0.data_ptr(), heads,
+            kv_heads, head_dim, int(window), float(scale), int(waves), int(columns), float(softcap),
+            *_more_arguments(heads, k_pages, v_pages, kv_heads, head_dim, value_dim or head_dim, window, extras, pooled),
+            ctypes.addressof(held), _stream()))
+        return out
     if pooled is not None:
         extras = extras or ScoreExtras()
         extras.check(heads)
@@ -1054,7 +1152,8 @@ def attention_prefill_bf16(q, out, k_pages, v_pages, block_table, tile_seq, tile
 
 def attention_decode_bf16(q, out, k_pages, v_pages, block_table, tok_slot, tok_pos, heads, kv_heads, head_dim, scale,
                           window=0, splits=1, partial=None, waves=1, kernel="auto", keep_runs=False, token_pages=None,
-                          value_dim=None, softcap=0.0, extras: Optional[ScoreExtras] = None, pooled: Optional[PooledBlocks] = None):
+                          value_dim=None, softcap=0.0, extras: Optional[ScoreExtras] = None, pooled: Optional[PooledBlocks] = None,
+                          terms: Optional[HeadTerms] = None):
     """One query token per sequence over its cached keys.  The keys are cut
     into ``splits`` runs, each a block of ``waves`` waves that deal its pages
     among themselves and merge in LDS; the runs are summed by a second kernel.
@@ -1085,8 +1184,19 @@ def attention_decode_bf16(q, out, k_pages, v_pages, block_table, tok_slot, tok_p
         if partial is None or partial.dtype != torch.float32 or partial.numel() < tokens * heads * splits * (value_dim + 4):
             raise KernelError("attention: splits need float32 scratch of tokens * heads * splits * (value channels + 4)")
         _dev(partial, "partial")
-    lib = attention_module(head_dim, value_dim, softcap, extras, pooled)
-    if pooled is not None:
+    lib = attention_module(head_dim, value_dim, softcap, extras, pooled, terms)
+    if terms:
+        if keep_runs and terms.gated:
+            raise KernelError("attention: gated heads are gated where their runs of keys are added up; the runs are not handed on")
+        held = terms.struct(tokens, heads)
+        _check(lib, lib.nnis_attention_decode_bf16_terms(
+            q.data_ptr(), out.data_ptr(), k_pages.data_ptr(), v_pages.data_ptr(), table.data_ptr(), table.shape[1],
+            tok_slot.data_ptr(), tok_pos.data_ptr(), tokens, heads, kv_heads, head_dim, int(window), float(scale), int(splits),
+            int(waves), _ptr(partial) if splits > 1 else None, _DECODE_KERNELS[kernel], 0 if (keep_runs and splits > 1) else 1,
+            1 if token_pages is not None else 0, float(softcap),
+            *_more_arguments(heads, k_pages, v_pages, kv_heads, head_dim, value_dim, window, extras, pooled),
+            ctypes.addressof(held), _stream()))
+    elif pooled is not None:
         extras = extras or ScoreExtras()
         extras.check(heads)
         pooled.check(k_pages, v_pages, kv_heads, head_dim, value_dim, window)
@@ -1177,8 +1287,8 @@ def decode_scratch_held(device):
     return _decode_scratch.get((device.type, device.index))
 
 
-def decode_max_waves(heads: int, kv_heads: int, head_dim: int, value_dim=None, softcap=0.0, extras=None, pooled=None) -> int:
-    return attention_module(head_dim, value_dim, softcap, extras, pooled).nnis_attention_decode_max_waves(heads, kv_heads)
+def decode_max_waves(heads: int, kv_heads: int, head_dim: int, value_dim=None, softcap=0.0, extras=None, pooled=None, terms=None) -> int:
+    return attention_module(head_dim, value_dim, softcap, extras, pooled, terms).nnis_attention_decode_max_waves(heads, kv_heads)
 
 
 def decode_plan(batch: int, kv_heads: int, longest: int, max_waves: int = 4, width: int = 0):
@@ -1334,7 +1444,7 @@ def prefill_tile_list(new_tokens, first_positions, padded, rows: int):
 def attention(q: torch.Tensor, out: torch.Tensor, view, ctx, heads: int, kv_heads: int, head_dim: int, scale: float,
               window: int = 0, keep_runs: bool = False, tables: Optional[StepTables] = None, plan=None,
               value_dim: Optional[int] = None, softcap: float = 0.0, extras: Optional[ScoreExtras] = None,
-              pooled: Optional[PooledBlocks] = None):
+              pooled: Optional[PooledBlocks] = None, terms: Optional[HeadTerms] = None):
     """Attention of the step's tokens over the cache ``view``: bfloat16 with a
     head size in steps of 16 runs on the matrix cores (one kernel for single
     tokens, one for runs of tokens); anything else takes the 32-bit kernel.
@@ -1348,7 +1458,7 @@ def attention(q: torch.Tensor, out: torch.Tensor, view, ctx, heads: int, kv_head
     size = max(head_dim, value_dim)  # what a wave's registers are sized by
     if fast and ctx.decode and heads // kv_heads <= 16 * (4 if size <= 64 else (2 if size <= 128 else 1)):
         splits, waves = plan or decode_plan(ctx.batch, kv_heads, ctx.planned_len, width=heads * value_dim)
-        waves = min(waves, decode_max_waves(heads, kv_heads, head_dim, value_dim, softcap, extras, pooled))
+        waves = min(waves, decode_max_waves(heads, kv_heads, head_dim, value_dim, softcap, extras, pooled, terms))
         partial = None
         if splits > 1:
             partial = decode_scratch(q.device, q.shape[0] * heads * splits * (value_dim + 4))
@@ -1356,19 +1466,19 @@ def attention(q: torch.Tensor, out: torch.Tensor, view, ctx, heads: int, kv_head
                                      kv_heads, head_dim, scale, window, splits, partial, waves,
                                      keep_runs=keep_runs and q.shape[0] <= KEY_RUNS_MOST_TOKENS,
                                      token_pages=tables.pages if tables is not None else None, value_dim=value_dim, softcap=softcap,
-                                     extras=extras, pooled=pooled)
+                                     extras=extras, pooled=pooled, terms=terms)
     if fast and not ctx.decode:
         # A tile's keys are a chain of dependent loads: the longest tile sets the kernel's time.  The waves of
         # a block deal the keys among themselves (their merge lives in LDS).
         waves, columns = plan or prefill_plan(ctx.planned_len, ctx.planned_rows, heads, size, kv_heads)
-        waves = min(waves, prefill_max_waves(heads, kv_heads, head_dim, columns, value_dim, softcap, extras, pooled))
-        rows = prefill_tile_rows(heads, kv_heads, head_dim, columns, value_dim, softcap, extras, pooled)
+        waves = min(waves, prefill_max_waves(heads, kv_heads, head_dim, columns, value_dim, softcap, extras, pooled, terms))
+        rows = prefill_tile_rows(heads, kv_heads, head_dim, columns, value_dim, softcap, extras, pooled, terms)
         tiles = ctx.lists.device_list(("attention_tiles", rows), lambda new, first, padded: prefill_tile_list(new, first, padded, rows))
         return attention_prefill_bf16(q, out, view.k_pages, view.v_pages, view.block_table, tiles[0], tiles[1],
                                       ctx.seq_slot, ctx.seq_start, ctx.seq_pos0, heads, kv_heads, head_dim, scale, window,
-                                      waves, columns, value_dim, softcap, extras, pooled)
+                                      waves, columns, value_dim, softcap, extras, pooled, terms)
     return attention_rows(q, out, view.k_pages, view.v_pages, view.block_table, ctx.tok_slot, ctx.tok_pos, heads,
-                          kv_heads, head_dim, scale, window, value_dim, softcap, extras, pooled)
+                          kv_heads, head_dim, scale, window, value_dim, softcap, extras, pooled, terms)
 
 
 def attention_on_matrix_cores(q_dtype, cache_dtype, head_dim: int, value_dim: Optional[int] = None, softcap: float = 0.0,
@@ -2074,11 +2184,19 @@ def _route_groups(groups, n: int, what: str):
     return count, keep
 
 
+def _check_router_bias(bias: Optional[torch.Tensor], n: int, what: str) -> None:
+    if bias is not None:
+        _dev(bias, "router bias")
+        if bias.dtype != torch.float32 or bias.numel() != n:
+            raise KernelError(f"{what}: a float32 bias per output ({n}), got {tuple(bias.shape)} {bias.dtype}")
+
+
 def route_top(logits: torch.Tensor, correction: Optional[torch.Tensor], experts: int, top: int, gates: torch.Tensor,
-              keep: torch.Tensor, groups=None):
+              keep: torch.Tensor, groups=None, bias: Optional[torch.Tensor] = None, chosen_softmax: bool = False):
     """Scores softmax(logits) [rows, n]; the ``top`` largest of score + correction are chosen.  ``gates`` [rows, experts]
     gets the score of every chosen output below ``experts`` and 0 elsewhere; ``keep`` [rows] the summed scores of the
-    chosen outputs from ``experts`` on.  All float32."""
+    chosen outputs from ``experts`` on.  ``bias`` [n] joins the logits first.  ``chosen_softmax``: chosen are the ``top``
+    largest logits (+ correction), and their weights are the softmax over the chosen logits alone.  All float32."""
     _dev(logits, "logits"), _dev(gates, "gates"), _dev(keep, "keep")
     rows, n = logits.shape
     if logits.dtype != torch.float32 or gates.dtype != torch.float32 or keep.dtype != torch.float32 \
@@ -2090,9 +2208,11 @@ def route_top(logits: torch.Tensor, correction: Optional[torch.Tensor], experts:
             raise KernelError(f"route_top: a float32 correction per output ({n}), got {tuple(correction.shape)} {correction.dtype}")
     if not (0 < n <= ROUTE_MOST_OUTPUTS and 0 <= experts <= n and 0 < top <= n):
         raise KernelError(f"route_top: {experts} experts and the {top} largest of {n} outputs (at most {ROUTE_MOST_OUTPUTS})")
+    _check_router_bias(bias, n, "route_top")
     group_count, group_keep = _route_groups(groups, n, "route_top")
     lib = sublayer()
-    _check(lib, lib.nnis_route_top(logits.data_ptr(), _ptr(correction), rows, n, experts, top, gates.data_ptr(), keep.data_ptr(),
+    _check(lib, lib.nnis_route_top(logits.data_ptr(), _ptr(bias), _ptr(correction), rows, n, experts, top, 1 if chosen_softmax else 0,
+                                   gates.data_ptr(), keep.data_ptr(),
                                    group_count, group_keep, _stream()))
     return gates, keep
 
@@ -2101,7 +2221,7 @@ ROUTE_FUSED_MOST_CHANNELS = 8192
 
 
 def route(x: torch.Tensor, weight: torch.Tensor, correction: Optional[torch.Tensor], experts: int, top: int, gates: torch.Tensor,
-          keep: torch.Tensor, groups=None):
+          keep: torch.Tensor, groups=None, bias: Optional[torch.Tensor] = None, chosen_softmax: bool = False):
     """``router_logits`` and ``route_top`` in one kernel (rows of up to ``ROUTE_FUSED_MOST_CHANNELS`` channels).
     ``groups``: (count, keep): the outputs form ``count`` equal groups of neighbours, a group's mark is its largest
     corrected score, and only outputs of the ``keep`` groups with the largest marks can be chosen."""
@@ -2117,28 +2237,42 @@ def route(x: torch.Tensor, weight: torch.Tensor, correction: Optional[torch.Tens
             raise KernelError(f"route: a float32 correction per output ({n}), got {tuple(correction.shape)} {correction.dtype}")
     if not (0 < n <= ROUTE_MOST_OUTPUTS and 0 <= experts <= n and 0 < top <= n and width <= ROUTE_FUSED_MOST_CHANNELS):
         raise KernelError(f"route: {experts} experts and the {top} largest of {n} outputs (at most {ROUTE_MOST_OUTPUTS}) of rows of {width} channels")
+    _check_router_bias(bias, n, "route")
     group_count, group_keep = _route_groups(groups, n, "route")
     lib = sublayer()
-    _check(lib, lib.nnis_route(x.data_ptr(), _code(x), weight.data_ptr(), _ptr(correction), rows, n, width, experts, top, gates.data_ptr(),
-                               keep.data_ptr(), group_count, group_keep, _stream()))
+    _check(lib, lib.nnis_route(x.data_ptr(), _code(x), weight.data_ptr(), _ptr(bias), _ptr(correction), rows, n, width, experts, top,
+                               1 if chosen_softmax else 0, gates.data_ptr(), keep.data_ptr(), group_count, group_keep, _stream()))
     return gates, keep
 
 
-def routed_act(z: torch.Tensor, gates: torch.Tensor, out: torch.Tensor, form: str = "relu_squared") -> torch.Tensor:
+_ROUTED_FORMS = {"relu_squared": 0, "silu_gated": 1, "clamped_swiglu": 2}
+
+
+def routed_act(z: torch.Tensor, gates: Optional[torch.Tensor], out: torch.Tensor, form: str = "relu_squared", limit: float = 0.0,
+               inner: Optional[int] = None) -> torch.Tensor:
     """On the experts' fused up projection.  ``relu_squared``: out[row, e * ff + c] = gates[row, e] * relu(z[row, e * ff
     + c])^2.  ``silu_gated``: z [rows, experts * 2 * ff] holds, expert by expert, gate columns then up columns, and
-    out[row, e * ff + c] = gates[row, e] * silu(gate) * up."""
-    _dev(z, "z"), _dev(gates, "gates"), _dev(out, "out")
-    rows, experts = gates.shape
-    if form not in ("relu_squared", "silu_gated"):
+    out[row, e * ff + c] = gates[row, e] * silu(gate) * up.  ``clamped_swiglu``: the same columns; gate held at most at
+    ``limit``, up within plus or minus ``limit`` (0: not held), out = gates * gate * sigmoid(1.702 gate) * (up + 1).
+    ``inner`` (ff): given where ``z`` and ``out`` are views whose rows are further apart.  ``gates`` None: one expert of
+    weight one."""
+    rows, experts = (z.shape[0], 1) if gates is None else gates.shape
+    if form not in _ROUTED_FORMS:
         raise KernelError(f"routed_act: unknown form {form!r}")
-    per = 2 if form == "silu_gated" else 1
-    if (gates.dtype != torch.float32 or z.dim() != 2 or z.shape[0] != rows or z.shape[1] % max(per * experts, 1)
-            or tuple(out.shape) != (rows, z.shape[1] // per) or not z.is_contiguous() or not out.is_contiguous()):
-        raise KernelError(f"routed_act: z {tuple(z.shape)} and out {tuple(out.shape)} against gates {tuple(gates.shape)}")
+    per = 1 if form == "relu_squared" else 2
+    if gates is not None:
+        _dev(gates, "gates")
+    if inner is None:
+        _dev(z, "z"), _dev(out, "out")
+    if ((gates is not None and gates.dtype != torch.float32) or z.dim() != 2 or z.shape[0] != rows or z.shape[1] % max(per * experts, 1)
+            or tuple(out.shape) != (rows, z.shape[1] // per) or not z.is_cuda or not out.is_cuda
+            or z.stride(1) != 1 or out.stride(1) != 1 or (inner is not None and z.shape[1] != per * experts * inner)):
+        raise KernelError(f"routed_act: z {tuple(z.shape)} and out {tuple(out.shape)} for {rows} rows of {experts} experts")
     lib = sublayer()
-    _check(lib, lib.nnis_routed_act(z.data_ptr(), _code(z), gates.data_ptr(), out.data_ptr(), _code(out), rows, experts,
-                                    z.shape[1] // (per * experts), per - 1, _stream()))
+    z_stride = z.stride(0) if rows > 1 else z.shape[1]
+    out_stride = out.stride(0) if rows > 1 else out.shape[1]
+    _check(lib, lib.nnis_routed_act(z.data_ptr(), _code(z), z_stride, _ptr(gates), out.data_ptr(), _code(out), out_stride, rows, experts,
+                                    z.shape[1] // (per * experts), _ROUTED_FORMS[form], float(limit), _stream()))
     return out
 
 
@@ -2169,9 +2303,11 @@ HEAD_NORM_MOST_CHANNELS = 1024
 def head_norm_write(rows: torch.Tensor, columns, q_out: torch.Tensor, q_weight: Optional[torch.Tensor], k_weight: Optional[torch.Tensor],
                     eps: float, cos: Optional[torch.Tensor], sin: Optional[torch.Tensor], rot_dim: int, neighbours: bool,
                     tok_slot: torch.Tensor, tok_pos: torch.Tensor, k_pages: Optional[torch.Tensor], v_pages: Optional[torch.Tensor],
-                    block_table: Optional[torch.Tensor], heads: int, kv_heads: int, head_dim: int, value_dim: int) -> torch.Tensor:
+                    block_table: Optional[torch.Tensor], heads: int, kv_heads: int, head_dim: int, value_dim: int,
+                    unit: bool = False, q_factor: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Queries and keys of a fused projection's ``rows`` head by head: an RMS norm over the head with a weight that the
-    heads share (None: no norm), then the rotation of the first ``rot_dim`` channels by the token's position (channel
+    heads share (None: no norm, or with ``unit`` the norm without a weight; ``q_factor``, float32 [heads]: a query
+    head's own factor on top), then the rotation of the first ``rot_dim`` channels by the token's position (channel
     2i with 2i + 1 if ``neighbours``, else i with i + rot_dim / 2); queries to ``q_out``, keys and values into the
     pages.  ``columns``: (first column of the queries, of the keys, of the values) in a row; with ``k_pages`` None the
     rows bring queries only."""
@@ -2195,6 +2331,12 @@ def head_norm_write(rows: torch.Tensor, columns, q_out: torch.Tensor, q_weight: 
             w_code = _code(weight)
     if q_weight is not None and k_weight is not None and q_weight.dtype != k_weight.dtype:
         raise KernelError("head_norm_write: the two norm weights differ in type")
+    if unit and (q_weight is not None or k_weight is not None):
+        raise KernelError("head_norm_write: a norm without a weight was handed a weight")
+    if q_factor is not None:
+        _dev(q_factor, "q_factor")
+        if q_factor.dtype != torch.float32 or q_factor.numel() != heads:
+            raise KernelError(f"head_norm_write: query factors are float32, one a head ({heads})")
     table_positions = 0
     if cos is not None:
         _dev(cos, "cos"), _dev(sin, "sin")
@@ -2215,7 +2357,7 @@ def head_norm_write(rows: torch.Tensor, columns, q_out: torch.Tensor, q_weight: 
                                          _ptr(k_weight), w_code, float(eps), _ptr(cos), _ptr(sin), table_positions, int(rot_dim),
                                          1 if neighbours else 0, tok_slot.data_ptr(), tok_pos.data_ptr(), _ptr(k_pages) if keys else None,
                                          _ptr(v_pages) if keys else None, cache_code, _ptr(block_table) if keys else None, max_pages,
-                                         tokens, heads, keys, head_dim, int(value_dim), _stream()))
+                                         tokens, heads, keys, head_dim, int(value_dim), 1 if unit else 0, _ptr(q_factor), _stream()))
     return q_out
 
 

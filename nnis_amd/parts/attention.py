@@ -15,7 +15,11 @@ query (``keep_first``); a learned bias by distance added to the scaled score
 (``distance_bias``, ``bias_reach``); a sink in the softmax's denominator
 (``sink``); values that are the keys as projected, before their rotation, with
 no projection of their own (``values_from_keys``); a gate per head, sigmoid of
-a projection of the mixer's input, on the head's output (``head_gate``).
+a projection of the mixer's input, on the head's output (``head_gate``);
+queries and keys divided, head by head, by their root mean square
+(``unit_heads``), a learned factor per head on the queries behind that
+(``temperature``), and scores that fall with the logarithm of the distance by
+two learned numbers per head (``decay``).
 """
 
 from __future__ import annotations
@@ -25,6 +29,7 @@ import math
 import torch
 
 from ..errors import InvalidInput
+from ..weights.random_init import register_init_rule
 from .base import KVRequest, Mixer, TensorSpec, register_part
 from .linear import Projection
 
@@ -46,14 +51,20 @@ class CausalSelfAttention(Mixer):
     def __init__(self, width, heads, kv_heads, head_dim, q, k, v, o, position=None, window=None, positions=None,
                  value_dim=None, scale=None, softcap=None, q_bias=None, k_bias=None, v_bias=None, o_bias=None,
                  keep_first=None, distance_bias=None, bias_reach=None, bias_buckets=None, sink=None, values_from_keys=False,
-                 head_gate=None):
+                 head_gate=None, unit_heads=None,
+                 temperature=None, decay=None):
         """``keep_first``: with a ``window``, keys at positions below it stay
         visible.  ``distance_bias``: the name of a table [buckets, heads]; the
         scaled score of a key n positions back gets row ``distance_bucket(n,
         buckets, bias_reach)`` of its head's column added (the table's length
         is the checkpoint's; a random model names it as ``bias_buckets``).
         ``sink``: "zero" for a score of 0, or the name of a tensor [heads] of
-        learned scores, that joins the softmax's denominator and has no value."""
+        learned scores, that joins the softmax's denominator and has no value.
+        ``unit_heads``: the eps inside the root of the norm without a weight
+        that every head's query and key go through.  ``temperature``: the name
+        of a tensor [heads], a factor of the head's scores.  ``decay``: the
+        names of two tensors [heads], r1 and r2: the scaled score of a key n
+        positions back loses r1 * ln(1 + r2 * n)."""
         if heads % kv_heads != 0:
             raise InvalidInput(f"{heads} query heads do not divide into {kv_heads} key/value heads")
         self.width, self.heads, self.kv_heads, self.head_dim = int(width), int(heads), int(kv_heads), int(head_dim)
@@ -93,6 +104,13 @@ class CausalSelfAttention(Mixer):
         self.extras = None  # ``ops.ScoreExtras``, made when the weights are bound
         self.qkv = None
         self.out = None
+        self.unit_eps = None if unit_heads is None else float(unit_heads)
+        self.temperature_name, self.decay_names = temperature, None if decay is None else tuple(decay)
+        self.temperature = self.terms = None
+        if self.unit_eps is None and (temperature is not None or decay is not None):
+            raise InvalidInput("a temperature and a decay by distance are built for heads that are normed without a weight (unit_heads)")
+        if self.unit_eps is not None and (q_bias is not None or values_from_keys):
+            raise InvalidInput("heads that are normed without a weight have projections without biases and values of their own")
 
     def tensors(self):
         q_width, kv_width = self.heads * self.head_dim, self.kv_heads * self.head_dim
@@ -114,14 +132,25 @@ class CausalSelfAttention(Mixer):
             out.append(TensorSpec(self.bias_name, (self.bias_buckets, self.heads)))
         if self.sink_name and self.sink_name != "zero":
             out.append(TensorSpec(self.sink_name, (self.heads,)))
+        if self.temperature_name:
+            out.append(TensorSpec(self.temperature_name, (self.heads,), init="head_number"))
+        if self.decay_names:
+            out += [TensorSpec(name, (self.heads,), init="head_number") for name in self.decay_names]
         return out
 
     def bind(self, weights, rt):
         # one projection for queries, keys and values: rows q heads, k heads, v heads
         rows = ("q", "k") if self.values_from_keys else ("q", "k", "v")
-        self.qkv = Projection(torch.cat([weights[self.names[key]] for key in rows], dim=0), rt)
+        parts = [weights[self.names[key]] for key in rows]
+        if self.unit_eps is not None and self.gate_name:
+            parts.append(weights[self.gate_name])  # (the gates' logits are columns of the same product)
+        self.qkv = Projection(torch.cat(parts, dim=0), rt)
         self.out = Projection(weights[self.names["o"]], rt)
-        if self.gate_name:
+        if self.unit_eps is not None:
+            self.temperature = weights[self.temperature_name].float().contiguous() if self.temperature_name else None
+            decay = tuple(weights[name].float().contiguous() for name in self.decay_names) if self.decay_names else None
+            self.terms = rt.ops.HeadTerms(decay, gated=bool(self.gate_name))
+        elif self.gate_name:
             self.gate = Projection(weights[self.gate_name], rt)
         if self.bias_names["q"]:
             self.qkv_bias = torch.cat([weights[self.bias_names[key]] for key in rows]).contiguous()
@@ -167,6 +196,8 @@ class CausalSelfAttention(Mixer):
         # (runs of the keys, waves of a block) of a step of single tokens with these sizes
         if not self._matrix_cores(rt):
             return None
+        if self.window:  # (a window of n tokens touches the pages of at most n + 63)
+            longest = min(longest, self.window + 63)
         return rt.ops.decode_plan(batch, self.kv_heads, longest, width=self.heads * self.value_dim)
 
     def prompt_plan(self, batch, rows, longest, rt):
@@ -213,6 +244,27 @@ class CausalSelfAttention(Mixer):
         )
         return q
 
+    def _project_norm_store(self, x, ctx, view, rt):
+        """The same with heads that are normed without a weight; also the gates' logits [tokens, heads], a view (None without gates)."""
+        from .lazy import PendingNorm
+
+        tables = self.position.rotary() if self.position is not None else None
+        if isinstance(x, PendingNorm) and x.can_fuse(self.qkv.weight):
+            rows = x.fused(self.qkv.weight, rt.empty(x.rows, self.qkv.out_features), rt.ops.EPILOGUE_STORE)
+        else:
+            rows = self.qkv(x.materialize() if isinstance(x, PendingNorm) else x, rt)
+        keys_at = self.heads * self.head_dim
+        values_at = keys_at + self.kv_heads * self.head_dim
+        gates_at = values_at + self.kv_heads * self.value_dim
+        writes = not view.read_only
+        q = rt.ops.head_norm_write(
+            rows, (0, keys_at, values_at), rt.empty(rows.shape[0], keys_at), None, None, self.unit_eps,
+            tables.cos if tables else None, tables.sin if tables else None, tables.rot_dim if tables else 0,
+            getattr(self.position, "pairing", None) == "neighbours", ctx.tok_slot, ctx.tok_pos,
+            view.k_pages if writes else None, view.v_pages if writes else None, view.block_table if writes else None,
+            self.heads, self.kv_heads, self.head_dim, self.value_dim, unit=True, q_factor=self.temperature)
+        return q, rows[:, gates_at:gates_at + self.heads] if self.gate_name else None
+
     can_leave_bias = True  # ``forward(..., bias_later=True)`` leaves ``output_bias`` to a consumer that adds it in a kernel of its own
 
     def forward(self, x, ctx, view, rt, into=None, bias_later=False):
@@ -223,7 +275,12 @@ class CausalSelfAttention(Mixer):
                 x = x.materialize()
             gate = self.gate(x, rt, out_dtype=torch.float32)
             into = None  # the heads are gated before the output projection, which then takes plain rows
-        q = self._project_rotate_store(x, ctx, view, rt)
+        terms = None
+        if self.unit_eps is not None:
+            q, logits = self._project_norm_store(x, ctx, view, rt)
+            terms = self.terms.with_gate(logits)
+        else:
+            q = self._project_rotate_store(x, ctx, view, rt)
         tokens = q.shape[0]
         attn = rt.empty(tokens, self.heads * self.value_dim)
         # a decode step over long sequences leaves its runs of keys to the output projection, if that takes them
@@ -236,8 +293,8 @@ class CausalSelfAttention(Mixer):
             plan = (self.decode_plan(ctx.batch, ctx.planned_len, rt) if ctx.decode
                     else self.prompt_plan(ctx.batch, ctx.planned_rows, ctx.planned_len, rt))
         attn = rt.ops.attention(q, attn, view, ctx, self.heads, self.kv_heads, self.head_dim, self.scale, self.window or 0,
-                                keep_runs=into is not None and self.output_bias is None, tables=step, plan=plan,
-                                value_dim=self.value_dim, softcap=self.softcap, extras=self.extras)
+                                keep_runs=into is not None and self.output_bias is None and not (terms and terms.gated), tables=step,
+                                plan=plan, value_dim=self.value_dim, softcap=self.softcap, extras=self.extras, terms=terms)
         if isinstance(attn, rt.ops.KeyRuns) and not (into.can_take(attn, self.out.weight) and attn.fits(self.out.weight.shape[0])):
             attn = attn.combine()
         if gate is not None:
@@ -250,6 +307,8 @@ class CausalSelfAttention(Mixer):
         return y
 
 
+# what a random model draws for a number per head (a temperature, a decay's two numbers): around one half, never near zero
+register_init_rule("head_number", lambda spec, generator, dtype: (0.5 + torch.rand(tuple(spec.shape), generator=generator)).to(dtype), replace=True)
 register_part("mixer", "causal_attention", CausalSelfAttention)
 
 

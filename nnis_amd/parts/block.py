@@ -31,13 +31,17 @@ def _joined(plans):
 
 
 class PreNormBlock(Block):
-    def __init__(self, width, norm1, mixer, norm2, feed_forward, positions=None):
+    """Without a feed-forward (and its norm) the layer is its mixer alone."""
+
+    def __init__(self, width, norm1, mixer, norm2=None, feed_forward=None, positions=None):
         self.width = int(width)
+        if (feed_forward is None) != (norm2 is None):
+            raise InvalidInput("a feed-forward comes with its norm, or neither")
         self.norm1 = build_part("norm", norm1)
         self.mixer = build_part("mixer", mixer, positions=positions)
-        self.norm2 = build_part("norm", norm2)
-        self.feed_forward = build_part("feed_forward", feed_forward)
-        self._parts = [self.norm1, self.mixer, self.norm2, self.feed_forward]
+        self.norm2 = build_part("norm", norm2) if norm2 is not None else None
+        self.feed_forward = build_part("feed_forward", feed_forward) if feed_forward is not None else None
+        self._parts = [part for part in (self.norm1, self.mixer, self.norm2, self.feed_forward) if part is not None]
         self.graph_safe = all(getattr(part, "graph_safe", False) for part in self._parts)
 
     def tensors(self):
@@ -98,6 +102,8 @@ class PreNormBlock(Block):
         else:
             x, pending = stream
             normed = self.norm1.defer(x, pending, rt)
+        if self.feed_forward is None:
+            return self._run(self.mixer, normed, (ctx, view, rt), following, rt)
         normed = self._run(self.mixer, normed, (ctx, view, rt), self.norm2, rt)
         return self._run(self.feed_forward, normed, (ctx, rt), following, rt)
 

@@ -8,23 +8,30 @@ from __future__ import annotations
 
 import torch
 
-from .base import Part, StateRequest, TensorSpec, register_part
+from ..errors import InvalidInput
+from .base import Part, StateRequest, TensorSpec, build_part, register_part
 from .linear import Projection
 
 
 class TokenEmbedding(Part):
     graph_safe = True
 
-    def __init__(self, vocab_size, width, weight, scale=1.0):
-        """``scale``: every row is multiplied by it on the way out (in 32-bit)."""
+    def __init__(self, vocab_size, width, weight, scale=1.0, norm=None):
+        """``scale``: every row is multiplied by it on the way out (in 32-bit).  ``norm``: the description of an RMS norm
+        (``width``, ``eps``, ``weight``) of every row behind that, in the same kernel."""
         self.vocab_size, self.width, self.weight_name, self.scale = int(vocab_size), int(width), weight, float(scale)
         self.table = None
+        self.norm = build_part("norm", norm) if norm is not None else None
+        if self.norm is not None and not getattr(self.norm, "fusable_rms", False):
+            raise InvalidInput("an embedding is normed by a plain RMS norm")
 
     def tensors(self):
-        return [TensorSpec(self.weight_name, (self.vocab_size, self.width))]
+        return [TensorSpec(self.weight_name, (self.vocab_size, self.width))] + (self.norm.tensors() if self.norm is not None else [])
 
     def bind(self, weights, rt):
         self.table = weights[self.weight_name].contiguous()
+        if self.norm is not None:
+            self.norm.bind(weights, rt)
 
     def adopt_packed(self, source, packed) -> bool:
         """A part of the model has packed the tensor at ``source`` (address,
@@ -38,7 +45,10 @@ class TokenEmbedding(Part):
 
     def forward(self, ids, tokens, rt):
         """ids: int32 on the device -> the 32-bit residual stream [tokens, width]."""
-        return rt.ops.embed(ids, self.table, rt.empty(tokens, self.width, dtype=torch.float32), self.scale)
+        out = rt.empty(tokens, self.width, dtype=torch.float32)
+        if self.norm is not None:
+            return rt.ops.embed_norm(ids, self.table, self.norm.weight, self.norm.eps, out, self.scale)
+        return rt.ops.embed(ids, self.table, out, self.scale)
 
 
 class PairHashEmbedding(Part):

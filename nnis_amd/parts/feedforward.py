@@ -108,7 +108,13 @@ class RoutedFeedForward(FeedForward):
         out = sum over chosen e of s_e * expert_e(x),            expert_e(x) = x for the last ``identity`` outputs
 
     The weights are the scores themselves, not renormalised; ``correction`` (a tensor's name or None) enters the
-    choice only.  ``groups`` (count, keep): the outputs, identity outputs included, form ``count`` equal groups of
+    choice only.  ``scoring="chosen_softmax"``: chosen are the ``top`` largest logits instead, and the weights are the
+    softmax over the chosen logits alone; ``router_bias`` (a name): joins the logits.  ``activation="clamped_swiglu"``:
+    down_e(a sigmoid(1.702 a) (u + 1)), a = min(gate_e x, limit), u = up_e x held within plus or minus ``limit`` (None:
+    not held).  ``shared`` (``inner``, ``limit``, ``gate``, ``up``, ``down``): one more expert of the same form, with an
+    inner size and a limit of its own, that every token uses with weight one.
+
+    ``groups`` (count, keep): the outputs, identity outputs included, form ``count`` equal groups of
     neighbours; a group's mark is its largest corrected score, and only outputs of the ``keep`` groups with the largest
     marks can be chosen.  The experts' up projections are one product over all experts, gated row by row with the
     scores (zero for the experts not chosen) before one down projection over all of them."""
@@ -116,14 +122,22 @@ class RoutedFeedForward(FeedForward):
     graph_safe = True
 
     def __init__(self, width, inner, experts, top, router, up, down, identity=0, correction=None, activation="relu_squared", gate=None,
-                 groups=None):
+                 groups=None, scoring="softmax", router_bias=None, limit=None, shared=None):
         """``up``, ``down`` and ``gate``: names with ``{}`` in the expert's place."""
         self.width, self.inner, self.experts, self.top, self.identity = int(width), int(inner), int(experts), int(top), int(identity or 0)
         if min(self.width, self.inner, self.experts, self.top) <= 0 or self.identity < 0 or self.top > self.experts + self.identity:
             raise InvalidInput(f"a router of {experts} experts and {identity} identity outputs cannot choose {top}")
-        if activation not in ("relu_squared", "silu_gated") or (activation == "silu_gated") != (gate is not None):
-            raise InvalidInput(f"experts are relu_squared, or silu_gated with gate projections; got {activation!r}")
-        self.activation = activation
+        if activation not in ("relu_squared", "silu_gated", "clamped_swiglu") or (activation != "relu_squared") != (gate is not None):
+            raise InvalidInput(f"experts are relu_squared, or silu_gated or clamped_swiglu with gate projections; got {activation!r}")
+        self.activation, self.limit = activation, 0.0 if limit is None else float(limit)
+        if scoring not in ("softmax", "chosen_softmax"):
+            raise InvalidInput(f"a router weighs by softmax or chosen_softmax; got {scoring!r}")
+        if self.limit < 0.0 or (limit is not None and (activation != "clamped_swiglu" or self.limit == 0.0)):
+            raise InvalidInput(f"a positive limit belongs to clamped_swiglu experts; got {limit!r} with {activation!r}")
+        self.scoring = scoring
+        self.shared = None if shared is None else dict(shared, inner=int(shared["inner"]), limit=float(shared.get("limit") or 0.0))
+        if self.shared is not None and (activation == "relu_squared" or self.shared["inner"] <= 0):
+            raise InvalidInput("a shared expert has the form of gated experts and a size of its own")
         self.groups = None
         if groups is not None and int(groups[0]) > 1:
             count, keep = int(groups[0]), int(groups[1])
@@ -131,13 +145,19 @@ class RoutedFeedForward(FeedForward):
             if outputs % count or not 1 <= keep <= count or self.top > keep * (outputs // count):
                 raise InvalidInput(f"{outputs} router outputs in {count} equal groups of which {keep} are kept cannot choose {top}")
             self.groups = (count, keep)
-        self.names = {"router": router, "up": up, "down": down, "correction": correction, "gate": gate}
+        self.names = {"router": router, "up": up, "down": down, "correction": correction, "gate": gate, "router_bias": router_bias}
 
     def tensors(self):
         n, outputs = self.names, self.experts + self.identity
         out = [TensorSpec(n["router"], (outputs, self.width), init="router")]
         if n["correction"]:
             out.append(TensorSpec(n["correction"], (outputs,), init="small"))
+        if n["router_bias"]:
+            out.append(TensorSpec(n["router_bias"], (outputs,), init="small"))
+        if self.shared is not None:
+            inner = self.shared["inner"]
+            out += [TensorSpec(self.shared["gate"], (inner, self.width)), TensorSpec(self.shared["up"], (inner, self.width)),
+                    TensorSpec(self.shared["down"], (self.width, inner))]
         for e in range(self.experts):
             if n["gate"]:
                 out.append(TensorSpec(n["gate"].format(e), (self.inner, self.width)))
@@ -154,9 +174,14 @@ class RoutedFeedForward(FeedForward):
         self.router = weights[n["router"]].float().contiguous()  # its logits are a 32-bit product under either runtime
         self.correction = weights[n["correction"]].float().contiguous() if n["correction"] else None
         # one product over all experts: expert by expert its up rows (behind its gate rows, where it has them)
+        self.router_bias = weights[n["router_bias"]].float().contiguous() if n["router_bias"] else None
         rows = [weights[name.format(e)] for e in range(self.experts) for name in ((n["gate"], n["up"]) if n["gate"] else (n["up"],))]
+        columns = [weights[n["down"].format(e)] for e in range(self.experts)]
+        if self.shared is not None:  # (its rows and columns lie behind the experts')
+            rows += [weights[self.shared["gate"]], weights[self.shared["up"]]]
+            columns.append(weights[self.shared["down"]])
         self.up = Projection(torch.cat(rows, dim=0), rt)
-        self.down = Projection(torch.cat([weights[n["down"].format(e)] for e in range(self.experts)], dim=1), rt)
+        self.down = Projection(torch.cat(columns, dim=1), rt)
 
     def weight_bytes(self):
         return self.up.weight_bytes() + self.down.weight_bytes() + self.router.numel() * 4
@@ -167,13 +192,21 @@ class RoutedFeedForward(FeedForward):
         """With ``share_later`` and identity outputs: returns (y, (keep, x)), where the output is y + keep[row] * x[row]."""
         tokens = x.shape[0]
         gates, keep = rt.empty(tokens, self.experts, dtype=torch.float32), rt.empty(tokens, dtype=torch.float32)
+        rule = dict(groups=self.groups, bias=self.router_bias, chosen_softmax=self.scoring == "chosen_softmax")
         if self.width <= rt.ops.ROUTE_FUSED_MOST_CHANNELS:
-            rt.ops.route(x, self.router, self.correction, self.experts, self.top, gates, keep, groups=self.groups)
+            rt.ops.route(x, self.router, self.correction, self.experts, self.top, gates, keep, **rule)
         else:
             logits = rt.ops.router_logits(x, self.router, rt.empty(tokens, self.experts + self.identity, dtype=torch.float32))
-            rt.ops.route_top(logits, self.correction, self.experts, self.top, gates, keep, groups=self.groups)
+            rt.ops.route_top(logits, self.correction, self.experts, self.top, gates, keep, **rule)
         z = self.up(x, rt)
-        y = self.down(rt.ops.routed_act(z, gates, rt.empty(tokens, self.experts * self.inner), self.activation), rt)
+        inner, extra = self.experts * self.inner, 0 if self.shared is None else self.shared["inner"]
+        hidden = rt.empty(tokens, inner + extra)
+        if not extra:
+            rt.ops.routed_act(z, gates, hidden, self.activation, self.limit)
+        else:
+            rt.ops.routed_act(z[:, :2 * inner], gates, hidden[:, :inner], self.activation, self.limit, inner=self.inner)
+            rt.ops.routed_act(z[:, 2 * inner:], None, hidden[:, inner:], self.activation, self.shared["limit"], inner=extra)
+        y = self.down(hidden, rt)
         if self.identity and share_later:
             return y, (keep, x)
         if self.identity:
