@@ -51,6 +51,14 @@ over a cached latent in a window with a gate element by element; experts chosen
 among groups; RMS norms before and after every sublayer) beside a Zifunex of
 the same width, layers, heads, state sizes, inner size and vocabulary.
 
+``--workload tonanex`` measures the Tonanex design (windowed attention whose
+heads are normed without a weight, with a temperature, scores that fall with
+the logarithm of the distance and a gate a head; clamped experts weighted over
+the chosen logits beside a shared expert; RMS norms before every sublayer)
+beside a Robopel of windowed attention layers and routed feed-forwards of the
+same width, layers, heads, window and vocabulary, its inner sizes chosen so
+that both have the same number of weights.
+
 Peaks used for the fractions are the published MI355X ones: HBM 8 TB/s; dense
 matrix rate 2.5 PFLOP/s for bfloat16, 157.3 TFLOP/s for 32-bit.
 """
@@ -195,7 +203,7 @@ def decode_run(shape, rng, batch, steps, warmup, prompt_min, prompt_max, windows
     finish(pending)
     sync()
     each = sorted(marks[i].elapsed_time(marks[i + 1]) for i in range(spread)) or [1000.0 * seconds / steps]
-    step_bytes = engine.model.step_weight_bytes() + engine.cache.bytes_per_token() * context_tokens
+    step_bytes = engine.model.step_weight_bytes(batch) + engine.cache.bytes_per_token() * context_tokens
     del engine, selector
     torch.cuda.empty_cache()
     per_step = seconds / steps
@@ -233,7 +241,7 @@ def prefill_run(shape, rng, tokens=2048):
     torch.cuda.empty_cache()
     seconds = sorted(times[3:])[3]  # the median of seven runs of a shape that has come before (and is captured, where it is)
     flops = {"Zifunex": zifunex_step_flops, "Mutedra": mutedra_step_flops, "Robopel": robopel_step_flops,
-             "Mafalorn": mafalorn_step_flops}.get(shape.config.get("architecture"), step_flops)(
+             "Mafalorn": mafalorn_step_flops, "Tonanex": tonanex_step_flops}.get(shape.config.get("architecture"), step_flops)(
         shape.config, [tokens], 1)
     return {"value": round(tokens / seconds, 1), "tokens": tokens, "ms": round(1000.0 * seconds, 3),
             "frac": round(flops / seconds / FLOP_PEAK[shape.dtype], 5), "first_ms": round(1000.0 * times[0], 3)}
@@ -436,8 +444,8 @@ def robopel_step_flops(config, tokens_per_sequence, wanted_rows):
             if layer["type"] == "attention":
                 own = 0 if m.get("kv_from") is not None else m["kv_heads"] * (m["dim"] + m["vdim"])
                 per_token = (m["heads"] * m["dim"] + own + 2 * m["heads"] * m["vdim"]) * w
-                size, pool = m["mask"]["size"], m["mask"]["pool"]
-                keys = sum(min(i + 1, size) + max(0, i + 1 - size) // pool for i in range(n))
+                size, pool = m["mask"]["size"], m["mask"].get("pool")
+                keys = sum(min(i + 1, size) + (max(0, i + 1 - size) // pool if pool else 0) for i in range(n))
                 total += 2 * per_token * n + 2 * m["heads"] * (m["dim"] + m["vdim"]) * keys
             else:
                 total += 2 * 4 * m["width"] * w * n
@@ -446,7 +454,7 @@ def robopel_step_flops(config, tokens_per_sequence, wanted_rows):
                 total += 2 * 2 * w * mlp["ff"] * n
             elif mlp is not None:
                 router = mlp["router"]
-                total += 2 * (2 * w * mlp["expert"]["ff"] * router["top"] + (router["experts"] + router["identity"]) * w) * n
+                total += 2 * (2 * w * mlp["expert"]["ff"] * router["top"] + (router["experts"] + router.get("identity", 0)) * w) * n
     return total + 2 * wanted_rows * w * config["vocab"]
 
 
@@ -545,6 +553,57 @@ def mafalorn_twin_config(sizes):
     return config
 
 
+# Tonanex at two sets of layer sizes: D = a dense feed-forward, M = experts (experts, chosen, inner size, the shared
+# expert's inner size); every layer attention in a window.
+TONANEX_SETS = {
+    "w1024": dict(width=1024, ff=2816, attention=(16, 4, 64, 64), window=512, moe=(16, 2, 352, 704)),
+    "w2048": dict(width=2048, ff=5632, attention=(16, 4, 128, 128), window=1024, moe=(16, 2, 704, 1408)),
+}
+TONANEX_LAYERS = "DMMMMMMM"
+
+
+def tonanex_config(sizes):
+    heads, kv_heads, dim, vdim = sizes["attention"]
+    experts, top, expert_ff, shared_ff = sizes["moe"]
+    mixer = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": dim ** -0.5, "mask": {"size": sizes["window"]}}
+    mlps = {"D": {"kind": "dense", "ff": sizes["ff"]},
+            "M": {"kind": "moe", "expert": {"ff": expert_ff, "limit": 7.0}, "router": {"experts": experts, "top": top},
+                  "shared": {"ff": shared_ff, "limit": 7.0}}}
+    return {"architecture": "Tonanex", "vocab": ZIFUNEX_VOCAB, "width": sizes["width"], "norm": {"eps": 1e-6}, "logit_softcap": 30.0,
+            "layers": [{"type": "attention", "mixer": mixer, "mlp": mlps[kind]} for kind in TONANEX_LAYERS]}
+
+
+def tonanex_step_flops(config, tokens_per_sequence, wanted_rows):
+    """Multiply-adds x2 of one step over whole prompts from empty slots: the projections, a window's keys, and of the
+    experts those that a token has chosen, and the shared one."""
+    w = config["width"]
+    total = 0
+    for n in tokens_per_sequence:
+        for layer in config["layers"]:
+            m, mlp = layer["mixer"], layer["mlp"]
+            per_token = (m["heads"] * (m["dim"] + m["vdim"] + 1) + m["kv_heads"] * (m["dim"] + m["vdim"])) * w
+            keys = sum(min(i + 1, m["mask"]["size"]) for i in range(n))
+            total += 2 * per_token * n + 2 * m["heads"] * (m["dim"] + m["vdim"]) * keys
+            if mlp["kind"] == "dense":
+                total += 2 * 3 * w * mlp["ff"] * n
+            else:
+                total += 2 * (3 * w * (mlp["expert"]["ff"] * mlp["router"]["top"] + mlp["shared"]["ff"]) + mlp["router"]["experts"] * w) * n
+    return total + 2 * wanted_rows * w * config["vocab"]
+
+
+def tonanex_twin_config(sizes):
+    """The closest model the library had: a Robopel of windowed attention layers (normed heads, a sink, gates) whose
+    feed-forwards, of two matrices an expert instead of three, have as many weights between them."""
+    heads, kv_heads, dim, vdim = sizes["attention"]
+    experts, top, expert_ff, shared_ff = sizes["moe"]
+    mixer = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": dim ** -0.5, "mask": {"size": sizes["window"]}}
+    inner = (3 * (experts * expert_ff + shared_ff) // (2 * experts) + 8) // 16 * 16
+    mlps = {"D": {"kind": "dense", "ff": 3 * sizes["ff"] // 2},
+            "M": {"kind": "moe", "expert": {"ff": inner}, "router": {"experts": experts, "top": top}}}
+    return {"architecture": "Robopel", "vocab": ZIFUNEX_VOCAB, "width": sizes["width"], "norm": {"eps": 1e-6}, "embedding": {"scale": 8.0},
+            "layers": [{"type": "attention", "mixer": mixer, "mlp": mlps[kind]} for kind in TONANEX_LAYERS]}
+
+
 def design_run(args, rng, design, sets, config_of, twin_of, twin="llama"):
     """Each set of sizes: the design's model and its Llama twin, a prompt of 2,048 tokens and decode at batch 1, 8, 64."""
     import torch
@@ -597,7 +656,7 @@ def main() -> int:
     parser.add_argument("--no-other-shapes", action="store_true", help="points of the headline's shape only")
     parser.add_argument("--prompt-min", type=int, default=128, help="shortest prompt of the decode batches")
     parser.add_argument("--prompt-max", type=int, default=2048, help="longest prompt of the decode batches (within the context)")
-    parser.add_argument("--workload", choices=["tinyllama-ragged", "zifunex", "mutedra", "robopel", "mafalorn"], help="run this workload alone")
+    parser.add_argument("--workload", choices=["tinyllama-ragged", "zifunex", "mutedra", "robopel", "mafalorn", "tonanex"], help="run this workload alone")
     args = parser.parse_args()
     if args.gpus != 1:
         print(f"bench.py: this library runs on one GPU; --gpus {args.gpus} is not supported")
@@ -651,6 +710,18 @@ def main() -> int:
             "ms_per_step": head["ms_per_step"], "higher_is_better": True, "dtype": "bf16" if args.dtype == "bfloat16" else "fp32",
             "data": "synthetic: random weights from a seed, uniform-random token ids",
             "config": {"model": "Mafalorn, 8 layers of width 2048 (decode at batch 8)", "sets": MAFALORN_SETS, "layers": MAFALORN_LAYERS,
+                       "vocab": ZIFUNEX_VOCAB, "context": ZIFUNEX_CONTEXT, "prompt_min": args.prompt_min, "prompt_max": args.prompt_max},
+            "models": models, "env": environment()}))
+        return 0
+    if args.workload == "tonanex":
+        models = design_run(args, rng, "tonanex", TONANEX_SETS, tonanex_config, tonanex_twin_config, twin="robopel")
+        head = models["tonanex-w2048"]["decode_b8"]
+        print(json.dumps({
+            "metric": "Tonanex at two sets of layer sizes beside a Robopel of windowed attention of the same sizes: prefill of 2,048 tokens, decode at batch 1, 8, 64",
+            "value": head["tokens_per_second"], "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
+            "ms_per_step": head["ms_per_step"], "higher_is_better": True, "dtype": "bf16" if args.dtype == "bfloat16" else "fp32",
+            "data": "synthetic: random weights from a seed, uniform-random token ids",
+            "config": {"model": "Tonanex, 8 layers of width 2048 (decode at batch 8)", "sets": TONANEX_SETS, "layers": TONANEX_LAYERS,
                        "vocab": ZIFUNEX_VOCAB, "context": ZIFUNEX_CONTEXT, "prompt_min": args.prompt_min, "prompt_max": args.prompt_max},
             "models": models, "env": environment()}))
         return 0

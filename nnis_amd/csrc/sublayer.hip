@@ -342,6 +342,8 @@ struct RouteRule {
   const float* bias;
   const float* correction;
   int chosen_softmax, group_count, group_keep;
+  int* chosen;     // [rows, top] or null: the chosen outputs, best first
+  float* weights;  // [rows, top], with `chosen`: their weights
 };
 
 __device__ __forceinline__ void route_row(const float* logits, const RouteRule& rule, int row, int n, int experts, int top,
@@ -410,6 +412,8 @@ __device__ __forceinline__ void route_row(const float* logits, const RouteRule& 
   }
   float kept = 0.0f;
   float weight = 0.0f;  // of this lane's chosen outputs together
+  int picked = 0;       // lane i: the i-th choice and its weight
+  float picked_weight = 0.0f;
   for (int round = 0; round < top; ++round) {
     float best = -INFINITY;
     int best_e = 0x7fffffff;
@@ -431,15 +435,24 @@ __device__ __forceinline__ void route_row(const float* logits, const RouteRule& 
       }
     }
     if (best_e == 0x7fffffff) break;  // fewer outputs than `top`
+    float mine = 0.0f;
     if (best_e % kWave == lane) {
       const int i = best_e / kWave;
       chosen |= 1u << i;
 #pragma unroll
       for (int k = 0; k < kRouteMost; ++k)
         if (k == i) {
+          mine = s[k];
           weight += s[k];
           if (best_e >= experts) kept += s[k];
         }
+    }
+    if (rule.chosen) {
+      mine = __shfl(mine, best_e % kWave, kWave);
+      if (round == lane) {
+        picked = best_e;
+        picked_weight = mine;
+      }
     }
   }
   const float share = rule.chosen_softmax ? 1.0f / wave_sum(weight) : 1.0f;
@@ -447,6 +460,10 @@ __device__ __forceinline__ void route_row(const float* logits, const RouteRule& 
   for (int i = 0; i < kRouteMost; ++i) {
     const int e = i * kWave + lane;
     if (e < experts) gates[(size_t)row * experts + e] = (chosen >> i & 1u) ? s[i] * share : 0.0f;
+  }
+  if (rule.chosen && lane < top) {  // (the host asks for them for up to a wave's lanes of choices)
+    rule.chosen[(size_t)row * top + lane] = picked;
+    rule.weights[(size_t)row * top + lane] = picked_weight * share;
   }
   kept = wave_sum(kept) * share;
   if (lane == 0) keep[row] = kept;
@@ -515,6 +532,84 @@ __global__ __launch_bounds__(R == 1 ? 1024 : 256) void route_kernel(const void* 
   const int wave = threadIdx.x / kWave;
   if (wave < R && row0 + wave < rows)
     route_row(lg + wave * n, rule, row0 + wave, n, experts, top, gates, keep, threadIdx.x % kWave);
+}
+
+// The same behind an RMS norm of the 32-bit stream, in one kernel: x[row] (+ delta[row], summed into x), its norm with
+// weight `gain` as floats into LDS and in the activation type to h, the router's logits and choice from the floats.
+// R rows a block; with R == 1 all waves norm the row together, else wave r norms row r.
+struct RouteNormArgs {
+  float* x;
+  const void* delta;  // null: nothing to add
+  int delta_dtype;
+  const void* gain;
+  int gain_dtype;
+  float eps;
+  void* h;
+  int h_dtype;
+};
+
+template <int R>
+__global__ __launch_bounds__(R == 1 ? 1024 : 64 * R) void route_norm_kernel(RouteNormArgs a, const float* __restrict__ w, RouteRule rule, int rows, int n,
+                                                                       int width, int experts, int top, float* __restrict__ gates,
+                                                                       float* __restrict__ keep) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];  // [R][width] rows, then [R][n] logits
+  __shared__ float scratch[16];
+  float* lg = lds + (size_t)R * width;
+  const int row0 = blockIdx.x * R;
+  const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
+  const int first = R == 1 ? threadIdx.x : lane, step = R == 1 ? blockDim.x : kWave;
+  const int mine = R == 1 ? 0 : wave, row = row0 + mine;  // the row this thread norms
+  float* xs = lds + (size_t)mine * width;
+  const bool live = row < rows;
+  const size_t base = (size_t)(live ? row : rows - 1) * width;
+  float ss = 0.0f;
+  if (width % 4 == 0) {
+    for (int c = 4 * first; c < width; c += 4 * step) {
+      float4 v = *(const float4*)(a.x + base + c);
+      if (a.delta) {
+        v.x += load_as_f32(a.delta, a.delta_dtype, base + c);
+        v.y += load_as_f32(a.delta, a.delta_dtype, base + c + 1);
+        v.z += load_as_f32(a.delta, a.delta_dtype, base + c + 2);
+        v.w += load_as_f32(a.delta, a.delta_dtype, base + c + 3);
+        if (live) *(float4*)(a.x + base + c) = v;
+      }
+      *(float4*)(xs + c) = v;
+      ss = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, ss))));
+    }
+  } else {
+    for (int c = first; c < width; c += step) {
+      float v = a.x[base + c];
+      if (a.delta) {
+        v += load_as_f32(a.delta, a.delta_dtype, base + c);
+        if (live) a.x[base + c] = v;
+      }
+      xs[c] = v;
+      ss = fmaf(v, v, ss);
+    }
+  }
+  const float inv = 1.0f / sqrtf((R == 1 ? block_sum(ss, scratch) : wave_sum(ss)) / (float)width + a.eps);
+  if (width % 4 == 0) {
+    for (int c = 4 * first; c < width; c += 4 * step) {
+      float4 v = *(const float4*)(xs + c);
+      v.x *= inv * load_as_f32(a.gain, a.gain_dtype, c);
+      v.y *= inv * load_as_f32(a.gain, a.gain_dtype, c + 1);
+      v.z *= inv * load_as_f32(a.gain, a.gain_dtype, c + 2);
+      v.w *= inv * load_as_f32(a.gain, a.gain_dtype, c + 3);
+      *(float4*)(xs + c) = v;
+      if (live && a.h_dtype == NNIS_F32) *(float4*)((float*)a.h + base + c) = v;
+      else if (live) store4((bf16_t*)a.h + base + c, v);
+    }
+  } else {
+    for (int c = first; c < width; c += step) {
+      const float v = xs[c] * inv * load_as_f32(a.gain, a.gain_dtype, c);
+      xs[c] = v;
+      if (live) store_from_f32(a.h, a.h_dtype, base + c, v);
+    }
+  }
+  __syncthreads();
+  router_dots<R>(lds, w, lg, n, width);
+  __syncthreads();
+  if (wave < R && row0 + wave < rows) route_row(lg + wave * n, rule, row0 + wave, n, experts, top, gates, keep, lane);
 }
 
 // the logits alone, to global memory [rows, n]
@@ -969,7 +1064,9 @@ extern "C" int nnis_router_logits(const void* x, int x_dtype, const float* w, fl
 }
 
 extern "C" int nnis_route(const void* x, int x_dtype, const float* w, const float* bias, const float* correction, int rows, int n, int width,
-                          int experts, int top, int chosen_softmax, float* gates, float* keep, int group_count, int group_keep, void* stream) {
+                          int experts, int top, int chosen_softmax, float* gates, float* keep, int* chosen, float* weights, int group_count,
+                          int group_keep, void* stream) {
+  NNIS_REQUIRE((chosen == nullptr) == (weights == nullptr) && (chosen == nullptr || top <= kWave), "route: up to %d choices are listed", kWave);
   NNIS_REQUIRE(x && w && gates && keep && n > 0 && width > 0, "route: missing operand");
   NNIS_REQUIRE(group_count >= 1 && group_count <= kWave && n % group_count == 0 && group_keep >= 1 && group_keep <= group_count,
                "route: %d outputs in %d groups (up to %d, equal ones) of which %d are kept", n, group_count, kWave, group_keep);
@@ -983,7 +1080,7 @@ extern "C" int nnis_route(const void* x, int x_dtype, const float* w, const floa
   const size_t lds = (size_t)together * (width + n) * sizeof(float);
   const dim3 grid((rows + together - 1) / together);
   hipStream_t s = (hipStream_t)stream;
-  const RouteRule rule = {bias, correction, chosen_softmax ? 1 : 0, group_count, group_keep};
+  const RouteRule rule = {bias, correction, chosen_softmax ? 1 : 0, group_count, group_keep, chosen, weights};
   if (together == 4) {
     hipLaunchKernelGGL((route_kernel<4>), grid, dim3(256), lds, s, x, x_dtype, w, rule, rows, n, width, experts, top, gates, keep);
   } else if (together == 2) {
@@ -997,6 +1094,38 @@ extern "C" int nnis_route(const void* x, int x_dtype, const float* w, const floa
   return 0;
 }
 
+// see RouteNormArgs; chosen (null, or [rows, top] for up to 64 choices) and weights: the choices as a list beside the gates
+extern "C" int nnis_route_norm(float* x, const void* delta, int delta_dtype, const void* gain, int gain_dtype, float eps, void* h, int h_dtype,
+                               const float* w, const float* bias, const float* correction, int rows, int n, int width, int experts, int top,
+                               int chosen_softmax, float* gates, float* keep, int* chosen, float* weights, int group_count, int group_keep,
+                               void* stream) {
+  NNIS_REQUIRE(x && gain && h && w && gates && keep && n > 0 && width > 0, "route_norm: missing operand");
+  NNIS_REQUIRE(group_count >= 1 && group_count <= kWave && n % group_count == 0 && group_keep >= 1 && group_keep <= group_count,
+               "route_norm: %d outputs in %d groups (up to %d, equal ones) of which %d are kept", n, group_count, kWave, group_keep);
+  NNIS_REQUIRE(nnis_dtype_ok(gain_dtype) && nnis_dtype_ok(h_dtype) && (delta == nullptr || nnis_dtype_ok(delta_dtype)), "route_norm: unknown dtype");
+  NNIS_REQUIRE(n <= kWave * kRouteMost && width <= 8192, "route_norm: up to %d outputs of rows of up to 8192 channels, got %d and %d",
+               kWave * kRouteMost, n, width);
+  NNIS_REQUIRE(experts >= 0 && experts <= n && top > 0 && top <= n, "route_norm: %d experts and the %d largest of %d outputs", experts, top, n);
+  NNIS_REQUIRE((chosen == nullptr) == (weights == nullptr) && (chosen == nullptr || top <= kWave), "route_norm: up to %d choices are listed", kWave);
+  if (rows <= 0) return 0;
+  const int together = rows <= 256 ? 1 : ((size_t)4 * (width + n) * 4 <= 49152 ? 4 : ((size_t)2 * (width + n) * 4 <= 49152 ? 2 : 1));
+  const size_t lds = (size_t)together * (width + n) * sizeof(float);
+  const dim3 grid((rows + together - 1) / together);
+  hipStream_t s = (hipStream_t)stream;
+  const RouteRule rule = {bias, correction, chosen_softmax ? 1 : 0, group_count, group_keep, chosen, weights};
+  const RouteNormArgs a = {x, delta, delta_dtype, gain, gain_dtype, eps, h, h_dtype};
+  if (together == 4) {
+    hipLaunchKernelGGL((route_norm_kernel<4>), grid, dim3(256), lds, s, a, w, rule, rows, n, width, experts, top, gates, keep);
+  } else if (together == 2) {
+    hipLaunchKernelGGL((route_norm_kernel<2>), grid, dim3(128), lds, s, a, w, rule, rows, n, width, experts, top, gates, keep);
+  } else {
+    const int threads = n > 8 ? 1024 : (n > 4 ? 512 : 256);
+    hipLaunchKernelGGL((route_norm_kernel<1>), grid, dim3(threads), lds, s, a, w, rule, rows, n, width, experts, top, gates, keep);
+  }
+  NNIS_LAUNCH_CHECK("route_norm");
+  return 0;
+}
+
 extern "C" int nnis_route_top(const float* logits, const float* bias, const float* correction, int rows, int n, int experts, int top,
                               int chosen_softmax, float* gates, float* keep, int group_count, int group_keep, void* stream) {
   NNIS_REQUIRE(logits && gates && keep, "route_top: missing operand");
@@ -1005,7 +1134,7 @@ extern "C" int nnis_route_top(const float* logits, const float* bias, const floa
   NNIS_REQUIRE(n > 0 && n <= kWave * kRouteMost, "route_top: 1 to %d router outputs, got %d", kWave * kRouteMost, n);
   NNIS_REQUIRE(experts >= 0 && experts <= n && top > 0 && top <= n, "route_top: %d experts and the %d largest of %d outputs", experts, top, n);
   if (rows <= 0) return 0;
-  const RouteRule rule = {bias, correction, chosen_softmax ? 1 : 0, group_count, group_keep};
+  const RouteRule rule = {bias, correction, chosen_softmax ? 1 : 0, group_count, group_keep, nullptr, nullptr};
   hipLaunchKernelGGL(route_top_kernel, dim3((rows + 3) / 4), dim3(256), 0, (hipStream_t)stream, logits, rule, rows, n, experts, top, gates,
                      keep);
   NNIS_LAUNCH_CHECK("route_top");

@@ -62,7 +62,9 @@ PREBUILT_WIDE_VALUES = ("attn_hd7v5c", "attn_hd32v16c", "attn_hd16v48c", "attn_h
                         "attn_hd24v40x", "attn_hd24v40cx", "attn_hd24v40xp", "attn_hd24v40cxp", "attn_hd16cx", "attn_hd16xp", "attn_hd16cxp",
                         "attn_hd20v12xp", "attn_hd32xp", "attn_hd64cxp", "attn_hd128cxp",
                         # latents as the one key/value head without any extras, in a window or not: the tests' sizes and the measurements'
-                        "attn_hd48v40", "attn_hd64v48", "attn_hd32v24", "attn_hd20v16", "attn_hd160v128", "attn_hd256v192")
+                        "attn_hd48v40", "attn_hd64v48", "attn_hd32v24", "attn_hd20v16", "attn_hd160v128", "attn_hd256v192",
+                        # scores that fall with the logarithm of the distance and gated heads: the tests' sizes and the measurements'
+                        "attn_hd32v16lg", "attn_hd16v48lg", "attn_hd24v40lg", "attn_hd16lg", "attn_hd32v16clgx", "attn_hd64lg", "attn_hd128lg")
 
 _loaded: Dict[str, ctypes.CDLL] = {}
 _lock = threading.Lock()
@@ -155,7 +157,7 @@ def _attention_recipe(rest: str) -> ModuleRecipe:
 
 # the library's own modules: ``core`` holds the kernels whose sizes are run-time arguments; attention is compiled per head size
 register_module("core", ["elementwise.hip", "residual.hip", "gemm.hip", "gemm_mfma.hip", "gemm_fused.hip", "sampling.hip"],
-                headers=["common.h", "epilogue.h", "nnis_noalloc.h"], source_flags={"gemm_mfma.hip": _VECTOR_SUMS})
+                headers=["common.h", "epilogue.h", "product.h", "nnis_noalloc.h"], source_flags={"gemm_mfma.hip": _VECTOR_SUMS})
 register_module_family("attn_hd", _attention_recipe)
 # the mixers that carry a state of fixed size (convolution, selective scan, gated linear attention and retention, minGRU, gated delta rule)
 register_module("recurrent", ["recurrent.hip"], headers=["common.h"])
@@ -163,6 +165,8 @@ register_module("recurrent", ["recurrent.hip"], headers=["common.h"])
 register_module("latent", ["latent.hip"], headers=["common.h"])
 # what lies between the projections of sublayers that norm their outputs, gate or pool their heads, or route their tokens
 register_module("sublayer", ["sublayer.hip"], headers=["common.h"])
+# the products of a routed feed-forward over the experts that the router chose
+register_module("experts", ["experts.hip"], headers=["common.h", "product.h"], source_flags={"experts.hip": _VECTOR_SUMS})
 # plain host references of the kernels' operations, for the tests (no device code: the host compiler builds them)
 register_module("reference", ["reference.cpp"], host_only=True)
 HOST_FLAGS = ["-O2", "-std=c++17", "-fPIC", "-ffp-contract=off"]  # a multiply-add is fused only where the source says fmaf
@@ -336,7 +340,7 @@ def load_module(module: str, build_if_missing: bool = True) -> ctypes.CDLL:
 
 
 def all_prebuilt_modules() -> List[str]:
-    return ["core", "reference", "recurrent", "latent", "sublayer"] + [f"attn_hd{d}" for d in PREBUILT_HEAD_DIMS] + list(PREBUILT_WIDE_VALUES)
+    return ["core", "reference", "recurrent", "latent", "sublayer", "experts"] + [f"attn_hd{d}" for d in PREBUILT_HEAD_DIMS] + list(PREBUILT_WIDE_VALUES)
 
 
 def build_all(force: bool = True, jobs: int = 4) -> List[str]:

@@ -123,7 +123,9 @@ _SUBLAYER_SIGNATURES = {
     "nnis_cast_rows": [_VOID, _INT, _VOID, _INT, _VOID, _INT, _INT, _VOID],
     "nnis_rms_post_step": [_VOID, _VOID, _INT, _VOID, _INT, _FLT, _FLT, _VOID, _INT, _INT, _INT, _VOID, _VOID, _INT, _VOID],
     "nnis_rms_between": [_VOID, _VOID, _INT, _VOID, _VOID, _INT, _FLT, _VOID, _INT, _INT, _INT, _VOID, _VOID, _INT, _VOID],
-    "nnis_route": [_VOID, _INT, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _VOID, _VOID, _INT, _INT, _VOID],
+    "nnis_route": [_VOID, _INT, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _VOID, _VOID, _VOID, _VOID, _INT, _INT, _VOID],
+    "nnis_route_norm": [_VOID, _VOID, _INT, _VOID, _INT, _FLT, _VOID, _INT, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _VOID,
+                        _VOID, _VOID, _VOID, _INT, _INT, _VOID],
     "nnis_poly_norm": [_VOID, _INT, _VOID, _FLT, _VOID, _INT, _INT, _INT, _VOID],
     "nnis_router_logits": [_VOID, _INT, _VOID, _VOID, _INT, _INT, _INT, _VOID],
     "nnis_route_top": [_VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _VOID, _VOID, _INT, _INT, _VOID],
@@ -134,6 +136,14 @@ _SUBLAYER_SIGNATURES = {
                              _VOID, _VOID, _VOID, _VOID, _INT, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _INT, _VOID, _VOID],
     "nnis_pool_blocks": [_VOID, _VOID, _INT, _VOID, _INT, _VOID, _VOID, _VOID, _INT, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT,
                          _VOID],
+}
+
+_EXPERTS_SIGNATURES = {
+    "nnis_experts_up_few": [_VOID, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _FLT, _FLT, _VOID],
+    "nnis_experts_down_few": [_VOID, _VOID, _VOID, _VOID, _VOID, _VOID, _INT, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _VOID],
+    "nnis_experts_lists": [_VOID, _INT, _INT, _INT, _VOID, _VOID, _VOID],
+    "nnis_experts_many": [_INT, _VOID, _VOID, _VOID, _VOID, _VOID, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _INT, _FLT, _FLT, _VOID],
+    "nnis_experts_combine": [_VOID, _VOID, _VOID, _VOID, _VOID, _INT, _VOID, _VOID, _INT, _INT, _INT, _VOID],
 }
 
 _LATENT_SIGNATURES = {
@@ -216,6 +226,7 @@ def latent():
 
 
 _sublayer = None
+_experts = None
 
 
 def sublayer():
@@ -225,6 +236,14 @@ def sublayer():
     if _sublayer is None:
         _sublayer = _bind("sublayer", _SUBLAYER_SIGNATURES)
     return _sublayer
+
+
+def experts():
+    """The module of the products over chosen experts."""
+    global _experts
+    if _experts is None:
+        _experts = _bind("experts", _EXPERTS_SIGNATURES)
+    return _experts
 
 
 def core():
@@ -2221,10 +2240,11 @@ ROUTE_FUSED_MOST_CHANNELS = 8192
 
 
 def route(x: torch.Tensor, weight: torch.Tensor, correction: Optional[torch.Tensor], experts: int, top: int, gates: torch.Tensor,
-          keep: torch.Tensor, groups=None, bias: Optional[torch.Tensor] = None, chosen_softmax: bool = False):
+          keep: torch.Tensor, groups=None, bias: Optional[torch.Tensor] = None, chosen_softmax: bool = False, chosen=None):
     """``router_logits`` and ``route_top`` in one kernel (rows of up to ``ROUTE_FUSED_MOST_CHANNELS`` channels).
     ``groups``: (count, keep): the outputs form ``count`` equal groups of neighbours, a group's mark is its largest
-    corrected score, and only outputs of the ``keep`` groups with the largest marks can be chosen."""
+    corrected score, and only outputs of the ``keep`` groups with the largest marks can be chosen.  ``chosen``: (int32 [rows, top],
+    float32 [rows, top]) that take the choices and their weights as lists, best first."""
     _dev(x, "x"), _dev(weight, "router weight"), _dev(gates, "gates"), _dev(keep, "keep")
     rows, width = x.shape
     n = weight.shape[0]
@@ -2241,8 +2261,55 @@ def route(x: torch.Tensor, weight: torch.Tensor, correction: Optional[torch.Tens
     group_count, group_keep = _route_groups(groups, n, "route")
     lib = sublayer()
     _check(lib, lib.nnis_route(x.data_ptr(), _code(x), weight.data_ptr(), _ptr(bias), _ptr(correction), rows, n, width, experts, top,
-                               1 if chosen_softmax else 0, gates.data_ptr(), keep.data_ptr(), group_count, group_keep, _stream()))
+                               1 if chosen_softmax else 0, gates.data_ptr(), keep.data_ptr(), *_chosen_lists(chosen, rows, top, "route"),
+                               group_count, group_keep, _stream()))
     return gates, keep
+
+
+ROUTE_MOST_LISTED = 64  # choices a row that the router's kernels list
+
+
+def _chosen_lists(chosen, rows: int, top: int, what: str):
+    if chosen is None:
+        return None, None
+    ids, weights = chosen
+    _dev(ids, "chosen"), _dev(weights, "weights")
+    if (ids.dtype != torch.int32 or weights.dtype != torch.float32 or tuple(ids.shape) != (rows, top) or tuple(weights.shape) != (rows, top)
+            or top > ROUTE_MOST_LISTED):
+        raise KernelError(f"{what}: choices as int32 [rows, top] and float32 [rows, top], up to {ROUTE_MOST_LISTED}; got {tuple(ids.shape)}")
+    return ids.data_ptr(), weights.data_ptr()
+
+
+def route_norm(x: torch.Tensor, delta: Optional[torch.Tensor], gain: torch.Tensor, eps: float, h: torch.Tensor, weight: torch.Tensor,
+               correction: Optional[torch.Tensor], experts: int, top: int, gates: torch.Tensor, keep: torch.Tensor, groups=None,
+               bias: Optional[torch.Tensor] = None, chosen_softmax: bool = False, chosen=None):
+    """``route`` behind the RMS norm of the 32-bit stream ``x`` (+ ``delta``, summed into ``x``), in one kernel: ``h`` takes
+    the normed rows, the router reads them in 32-bit."""
+    _dev(x, "x"), _dev(gain, "norm weight"), _dev(h, "h"), _dev(weight, "router weight"), _dev(gates, "gates"), _dev(keep, "keep")
+    rows, width = x.shape
+    n = weight.shape[0]
+    if (x.dtype != torch.float32 or h.shape != x.shape or gain.numel() != width or weight.dtype != torch.float32 or weight.dim() != 2
+            or weight.shape[1] != width or gates.dtype != torch.float32 or keep.dtype != torch.float32
+            or tuple(gates.shape) != (rows, experts) or keep.numel() != rows):
+        raise KernelError(f"route_norm: float32 x {tuple(x.shape)}, h {tuple(h.shape)}, weight {tuple(weight.shape)}, gates {tuple(gates.shape)}")
+    if delta is not None:
+        _dev(delta, "delta")
+        if delta.shape != x.shape:
+            raise KernelError(f"route_norm: delta {tuple(delta.shape)} against x {tuple(x.shape)}")
+    if correction is not None:
+        _dev(correction, "correction")
+        if correction.dtype != torch.float32 or correction.numel() != n:
+            raise KernelError(f"route_norm: a float32 correction per output ({n}), got {tuple(correction.shape)} {correction.dtype}")
+    if not (0 < n <= ROUTE_MOST_OUTPUTS and 0 <= experts <= n and 0 < top <= n and width <= ROUTE_FUSED_MOST_CHANNELS):
+        raise KernelError(f"route_norm: {experts} experts and the {top} largest of {n} outputs (at most {ROUTE_MOST_OUTPUTS}) of rows of {width} channels")
+    _check_router_bias(bias, n, "route_norm")
+    group_count, group_keep = _route_groups(groups, n, "route_norm")
+    lib = sublayer()
+    _check(lib, lib.nnis_route_norm(x.data_ptr(), _ptr(delta), _code(delta) if delta is not None else 0, gain.data_ptr(), _code(gain), float(eps),
+                                    h.data_ptr(), _code(h), weight.data_ptr(), _ptr(bias), _ptr(correction), rows, n, width, experts, top,
+                                    1 if chosen_softmax else 0, gates.data_ptr(), keep.data_ptr(), *_chosen_lists(chosen, rows, top, "route_norm"),
+                                    group_count, group_keep, _stream()))
+    return h
 
 
 _ROUTED_FORMS = {"relu_squared": 0, "silu_gated": 1, "clamped_swiglu": 2}
@@ -2410,3 +2477,110 @@ def min_gru(rows: torch.Tensor, z_bias: Optional[torch.Tensor], x_bias: Optional
                                  ctx.seq_start.data_ptr(), ctx.batch, width, out.data_ptr(), _code(out), piece, pieces, _ptr(decay),
                                  _ptr(ends), _stream()))
     return out
+
+
+# ---------------------------------------------------------------------------
+# the products of a routed feed-forward over the experts that were chosen
+# ---------------------------------------------------------------------------
+
+EXPERTS_MOST = 1024
+EXPERTS_FEW_ROWS = 16  # rows that the kernels for few tokens take
+
+
+class ExpertRegions:
+    """Sizes and constants of gated experts whose projections are kept as
+    regions of two packed weights: ``up`` [experts * 2 * inner + 2 * shared,
+    width], expert by expert its gate rows then its up rows, the shared
+    expert's behind them; ``down`` [width, experts * inner + shared].
+    ``inner`` and ``shared`` (0: none) are padded to steps of ``STEP``
+    channels with zeros.  ``form``: "silu_gated" or "clamped_swiglu" with the
+    limits (0: not held)."""
+
+    STEP = 64
+
+    def __init__(self, experts: int, inner: int, shared: int, form: str, limit: float, shared_limit: float):
+        self.experts, self.inner, self.shared, self.form = int(experts), int(inner), int(shared), _ROUTED_FORMS[form]
+        self.limit, self.shared_limit = float(limit), float(shared_limit)
+
+    @property
+    def hidden(self) -> int:
+        return self.experts * self.inner + self.shared
+
+    def check(self, up, down, width: int) -> None:
+        _packed(up, "experts"), _packed(down, "experts")
+        if tuple(up.shape) != (2 * self.hidden, width) or tuple(down.shape) != (width, self.hidden):
+            raise KernelError(f"experts: weights {tuple(up.shape)} and {tuple(down.shape)} do not fit {self.experts} experts of {self.inner} "
+                              f"(shared {self.shared}) on rows of {width}")
+
+
+def _into_stream(residual, gain, scaled, ss, rows: int, width: int, parts: int, what: str):
+    """The pointers of a product that ends in the residual stream, checked."""
+    for t, name in ((residual, "residual"), (gain, "gain"), (scaled, "scaled"), (ss, "ss")):
+        _dev(t, name)
+    if (residual.dtype != torch.float32 or tuple(residual.shape) != (rows, width) or scaled.dtype != torch.bfloat16
+            or tuple(scaled.shape) != (rows, width) or gain.numel() != width or ss.dtype != torch.float32 or ss.numel() < parts * rows):
+        raise KernelError(f"{what}: the stream {tuple(residual.shape)}, scaled {tuple(scaled.shape)} and ss do not fit {rows} rows of {width}")
+    return [residual.data_ptr(), gain.data_ptr(), _code(gain), scaled.data_ptr(), ss.data_ptr()]
+
+
+def experts_few(x: torch.Tensor, up, down, regions: ExpertRegions, gates: torch.Tensor, out: Optional[torch.Tensor], into=None) -> int:
+    """out = the weighted sum of the chosen experts' outputs and the shared
+    one's, for up to ``EXPERTS_FEW_ROWS`` rows: two kernels that read the
+    weights of experts somebody chose (``gates`` [rows, experts], zero where
+    not) and no others.  ``into``: (residual, gain, scaled, ss) as
+    ``gemm_residual`` takes them, in place of ``out``; returns the parts of ss
+    written."""
+    _dev(x, "x"), _dev(gates, "gates")
+    rows, width = x.shape
+    regions.check(up, down, width)
+    if x.dtype != torch.bfloat16 or gates.dtype != torch.float32 or tuple(gates.shape) != (rows, regions.experts) or rows > EXPERTS_FEW_ROWS:
+        raise KernelError(f"experts_few: bfloat16 x {tuple(x.shape)} (up to {EXPERTS_FEW_ROWS} rows) and float32 gates {tuple(gates.shape)}")
+    parts = (width + 15) // 16
+    if into is not None:
+        ends = [None] + _into_stream(*into, rows, width, parts, "experts_few")
+    else:
+        _dev(out, "out")
+        if out.dtype != torch.bfloat16 or tuple(out.shape) != (rows, width):
+            raise KernelError(f"experts_few: out {tuple(out.shape)} {out.dtype}")
+        ends = [out.data_ptr(), None, None, 0, None, None]
+    hidden = torch.empty(rows, regions.hidden, dtype=torch.bfloat16, device=x.device)
+    lib = experts()
+    _check(lib, lib.nnis_experts_up_few(x.data_ptr(), up.data_ptr(), gates.data_ptr(), hidden.data_ptr(), rows, width, regions.experts,
+                                        regions.inner, regions.shared, regions.form, regions.limit, regions.shared_limit, _stream()))
+    _check(lib, lib.nnis_experts_down_few(hidden.data_ptr(), down.data_ptr(), gates.data_ptr(), *ends, rows, width, regions.experts,
+                                          regions.inner, regions.shared, regions.form, _stream()))
+    return parts
+
+
+def experts_many(x: torch.Tensor, up, down, regions: ExpertRegions, chosen: torch.Tensor, weights: torch.Tensor,
+                 out: Optional[torch.Tensor], into=None) -> int:
+    """The same for any number of rows: every expert's products run over the
+    rows that chose it (``chosen`` int32 and ``weights`` float32 [rows, top]),
+    gathered by lists that are made on the device."""
+    _dev(x, "x"), _dev(chosen, "chosen"), _dev(weights, "weights")
+    rows, width = x.shape
+    regions.check(up, down, width)
+    top = chosen.shape[1]
+    if (x.dtype != torch.bfloat16 or chosen.dtype != torch.int32 or weights.dtype != torch.float32 or chosen.shape[0] != rows
+            or weights.shape != chosen.shape or not 0 < top <= regions.experts):
+        raise KernelError(f"experts_many: bfloat16 x {tuple(x.shape)}, int32 chosen {tuple(chosen.shape)}, float32 weights {tuple(weights.shape)}")
+    if into is not None:
+        ends = [None] + _into_stream(*into, rows, width, 1, "experts_many")
+    else:
+        _dev(out, "out")
+        if out.dtype != torch.bfloat16 or tuple(out.shape) != (rows, width):
+            raise KernelError(f"experts_many: out {tuple(out.shape)} {out.dtype}")
+        ends = [out.data_ptr(), None, None, 0, None, None]
+    make = lambda *shape, dtype=torch.bfloat16: torch.empty(shape, dtype=dtype, device=x.device)  # noqa: E731
+    counts, lists = make(regions.experts, dtype=torch.int32), make(regions.experts, rows, dtype=torch.int32)
+    hidden, pairs = make(rows * top, regions.inner), make(rows * top, width)
+    hidden_shared, shared = (make(rows, regions.shared), make(rows, width)) if regions.shared else (None, None)
+    lib = experts()
+    sizes = (rows, top, width, regions.experts, regions.inner, regions.shared, regions.form, regions.limit, regions.shared_limit)
+    _check(lib, lib.nnis_experts_lists(chosen.data_ptr(), rows, top, regions.experts, counts.data_ptr(), lists.data_ptr(), _stream()))
+    _check(lib, lib.nnis_experts_many(0, x.data_ptr(), None, up.data_ptr(), hidden.data_ptr(), _ptr(hidden_shared), weights.data_ptr(),
+                                      counts.data_ptr(), lists.data_ptr(), *sizes, _stream()))
+    _check(lib, lib.nnis_experts_many(1, hidden.data_ptr(), _ptr(hidden_shared), down.data_ptr(), pairs.data_ptr(), _ptr(shared),
+                                      weights.data_ptr(), counts.data_ptr(), lists.data_ptr(), *sizes, _stream()))
+    _check(lib, lib.nnis_experts_combine(pairs.data_ptr(), _ptr(shared), *ends, rows, top, width, _stream()))
+    return 1

@@ -55,10 +55,15 @@ class DecoderModel:
                         part.adopt_packed(source, packed)
         self.bound = True
 
-    def step_weight_bytes(self) -> int:
+    def step_weight_bytes(self, rows=None) -> int:
         """Bytes of weights a decode step reads: every layer each time the
-        schedule runs it, the head, and no embedding table (a row per token)."""
-        total = sum(self.layers[entry.layer].weight_bytes() for entry in self.spec.schedule)
+        schedule runs it, the head, and no embedding table (a row per token).
+        ``rows``: the step's tokens, for parts that read by them (experts that
+        no token chose; None: all that there is)."""
+        def of(block):
+            return block.weight_bytes() if rows is None else block.weight_bytes_for(rows)
+
+        total = sum(of(self.layers[entry.layer]) for entry in self.spec.schedule)
         total += sum(part.weight_bytes() for part in self.entries.values())
         return total + self.final_norm.weight_bytes() + self.head.weight_bytes()
 

@@ -178,7 +178,10 @@ class CausalSelfAttention(Mixer):
         return KVRequest(self.kv_heads, self.head_dim, self.window, None if self.value_dim == self.head_dim else self.value_dim)
 
     def check(self, rt):
-        rt.ops.attention_check(self.head_dim, self.value_dim)
+        ops = rt.ops
+        # (normed heads wider than the matrix-core kernels carry take the row kernel, at its pace)
+        wide = self.unit_eps is not None and max(self.head_dim, self.value_dim) > ops.ATTENTION_MOST_CHANNELS
+        ops.attention_check(self.head_dim, self.value_dim, ops.ATTENTION_ROWS_MOST_CHANNELS if wide else ops.ATTENTION_MOST_CHANNELS)
         tables = self.position.rotary() if self.position is not None else None
         rot_dim = tables.rot_dim if tables is not None else getattr(self.position, "rot_dim", 0)
         if rot_dim > self.head_dim:

@@ -125,6 +125,10 @@ class Part:
         """Bytes of weights one step has to read through this part."""
         return 0
 
+    def weight_bytes_for(self, rows: int) -> int:
+        """The same for a step of ``rows`` tokens, where it depends on them."""
+        return self.weight_bytes()
+
     def check(self, rt) -> None:
         """Raises ``Unsupported`` if the kernels this part would launch under
         ``rt`` do not take its sizes.  Asked when a model is put together,

@@ -54,6 +54,9 @@ class PreNormBlock(Block):
     def weight_bytes(self):
         return sum(part.weight_bytes() for part in self._parts)
 
+    def weight_bytes_for(self, rows):
+        return sum(part.weight_bytes_for(rows) for part in self._parts)
+
     def cache_request(self):
         return self.mixer.cache_request()
 
@@ -152,6 +155,9 @@ class HyperConnectionBlock(Block):
     def weight_bytes(self):
         return sum(part.weight_bytes() for part in self._parts)
 
+    def weight_bytes_for(self, rows):
+        return sum(part.weight_bytes_for(rows) for part in self._parts)
+
     def cache_request(self):
         return self.mixer.cache_request()
 
@@ -239,6 +245,9 @@ class PrePostNormBlock(Block):
 
     def weight_bytes(self):
         return sum(part.weight_bytes() for part in self._parts)
+
+    def weight_bytes_for(self, rows):
+        return sum(part.weight_bytes_for(rows) for part in self._parts)
 
     def cache_request(self):
         return self.mixer.cache_request()
@@ -359,6 +368,9 @@ class PostNormBlock(Block):
 
     def weight_bytes(self):
         return sum(part.weight_bytes() for part in self._parts)
+
+    def weight_bytes_for(self, rows):
+        return sum(part.weight_bytes_for(rows) for part in self._parts)
 
     def cache_request(self):
         return self.mixer.cache_request()

@@ -170,42 +170,111 @@ class RoutedFeedForward(FeedForward):
                               f"{rt.ops.ROUTE_MOST_CHANNELS} channels, got {self.experts + self.identity} and {self.width}")
 
     def bind(self, weights, rt):
-        n = self.names
+        n, ops = self.names, rt.ops
         self.router = weights[n["router"]].float().contiguous()  # its logits are a 32-bit product under either runtime
         self.correction = weights[n["correction"]].float().contiguous() if n["correction"] else None
-        # one product over all experts: expert by expert its up rows (behind its gate rows, where it has them)
         self.router_bias = weights[n["router_bias"]].float().contiguous() if n["router_bias"] else None
-        rows = [weights[name.format(e)] for e in range(self.experts) for name in ((n["gate"], n["up"]) if n["gate"] else (n["up"],))]
-        columns = [weights[n["down"].format(e)] for e in range(self.experts)]
-        if self.shared is not None:  # (its rows and columns lie behind the experts')
-            rows += [weights[self.shared["gate"]], weights[self.shared["up"]]]
-            columns.append(weights[self.shared["down"]])
+        # one product over all experts: expert by expert its up rows (behind its gate rows, where it has them), the shared
+        # expert's behind them.  Where the experts' own kernels are to run, an inner size is filled up with zeros.
+        extra = 0 if self.shared is None else self.shared["inner"]
+        grouped = (rt.dtype == torch.bfloat16 and n["gate"] is not None and not self.identity and self.experts <= ops.EXPERTS_MOST
+                   and self.top <= ops.ROUTE_MOST_LISTED and self.width <= ops.ROUTE_FUSED_MOST_CHANNELS
+                   and ops.packs(weights[n["up"].format(0)]))
+        step = ops.ExpertRegions.STEP if grouped else 1
+        self.padded, extra = -(-self.inner // step) * step, -(-extra // step) * step
+
+        def filled(name, size, dim):
+            w = weights[name]
+            if w.shape[dim] == size:
+                return w
+            shape = list(w.shape)
+            shape[dim] = size - w.shape[dim]
+            return torch.cat([w, w.new_zeros(shape)], dim=dim)
+
+        names = (n["gate"], n["up"]) if n["gate"] else (n["up"],)
+        rows = [filled(name.format(e), self.padded, 0) for e in range(self.experts) for name in names]
+        columns = [filled(n["down"].format(e), self.padded, 1) for e in range(self.experts)]
+        if self.shared is not None:
+            rows += [filled(self.shared["gate"], extra, 0), filled(self.shared["up"], extra, 0)]
+            columns.append(filled(self.shared["down"], extra, 1))
         self.up = Projection(torch.cat(rows, dim=0), rt)
         self.down = Projection(torch.cat(columns, dim=1), rt)
+        self.extra = extra
+        self.regions = None
+        if grouped:
+            self.regions = ops.ExpertRegions(self.experts, self.padded, extra, self.activation, self.limit,
+                                             0.0 if self.shared is None else self.shared["limit"])
 
     def weight_bytes(self):
         return self.up.weight_bytes() + self.down.weight_bytes() + self.router.numel() * 4
 
+    def weight_bytes_for(self, rows):
+        """What a step of ``rows`` tokens reads: where experts that nobody chose are left out, the expected share of them
+        under a router that chooses evenly."""
+        if self.regions is None or rows > self.few_rows:
+            return self.weight_bytes()
+        unread = self.experts * (1.0 - self.top / self.experts) ** rows * self.padded
+        return self.weight_bytes() - int((self.up.weight_bytes() + self.down.weight_bytes()) * unread / self.regions.hidden)
+
+    few_rows = 16  # up to this many rows the experts that nobody chose are left out
+    many_rows = 192  # from this many on an expert's products run over the rows that chose it; in between all experts are multiplied
+    takes_pending_norm = True
+    adds_to_residual = True
     can_leave_share = True  # ``forward(..., share_later=True)`` leaves the identity outputs' share to a consumer that adds it in a kernel of its own
 
-    def forward(self, x, ctx, rt, share_later=False):
-        """With ``share_later`` and identity outputs: returns (y, (keep, x)), where the output is y + keep[row] * x[row]."""
-        tokens = x.shape[0]
+    def _route(self, x, rt, listed):
+        """(normed rows, gates, keep, choices as lists or None): the router's own kernel, with the norm before it where
+        that is still to run."""
+        from .lazy import PendingNorm
+
+        ops = rt.ops
+        pending = isinstance(x, PendingNorm)
+        tokens = x.rows if pending else x.shape[0]
         gates, keep = rt.empty(tokens, self.experts, dtype=torch.float32), rt.empty(tokens, dtype=torch.float32)
+        chosen = (rt.empty(tokens, self.top, dtype=torch.int32), rt.empty(tokens, self.top, dtype=torch.float32)) if listed else None
         rule = dict(groups=self.groups, bias=self.router_bias, chosen_softmax=self.scoring == "chosen_softmax")
-        if self.width <= rt.ops.ROUTE_FUSED_MOST_CHANNELS:
-            rt.ops.route(x, self.router, self.correction, self.experts, self.top, gates, keep, **rule)
+        if (pending and getattr(x.norm, "fusable_rms", False) and x.x.dtype == torch.float32 and x.x.is_contiguous()
+                and self.width <= ops.ROUTE_FUSED_MOST_CHANNELS):
+            h = ops.route_norm(x.x, x.delta, x.norm.weight, x.norm.eps, rt.empty(tokens, self.width), self.router, self.correction,
+                               self.experts, self.top, gates, keep, chosen=chosen, **rule)
+            x.residual = x.x
+            return h, gates, keep, chosen
+        if pending:
+            x = x.materialize()
+        if self.width <= ops.ROUTE_FUSED_MOST_CHANNELS:
+            ops.route(x, self.router, self.correction, self.experts, self.top, gates, keep, chosen=chosen, **rule)
         else:
-            logits = rt.ops.router_logits(x, self.router, rt.empty(tokens, self.experts + self.identity, dtype=torch.float32))
-            rt.ops.route_top(logits, self.correction, self.experts, self.top, gates, keep, **rule)
+            logits = ops.router_logits(x, self.router, rt.empty(tokens, self.experts + self.identity, dtype=torch.float32))
+            ops.route_top(logits, self.correction, self.experts, self.top, gates, keep, **rule)
+        return x, gates, keep, chosen
+
+    def forward(self, x, ctx, rt, share_later=False, into=None):
+        """With ``share_later`` and identity outputs: returns (y, (keep, x)), where the output is y + keep[row] * x[row]."""
+        ops = rt.ops
+        tokens = x.rows if hasattr(x, "rows") else x.shape[0]
+        many = self.regions is not None and tokens >= self.many_rows
+        x, gates, keep, chosen = self._route(x, rt, many)
+        if self.regions is not None and (many or tokens <= self.few_rows):
+            def run(out, stream=None):
+                if many:
+                    return ops.experts_many(x, self.up.weight, self.down.weight, self.regions, chosen[0], chosen[1], out, stream)
+                return ops.experts_few(x, self.up.weight, self.down.weight, self.regions, gates, out, stream)
+
+            if into is not None and hasattr(into, "take_by") and into.can_take(x, self.down.weight):
+                return into.take_by(lambda *stream: run(None, stream))  # (the last kernel adds to the stream itself)
+            y = rt.empty(tokens, self.width)
+            run(y)
+            return y
         z = self.up(x, rt)
-        inner, extra = self.experts * self.inner, 0 if self.shared is None else self.shared["inner"]
+        inner, extra = self.experts * self.padded, self.extra
         hidden = rt.empty(tokens, inner + extra)
         if not extra:
-            rt.ops.routed_act(z, gates, hidden, self.activation, self.limit)
+            ops.routed_act(z, gates, hidden, self.activation, self.limit)
         else:
-            rt.ops.routed_act(z[:, :2 * inner], gates, hidden[:, :inner], self.activation, self.limit, inner=self.inner)
-            rt.ops.routed_act(z[:, 2 * inner:], None, hidden[:, inner:], self.activation, self.shared["limit"], inner=extra)
+            ops.routed_act(z[:, :2 * inner], gates, hidden[:, :inner], self.activation, self.limit, inner=self.padded)
+            ops.routed_act(z[:, 2 * inner:], None, hidden[:, inner:], self.activation, self.shared["limit"], inner=extra)
+        if into is not None and not self.identity and into.can_take(hidden, self.down.weight):
+            return into.take(hidden, self.down.weight)
         y = self.down(hidden, rt)
         if self.identity and share_later:
             return y, (keep, x)

@@ -100,11 +100,17 @@ class ResidualInto:
 
     def take(self, x: torch.Tensor, weight) -> PendingNorm:
         """residual += x @ weight^T; returns the next norm, prepared."""
+        return self.take_by(lambda residual, gain, scaled, ss: self.rt.ops.gemm_residual(x, weight, residual, gain, scaled, ss))
+
+    def take_by(self, write) -> PendingNorm:
+        """The same by a kernel of the part's own: ``write(residual, gain,
+        scaled, ss)`` adds to the stream and returns how many parts of the
+        rows' sums of squares it left in ``ss``."""
         rt, residual = self.rt, self.source.residual
         rows, width = residual.shape
         scaled = rt.empty(rows, width)
         ss = rt.empty(rt.ops.gemm_residual_parts(rows, width), rows, dtype=torch.float32)
-        parts = rt.ops.gemm_residual(x, weight, residual, self.norm.weight, scaled, ss)
+        parts = write(residual, self.norm.weight, scaled, ss)
         return PendingNorm.prepared(self.norm, residual, scaled, ss, parts, rt)
 
 

@@ -74,6 +74,7 @@ def dense_feed_forward(h, w, rnd=identity):
 
 def clamped_expert(h, w, limit, rnd=identity):
     """g = min(Wgate h, limit), u = Wup h held in [-limit, limit]; Wdown (g sigmoid(1.702 g) (u + 1))."""
+    limit = math.inf if limit is None else limit
     g = torch.clamp(rnd(h @ w["gate"].T), max=limit)
     u = torch.clamp(rnd(h @ w["up"].T), min=-limit, max=limit)
     return rnd(g * sigmoid(1.702 * g) * (u + 1.0)) @ w["down"].T
@@ -94,9 +95,9 @@ def routed_feed_forward(h, w, mlp, rnd=identity):
     for e in range(mlp["router"]["experts"]):
         rows, place = torch.nonzero(chosen == e, as_tuple=True)
         if rows.numel():
-            out[rows] += weights[rows, place, None] * clamped_expert(h[rows], _sub(w, f"e{e}."), mlp["expert"]["limit"], rnd)
+            out[rows] += weights[rows, place, None] * clamped_expert(h[rows], _sub(w, f"e{e}."), mlp["expert"].get("limit"), rnd)
     if mlp.get("shared"):
-        out = out + clamped_expert(h, _sub(w, "shared."), mlp["shared"]["limit"], rnd)
+        out = out + clamped_expert(h, _sub(w, "shared."), mlp["shared"].get("limit"), rnd)
     return out, chosen
 
 
