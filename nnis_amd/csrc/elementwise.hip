@@ -110,11 +110,23 @@ __global__ __launch_bounds__(256) void embed_norm_kernel(const int* __restrict__
     for (int k = threadIdx.x * 8; k < width; k += blockDim.x * 8) {
       const uint4 p = piece(k);
       const uint32_t words[4] = {p.x, p.y, p.z, p.w};
+      float m[8];
+      if (weight_dtype == NNIS_BF16) {
+        const uint4 wp = *(const uint4*)((const bf16_t*)weight + k);
+        const uint32_t ww[4] = {wp.x, wp.y, wp.z, wp.w};
+#pragma unroll
+        for (int i = 0; i < 4; ++i) m[2 * i] = __uint_as_float(ww[i] << 16), m[2 * i + 1] = __uint_as_float(ww[i] & 0xffff0000u);
+      } else {
+        *(float4*)m = *(const float4*)((const float*)weight + k);
+        *(float4*)(m + 4) = *(const float4*)((const float*)weight + k + 4);
+      }
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        dst[k + 2 * i] = __uint_as_float(words[i] << 16) * inv * load_as_f32(weight, weight_dtype, k + 2 * i);
-        dst[k + 2 * i + 1] = __uint_as_float(words[i] & 0xffff0000u) * inv * load_as_f32(weight, weight_dtype, k + 2 * i + 1);
+        m[2 * i] *= __uint_as_float(words[i] << 16) * inv;
+        m[2 * i + 1] *= __uint_as_float(words[i] & 0xffff0000u) * inv;
       }
+      *(float4*)(dst + k) = *(const float4*)m;
+      *(float4*)(dst + k + 4) = *(const float4*)(m + 4);
     }
     return;
   }
@@ -134,6 +146,7 @@ extern "C" int nnis_embed_norm(const int* ids, const void* table, int table_dtyp
   NNIS_REQUIRE(nnis_dtype_ok(table_dtype) && nnis_dtype_ok(weight_dtype) && weight, "embed_norm: unknown types or no weight");
   NNIS_REQUIRE(tokens >= 0 && width > 0 && vocab > 0, "embed_norm: bad sizes tokens=%d width=%d vocab=%d", tokens, width, vocab);
   NNIS_REQUIRE(!packed || (width % 8 == 0 && table_dtype == NNIS_BF16), "embed_norm: a packed table is bfloat16 with a width that is a multiple of 8");
+  NNIS_REQUIRE(!packed || ((uintptr_t)weight % 16 == 0 && (uintptr_t)out % 16 == 0), "embed_norm: operands must be 16-byte aligned");
   if (tokens == 0) return 0;
   hipLaunchKernelGGL(embed_norm_kernel, dim3(tokens), dim3(256), 0, (hipStream_t)stream, ids, table, table_dtype, packed ? 1 : 0, weight,
                      weight_dtype, eps, out, width, vocab, scale);

@@ -121,16 +121,19 @@ __global__ __launch_bounds__(64 * KSPLIT) void experts_up_few_kernel(const bf16_
   *(bf16x4*)(hidden + row + (size_t)region * reg.inner + unit * 16 + 4 * g) = out;
 }
 
-// A block of KSPLIT waves takes 16 output channels (or, with PAIR, two blocks share them and meet as the library's paired
-// products do): the chunks of the regions that somebody chose, and of the shared one, dealt to the waves.
+// Two blocks of KSPLIT waves take 16 output channels between them (the strips alone would leave half the chip without a block)
+// and meet as the library's paired products do: the chunks of the regions that somebody chose, and of the shared one,
+// dealt to the waves of both.
 template <int KSPLIT, typename OutT>
 __global__ __launch_bounds__(64 * KSPLIT) void experts_down_few_kernel(const bf16_t* __restrict__ hidden, const bf16_t* __restrict__ w,
-                                                                       const float* __restrict__ gates, OutT y, Regions reg, int m, int n) {
+                                                                       const float* __restrict__ gates, OutT y, Regions reg, int m, int n,
+                                                                       PairScratch pair) {
+  constexpr int kShares = 2 * KSPLIT;
   __shared__ float partial[KSPLIT][kWave][4];
   __shared__ short active[kMostExperts];
   __shared__ int active_count;
   const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave, r = lane % 16, g = lane / 16;
-  const int strip = blockIdx.x;
+  const int strip = blockIdx.x / 2, share = 2 * wave + (int)(blockIdx.x % 2);
   const int k = reg.experts * reg.inner + reg.shared;
   constexpr bool kResidual = std::is_same<OutT, ResidualOut>::value;
   const int n0 = strip * 16 + g * 4;
@@ -158,13 +161,14 @@ __global__ __launch_bounds__(64 * KSPLIT) void experts_down_few_kernel(const bf1
   __syncthreads();
   const int per = reg.inner / 64, shared_chunks = reg.shared / 64;
   const int chunks = active_count * per + shared_chunks;
-  f32x4 acc = {0.0f, 0.0f, 0.0f, 0.0f};
+  f32x4 sums[1] = {{0.0f, 0.0f, 0.0f, 0.0f}};
+  f32x4& acc = sums[0];
   constexpr int DEPTH = 4;
-  for (int base = wave; base < chunks; base += KSPLIT * DEPTH) {
+  for (int base = share; base < chunks; base += kShares * DEPTH) {
     bf16x8 wv[DEPTH][2], xv[DEPTH][2];
 #pragma unroll
     for (int d = 0; d < DEPTH; ++d) {
-      int c = base + d * KSPLIT;
+      int c = base + d * kShares;
       const bool inside = c < chunks;
       c = inside ? c : chunks - 1;
       // the shared expert's chunks first, then the chosen regions'
@@ -185,6 +189,7 @@ __global__ __launch_bounds__(64 * KSPLIT) void experts_down_few_kernel(const bf1
   if (wave != 0) return;
 #pragma unroll
   for (int other = 1; other < KSPLIT; ++other) acc += *(const f32x4*)&partial[other][lane][0];
+  if (!pair_meets<1>(sums, pair, strip, blockIdx.x % 2, lane)) return;  // the first of the two: the other ends the strip
   if constexpr (kResidual) {
     float sq = 0.0f;
     if (valid > 0) sq = residual_take(y, held, (size_t)r * n + n0, acc, valid, vector_ok);
@@ -251,13 +256,16 @@ struct ManyArgs {
 };
 
 // A block of 8 waves (4 x 2) takes 128 of a region's rows and 128 weight rows -- UP: 64 channels' gate and up rows, strips
-// alternating between the two -- through a ring of three stages of 64 k in LDS, as the library's tiled product does
+// alternating between the two -- through a ring of NS stages of 64 k in LDS, as the library's tiled product does
 // (operands straight from memory into LDS, activations' chunks of 16 bytes swizzled by row; a step's second half is
 // multiplied behind the barrier).  The rows are gathered: a row's address is its list entry's.
+// Two stages let a compute unit run two blocks, one multiplying while the other begins or ends; three, where there are blocks
+// for one a unit only (both products of 16 experts of 704 and a shared one of 1,408 on rows of 2,048 channels, two and three
+// stages: 64 rows 68 / 51 us, 192 rows 70 / 58, 512 rows 79 / 84, 2,048 rows 144 / 155, 4,096 rows 244 / 263).
 // Items are dealt so that a die runs a run of neighbours, the row blocks of one block of weights one after another.
-template <bool UP>
+template <bool UP, int NS>
 __global__ __launch_bounds__(512) void experts_tiled_kernel(ManyArgs a) {
-  constexpr int BM = 128, BN = 128, BK = 64, NS = 3, W = 8, WGN = 2;
+  constexpr int BM = 128, BN = 128, BK = 64, W = 8, WGN = 2;
   constexpr int WM = 32, WN = 64, TM = 2, TN = 4;
   constexpr int A_LOADS = BM / (8 * W), B_LOADS = BN / (8 * W), LOADS = A_LOADS + B_LOADS;
   constexpr int A_BYTES = BM * BK * 2, STAGE_BYTES = (BM + BN) * BK * 2;
@@ -519,7 +527,9 @@ extern "C" int nnis_experts_up_few(const void* x, const void* w, const float* ga
 #define NNIS_UP_FEW(SPLIT_)                                                                                                          \
   hipLaunchKernelGGL((experts_up_few_kernel<SPLIT_>), dim3(blocks), dim3(64 * SPLIT_), 0, s, (const bf16_t*)x, (const bf16_t*)w, gates, \
                      (bf16_t*)hidden, reg, m, k)
-  if (chunks > 16) NNIS_UP_FEW(8);
+  // (rows of 2,048 channels, 16 experts of 704: 11 of them chosen 17.7 us with 8 waves, 19.8 with 4 and 20.7 with 16; 2 of them
+  // 7.8, 6.3 and 8.1)
+  if (chunks > 16 && m > 2) NNIS_UP_FEW(8);
   else if (chunks > 4) NNIS_UP_FEW(4);
   else NNIS_UP_FEW(2);
 #undef NNIS_UP_FEW
@@ -528,9 +538,11 @@ extern "C" int nnis_experts_up_few(const void* x, const void* w, const float* ga
 }
 
 // hidden as above, the product [m, n] into y: bfloat16 rows (resid null), or into the stream with the following norm prepared
-// (resid float32 [m, n], gain, scaled bfloat16 [m, n], ss float32 [(n + 15) / 16, m])
+// (resid float32 [m, n], gain, scaled bfloat16 [m, n], ss float32 [(n + 15) / 16, m]).  pair_sums: scratch of 2 KB a strip of 16
+// channels; pair_counts: a word a strip, zero between calls; pair_strips: for how many strips both are.
 extern "C" int nnis_experts_down_few(const void* hidden, const void* w, const float* gates, void* y, float* resid, const void* gain, int gain_dtype,
-                                     void* scaled, float* ss, int m, int n, int experts, int inner, int shared, int form, void* stream) {
+                                     void* scaled, float* ss, int m, int n, int experts, int inner, int shared, int form, float* pair_sums,
+                                     int* pair_counts, int pair_strips, void* stream) {
   const Regions reg = {experts, inner, shared, form, 0.0f, 0.0f};
   if (check_regions("experts_down_few", reg)) return 1;
   NNIS_REQUIRE(hidden && w && gates && m >= 0 && m <= 16 && n > 0, "experts_down_few: up to 16 rows, got %d", m);
@@ -538,17 +550,19 @@ extern "C" int nnis_experts_down_few(const void* hidden, const void* w, const fl
   NNIS_REQUIRE((uintptr_t)hidden % 16 == 0 && (uintptr_t)w % 16 == 0 && (uintptr_t)y % 16 == 0 && (uintptr_t)resid % 16 == 0 &&
                    (uintptr_t)scaled % 16 == 0 && (uintptr_t)gain % 16 == 0,
                "experts_down_few: operands must be 16-byte aligned");
-  if (m == 0) return 0;
   const unsigned strips = (unsigned)((n + 15) / 16);
+  NNIS_REQUIRE(pair_sums && pair_counts && (int)strips <= pair_strips, "experts_down_few: scratch for %u strips is needed, not %d", strips, pair_strips);
+  if (m == 0) return 0;
+  const PairScratch pair = {pair_sums, pair_counts};
   hipStream_t s = (hipStream_t)stream;
   if (resid) {
     ResidualOut out;
     out.resid = resid; out.gain = gain; out.gain_dtype = gain_dtype; out.scaled = (bf16_t*)scaled; out.ss = ss;
-    hipLaunchKernelGGL((experts_down_few_kernel<16, ResidualOut>), dim3(strips), dim3(64 * 16), 0, s, (const bf16_t*)hidden, (const bf16_t*)w, gates,
-                       out, reg, m, n);
+    hipLaunchKernelGGL((experts_down_few_kernel<8, ResidualOut>), dim3(2 * strips), dim3(64 * 8), 0, s, (const bf16_t*)hidden, (const bf16_t*)w, gates,
+                       out, reg, m, n, pair);
   } else {
-    hipLaunchKernelGGL((experts_down_few_kernel<16, bf16_t*>), dim3(strips), dim3(64 * 16), 0, s, (const bf16_t*)hidden, (const bf16_t*)w, gates,
-                       (bf16_t*)y, reg, m, n);
+    hipLaunchKernelGGL((experts_down_few_kernel<8, bf16_t*>), dim3(2 * strips), dim3(64 * 8), 0, s, (const bf16_t*)hidden, (const bf16_t*)w, gates,
+                       (bf16_t*)y, reg, m, n, pair);
   }
   NNIS_LAUNCH_CHECK("experts_down_few");
   return 0;
@@ -588,18 +602,22 @@ extern "C" int nnis_experts_many(int which, const void* x, const void* x_shared,
   ManyArgs a;
   a.x = (const bf16_t*)x; a.x_shared = (const bf16_t*)x_shared; a.w = (const bf16_t*)w; a.y = (bf16_t*)y; a.y_shared = (bf16_t*)y_shared;
   a.weights = weights; a.counts = counts; a.lists = lists; a.reg = reg; a.tokens = tokens; a.top = top; a.width = width;
-  constexpr int lds_bytes = 3 * (128 + 128) * 64 * 2;
   hipStream_t s = (hipStream_t)stream;
   // (beyond 64 KB a kernel has to be told once; a refusal shows as the launch's failure)
-  if (which == 0) {
-    static const hipError_t allowed = hipFuncSetAttribute((const void*)experts_tiled_kernel<true>, hipFuncAttributeMaxDynamicSharedMemorySize, lds_bytes);
-    (void)allowed;
-    hipLaunchKernelGGL((experts_tiled_kernel<true>), dim3((unsigned)blocks), dim3(512), lds_bytes, s, a);
-  } else {
-    static const hipError_t allowed = hipFuncSetAttribute((const void*)experts_tiled_kernel<false>, hipFuncAttributeMaxDynamicSharedMemorySize, lds_bytes);
-    (void)allowed;
-    hipLaunchKernelGGL((experts_tiled_kernel<false>), dim3((unsigned)blocks), dim3(512), lds_bytes, s, a);
-  }
+#define NNIS_EXPERTS_TILED(UP_, NS_)                                                                                          \
+  do {                                                                                                                        \
+    constexpr int lds_bytes = NS_ * (128 + 128) * 64 * 2;                                                                     \
+    static const hipError_t allowed = hipFuncSetAttribute((const void*)experts_tiled_kernel<UP_, NS_>,                        \
+                                                          hipFuncAttributeMaxDynamicSharedMemorySize, lds_bytes);             \
+    (void)allowed;                                                                                                            \
+    hipLaunchKernelGGL((experts_tiled_kernel<UP_, NS_>), dim3((unsigned)blocks), dim3(512), lds_bytes, s, a);                 \
+  } while (0)
+  const bool deep = tokens <= 320;
+  if (which == 0 && deep) NNIS_EXPERTS_TILED(true, 3);
+  else if (which == 0) NNIS_EXPERTS_TILED(true, 2);
+  else if (deep) NNIS_EXPERTS_TILED(false, 3);
+  else NNIS_EXPERTS_TILED(false, 2);
+#undef NNIS_EXPERTS_TILED
   NNIS_LAUNCH_CHECK("experts_many");
   return 0;
 }

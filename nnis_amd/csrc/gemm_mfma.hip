@@ -156,11 +156,6 @@ __device__ __forceinline__ void make_activations(const RunsIn& runs, bf16_t* x_t
 // in `pair.sums`; the one that finds the other's already there (a count per strip in `pair.count`, which it sets
 // back to zero) adds them to its own and ends the strip.  Nobody waits for anybody.  For strips so few that they
 // leave half the chip without a block, on a K long enough that a compute unit's own rate of reading bounds the kernel.
-struct PairScratch {
-  float* sums;  // [strips][2][MT][64 lanes][4]
-  int* count;   // [strips], zero between calls
-};
-
 template <int MT, int KSPLIT, bool RUNS, typename OutT, bool PAIR = false>
 __global__ __launch_bounds__(KSPLIT > 4 ? 64 * KSPLIT : 256) void gemm_skinny_kernel(const bf16_t* __restrict__ x,
                                                                                    const bf16_t* __restrict__ w,
@@ -302,36 +297,8 @@ __global__ __launch_bounds__(KSPLIT > 4 ? 64 * KSPLIT : 256) void gemm_skinny_ke
   }
   if (!active) return;
   if constexpr (PAIR) {
-    // (one wave of the block is left.)  The sums go out past the caches, are waited for, and then the count:
-    // who finds it at one has the other block's sums in memory.  All of it with relaxed order at agent scope,
-    // which rests on three facts of this chip and not on the language's memory model: (1) a wave's stores are
-    // counted by vmcnt, and `s_waitcnt vmcnt(0)` below ends only when they have been written where agent-scope
-    // accesses see them; (2) atomic loads and stores at agent scope go past the dies' own L2 (each die has
-    // one), so the second block reads what the first wrote and not a line its die had kept; (3) a wave issues
-    // no load before the branch it stands behind is decided, so the sums are not read before the count.  The
-    // same with a release on the count and an acquire fence for the second block (the compiler then writes
-    // back and invalidates the L2 around them) was measured: 2048 x 5632 at 1 / 8 / 16 tokens 7.8 / 8.3 / 9.7
-    // -> 10.1 / 10.4 / 12.0 us, 2048 x 8192 9.7 / 10.2 / 11.7 -> 12.4 / 13.3 / 15.2: more than the second
-    // block gains.  The asm statements keep the compiler from moving memory accesses across them.
-    float* mine = pair.sums + ((size_t)strip * 2 + blockIdx.x % 2) * (MT * kWave * 4);
-    const float* theirs = pair.sums + ((size_t)strip * 2 + 1 - blockIdx.x % 2) * (MT * kWave * 4);
-#pragma unroll
-    for (int t = 0; t < MT; ++t)
-#pragma unroll
-      for (int e = 0; e < 4; ++e)
-        __hip_atomic_store(mine + (t * kWave + lane) * 4 + e, acc[t][e], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-    int before = 0;
-    if (lane == 0) before = __hip_atomic_fetch_add(pair.count + strip, 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-    before = __builtin_amdgcn_readfirstlane(before);
-    asm volatile("" ::: "memory");
-    if (before == 0) return;  // the first of the two: the other ends the strip
-#pragma unroll
-    for (int t = 0; t < MT; ++t)
-#pragma unroll
-      for (int e = 0; e < 4; ++e)
-        acc[t][e] += __hip_atomic_load(theirs + (t * kWave + lane) * 4 + e, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-    if (lane == 0) __hip_atomic_store(pair.count + strip, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    // (one wave of the block is left)
+    if (!pair_meets<MT>(acc, pair, strip, blockIdx.x % 2, lane)) return;  // the first of the two: the other ends the strip
   }
 
 #pragma unroll

@@ -162,4 +162,46 @@ __device__ __forceinline__ float residual_take(const ResidualOut& o, const Resid
   return sq;
 }
 
+struct PairScratch {
+  float* sums;  // [strips][2][MT][64 lanes][4]
+  int* count;   // [strips], zero between calls
+};
+
+// Where two blocks that share a strip meet, called by the one wave of either that is left with the block's sums: true for
+// the second, whose acc then holds both blocks' sums; false for the first, which is done.
+template <int MT>
+__device__ __forceinline__ bool pair_meets(f32x4 (&acc)[MT], const PairScratch& pair, int strip, int which, int lane) {
+  // The sums go out past the caches, are waited for, and then the count:
+  // who finds it at one has the other block's sums in memory.  All of it with relaxed order at agent scope,
+  // which rests on three facts of this chip and not on the language's memory model: (1) a wave's stores are
+  // counted by vmcnt, and `s_waitcnt vmcnt(0)` below ends only when they have been written where agent-scope
+  // accesses see them; (2) atomic loads and stores at agent scope go past the dies' own L2 (each die has
+  // one), so the second block reads what the first wrote and not a line its die had kept; (3) a wave issues
+  // no load before the branch it stands behind is decided, so the sums are not read before the count.  The
+  // same with a release on the count and an acquire fence for the second block (the compiler then writes
+  // back and invalidates the L2 around them) was measured: 2048 x 5632 at 1 / 8 / 16 tokens 7.8 / 8.3 / 9.7
+  // -> 10.1 / 10.4 / 12.0 us, 2048 x 8192 9.7 / 10.2 / 11.7 -> 12.4 / 13.3 / 15.2: more than the second
+  // block gains.  The asm statements keep the compiler from moving memory accesses across them.
+  float* mine = pair.sums + ((size_t)strip * 2 + which) * (MT * kWave * 4);
+  const float* theirs = pair.sums + ((size_t)strip * 2 + 1 - which) * (MT * kWave * 4);
+#pragma unroll
+  for (int t = 0; t < MT; ++t)
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+      __hip_atomic_store(mine + (t * kWave + lane) * 4 + e, acc[t][e], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+  int before = 0;
+  if (lane == 0) before = __hip_atomic_fetch_add(pair.count + strip, 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  before = __builtin_amdgcn_readfirstlane(before);
+  asm volatile("" ::: "memory");
+  if (before == 0) return false;
+#pragma unroll
+  for (int t = 0; t < MT; ++t)
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+      acc[t][e] += __hip_atomic_load(theirs + (t * kWave + lane) * 4 + e, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  if (lane == 0) __hip_atomic_store(pair.count + strip, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  return true;
+}
+
 }  // namespace

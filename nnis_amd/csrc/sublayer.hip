@@ -346,14 +346,16 @@ struct RouteRule {
   float* weights;  // [rows, top], with `chosen`: their weights
 };
 
-__device__ __forceinline__ void route_row(const float* logits, const RouteRule& rule, int row, int n, int experts, int top,
+// SLOTS: outputs a lane holds, n <= 64 * SLOTS
+template <int SLOTS>
+__device__ __forceinline__ void route_row_slots(const float* logits, const RouteRule& rule, int row, int n, int experts, int top,
                                           float* __restrict__ gates, float* __restrict__ keep, int lane) {
   const float* __restrict__ correction = rule.correction;
   const int group_count = rule.group_count, group_keep = rule.group_keep;
-  float s[kRouteMost], choice[kRouteMost];
+  float s[SLOTS], choice[SLOTS];
   float top_logit = -INFINITY;
 #pragma unroll
-  for (int i = 0; i < kRouteMost; ++i) {
+  for (int i = 0; i < SLOTS; ++i) {
     const int e = i * kWave + lane;
     s[i] = e < n ? logits[e] + (rule.bias ? rule.bias[e] : 0.0f) : -INFINITY;
     choice[i] = s[i];  // (stays where outputs are chosen by logit)
@@ -362,14 +364,14 @@ __device__ __forceinline__ void route_row(const float* logits, const RouteRule& 
   top_logit = wave_max(top_logit);
   float sum = 0.0f;
 #pragma unroll
-  for (int i = 0; i < kRouteMost; ++i) {
+  for (int i = 0; i < SLOTS; ++i) {
     s[i] = (i * kWave + lane) < n ? expf(s[i] - top_logit) : 0.0f;
     sum += s[i];
   }
   const float inv = rule.chosen_softmax ? 1.0f : 1.0f / wave_sum(sum);
   unsigned chosen = 0;
 #pragma unroll
-  for (int i = 0; i < kRouteMost; ++i) {
+  for (int i = 0; i < SLOTS; ++i) {
     const int e = i * kWave + lane;
     s[i] *= inv;
     choice[i] = e < n ? (rule.chosen_softmax ? choice[i] : s[i]) + (correction ? correction[e] : 0.0f) : -INFINITY;
@@ -381,7 +383,7 @@ __device__ __forceinline__ void route_row(const float* logits, const RouteRule& 
     for (int g = 0; g < group_count; ++g) {
       float best = -INFINITY;
 #pragma unroll
-      for (int i = 0; i < kRouteMost; ++i) {
+      for (int i = 0; i < SLOTS; ++i) {
         const int e = i * kWave + lane;
         if (e < n && e / size == g) best = fmaxf(best, choice[i]);
       }
@@ -405,7 +407,7 @@ __device__ __forceinline__ void route_row(const float* logits, const RouteRule& 
       allowed |= 1ull << best_g;
     }
 #pragma unroll
-    for (int i = 0; i < kRouteMost; ++i) {
+    for (int i = 0; i < SLOTS; ++i) {
       const int e = i * kWave + lane;
       if (e < n && !(allowed >> (e / size) & 1ull)) choice[i] = -INFINITY;
     }
@@ -418,7 +420,7 @@ __device__ __forceinline__ void route_row(const float* logits, const RouteRule& 
     float best = -INFINITY;
     int best_e = 0x7fffffff;
 #pragma unroll
-    for (int i = 0; i < kRouteMost; ++i) {
+    for (int i = 0; i < SLOTS; ++i) {
       const int e = i * kWave + lane;
       if (!(chosen >> i & 1u) && e < n && choice[i] > -INFINITY && (choice[i] > best || (choice[i] == best && e < best_e))) {
         best = choice[i];
@@ -440,7 +442,7 @@ __device__ __forceinline__ void route_row(const float* logits, const RouteRule& 
       const int i = best_e / kWave;
       chosen |= 1u << i;
 #pragma unroll
-      for (int k = 0; k < kRouteMost; ++k)
+      for (int k = 0; k < SLOTS; ++k)
         if (k == i) {
           mine = s[k];
           weight += s[k];
@@ -457,7 +459,7 @@ __device__ __forceinline__ void route_row(const float* logits, const RouteRule& 
   }
   const float share = rule.chosen_softmax ? 1.0f / wave_sum(weight) : 1.0f;
 #pragma unroll
-  for (int i = 0; i < kRouteMost; ++i) {
+  for (int i = 0; i < SLOTS; ++i) {
     const int e = i * kWave + lane;
     if (e < experts) gates[(size_t)row * experts + e] = (chosen >> i & 1u) ? s[i] * share : 0.0f;
   }
@@ -467,6 +469,12 @@ __device__ __forceinline__ void route_row(const float* logits, const RouteRule& 
   }
   kept = wave_sum(kept) * share;
   if (lane == 0) keep[row] = kept;
+}
+
+__device__ __forceinline__ void route_row(const float* logits, const RouteRule& rule, int row, int n, int experts, int top,
+                                          float* __restrict__ gates, float* __restrict__ keep, int lane) {
+  if (n <= kWave) route_row_slots<1>(logits, rule, row, n, experts, top, gates, keep, lane);
+  else route_row_slots<kRouteMost>(logits, rule, row, n, experts, top, gates, keep, lane);
 }
 
 __global__ __launch_bounds__(256) void route_top_kernel(const float* __restrict__ logits, RouteRule rule, int rows, int n, int experts,
@@ -610,6 +618,126 @@ __global__ __launch_bounds__(R == 1 ? 1024 : 64 * R) void route_norm_kernel(Rout
   router_dots<R>(lds, w, lg, n, width);
   __syncthreads();
   if (wave < R && row0 + wave < rows) route_row(lg + wave * n, rule, row0 + wave, n, experts, top, gates, keep, lane);
+}
+
+// The same for few rows, a row a block, rows of a multiple of 4 channels: nothing waits for the norm's sum.  A wave takes two
+// outputs at a time and makes, from one round of loads, the row's sum of squares and both sums x gain w; a logit is such a sum
+// over the root mean square.  The row's share of `h` that a wave writes is its own slice of the channels.
+__global__ __launch_bounds__(512) void route_norm_few_kernel(RouteNormArgs a, const float* __restrict__ w, RouteRule rule, int n, int width,
+                                                             int experts, int top, float* __restrict__ gates, float* __restrict__ keep) {
+  __shared__ float lg[kWave * kRouteMost];
+  const int row = blockIdx.x, wave = threadIdx.x / kWave, lane = threadIdx.x % kWave, waves = blockDim.x / kWave;
+  const float* __restrict__ x = a.x + (size_t)row * width;
+  auto gain_at = [&](int c) { return a.gain_dtype == NNIS_F32 ? load4((const float*)a.gain + c) : load4((const bf16_t*)a.gain + c); };
+  float inv = 0.0f;
+  for (int e = 2 * wave; e < n; e += 2 * waves) {
+    const float* __restrict__ w0 = w + (size_t)e * width;
+    const float* __restrict__ w1 = w + (size_t)(e + 1 < n ? e + 1 : e) * width;
+    float ss = 0.0f, dot0 = 0.0f, dot1 = 0.0f;
+#pragma unroll 8
+    for (int c = 4 * lane; c < width; c += 4 * kWave) {
+      const float4 v = *(const float4*)(x + c), m = *(const float4*)(w0 + c), o = *(const float4*)(w1 + c);
+      const float4 g = gain_at(c);
+      ss = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, ss))));
+      const float4 y = make_float4(v.x * g.x, v.y * g.y, v.z * g.z, v.w * g.w);
+      dot0 = fmaf(y.x, m.x, fmaf(y.y, m.y, fmaf(y.z, m.z, fmaf(y.w, m.w, dot0))));
+      dot1 = fmaf(y.x, o.x, fmaf(y.y, o.y, fmaf(y.z, o.z, fmaf(y.w, o.w, dot1))));
+    }
+#pragma unroll
+    for (int offset = kWave / 2; offset > 0; offset >>= 1) {
+      ss += __shfl_xor(ss, offset, kWave);
+      dot0 += __shfl_xor(dot0, offset, kWave);
+      dot1 += __shfl_xor(dot1, offset, kWave);
+    }
+    inv = 1.0f / sqrtf(ss / (float)width + a.eps);
+    if (lane == 0) {
+      lg[e] = dot0 * inv;
+      if (e + 1 < n) lg[e + 1] = dot1 * inv;
+    }
+  }
+  __syncthreads();
+  if (wave == 0) route_row(lg, rule, row, n, experts, top, gates, keep, lane);
+  const size_t base = (size_t)row * width;
+  for (int c = 4 * threadIdx.x; c < width; c += 4 * blockDim.x) {  // (the host asks for no more waves than there are pairs of outputs)
+    float4 v = *(const float4*)(x + c);
+    const float4 g = gain_at(c);
+    v.x *= inv * g.x; v.y *= inv * g.y; v.z *= inv * g.z; v.w *= inv * g.w;
+    if (a.h_dtype == NNIS_F32) store4((float*)a.h + base + c, v);
+    else store4((bf16_t*)a.h + base + c, v);
+  }
+}
+
+// The same for many rows, bfloat16 rows out and a bfloat16 router weight [n, width], n up to 64: a block of 8 waves norms a
+// row a wave (kept in registers between the two passes), leaves the rounded rows in LDS, and takes the logits on the
+// matrix cores with 32-bit sums, K dealt to the waves; wave r routes row r.  width: a multiple of 32 up to kRouteManyMost.
+constexpr int kRouteManyKeep = 14;  // groups of 4 channels of a row that a lane keeps
+constexpr int kRouteManyMost = kRouteManyKeep * 4 * kWave;
+
+__global__ __launch_bounds__(512) void route_norm_many_kernel(RouteNormArgs a, const bf16_t* __restrict__ w, RouteRule rule, int rows, int n,
+                                                              int width, int experts, int top, float* __restrict__ gates,
+                                                              float* __restrict__ keep) {
+  typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8_t;
+  typedef __attribute__((ext_vector_type(4))) float f32x4_t;
+  extern __shared__ __attribute__((aligned(16))) float lds[];  // [8][width + 8] bfloat16
+  __shared__ __attribute__((aligned(16))) float partial[8][kWave][8];  // [wave][output][row]
+  __shared__ float lg[8][kWave];
+  bf16_t* hs = (bf16_t*)lds;
+  const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave, r = lane % 16, g = lane / 16;
+  const int row = blockIdx.x * 8 + wave, stride = width + 8;
+  const bool live = row < rows;
+  const size_t base = (size_t)(live ? row : rows - 1) * width;
+  float4 v[kRouteManyKeep];
+  float ss = 0.0f;
+#pragma unroll
+  for (int i = 0; i < kRouteManyKeep; ++i) {
+    const int c = 4 * (lane + i * kWave);
+    if (c < width) v[i] = load4(a.x + base + c);
+  }
+  if (a.delta) {
+#pragma unroll
+    for (int i = 0; i < kRouteManyKeep; ++i) {
+      const int c = 4 * (lane + i * kWave);
+      if (c < width) {
+        const float4 d = a.delta_dtype == NNIS_F32 ? load4((const float*)a.delta + base + c) : load4((const bf16_t*)a.delta + base + c);
+        v[i].x += d.x; v[i].y += d.y; v[i].z += d.z; v[i].w += d.w;
+        if (live) store4(a.x + base + c, v[i]);
+      }
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < kRouteManyKeep; ++i)
+    if (4 * (lane + i * kWave) < width) ss = fmaf(v[i].x, v[i].x, fmaf(v[i].y, v[i].y, fmaf(v[i].z, v[i].z, fmaf(v[i].w, v[i].w, ss))));
+  const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)width + a.eps);
+#pragma unroll
+  for (int i = 0; i < kRouteManyKeep; ++i) {
+    const int c = 4 * (lane + i * kWave);
+    if (c < width) {
+      const float4 m = a.gain_dtype == NNIS_F32 ? load4((const float*)a.gain + c) : load4((const bf16_t*)a.gain + c);
+      v[i].x *= inv * m.x; v[i].y *= inv * m.y; v[i].z *= inv * m.z; v[i].w *= inv * m.w;
+      store4(hs + (size_t)wave * stride + c, v[i]);
+      if (live) store4((bf16_t*)a.h + base + c, v[i]);
+    }
+  }
+  __syncthreads();
+  for (int o0 = 0; o0 < n; o0 += 16) {
+    const bf16_t* w_row = w + (size_t)(o0 + r < n ? o0 + r : n - 1) * width + 8 * g;
+    const bf16_t* x_row = hs + (size_t)(r % 8) * stride + 8 * g;
+    f32x4_t acc = {0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll 4
+    for (int k = wave * 32; k < width; k += 8 * 32)
+      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8_t*)(w_row + k), *(const bf16x8_t*)(x_row + k), acc, 0, 0, 0);
+    if (r < 8) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) partial[wave][o0 + 4 * g + e][r] = acc[e];  // (outputs beyond n: nobody reads them)
+    }
+  }
+  __syncthreads();
+  if (!live) return;
+  float logit = 0.0f;
+#pragma unroll
+  for (int o = 0; o < 8; ++o) logit += lane < n ? partial[o][lane][wave] : 0.0f;
+  if (lane < n) lg[wave][lane] = logit;
+  route_row_slots<1>(lg[wave], rule, row, n, experts, top, gates, keep, lane);  // (a lane reads what it wrote itself)
 }
 
 // the logits alone, to global memory [rows, n]
@@ -832,6 +960,45 @@ __global__ __launch_bounds__(64) void head_norm_write_kernel(HeadWriteArgs a) {
     for (int d = lane; d < vd; d += kWave)
       store_from_f32(a.v_pages, a.cache_dtype, dst + nnis_v_offset(d, in_page), load_as_f32(a.rows, a.dtype, src + d));
   }
+}
+
+// The same without a rotation and without weights (unit norm, query factors), bfloat16 throughout, heads in steps of 8 channels up to
+// 512: a lane holds 8 channels, the lanes of a head (a power of two of them, LANES) add up their squares among themselves, a
+// wave takes 64 / LANES heads of a token, a block the heads of a token four waves at a time.
+template <int LANES>
+__global__ __launch_bounds__(256) void head_unit_write_kernel(HeadWriteArgs a) {
+  typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8_t;
+  const int token = blockIdx.x;
+  const int slot = a.tok_slot[token];
+  const int head = blockIdx.y * (256 / LANES) + threadIdx.x / LANES, at = (threadIdx.x % LANES) * 8;
+  const int hd = a.head_dim, all = a.heads + a.kv_heads;
+  if (slot < 0) return;
+  const bool is_key = head >= a.heads, live = head < all && at < hd;
+  const bf16_t* row = (const bf16_t*)a.rows + (size_t)token * a.stride;
+  bf16x8_t in = {};
+  if (live) in = *(const bf16x8_t*)(row + (is_key ? a.k_col + (head - a.heads) * hd : a.q_col + head * hd) + at);
+  int page = -1, in_page = 0;
+  if (is_key && head < all) {
+    const int pos = a.tok_pos[token];
+    page = a.block_table[(size_t)slot * a.max_pages + pos / kPageTokens];
+    in_page = pos % kPageTokens;
+  }
+  float factor = !is_key && a.q_factor && live ? a.q_factor[head] : 1.0f;
+  float ss = 0.0f;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) ss = fmaf((float)in[e], (float)in[e], ss);
+#pragma unroll
+  for (int offset = LANES / 2; offset > 0; offset >>= 1) ss += __shfl_xor(ss, offset, kWave);
+  if (a.unit) factor *= 1.0f / sqrtf(ss / (float)hd + a.eps);
+  bf16x8_t out;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) out[e] = (__bf16)((float)in[e] * factor);
+  if (live && !is_key) *(bf16x8_t*)((bf16_t*)a.q_out + ((size_t)token * a.heads + head) * hd + at) = out;
+  if (!is_key || head >= all) return;
+  const int kv_head = head - a.heads, vd = a.value_dim;
+  if (live) *(bf16x8_t*)((bf16_t*)a.k_pages + ((size_t)page * a.kv_heads + kv_head) * nnis_k_page_elems(hd) + nnis_k_offset(in_page, at)) = out;
+  bf16_t* values = (bf16_t*)a.v_pages + ((size_t)page * a.kv_heads + kv_head) * nnis_v_page_elems(vd);
+  for (int d = threadIdx.x % LANES; d < vd; d += LANES) values[nnis_v_offset(d, in_page)] = row[a.v_col + kv_head * vd + d];
 }
 
 // -----------------------------------------------------------------------------
@@ -1094,10 +1261,11 @@ extern "C" int nnis_route(const void* x, int x_dtype, const float* w, const floa
   return 0;
 }
 
-// see RouteNormArgs; chosen (null, or [rows, top] for up to 64 choices) and weights: the choices as a list beside the gates
+// see RouteNormArgs; w_bf16: the router's weight in bfloat16 where that is what it is stored in (null: none, many rows then take the
+// 32-bit products too); chosen (null, or [rows, top] for up to 64 choices) and weights: the choices as a list beside the gates
 extern "C" int nnis_route_norm(float* x, const void* delta, int delta_dtype, const void* gain, int gain_dtype, float eps, void* h, int h_dtype,
-                               const float* w, const float* bias, const float* correction, int rows, int n, int width, int experts, int top,
-                               int chosen_softmax, float* gates, float* keep, int* chosen, float* weights, int group_count, int group_keep,
+                               const float* w, const void* w_bf16, const float* bias, const float* correction, int rows, int n, int width,
+                               int experts, int top, int chosen_softmax, float* gates, float* keep, int* chosen, float* weights, int group_count, int group_keep,
                                void* stream) {
   NNIS_REQUIRE(x && gain && h && w && gates && keep && n > 0 && width > 0, "route_norm: missing operand");
   NNIS_REQUIRE(group_count >= 1 && group_count <= kWave && n % group_count == 0 && group_keep >= 1 && group_keep <= group_count,
@@ -1114,6 +1282,24 @@ extern "C" int nnis_route_norm(float* x, const void* delta, int delta_dtype, con
   hipStream_t s = (hipStream_t)stream;
   const RouteRule rule = {bias, correction, chosen_softmax ? 1 : 0, group_count, group_keep, chosen, weights};
   const RouteNormArgs a = {x, delta, delta_dtype, gain, gain_dtype, eps, h, h_dtype};
+  const bool fours = width % 4 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)gain % 16 == 0 && (uintptr_t)h % 16 == 0 && (uintptr_t)w % 16 == 0;
+  if (rows > 256 && fours && w_bf16 && h_dtype == NNIS_BF16 && n <= kWave && width % 32 == 0 && width <= kRouteManyMost &&
+      (uintptr_t)w_bf16 % 16 == 0 && (uintptr_t)delta % 16 == 0) {
+    const size_t bytes = (size_t)8 * (width + 8) * sizeof(bf16_t);
+    static const hipError_t allowed = hipFuncSetAttribute((const void*)route_norm_many_kernel, hipFuncAttributeMaxDynamicSharedMemorySize,
+                                                          8 * (kRouteManyMost + 8) * (int)sizeof(bf16_t));
+    (void)allowed;  // (a refusal shows as the launch's failure)
+    hipLaunchKernelGGL(route_norm_many_kernel, dim3((rows + 7) / 8), dim3(512), bytes, s, a, (const bf16_t*)w_bf16, rule, rows, n, width, experts,
+                       top, gates, keep);
+    NNIS_LAUNCH_CHECK("route_norm");
+    return 0;
+  }
+  if (rows <= 256 && fours && delta == nullptr) {
+    const int waves = n < 16 ? (n + 1) / 2 : 8;  // (each has outputs of its own, and with them the row's root mean square)
+    hipLaunchKernelGGL(route_norm_few_kernel, dim3(rows), dim3(kWave * waves), 0, s, a, w, rule, n, width, experts, top, gates, keep);
+    NNIS_LAUNCH_CHECK("route_norm");
+    return 0;
+  }
   if (together == 4) {
     hipLaunchKernelGGL((route_norm_kernel<4>), grid, dim3(256), lds, s, a, w, rule, rows, n, width, experts, top, gates, keep);
   } else if (together == 2) {
@@ -1218,6 +1404,26 @@ extern "C" int nnis_head_norm_write(const void* rows, int dtype, int stride, int
   a.cache_dtype = cache_dtype; a.block_table = block_table; a.max_pages = max_pages;
   a.heads = heads; a.kv_heads = kv_heads; a.head_dim = head_dim; a.value_dim = value_dim;
   a.unit = unit ? 1 : 0; a.q_factor = q_factor;
+  if (!cos_table && !q_weight && !k_weight && dtype == NNIS_BF16 && q_dtype == NNIS_BF16 && (kv_heads == 0 || cache_dtype == NNIS_BF16) &&
+      head_dim % 8 == 0 && head_dim <= 512 && stride % 8 == 0 && q_col % 8 == 0 && (kv_heads == 0 || k_col % 8 == 0) &&
+      (uintptr_t)rows % 16 == 0 && (uintptr_t)q_out % 16 == 0 && (uintptr_t)k_pages % 16 == 0) {
+    int lanes = 1;
+    while (lanes * 8 < head_dim) lanes *= 2;
+    const int per_block = 256 / lanes;
+    const dim3 grid(tokens, (heads + kv_heads + per_block - 1) / per_block);
+    hipStream_t s = (hipStream_t)stream;
+    switch (lanes) {
+      case 1: hipLaunchKernelGGL(head_unit_write_kernel<1>, grid, dim3(256), 0, s, a); break;
+      case 2: hipLaunchKernelGGL(head_unit_write_kernel<2>, grid, dim3(256), 0, s, a); break;
+      case 4: hipLaunchKernelGGL(head_unit_write_kernel<4>, grid, dim3(256), 0, s, a); break;
+      case 8: hipLaunchKernelGGL(head_unit_write_kernel<8>, grid, dim3(256), 0, s, a); break;
+      case 16: hipLaunchKernelGGL(head_unit_write_kernel<16>, grid, dim3(256), 0, s, a); break;
+      case 32: hipLaunchKernelGGL(head_unit_write_kernel<32>, grid, dim3(256), 0, s, a); break;
+      default: hipLaunchKernelGGL(head_unit_write_kernel<64>, grid, dim3(256), 0, s, a); break;
+    }
+    NNIS_LAUNCH_CHECK("head_norm_write");
+    return 0;
+  }
   hipLaunchKernelGGL(head_norm_write_kernel, dim3(tokens, heads + kv_heads), dim3(64), 0, (hipStream_t)stream, a);
   NNIS_LAUNCH_CHECK("head_norm_write");
   return 0;

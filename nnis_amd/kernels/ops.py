@@ -124,7 +124,7 @@ _SUBLAYER_SIGNATURES = {
     "nnis_rms_post_step": [_VOID, _VOID, _INT, _VOID, _INT, _FLT, _FLT, _VOID, _INT, _INT, _INT, _VOID, _VOID, _INT, _VOID],
     "nnis_rms_between": [_VOID, _VOID, _INT, _VOID, _VOID, _INT, _FLT, _VOID, _INT, _INT, _INT, _VOID, _VOID, _INT, _VOID],
     "nnis_route": [_VOID, _INT, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _VOID, _VOID, _VOID, _VOID, _INT, _INT, _VOID],
-    "nnis_route_norm": [_VOID, _VOID, _INT, _VOID, _INT, _FLT, _VOID, _INT, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _VOID,
+    "nnis_route_norm": [_VOID, _VOID, _INT, _VOID, _INT, _FLT, _VOID, _INT, _VOID, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _VOID,
                         _VOID, _VOID, _VOID, _INT, _INT, _VOID],
     "nnis_poly_norm": [_VOID, _INT, _VOID, _FLT, _VOID, _INT, _INT, _INT, _VOID],
     "nnis_router_logits": [_VOID, _INT, _VOID, _VOID, _INT, _INT, _INT, _VOID],
@@ -140,7 +140,8 @@ _SUBLAYER_SIGNATURES = {
 
 _EXPERTS_SIGNATURES = {
     "nnis_experts_up_few": [_VOID, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _FLT, _FLT, _VOID],
-    "nnis_experts_down_few": [_VOID, _VOID, _VOID, _VOID, _VOID, _VOID, _INT, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _VOID],
+    "nnis_experts_down_few": [_VOID, _VOID, _VOID, _VOID, _VOID, _VOID, _INT, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _VOID, _VOID,
+                              _INT, _VOID],
     "nnis_experts_lists": [_VOID, _INT, _INT, _INT, _VOID, _VOID, _VOID],
     "nnis_experts_many": [_INT, _VOID, _VOID, _VOID, _VOID, _VOID, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _INT, _FLT, _FLT, _VOID],
     "nnis_experts_combine": [_VOID, _VOID, _VOID, _VOID, _VOID, _INT, _VOID, _VOID, _INT, _INT, _INT, _VOID],
@@ -2282,9 +2283,10 @@ def _chosen_lists(chosen, rows: int, top: int, what: str):
 
 def route_norm(x: torch.Tensor, delta: Optional[torch.Tensor], gain: torch.Tensor, eps: float, h: torch.Tensor, weight: torch.Tensor,
                correction: Optional[torch.Tensor], experts: int, top: int, gates: torch.Tensor, keep: torch.Tensor, groups=None,
-               bias: Optional[torch.Tensor] = None, chosen_softmax: bool = False, chosen=None):
+               bias: Optional[torch.Tensor] = None, chosen_softmax: bool = False, chosen=None, weight_bf16: Optional[torch.Tensor] = None):
     """``route`` behind the RMS norm of the 32-bit stream ``x`` (+ ``delta``, summed into ``x``), in one kernel: ``h`` takes
-    the normed rows, the router reads them in 32-bit."""
+    the normed rows, the router's logits are 32-bit sums over them.  ``weight_bf16``: the router's weight as it is stored,
+    where that is bfloat16: many rows then take their logits on the matrix cores, from the rows as ``h`` rounds them."""
     _dev(x, "x"), _dev(gain, "norm weight"), _dev(h, "h"), _dev(weight, "router weight"), _dev(gates, "gates"), _dev(keep, "keep")
     rows, width = x.shape
     n = weight.shape[0]
@@ -2303,10 +2305,14 @@ def route_norm(x: torch.Tensor, delta: Optional[torch.Tensor], gain: torch.Tenso
     if not (0 < n <= ROUTE_MOST_OUTPUTS and 0 <= experts <= n and 0 < top <= n and width <= ROUTE_FUSED_MOST_CHANNELS):
         raise KernelError(f"route_norm: {experts} experts and the {top} largest of {n} outputs (at most {ROUTE_MOST_OUTPUTS}) of rows of {width} channels")
     _check_router_bias(bias, n, "route_norm")
+    if weight_bf16 is not None:
+        _dev(weight_bf16, "router weight")
+        if weight_bf16.dtype != torch.bfloat16 or weight_bf16.shape != weight.shape:
+            raise KernelError(f"route_norm: a bfloat16 router weight {tuple(weight.shape)}, got {tuple(weight_bf16.shape)} {weight_bf16.dtype}")
     group_count, group_keep = _route_groups(groups, n, "route_norm")
     lib = sublayer()
     _check(lib, lib.nnis_route_norm(x.data_ptr(), _ptr(delta), _code(delta) if delta is not None else 0, gain.data_ptr(), _code(gain), float(eps),
-                                    h.data_ptr(), _code(h), weight.data_ptr(), _ptr(bias), _ptr(correction), rows, n, width, experts, top,
+                                    h.data_ptr(), _code(h), weight.data_ptr(), _ptr(weight_bf16), _ptr(bias), _ptr(correction), rows, n, width, experts, top,
                                     1 if chosen_softmax else 0, gates.data_ptr(), keep.data_ptr(), *_chosen_lists(chosen, rows, top, "route_norm"),
                                     group_count, group_keep, _stream()))
     return h
@@ -2544,11 +2550,15 @@ def experts_few(x: torch.Tensor, up, down, regions: ExpertRegions, gates: torch.
             raise KernelError(f"experts_few: out {tuple(out.shape)} {out.dtype}")
         ends = [out.data_ptr(), None, None, 0, None, None]
     hidden = torch.empty(rows, regions.hidden, dtype=torch.bfloat16, device=x.device)
+    work = _gemm_workspace(x.device)  # (the strips' counts behind it are zero between calls, as the products leave them)
+    if work is None:
+        raise KernelError("experts_few: the products' workspace would have to be made inside a graph capture")
     lib = experts()
     _check(lib, lib.nnis_experts_up_few(x.data_ptr(), up.data_ptr(), gates.data_ptr(), hidden.data_ptr(), rows, width, regions.experts,
                                         regions.inner, regions.shared, regions.form, regions.limit, regions.shared_limit, _stream()))
     _check(lib, lib.nnis_experts_down_few(hidden.data_ptr(), down.data_ptr(), gates.data_ptr(), *ends, rows, width, regions.experts,
-                                          regions.inner, regions.shared, regions.form, _stream()))
+                                          regions.inner, regions.shared, regions.form, work.data_ptr(), work.data_ptr() + GEMM_WORKSPACE_BYTES,
+                                          min(PAIR_COUNTS, GEMM_WORKSPACE_BYTES // 2048), _stream()))
     return parts
 
 

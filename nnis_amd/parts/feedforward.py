@@ -172,6 +172,8 @@ class RoutedFeedForward(FeedForward):
     def bind(self, weights, rt):
         n, ops = self.names, rt.ops
         self.router = weights[n["router"]].float().contiguous()  # its logits are a 32-bit product under either runtime
+        stored = weights[n["router"]]
+        self.router_stored = stored.contiguous() if stored.dtype == torch.bfloat16 else None
         self.correction = weights[n["correction"]].float().contiguous() if n["correction"] else None
         self.router_bias = weights[n["router_bias"]].float().contiguous() if n["router_bias"] else None
         # one product over all experts: expert by expert its up rows (behind its gate rows, where it has them), the shared
@@ -217,7 +219,7 @@ class RoutedFeedForward(FeedForward):
         return self.weight_bytes() - int((self.up.weight_bytes() + self.down.weight_bytes()) * unread / self.regions.hidden)
 
     few_rows = 16  # up to this many rows the experts that nobody chose are left out
-    many_rows = 192  # from this many on an expert's products run over the rows that chose it; in between all experts are multiplied
+    many_rows = 96  # from this many on an expert's products run over the rows that chose it; in between all experts are multiplied
     takes_pending_norm = True
     adds_to_residual = True
     can_leave_share = True  # ``forward(..., share_later=True)`` leaves the identity outputs' share to a consumer that adds it in a kernel of its own
@@ -236,7 +238,7 @@ class RoutedFeedForward(FeedForward):
         if (pending and getattr(x.norm, "fusable_rms", False) and x.x.dtype == torch.float32 and x.x.is_contiguous()
                 and self.width <= ops.ROUTE_FUSED_MOST_CHANNELS):
             h = ops.route_norm(x.x, x.delta, x.norm.weight, x.norm.eps, rt.empty(tokens, self.width), self.router, self.correction,
-                               self.experts, self.top, gates, keep, chosen=chosen, **rule)
+                               self.experts, self.top, gates, keep, chosen=chosen, weight_bf16=self.router_stored, **rule)
             x.residual = x.x
             return h, gates, keep, chosen
         if pending:
