@@ -78,8 +78,9 @@ extern "C" int nnis_embed_packed(const int* ids, const void* packed, float* out,
 }
 
 // The row copy with an RMS norm behind it: out[t, :] = e / sqrt(mean(e^2) + eps) * weight, e = table[ids[t], :] * scale.
-// A block a token; the row is read twice, the second time from the caches.  Eight channels a thread and access where the
-// table is packed (its pieces of a row), one otherwise.
+// A block a token.  Where the table is packed a thread takes pieces of eight channels and keeps the first kEmbedKeep between the
+// two passes; otherwise the row is read twice, a channel a thread, the second time from the caches.
+constexpr int kEmbedKeep = 4;
 __global__ __launch_bounds__(256) void embed_norm_kernel(const int* __restrict__ ids, const void* __restrict__ table, int table_dtype,
                                                          int packed, const void* __restrict__ weight, int weight_dtype, float eps,
                                                          float* __restrict__ out, int width, int vocab, float scale) {
@@ -97,18 +98,25 @@ __global__ __launch_bounds__(256) void embed_norm_kernel(const int* __restrict__
       return *(const uint4*)(strip + (size_t)(k / 64) * kPackedChunkElems + (size_t)((k % 16) / 8) * kPackedHalfElems + (size_t)((k % 64) / 16) * 128);
     };
     float ss = 0.0f;
-    for (int k = threadIdx.x * 8; k < width; k += blockDim.x * 8) {
-      const uint4 p = piece(k);
+    auto squares = [&](const uint4& p) {
       const uint32_t words[4] = {p.x, p.y, p.z, p.w};
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const float lo = __uint_as_float(words[i] << 16) * scale, hi = __uint_as_float(words[i] & 0xffff0000u) * scale;
         ss = fmaf(lo, lo, fmaf(hi, hi, ss));
       }
-    }
+    };
+    const int step = blockDim.x * 8;
+    uint4 held[kEmbedKeep];
+#pragma unroll
+    for (int i = 0; i < kEmbedKeep; ++i)
+      if (threadIdx.x * 8 + i * step < width) held[i] = piece(threadIdx.x * 8 + i * step);
+#pragma unroll
+    for (int i = 0; i < kEmbedKeep; ++i)
+      if (threadIdx.x * 8 + i * step < width) squares(held[i]);
+    for (int k = threadIdx.x * 8 + kEmbedKeep * step; k < width; k += step) squares(piece(k));
     const float inv = scale / sqrtf(block_sum(ss, scratch) / (float)width + eps);
-    for (int k = threadIdx.x * 8; k < width; k += blockDim.x * 8) {
-      const uint4 p = piece(k);
+    auto put = [&](int k, const uint4& p) {
       const uint32_t words[4] = {p.x, p.y, p.z, p.w};
       float m[8];
       if (weight_dtype == NNIS_BF16) {
@@ -127,7 +135,11 @@ __global__ __launch_bounds__(256) void embed_norm_kernel(const int* __restrict__
       }
       *(float4*)(dst + k) = *(const float4*)m;
       *(float4*)(dst + k + 4) = *(const float4*)(m + 4);
-    }
+    };
+#pragma unroll
+    for (int i = 0; i < kEmbedKeep; ++i)
+      if (threadIdx.x * 8 + i * step < width) put(threadIdx.x * 8 + i * step, held[i]);
+    for (int k = threadIdx.x * 8 + kEmbedKeep * step; k < width; k += step) put(k, piece(k));
     return;
   }
   const size_t base = (size_t)id * width;

@@ -83,7 +83,7 @@ def _run_in_steps(forward, cache, rt, xs, cuts):
 # ---------------------------------------------------------------------------------------------
 
 @pytest.mark.parametrize("packed", [False, True])
-@pytest.mark.parametrize("tokens, width, scale", [(1, 8, 1.0), (37, 56, 3.0), (5, 1032, 1.0), (3, 4096, 0.5)])
+@pytest.mark.parametrize("tokens, width, scale", [(1, 8, 1.0), (37, 56, 3.0), (5, 1032, 1.0), (3, 4096, 0.5), (2, 8456, 1.0)])
 def test_a_normed_embedding(packed, tokens, width, scale):
     from nnis_amd.kernels import ops
 
