@@ -255,26 +255,28 @@ struct ManyArgs {
   int tokens, top, width;
 };
 
-// A block of 8 waves (4 x 2) takes 128 of a region's rows and 128 weight rows -- UP: 64 channels' gate and up rows, strips
-// alternating between the two -- through a ring of NS stages of 64 k in LDS, as the library's tiled product does
+// A block of 8 waves takes 128 of a region's rows and BN weight rows -- UP: BN / 2 channels' gate and up rows, strips
+// alternating between the two -- through a ring of three stages of 64 k in LDS, as the library's tiled product does
 // (operands straight from memory into LDS, activations' chunks of 16 bytes swizzled by row; a step's second half is
 // multiplied behind the barrier).  The rows are gathered: a row's address is its list entry's.
-// Two stages let a compute unit run two blocks, one multiplying while the other begins or ends; three, where there are blocks
-// for one a unit only (both products of 16 experts of 704 and a shared one of 1,408 on rows of 2,048 channels, two and three
-// stages: 64 rows 68 / 51 us, 192 rows 70 / 58, 512 rows 79 / 84, 2,048 rows 144 / 155, 4,096 rows 244 / 263).
+// The wide tile brings three quarters of the narrow one's bytes through L2 a multiplication; the narrow one fills the chip
+// with few rows.  Up and down product of 16 experts of 704, 2 chosen, and a shared one of 1,408 on rows of 2,048 channels,
+// microseconds, narrow and wide: 192 rows 25 + 25 / 34 + 26; with two stages of the narrow one, two blocks a unit, against the
+// wide one: 512 rows 40 + 30 / 35 + 27, 2,048 rows 80 + 56 / 72 + 50, 8,192 rows 243 + 193 / 208 + 166.
 // Items are dealt so that a die runs a run of neighbours, the row blocks of one block of weights one after another.
-template <bool UP, int NS>
+template <bool UP, int BN>
 __global__ __launch_bounds__(512) void experts_tiled_kernel(ManyArgs a) {
-  constexpr int BM = 128, BN = 128, BK = 64, W = 8, WGN = 2;
-  constexpr int WM = 32, WN = 64, TM = 2, TN = 4;
+  constexpr int BM = 128, BK = 64, NS = 3, W = 8, WGN = BN / 64;
+  constexpr int WM = BM * WGN / W, WN = 64, TM = WM / 16, TN = WN / 16;
+  constexpr int CHANNELS = BN / 2;  // UP: of a tile
   constexpr int A_LOADS = BM / (8 * W), B_LOADS = BN / (8 * W), LOADS = A_LOADS + B_LOADS;
   constexpr int A_BYTES = BM * BK * 2, STAGE_BYTES = (BM + BN) * BK * 2;
   const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid / kWave), lane = tid % kWave;
   const int wave_m = wave / WGN, wave_n = wave % WGN, r = lane % 16, g = lane / 16;
   const Regions& reg = a.reg;
   // which item: the regions' row blocks are counted from the lists' lengths (every wave for itself)
-  const int cols = UP ? reg.inner / 64 : (a.width + BN - 1) / BN;
-  const int cols_shared = reg.shared == 0 ? 0 : (UP ? reg.shared / 64 : cols);
+  const int cols = UP ? (reg.inner + CHANNELS - 1) / CHANNELS : (a.width + BN - 1) / BN;
+  const int cols_shared = reg.shared == 0 ? 0 : (UP ? (reg.shared + CHANNELS - 1) / CHANNELS : cols);
   const int shared_items = (a.tokens + BM - 1) / BM * cols_shared;
   int total = shared_items;
   for (int e0 = 0; e0 < reg.experts; e0 += kWave) {
@@ -347,8 +349,11 @@ __global__ __launch_bounds__(512) void experts_tiled_kernel(ManyArgs a) {
   for (int o = 0; o < B_LOADS; ++o) {
     const int piece = o * W + wave, strip = piece / 2;
     int row;
-    if (UP) row = gate_row + (strip % 2 ? channels : 0) + col * 64 + (strip / 2) * 16 + r;
-    else row = col * BN + strip * 16 + r;
+    if (UP) {
+      int unit = col * CHANNELS + (strip / 2) * 16;  // (a tile's channels beyond the region's: multiplied again from its last, not stored)
+      unit = unit < channels ? unit : channels - 16;
+      row = gate_row + (strip % 2 ? channels : 0) + unit + r;
+    } else row = col * BN + strip * 16 + r;
     if (!UP) row = row < a.width ? row : a.width - 1;
     b_src[o] = a.w + nnis_packed_lane(row, g, w_k) + (size_t)first_chunk * kPackedChunkElems + (piece % 2) * kPackedHalfElems;
   }
@@ -443,10 +448,12 @@ __global__ __launch_bounds__(512) void experts_tiled_kernel(ManyArgs a) {
       if (out_row[i] < 0) continue;
 #pragma unroll
       for (int u = 0; u < TN / 2; ++u) {
+        const int unit = col * CHANNELS + wave_n * 32 + u * 16;
+        if (unit >= channels) continue;
         bf16x4 out;
 #pragma unroll
         for (int e = 0; e < 4; ++e) out[e] = (__bf16)gated_value(reg, acc[i][2 * u][e], acc[i][2 * u + 1][e], limit);
-        *(bf16x4*)(y + (size_t)out_row[i] * channels + col * 64 + wave_n * 32 + u * 16 + 4 * g) = out;
+        *(bf16x4*)(y + (size_t)out_row[i] * channels + unit + 4 * g) = out;
       }
     }
   } else {
@@ -594,8 +601,10 @@ extern "C" int nnis_experts_many(int which, const void* x, const void* x_shared,
   // row blocks of 128: as many as any choice can make
   const long long pairs = (long long)tokens * top;
   long long row_blocks = pairs / 128 + (experts < pairs ? experts : pairs);
-  const long long cols = which == 0 ? inner / 64 : (width + 127) / 128;
-  const long long cols_shared = shared == 0 ? 0 : (which == 0 ? shared / 64 : (width + 127) / 128);
+  const bool wide = tokens > 320;
+  const long long tile = wide ? 256 : 128;
+  const long long cols = which == 0 ? (inner + tile / 2 - 1) / (tile / 2) : (width + tile - 1) / tile;
+  const long long cols_shared = shared == 0 ? 0 : (which == 0 ? (shared + tile / 2 - 1) / (tile / 2) : cols);
   long long blocks = row_blocks * cols + (long long)((tokens + 127) / 128) * cols_shared;
   blocks = (blocks + 7) / 8 * 8;
   NNIS_REQUIRE(blocks <= 0x7fffffff, "experts_many: the step exceeds the grid limit");
@@ -604,19 +613,18 @@ extern "C" int nnis_experts_many(int which, const void* x, const void* x_shared,
   a.weights = weights; a.counts = counts; a.lists = lists; a.reg = reg; a.tokens = tokens; a.top = top; a.width = width;
   hipStream_t s = (hipStream_t)stream;
   // (beyond 64 KB a kernel has to be told once; a refusal shows as the launch's failure)
-#define NNIS_EXPERTS_TILED(UP_, NS_)                                                                                          \
+#define NNIS_EXPERTS_TILED(UP_, BN_)                                                                                          \
   do {                                                                                                                        \
-    constexpr int lds_bytes = NS_ * (128 + 128) * 64 * 2;                                                                     \
-    static const hipError_t allowed = hipFuncSetAttribute((const void*)experts_tiled_kernel<UP_, NS_>,                        \
+    constexpr int lds_bytes = 3 * (128 + BN_) * 64 * 2;                                                                       \
+    static const hipError_t allowed = hipFuncSetAttribute((const void*)experts_tiled_kernel<UP_, BN_>,                        \
                                                           hipFuncAttributeMaxDynamicSharedMemorySize, lds_bytes);             \
     (void)allowed;                                                                                                            \
-    hipLaunchKernelGGL((experts_tiled_kernel<UP_, NS_>), dim3((unsigned)blocks), dim3(512), lds_bytes, s, a);                 \
+    hipLaunchKernelGGL((experts_tiled_kernel<UP_, BN_>), dim3((unsigned)blocks), dim3(512), lds_bytes, s, a);                 \
   } while (0)
-  const bool deep = tokens <= 320;
-  if (which == 0 && deep) NNIS_EXPERTS_TILED(true, 3);
-  else if (which == 0) NNIS_EXPERTS_TILED(true, 2);
-  else if (deep) NNIS_EXPERTS_TILED(false, 3);
-  else NNIS_EXPERTS_TILED(false, 2);
+  if (which == 0 && wide) NNIS_EXPERTS_TILED(true, 256);
+  else if (which == 0) NNIS_EXPERTS_TILED(true, 128);
+  else if (wide) NNIS_EXPERTS_TILED(false, 256);
+  else NNIS_EXPERTS_TILED(false, 128);
 #undef NNIS_EXPERTS_TILED
   NNIS_LAUNCH_CHECK("experts_many");
   return 0;
