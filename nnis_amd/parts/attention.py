@@ -199,9 +199,13 @@ class CausalSelfAttention(Mixer):
         # (runs of the keys, waves of a block) of a step of single tokens with these sizes
         if not self._matrix_cores(rt):
             return None
-        if self.window:  # (a window of n tokens touches the pages of at most n + 63)
-            longest = min(longest, self.window + 63)
-        return rt.ops.decode_plan(batch, self.kv_heads, longest, width=self.heads * self.value_dim)
+        if not self.window:
+            return rt.ops.decode_plan(batch, self.kv_heads, longest, width=self.heads * self.value_dim)
+        longest = min(longest, self.window + 63)  # (a window of n tokens touches the pages of at most n + 63)
+        runs, waves = rt.ops.decode_plan(batch, self.kv_heads, longest, width=self.heads * self.value_dim)
+        # A window's keys in runs of a few pages: two waves a run (16/4 heads of 128 in a window of 1,024, whole steps of eight
+        # layers in four runs: batch 1 0.481 ms against 0.493 with four waves, batch 8 0.507 against 0.520).
+        return runs, min(waves, 2) if runs > 1 else waves
 
     def prompt_plan(self, batch, rows, longest, rt):
         # (waves of a block, columns a wave carries) of the matrix-core kernel; the 32-bit kernel has no plan
