@@ -253,6 +253,7 @@ struct ManyArgs {
   const int* lists;
   Regions reg;
   int tokens, top, width;
+  int run;                 // column blocks that a block takes one after the other
 };
 
 // A block of 8 waves takes 128 of a region's rows and BN weight rows -- UP: BN / 2 channels' gate and up rows, strips
@@ -263,7 +264,9 @@ struct ManyArgs {
 // with few rows.  Up and down product of 16 experts of 704, 2 chosen, and a shared one of 1,408 on rows of 2,048 channels,
 // microseconds, narrow and wide: 192 rows 25 + 25 / 34 + 26; with two stages of the narrow one, two blocks a unit, against the
 // wide one: 512 rows 40 + 30 / 35 + 27, 2,048 rows 80 + 56 / 72 + 50, 8,192 rows 243 + 193 / 208 + 166.
-// Items are dealt so that a die runs a run of neighbours, the row blocks of one block of weights one after another.
+// An item is a row block and a run of `run` column blocks: the ring goes on from one to the next, so that the next one's loads
+// are under way while the last one's rows go out, and a short K (an expert's inner size) pays for its beginning once.  Items
+// are dealt so that a die runs a run of neighbours, the row blocks of one block of weights one after another.
 template <bool UP, int BN>
 __global__ __launch_bounds__(512) void experts_tiled_kernel(ManyArgs a) {
   constexpr int BM = 128, BK = 64, NS = 3, W = 8, WGN = BN / 64;
@@ -277,14 +280,15 @@ __global__ __launch_bounds__(512) void experts_tiled_kernel(ManyArgs a) {
   // which item: the regions' row blocks are counted from the lists' lengths (every wave for itself)
   const int cols = UP ? (reg.inner + CHANNELS - 1) / CHANNELS : (a.width + BN - 1) / BN;
   const int cols_shared = reg.shared == 0 ? 0 : (UP ? (reg.shared + CHANNELS - 1) / CHANNELS : cols);
-  const int shared_items = (a.tokens + BM - 1) / BM * cols_shared;
+  const int runs = (cols + a.run - 1) / a.run;
+  const int shared_items = (a.tokens + BM - 1) / BM * ((cols_shared + a.run - 1) / a.run);
   int total = shared_items;
   for (int e0 = 0; e0 < reg.experts; e0 += kWave) {
     const int e = e0 + lane;
     int blocks = e < reg.experts ? (a.counts[e] + BM - 1) / BM : 0;
 #pragma unroll
     for (int offset = kWave / 2; offset > 0; offset >>= 1) blocks += __shfl_xor(blocks, offset, kWave);
-    total += blocks * cols;
+    total += blocks * runs;
   }
   total = __builtin_amdgcn_readfirstlane(total);
   int item;
@@ -301,7 +305,7 @@ __global__ __launch_bounds__(512) void experts_tiled_kernel(ManyArgs a) {
     for (int e0 = 0; e0 < reg.experts; e0 += kWave) {
       const int e = e0 + lane;
       const int count = e < reg.experts ? a.counts[e] : 0;
-      const int items = (count + BM - 1) / BM * cols;
+      const int items = (count + BM - 1) / BM * runs;
       int upto = items;  // inclusive sum over the lanes
 #pragma unroll
       for (int offset = 1; offset < kWave; offset <<= 1) {
@@ -326,7 +330,8 @@ __global__ __launch_bounds__(512) void experts_tiled_kernel(ManyArgs a) {
   item = __builtin_amdgcn_readfirstlane(item);
   blocks_here = __builtin_amdgcn_readfirstlane(blocks_here);
   const bool is_shared = region == reg.experts;
-  const int row0 = (item % blocks_here) * BM, col = item / blocks_here;
+  const int row0 = (item % blocks_here) * BM, col0 = item / blocks_here * a.run;
+  const int col_end = min(col0 + a.run, is_shared ? cols_shared : cols);
   const int* list = is_shared ? nullptr : a.lists + (size_t)region * a.tokens;
   const int k = UP ? a.width : (is_shared ? reg.shared : reg.inner);           // of this product
   const int w_k = UP ? a.width : reg.experts * reg.inner + reg.shared;         // of the packed weight's rows
@@ -345,32 +350,41 @@ __global__ __launch_bounds__(512) void experts_tiled_kernel(ManyArgs a) {
   }
   const int channels = is_shared ? reg.shared : reg.inner;  // UP: channels of the region
   const int gate_row = UP ? (is_shared ? reg.experts * 2 * reg.inner : region * 2 * reg.inner) : 0;
+  auto take_column = [&](int col) {  // the weight rows of a column block
 #pragma unroll
-  for (int o = 0; o < B_LOADS; ++o) {
-    const int piece = o * W + wave, strip = piece / 2;
-    int row;
-    if (UP) {
-      int unit = col * CHANNELS + (strip / 2) * 16;  // (a tile's channels beyond the region's: multiplied again from its last, not stored)
-      unit = unit < channels ? unit : channels - 16;
-      row = gate_row + (strip % 2 ? channels : 0) + unit + r;
-    } else row = col * BN + strip * 16 + r;
-    if (!UP) row = row < a.width ? row : a.width - 1;
-    b_src[o] = a.w + nnis_packed_lane(row, g, w_k) + (size_t)first_chunk * kPackedChunkElems + (piece % 2) * kPackedHalfElems;
-  }
-  const int steps = (k + BK - 1) / BK, chunks = steps;
+    for (int o = 0; o < B_LOADS; ++o) {
+      const int piece = o * W + wave, strip = piece / 2;
+      int row;
+      if (UP) {
+        int unit = col * CHANNELS + (strip / 2) * 16;  // (a tile's channels beyond the region's: multiplied again from its last, not stored)
+        unit = unit < channels ? unit : channels - 16;
+        row = gate_row + (strip % 2 ? channels : 0) + unit + r;
+      } else {
+        row = col * BN + strip * 16 + r;
+        row = row < a.width ? row : a.width - 1;
+      }
+      b_src[o] = a.w + nnis_packed_lane(row, g, w_k) + (size_t)first_chunk * kPackedChunkElems + (piece % 2) * kPackedHalfElems;
+    }
+  };
+  take_column(col0);
+  const int steps = (k + BK - 1) / BK;
   int last_chunk = k - 8 - chunk_k;  // offset of the row's last whole chunk from this lane's first
   last_chunk = last_chunk > -chunk_k ? last_chunk : -chunk_k;
-  auto ask = [&](int step, int stage) {
+  int ask_step = 0, ask_col = col0;  // what is asked for next
+  auto ask = [&](int stage) {
     char* base = tile_lds + stage * STAGE_BYTES + wave * 1024;
-    const int k0 = step * BK;
+    const int k0 = ask_step * BK;
     const int from = k0 <= last_chunk ? k0 : last_chunk;
 #pragma unroll
     for (int o = 0; o < A_LOADS; ++o)
       __builtin_amdgcn_global_load_lds((global_ptr_t)(a_src[o] + from), (lds_ptr_t)(base + o * W * 1024), 16, 0, 0);
-    const size_t from_chunk = (size_t)(step < chunks ? step : chunks - 1) * kPackedChunkElems;
+    const size_t from_chunk = (size_t)ask_step * kPackedChunkElems;
 #pragma unroll
     for (int o = 0; o < B_LOADS; ++o)
       __builtin_amdgcn_global_load_lds((global_ptr_t)(b_src[o] + from_chunk), (lds_ptr_t)(base + A_BYTES + o * W * 1024), 16, 0, 0);
+    if (ask_step + 1 < steps) ++ask_step;
+    else if (ask_col + 1 < col_end) take_column(++ask_col), ask_step = 0;
+    // (beyond the last column block: its last step again, a valid address that nobody reads, so that the count of loads holds)
   };
   f32x4 acc[TM][TN];
 #pragma unroll
@@ -378,7 +392,7 @@ __global__ __launch_bounds__(512) void experts_tiled_kernel(ManyArgs a) {
 #pragma unroll
     for (int j = 0; j < TN; ++j) acc[i][j] = (f32x4){0.0f, 0.0f, 0.0f, 0.0f};
 #pragma unroll
-  for (int s = 0; s < NS - 1; ++s) ask(s, s);
+  for (int s = 0; s < NS - 1; ++s) ask(s);
   // the rows this lane ends up with, asked for behind the first steps' loads
   int out_row[TM];
   float weight[TM];
@@ -420,56 +434,61 @@ __global__ __launch_bounds__(512) void experts_tiled_kernel(ManyArgs a) {
     }
     __builtin_amdgcn_sched_group_barrier(0x008, TM * TN - (TM + TN), 0);
   };
+  const float limit = is_shared ? reg.shared_limit : reg.limit;
+  bf16_t* y = is_shared ? a.y_shared : a.y;
+  const bool vector_ok = a.width % 4 == 0;
+  auto put = [&](int col) {  // a finished tile's rows; the sums begin again
+#pragma unroll
+    for (int i = 0; i < TM; ++i) {
+      if (out_row[i] < 0) continue;
+      if (UP) {
+#pragma unroll
+        for (int u = 0; u < TN / 2; ++u) {
+          const int unit = col * CHANNELS + wave_n * 32 + u * 16;
+          if (unit >= channels) continue;
+          bf16x4 out;
+#pragma unroll
+          for (int e = 0; e < 4; ++e) out[e] = (__bf16)gated_value(reg, acc[i][2 * u][e], acc[i][2 * u + 1][e], limit);
+          *(bf16x4*)(y + (size_t)out_row[i] * channels + unit + 4 * g) = out;
+        }
+      } else {
+#pragma unroll
+        for (int j = 0; j < TN; ++j) {
+          const int n0 = col * BN + wave_n * WN + j * 16 + 4 * g;
+          const int valid = a.width - n0 >= 4 ? 4 : (a.width - n0 > 0 ? a.width - n0 : 0);
+          if (valid > 0) store4(y, (size_t)out_row[i] * a.width + n0, acc[i][j] * weight[i], valid, vector_ok);
+        }
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < TM; ++i)
+#pragma unroll
+      for (int j = 0; j < TN; ++j) acc[i][j] = (f32x4){0.0f, 0.0f, 0.0f, 0.0f};
+  };
+  // (A column block's stores stand between two steps' loads in the order in which the counter below sees them end: the
+  // step after waits for them too, by when they have had a step's time.)
   int stage = 0;
   read_half(0, 0, a0, b0);
-  for (int step = 0; step < steps; ++step) {
-    ask(step + NS - 1, stage == 0 ? NS - 1 : stage - 1);
-    read_half(stage, 1, a1, b1);
-    multiply(a0, b0);
-    interleave();
-    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
-    wait_loads_but<(NS - 2) * LOADS>();
-    __builtin_amdgcn_sched_barrier(0);
-    __builtin_amdgcn_s_barrier();
-    __builtin_amdgcn_sched_barrier(0);
-    asm volatile("" ::: "memory");
-    stage = stage + 1 == NS ? 0 : stage + 1;
-    read_half(stage, 0, a0, b0);  // (after the last step: of a stage that nobody multiplies)
-    multiply(a1, b1);
-    interleave();
+  for (int col = col0; col < col_end; ++col) {
+    for (int step = 0; step < steps; ++step) {
+      ask(stage == 0 ? NS - 1 : stage - 1);
+      read_half(stage, 1, a1, b1);
+      multiply(a0, b0);
+      interleave();
+      asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+      wait_loads_but<(NS - 2) * LOADS>();
+      __builtin_amdgcn_sched_barrier(0);
+      __builtin_amdgcn_s_barrier();
+      __builtin_amdgcn_sched_barrier(0);
+      asm volatile("" ::: "memory");
+      stage = stage + 1 == NS ? 0 : stage + 1;
+      read_half(stage, 0, a0, b0);  // (after the last step: of a stage that nobody multiplies)
+      multiply(a1, b1);
+      interleave();
+    }
+    put(col);
   }
   wait_loads_but<0>();  // the steps asked for beyond the end: nothing of this block is in flight when it ends
-
-  if (UP) {
-    const float limit = is_shared ? reg.shared_limit : reg.limit;
-    bf16_t* y = is_shared ? a.y_shared : a.y;
-#pragma unroll
-    for (int i = 0; i < TM; ++i) {
-      if (out_row[i] < 0) continue;
-#pragma unroll
-      for (int u = 0; u < TN / 2; ++u) {
-        const int unit = col * CHANNELS + wave_n * 32 + u * 16;
-        if (unit >= channels) continue;
-        bf16x4 out;
-#pragma unroll
-        for (int e = 0; e < 4; ++e) out[e] = (__bf16)gated_value(reg, acc[i][2 * u][e], acc[i][2 * u + 1][e], limit);
-        *(bf16x4*)(y + (size_t)out_row[i] * channels + unit + 4 * g) = out;
-      }
-    }
-  } else {
-    bf16_t* y = is_shared ? a.y_shared : a.y;
-    const bool vector_ok = a.width % 4 == 0;
-#pragma unroll
-    for (int i = 0; i < TM; ++i) {
-      if (out_row[i] < 0) continue;
-#pragma unroll
-      for (int j = 0; j < TN; ++j) {
-        const int n0 = col * BN + wave_n * WN + j * 16 + 4 * g;
-        const int valid = a.width - n0 >= 4 ? 4 : (a.width - n0 > 0 ? a.width - n0 : 0);
-        if (valid > 0) store4(y, (size_t)out_row[i] * a.width + n0, acc[i][j] * weight[i], valid, vector_ok);
-      }
-    }
-  }
 }
 
 // The end: a token's pairs and its shared row added up, into the stream with the norm that follows prepared (ResidualOut:
@@ -605,12 +624,25 @@ extern "C" int nnis_experts_many(int which, const void* x, const void* x_shared,
   const long long tile = wide ? 256 : 128;
   const long long cols = which == 0 ? (inner + tile / 2 - 1) / (tile / 2) : (width + tile - 1) / tile;
   const long long cols_shared = shared == 0 ? 0 : (which == 0 ? (shared + tile / 2 - 1) / (tile / 2) : cols);
-  long long blocks = row_blocks * cols + (long long)((tokens + 127) / 128) * cols_shared;
+  const long long shared_rows = (tokens + 127) / 128;
+  // How many column blocks a block takes, one or two: what leaves the fewest (rounds of blocks) x (an item's steps and its beginning
+  // and end, worth eight steps), for the row blocks that a fairly even choice makes.  (The sizes above at 2,048 rows, one and two: 76
+  // + 50 us and 67 + 48; in longer runs, at 4,096 and 8,192 rows, what one product gained the other lost.)
+  const long long likely_rows = pairs / 128 + (experts < pairs ? experts : pairs) / 2;
+  const long long steps = which == 0 ? (width + 63) / 64 : inner / 64;
+  long long run = 1, best = -1;
+  for (long long r = 1; r <= 2; ++r) {
+    const long long items = likely_rows * ((cols + r - 1) / r) + shared_rows * ((cols_shared + r - 1) / r);
+    const long long cost = (items + 255) / 256 * (r * steps + 8);
+    if (best < 0 || cost < best) best = cost, run = r;
+  }
+  long long blocks = row_blocks * ((cols + run - 1) / run) + shared_rows * ((cols_shared + run - 1) / run);
   blocks = (blocks + 7) / 8 * 8;
   NNIS_REQUIRE(blocks <= 0x7fffffff, "experts_many: the step exceeds the grid limit");
   ManyArgs a;
   a.x = (const bf16_t*)x; a.x_shared = (const bf16_t*)x_shared; a.w = (const bf16_t*)w; a.y = (bf16_t*)y; a.y_shared = (bf16_t*)y_shared;
   a.weights = weights; a.counts = counts; a.lists = lists; a.reg = reg; a.tokens = tokens; a.top = top; a.width = width;
+  a.run = (int)run;
   hipStream_t s = (hipStream_t)stream;
   // (beyond 64 KB a kernel has to be told once; a refusal shows as the launch's failure)
 #define NNIS_EXPERTS_TILED(UP_, BN_)                                                                                          \
