@@ -377,6 +377,20 @@ def test_experts_under_uneven_routing(rows, who):
     _close(part.forward(x.to(torch.bfloat16).cuda(), None, rt), want, "bfloat16", f"{rows} rows, {who}", bf16=2e-2)
 
 
+def test_experts_with_more_tiles_than_blocks_at_once():
+    """So many rows that a block of the tiled products takes two column blocks one after the other, and the last run of a
+    row block (three column blocks, the last one part full) only one."""
+    rt, part, plain_w, mlp = _routed(648, 264, 20, 3, 1.0, 136, 2.0, "bfloat16")
+    x = torch.randn(3000, 648, generator=torch.Generator().manual_seed(6)).to(torch.bfloat16).double()
+    want = T.routed_feed_forward(x, plain_w, mlp, T.bf16_round)[0]
+    clear = _clear(x, plain_w, 3)
+    assert float(clear.float().mean()) > 0.8
+    got = part.forward(x.to(torch.bfloat16).cuda(), None, rt).float().cpu()
+    _close(got[clear], want[clear], "bfloat16", "3000 rows", bf16=2e-2)
+    apart = torch.cat([part.forward(x[i:i + 300].to(torch.bfloat16).cuda(), None, rt).float().cpu() for i in range(0, 3000, 300)])
+    _close(got, apart.double(), "bfloat16", "in ten parts", bf16=1e-2)
+
+
 @pytest.mark.parametrize("rows", [1, 9, 16, 40, 100, 333])
 def test_experts_end_in_the_residual_stream(rows):
     """The last kernel adds to the 32-bit stream and prepares the norm that follows: what the next projection then makes
