@@ -1,7 +1,8 @@
 // Causal attention over the paged cache, compiled for one head size
 // (-DNNIS_HEAD_DIM=<n>).  A query token at position p of the sequence in
-// `slot` reads keys [lo, p] of that slot, lo = 0 or p + 1 - window, whatever
-// the step brought: the current step's keys are in the cache before this runs.
+// `slot` reads keys [lo, p] of that slot, lo = 0, p + 1 - window, or the start
+// of p's chunk of the sequence, whatever the step brought: the current step's
+// keys are in the cache before this runs.
 //
 // Formula (/root/reference/crates/nnis-model/src/kernels.rs:66-125): query
 // head h reads KV head h / (heads / kv_heads); score = dot(q, k) * scale, the
@@ -95,7 +96,7 @@ struct AttnArgs {
   const int* tok_slot;
   const int* tok_pos;
   int tokens, heads, kv_heads;
-  int window;  // 0: all keys
+  int window;  // 0: all keys; n > 0: the last n; n < 0: those of the query's own chunk of -n positions (counted from position 0)
   float scale;
   float softcap;  // 0: none; else a score s becomes softcap * tanh(s / softcap)
   // Beyond the plain formula, each off when zero or null:
@@ -113,6 +114,12 @@ struct AttnArgs {
   int pool;
   NnisHeadTerms terms;
 };
+
+// the first key that a query at position `pos` (not negative) sees: see AttnArgs::window.  It never falls as pos rises.
+__device__ __forceinline__ int first_seen(int window, int pos) {
+  if (window < 0) return pos - pos % -window;
+  return (window > 0 && pos + 1 > window) ? pos + 1 - window : 0;
+}
 
 __device__ __forceinline__ float head_gate(const NnisHeadTerms& terms, size_t token, int head) {
   return 1.0f / (1.0f + expf(-load_as_f32(terms.gate, terms.gate_dtype, token * terms.gate_stride + head)));
@@ -139,7 +146,7 @@ __global__ __launch_bounds__(256) void attention_rows_kernel(AttnArgs a) {
   const int pos = a.tok_pos[token];
   const int kv_head = head / (a.heads / a.kv_heads);
   const int kv_len = pos + 1;
-  const int lo = (a.window > 0 && kv_len > a.window) ? kv_len - a.window : 0;
+  const int lo = first_seen(a.window, pos);
 
   float* qs = q_shared[wave];
   for (int d = lane; d < HD; d += kWave) qs[d] = load_as_f32(a.q, a.q_dtype, row + d);
@@ -1017,7 +1024,7 @@ __global__ __launch_bounds__(64 * kBlockWaves) void attention_prefill_kernel(Mfm
         q[c] = load_row_operand(a.q + ((size_t)(start + safe_row) * a.heads + safe_head) * HD, g);
         gates[c] = ask_gate(a.terms, start + safe_row, safe_head);
         hi[c] = live[c] ? pos0 + row : -1;
-        lo[c] = (a.window > 0 && hi[c] + 1 > a.window) ? hi[c] + 1 - a.window : 0;
+        lo[c] = live[c] ? first_seen(a.window, hi[c]) : 0;
         last = hi[c] > last ? hi[c] : last;
       }
     // the wave runs to the farthest key any of its columns reads, from the nearest
@@ -1186,7 +1193,7 @@ __global__ __launch_bounds__(64 * kBlockWaves) void attention_decode_kernel(Mfma
   }
   const int group = a.heads / a.kv_heads;
   const int pos = a.tok_pos[token];
-  const int first_key = (a.window > 0 && pos + 1 > a.window) ? pos + 1 - a.window : 0;
+  const int first_key = first_seen(a.window, pos);
   const int* pages = a.block_table + (size_t)(a.rows_by_token ? token : slot) * a.max_pages;
 
   QFrag q[C];
@@ -1285,7 +1292,7 @@ __global__ __launch_bounds__(64 * kKeysWaves) void attention_decode_keys_kernel(
   }
   const int group = a.heads / a.kv_heads;
   const int pos = a.tok_pos[token];
-  const int first_key = (a.window > 0 && pos + 1 > a.window) ? pos + 1 - a.window : 0;
+  const int first_key = first_seen(a.window, pos);
   const int* pages = a.block_table + (size_t)(a.rows_by_token ? token : slot) * a.max_pages;
 
   // the end's columns are the heads r of the group; the scores' are the heads j
@@ -1524,7 +1531,7 @@ extern "C" int nnis_attention_rows_terms(const void* q, int q_dtype, void* out, 
                "attention: unknown dtype (q %d, out %d, cache %d)", q_dtype, out_dtype, cache_dtype);
   NNIS_REQUIRE(heads > 0 && kv_heads > 0 && heads % kv_heads == 0, "attention: %d heads do not divide into %d kv heads",
                heads, kv_heads);
-  NNIS_REQUIRE(window >= 0 && max_pages > 0, "attention: bad window %d or block table width %d", window, max_pages);
+  NNIS_REQUIRE(window > -(1 << 30) && max_pages > 0, "attention: bad window %d or block table width %d", window, max_pages);
   NNIS_REQUIRE(keep_first >= 0 && (bias == nullptr || reach >= 0), "attention: bad keep_first %d or reach %d", keep_first, reach);
   if (tokens <= 0) return 0;
   AttnArgs a;
@@ -1589,7 +1596,7 @@ int fill_common(MfmaArgs& a, const void* q, void* out, const void* k_pages, cons
                "attention: this module is compiled %s a cap of the scores, got a cap of %g", NNIS_SCORE_CAP ? "with" : "without", (double)softcap);
   NNIS_REQUIRE(heads > 0 && kv_heads > 0 && heads % kv_heads == 0, "attention: %d heads do not divide into %d kv heads",
                heads, kv_heads);
-  NNIS_REQUIRE(window >= 0 && max_pages > 0, "attention: bad window %d or block table width %d", window, max_pages);
+  NNIS_REQUIRE(window > -(1 << 30) && max_pages > 0, "attention: bad window %d or block table width %d", window, max_pages);
   NNIS_REQUIRE(scale > 0.0f, "attention: the scale of the scores must be positive");
   NNIS_REQUIRE(((uintptr_t)q % 16 == 0) && ((uintptr_t)out % 16 == 0) && ((uintptr_t)k_pages % 16 == 0) &&
                    ((uintptr_t)v_pages % 16 == 0),

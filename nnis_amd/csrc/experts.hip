@@ -6,6 +6,7 @@
 // by both projections), so that regions begin at strips of `up` and at chunks of `down`:
 //   up    [experts x (gate rows | up rows) | shared gate rows | shared up rows][width]
 //   down  [width][experts x inner | shared inner]
+// The shared expert's weight may be a number a token instead of one (`shared_weights` [tokens]).
 // Between the two, a region's value is weight * act(gate, up), act by `form`: 1 silu(a) u; 2 the clamped gate
 // a sigmoid(1.702 a) (u + 1) with a held at most at the region's limit and u within plus or minus it (0: not held).
 //
@@ -54,8 +55,8 @@ constexpr int kMostExperts = 1024;
 // product does not read it).
 template <int KSPLIT>
 __global__ __launch_bounds__(64 * KSPLIT) void experts_up_few_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ w,
-                                                                     const float* __restrict__ gates, bf16_t* __restrict__ hidden, Regions reg,
-                                                                     int m, int k) {
+                                                                     const float* __restrict__ gates, const float* __restrict__ shared_weights,
+                                                                     bf16_t* __restrict__ hidden, Regions reg, int m, int k) {
   __shared__ float partial[KSPLIT][2][kWave][4];
   const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave, r = lane % 16, g = lane / 16;
   const int units = reg.inner / 16, shared_units = reg.shared / 16;
@@ -67,6 +68,8 @@ __global__ __launch_bounds__(64 * KSPLIT) void experts_up_few_kernel(const bf16_
   if (!is_shared) {
     weight = r < m ? gates[(size_t)r * reg.experts + region] : 0.0f;
     if (!__any(weight != 0.0f)) return;  // (all waves of the block see the same)
+  } else if (shared_weights) {
+    weight = r < m ? shared_weights[r] : 0.0f;
   }
   const int strip = is_shared ? reg.experts * 2 * units + unit : region * 2 * units + unit;
   const int strip_up = strip + (is_shared ? shared_units : units);
@@ -249,6 +252,7 @@ struct ManyArgs {
   bf16_t* y;               // UP: hidden rows of the pairs; DOWN: the pairs' outputs [tokens * top][width]
   bf16_t* y_shared;        // of the shared expert: [tokens][shared] or [tokens][width]
   const float* weights;    // [tokens * top]
+  const float* shared_weights;  // [tokens] or null: ones
   const int* counts;
   const int* lists;
   Regions reg;
@@ -402,7 +406,7 @@ __global__ __launch_bounds__(512) void experts_tiled_kernel(ManyArgs a) {
     const bool live = row < rows;
     row = live ? row : rows - 1;
     const int to = list ? list[row] : row;
-    weight[i] = !UP && list ? a.weights[to] : 1.0f;
+    weight[i] = UP ? 1.0f : (list ? a.weights[to] : (a.shared_weights ? a.shared_weights[to] : 1.0f));
     out_row[i] = live ? to : -1;
   }
   wait_loads_but<0>();
@@ -538,8 +542,8 @@ int check_regions(const char* what, const Regions& reg) {
 
 }  // namespace
 
-// x [m, k] bfloat16, gates float32 [m, experts], hidden [m, experts * inner + shared]; m <= 16
-extern "C" int nnis_experts_up_few(const void* x, const void* w, const float* gates, void* hidden, int m, int k, int experts, int inner, int shared,
+// x [m, k] bfloat16, gates float32 [m, experts], shared_weights float32 [m] or null, hidden [m, experts * inner + shared]; m <= 16
+extern "C" int nnis_experts_up_few(const void* x, const void* w, const float* gates, const float* shared_weights, void* hidden, int m, int k, int experts, int inner, int shared,
                                    int form, float limit, float shared_limit, void* stream) {
   const Regions reg = {experts, inner, shared, form, limit, shared_limit};
   if (check_regions("experts_up_few", reg)) return 1;
@@ -552,7 +556,7 @@ extern "C" int nnis_experts_up_few(const void* x, const void* w, const float* ga
   hipStream_t s = (hipStream_t)stream;
 #define NNIS_UP_FEW(SPLIT_)                                                                                                          \
   hipLaunchKernelGGL((experts_up_few_kernel<SPLIT_>), dim3(blocks), dim3(64 * SPLIT_), 0, s, (const bf16_t*)x, (const bf16_t*)w, gates, \
-                     (bf16_t*)hidden, reg, m, k)
+                     shared_weights, (bf16_t*)hidden, reg, m, k)
   // (rows of 2,048 channels, 16 experts of 704: 11 of them chosen 17.7 us with 8 waves, 19.8 with 4 and 20.7 with 16; 2 of them
   // 7.8, 6.3 and 8.1)
   if (chunks > 16 && m > 2) NNIS_UP_FEW(8);
@@ -605,9 +609,9 @@ extern "C" int nnis_experts_lists(const int* chosen, int tokens, int top, int ex
 
 // which 0: `up`, x [tokens, width] -> y [tokens * top, inner], y_shared [tokens, shared];
 // which 1: `down`, x [tokens * top, inner], x_shared [tokens, shared] -> y [tokens * top, width] (each row times its pair's
-// weight), y_shared [tokens, width].  Rows whose pair chose no expert of the lists do not exist: every pair has its expert.
+// weight, the shared expert's times its token's shared_weights where given), y_shared [tokens, width].  Rows whose pair chose no expert of the lists do not exist: every pair has its expert.
 extern "C" int nnis_experts_many(int which, const void* x, const void* x_shared, const void* w, void* y, void* y_shared, const float* weights,
-                                 const int* counts, const int* lists, int tokens, int top, int width, int experts, int inner, int shared, int form,
+                                 const float* shared_weights, const int* counts, const int* lists, int tokens, int top, int width, int experts, int inner, int shared, int form,
                                  float limit, float shared_limit, void* stream) {
   const Regions reg = {experts, inner, shared, form, limit, shared_limit};
   if (check_regions("experts_many", reg)) return 1;
@@ -641,7 +645,7 @@ extern "C" int nnis_experts_many(int which, const void* x, const void* x_shared,
   NNIS_REQUIRE(blocks <= 0x7fffffff, "experts_many: the step exceeds the grid limit");
   ManyArgs a;
   a.x = (const bf16_t*)x; a.x_shared = (const bf16_t*)x_shared; a.w = (const bf16_t*)w; a.y = (bf16_t*)y; a.y_shared = (bf16_t*)y_shared;
-  a.weights = weights; a.counts = counts; a.lists = lists; a.reg = reg; a.tokens = tokens; a.top = top; a.width = width;
+  a.weights = weights; a.shared_weights = shared_weights; a.counts = counts; a.lists = lists; a.reg = reg; a.tokens = tokens; a.top = top; a.width = width;
   a.run = (int)run;
   hipStream_t s = (hipStream_t)stream;
   // (beyond 64 KB a kernel has to be told once; a refusal shows as the launch's failure)

@@ -2,7 +2,8 @@
 // selective scan (a diagonal recurrence per channel with input-dependent steps), gated linear attention (a
 // matrix state per head with a decay per key channel; with one fixed decay a head and turned queries and keys it
 // is retention), the per-head norm and gate behind it, the minGRU, and the gated delta rule (a matrix state per
-// head whose every token first takes back what the state already holds under its key).
+// head whose every token first takes back what the state already holds under its key), and the real-gated linear
+// recurrent unit.
 //
 // A step's rows are packed: sequence b of the step owns rows seq_start[b] .. seq_start[b + 1] - 1, which
 // continue the sequence in slot seq_slot[b] (negative: padding, nothing is read or written for it).  State
@@ -33,9 +34,11 @@ __device__ __forceinline__ float softplus_f(float z) {
 __device__ __forceinline__ float log_sigmoid_f(float z) { return fminf(z, 0.0f) - log1pf(expf(-fabsf(z))); }
 
 // -----------------------------------------------------------------------------
-// Causal convolution per channel with SiLU: y[t, c] = silu(b[c] + sum_j w[c, j] x[t - (taps - 1) + j, c]),
-// the last tap on the token itself, zeros before the sequence's start.  Inputs older than the step's first
-// row come from `state` [slots, taps - 1, channels] (the sequence's last taps - 1 inputs, oldest first).
+// Causal convolution per channel: y[t, c] = act(b[c] + sum_j w[c, j] x[t - (taps - 1) + j, c]), act SiLU or the
+// identity, the last tap on the token itself, zeros before the sequence's start.  With x_bias an input is x + x_bias[c].
+// Inputs older than the step's first row come from `state` [slots, taps - 1, channels] (the sequence's last taps - 1
+// inputs, oldest first), or, with `ring`, from [slots, taps, channels]: position p's input is row p % taps, so that a
+// step of single tokens writes a row that nobody reads in it (kernels that take the convolution in count on that).
 // -----------------------------------------------------------------------------
 constexpr int kMostTaps = 16;
 
@@ -54,15 +57,24 @@ struct ConvArgs {
   int tokens, batch, channels, taps;
   void* y;  // [tokens, channels]
   int y_dtype;
+  const float* x_bias;  // [channels] or null
+  int plain;            // 1: no activation
+  int ring;
 };
+
+__device__ __forceinline__ float conv_fresh(const ConvArgs& a, int token, int c) {
+  const float x = load_as_f32(a.x, a.x_dtype, (size_t)token * a.x_stride + c);
+  return a.x_bias ? x + a.x_bias[c] : x;
+}
+__device__ __forceinline__ float conv_act(const ConvArgs& a, float v) { return a.plain ? v : v * sigmoid_f(v); }
 
 // the input `back` tokens before row `token` of the sequence in `slot` at position `pos` (back <= pos): a row of
 // this step while the rows belong to the sequence, then the state's rows, newest last
-__device__ __forceinline__ float conv_input(const ConvArgs& a, int token, int slot, int back, int c, bool& in_step, int& behind) {
-  if (in_step && token - back >= 0 && a.tok_slot[token - back] == slot)
-    return load_as_f32(a.x, a.x_dtype, (size_t)(token - back) * a.x_stride + c);
+__device__ __forceinline__ float conv_input(const ConvArgs& a, int token, int slot, int pos, int back, int c, bool& in_step, int& behind) {
+  if (in_step && token - back >= 0 && a.tok_slot[token - back] == slot) return conv_fresh(a, token - back, c);
   in_step = false;
   ++behind;
+  if (a.ring) return a.state[((size_t)slot * a.taps + (pos - back) % a.taps) * a.channels + c];
   return a.state[((size_t)slot * (a.taps - 1) + (a.taps - 1 - behind)) * a.channels + c];
 }
 
@@ -83,7 +95,7 @@ __global__ __launch_bounds__(256) void conv_silu_kernel(ConvArgs a) {
   const float bias = a.bias ? load_as_f32(a.bias, a.weight_dtype, c) : 0.0f;
   float fresh[kConvStrip];  // the strip's own inputs, all asked for at once
 #pragma unroll
-  for (int i = 0; i < kConvStrip; ++i) fresh[i] = begin + i < end ? load_as_f32(a.x, a.x_dtype, (size_t)(begin + i) * a.x_stride + c) : 0.0f;
+  for (int i = 0; i < kConvStrip; ++i) fresh[i] = begin + i < end ? conv_fresh(a, begin + i, c) : 0.0f;
   int before = -2;  // the slot of the row before, if its inputs are held
 #pragma unroll
   for (int i = 0; i < kConvStrip; ++i) {
@@ -109,7 +121,7 @@ __global__ __launch_bounds__(256) void conv_silu_kernel(ConvArgs a) {
 #pragma unroll
       for (int back = 0; back < kMostTaps; ++back) {
         if (back < a.taps) {
-          const float v = back <= pos ? conv_input(a, token, slot, back, c, in_step, behind) : 0.0f;  // zeros before the start
+          const float v = back <= pos ? conv_input(a, token, slot, pos, back, c, in_step, behind) : 0.0f;  // zeros before the start
 #pragma unroll
           for (int j = 0; j < kMostTaps; ++j)
             if (j == a.taps - 1 - back) held[j] = v;
@@ -120,7 +132,7 @@ __global__ __launch_bounds__(256) void conv_silu_kernel(ConvArgs a) {
     float acc = bias;
 #pragma unroll
     for (int j = 0; j < kMostTaps; ++j) acc = fmaf(w[j], held[j], acc);  // (beyond the taps: zeros)
-    store_from_f32(a.y, a.y_dtype, (size_t)token * a.channels + c, acc * sigmoid_f(acc));
+    store_from_f32(a.y, a.y_dtype, (size_t)token * a.channels + c, conv_act(a, acc));
   }
 }
 
@@ -137,8 +149,21 @@ __global__ __launch_bounds__(256) void conv_single_kernel(ConvArgs a) {
     return;
   }
   const int keep = a.taps - 1;
+  const float now = conv_fresh(a, token, c);
+  if (a.ring) {
+    const int pos = a.tok_pos[token];
+    float* rows = a.state + (size_t)slot * a.taps * a.channels + c;
+    float sum = a.bias ? load_as_f32(a.bias, a.weight_dtype, c) : 0.0f;
+    for (int j = 0; j < keep; ++j) {
+      const int at = pos - keep + j;
+      if (at >= 0) sum = fmaf(load_as_f32(a.weight, a.weight_dtype, (size_t)c * a.taps + j), rows[(size_t)(at % a.taps) * a.channels], sum);
+    }
+    sum = fmaf(load_as_f32(a.weight, a.weight_dtype, (size_t)c * a.taps + keep), now, sum);
+    store_from_f32(a.y, a.y_dtype, (size_t)token * a.channels + c, conv_act(a, sum));
+    rows[(size_t)(pos % a.taps) * a.channels] = now;
+    return;
+  }
   float* state = a.state + (size_t)slot * keep * a.channels + c;
-  const float now = load_as_f32(a.x, a.x_dtype, (size_t)token * a.x_stride + c);
   float acc = a.bias ? load_as_f32(a.bias, a.weight_dtype, c) : 0.0f;
   float older[kMostTaps];
 #pragma unroll
@@ -147,7 +172,7 @@ __global__ __launch_bounds__(256) void conv_single_kernel(ConvArgs a) {
     if (j < keep) acc = fmaf(load_as_f32(a.weight, a.weight_dtype, (size_t)c * a.taps + j), older[j], acc);
   }
   acc = fmaf(load_as_f32(a.weight, a.weight_dtype, (size_t)c * a.taps + keep), now, acc);
-  store_from_f32(a.y, a.y_dtype, (size_t)token * a.channels + c, acc * sigmoid_f(acc));
+  store_from_f32(a.y, a.y_dtype, (size_t)token * a.channels + c, conv_act(a, acc));
 #pragma unroll
   for (int j = 0; j < kMostTaps; ++j)
     if (j < keep) state[(size_t)j * a.channels] = j + 1 < keep ? older[j + 1] : now;
@@ -162,6 +187,12 @@ __global__ void conv_state_kernel(ConvArgs a) {
   if (slot < 0 || c >= a.channels) return;
   const int first = a.seq_start[b], count = a.seq_start[b + 1] - first;
   if (count <= 0) return;
+  if (a.ring) {
+    const int pos0 = a.tok_pos[first];
+    for (int i = max(0, count - a.taps); i < count; ++i)
+      a.state[((size_t)slot * a.taps + (pos0 + i) % a.taps) * a.channels + c] = conv_fresh(a, first + i, c);
+    return;
+  }
   const int keep = a.taps - 1;
   float* state = a.state + (size_t)slot * keep * a.channels + c;
   float fresh[kMostTaps];
@@ -169,7 +200,7 @@ __global__ void conv_state_kernel(ConvArgs a) {
   for (int j = 0; j < kMostTaps; ++j) {
     if (j < keep) {
       const int back = keep - 1 - j;  // new row j holds the input `back` tokens before the run's last
-      fresh[j] = back < count ? load_as_f32(a.x, a.x_dtype, (size_t)(first + count - 1 - back) * a.x_stride + c)
+      fresh[j] = back < count ? conv_fresh(a, first + count - 1 - back, c)
                               : state[(size_t)(j + count) * a.channels];
     }
   }
@@ -592,16 +623,17 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __rest
 
 extern "C" int nnis_conv_silu(const void* x, int x_dtype, int x_stride, const void* weight, const void* bias, int weight_dtype,
                               float* state, const int* tok_slot, const int* tok_pos, const int* seq_slot, const int* seq_start,
-                              int tokens, int batch, int channels, int taps, void* y, int y_dtype, int single, void* stream) {
+                              int tokens, int batch, int channels, int taps, void* y, int y_dtype, int single, const float* x_bias, int plain, int ring,
+                              void* stream) {
   NNIS_REQUIRE(nnis_dtype_ok(x_dtype) && nnis_dtype_ok(weight_dtype) && nnis_dtype_ok(y_dtype), "conv: unknown dtype");
   NNIS_REQUIRE(taps >= 1 && taps <= kMostTaps, "conv: 1 to %d taps are taken, got %d", kMostTaps, taps);
   NNIS_REQUIRE(channels > 0 && x_stride >= channels && tokens >= 0 && batch >= 0, "conv: bad sizes");
-  NNIS_REQUIRE(x && weight && tok_slot && tok_pos && seq_slot && seq_start && y && (state || taps == 1), "conv: a pointer is missing");
+  NNIS_REQUIRE(x && weight && tok_slot && tok_pos && seq_slot && seq_start && y && (state || (taps == 1 && !ring)), "conv: a pointer is missing");
   if (tokens == 0 || batch == 0) return 0;
   ConvArgs a;
   a.x = x; a.x_dtype = x_dtype; a.x_stride = x_stride; a.weight = weight; a.bias = bias; a.weight_dtype = weight_dtype; a.state = state;
   a.tok_slot = tok_slot; a.tok_pos = tok_pos; a.seq_slot = seq_slot; a.seq_start = seq_start; a.tokens = tokens; a.batch = batch;
-  a.channels = channels; a.taps = taps; a.y = y; a.y_dtype = y_dtype;
+  a.channels = channels; a.taps = taps; a.y = y; a.y_dtype = y_dtype; a.x_bias = x_bias; a.plain = plain; a.ring = ring;
   NNIS_REQUIRE(batch <= 65535 && (tokens + kConvStrip - 1) / kConvStrip <= 65535, "conv: too many rows or sequences for the grid");
   const int width = channels >= 256 ? 256 : 64;
   if (single) {  // every sequence brings one token: row b is sequence b's
@@ -613,7 +645,7 @@ extern "C" int nnis_conv_silu(const void* x, int x_dtype, int x_stride, const vo
   hipLaunchKernelGGL(conv_silu_kernel, dim3((channels + width - 1) / width, (tokens + kConvStrip - 1) / kConvStrip), dim3(width), 0,
                      (hipStream_t)stream, a);
   NNIS_LAUNCH_CHECK("conv_silu");
-  if (taps > 1) {
+  if (taps > 1 || ring) {
     const int threads = channels >= 256 ? 256 : 64;
     hipLaunchKernelGGL(conv_state_kernel, dim3((channels + threads - 1) / threads, batch), dim3(threads), 0, (hipStream_t)stream, a);
     NNIS_LAUNCH_CHECK("conv_state");
@@ -1169,5 +1201,122 @@ extern "C" int nnis_gated_delta(const void* rows, int dtype, int stride, const f
     default: hipLaunchKernelGGL(gated_delta_kernel<32>, grid, dim3(256), lds, s, a); break;
   }
   NNIS_LAUNCH_CHECK("gated_delta");
+  return 0;
+}
+
+// -----------------------------------------------------------------------------
+// The real-gated linear recurrent unit's recurrence.  Per channel c of row t, with the gates' logits zr and zi:
+//     log a = -8 sigmoid(zr + br) rate,   rate = softplus(lam) ready-made
+//     S <- a S + sqrt(1 - a^2) sigmoid(zi + bi) u,   out = S * gelu_tanh(y + by)
+// over each sequence's rows, from and into state [slots, width] (32-bit).  logits [tokens, blocks, 2, width / blocks]: a
+// block's zr, then its zi.  A thread a channel; a long run is cut into pieces as the minGRU's.
+// -----------------------------------------------------------------------------
+namespace {
+
+struct UnitArgs {
+  const float* logits;
+  const float* r_bias;
+  const float* i_bias;
+  const float* rate;
+  const void* u;  // [tokens, u_stride]
+  int u_dtype, u_stride;
+  const void* y;  // [tokens, y_stride]
+  int y_dtype, y_stride;
+  const float* y_bias;
+  float* state;
+  const int* seq_slot;
+  const int* seq_start;
+  int batch, width, block;  // block: channels of one of the gates' maps
+  void* out;
+  int out_dtype;
+  int piece, pieces;
+  float* decay;  // [batch, pieces, width]: a piece's sum of log a
+  float* ends;   // [batch, pieces, width]: a piece's end state from zero
+};
+
+__device__ __forceinline__ float gelu_tanh_f(float z) {
+  const float t = 0.7978845608028654f * fmaf(0.044715f * z * z, z, z);
+  return z * sigmoid_f(2.0f * t);  // (1 + tanh t) / 2 = sigmoid(2 t)
+}
+
+template <int PASS>
+__global__ __launch_bounds__(256) void rg_lru_kernel(UnitArgs a) {
+  const int c = blockIdx.x * blockDim.x + threadIdx.x;
+  const int b = blockIdx.y / a.pieces, piece = blockIdx.y % a.pieces;
+  const int slot = a.seq_slot[b];
+  if (slot < 0 || c >= a.width) return;
+  const int start = a.seq_start[b], stop = a.seq_start[b + 1];
+  int first = start, last = stop;
+  if (a.pieces > 1) {
+    first = start + piece * a.piece;
+    last = min(stop, first + a.piece);
+    if (first >= stop) return;
+    if (PASS == 1 && last == stop && piece > 0) return;
+  }
+  const float br = a.r_bias[c], bi = a.i_bias[c], by = a.y_bias ? a.y_bias[c] : 0.0f, rate = -8.0f * a.rate[c];
+  const size_t gate_at = (size_t)(c / a.block) * 2 * a.block + c % a.block;
+  float s = 0.0f, logs = 0.0f;
+  const size_t mine = ((size_t)b * a.pieces + piece) * a.width + c;
+  if (a.pieces == 1) {
+    s = a.state[(size_t)slot * a.width + c];
+  } else if (PASS == 1) {
+    if (piece == 0) a.decay[mine] = s = a.state[(size_t)slot * a.width + c];  // (a copy of the state: see the minGRU)
+  } else if (piece == 0) {
+    s = a.decay[mine];
+  } else {
+    s = a.ends[(size_t)b * a.pieces * a.width + c];
+#pragma unroll 8
+    for (int k = 1; k < piece; ++k) {
+      const size_t at = ((size_t)b * a.pieces + k) * a.width + c;
+      s = fmaf(expf(a.decay[at]), s, a.ends[at]);
+    }
+  }
+#pragma unroll 4
+  for (int t = first; t < last; ++t) {
+    const float zr = a.logits[(size_t)t * 2 * a.width + gate_at] + br;
+    const float zi = a.logits[(size_t)t * 2 * a.width + gate_at + a.block] + bi;
+    const float u = load_as_f32(a.u, a.u_dtype, (size_t)t * a.u_stride + c);
+    const float log_a = rate / (1.0f + expf(-zr));
+    const float keep = expf(log_a);
+    s = fmaf(keep, s, sqrtf(-expm1f(2.0f * log_a)) * (u / (1.0f + expf(-zi))));
+    if (PASS == 1) {
+      logs += log_a;
+    } else {
+      const float y = load_as_f32(a.y, a.y_dtype, (size_t)t * a.y_stride + c) + by;
+      store_from_f32(a.out, a.out_dtype, (size_t)t * a.width + c, s * gelu_tanh_f(y));
+    }
+  }
+  if (PASS == 1) {
+    if (piece > 0) a.decay[mine] = logs;
+    a.ends[mine] = s;
+  } else if (last == stop) {
+    a.state[(size_t)slot * a.width + c] = s;
+  }
+}
+
+}  // namespace
+
+extern "C" int nnis_rg_lru(const float* logits, const float* r_bias, const float* i_bias, const float* rate, const void* u, int u_dtype,
+                           int u_stride, const void* y, int y_dtype, int y_stride, const float* y_bias, float* state, const int* seq_slot,
+                           const int* seq_start, int batch, int width, int block, void* out, int out_dtype, int piece, int pieces,
+                           float* decay, float* ends, void* stream) {
+  NNIS_REQUIRE(logits && r_bias && i_bias && rate && u && y && state && seq_slot && seq_start && out, "rg_lru: missing operand");
+  NNIS_REQUIRE(nnis_dtype_ok(u_dtype) && nnis_dtype_ok(y_dtype) && nnis_dtype_ok(out_dtype), "rg_lru: unknown dtype");
+  NNIS_REQUIRE(width > 0 && block > 0 && width % block == 0 && u_stride >= width && y_stride >= width, "rg_lru: bad sizes (%d channels in blocks of %d)", width, block);
+  NNIS_REQUIRE(pieces >= 1 && (pieces == 1 || (piece > 0 && decay && ends)) && (long long)batch * pieces <= 65535, "rg_lru: bad pieces");
+  if (batch <= 0) return 0;
+  UnitArgs a;
+  a.logits = logits; a.r_bias = r_bias; a.i_bias = i_bias; a.rate = rate; a.u = u; a.u_dtype = u_dtype; a.u_stride = u_stride;
+  a.y = y; a.y_dtype = y_dtype; a.y_stride = y_stride; a.y_bias = y_bias; a.state = state; a.seq_slot = seq_slot; a.seq_start = seq_start;
+  a.batch = batch; a.width = width; a.block = block; a.out = out; a.out_dtype = out_dtype; a.piece = piece; a.pieces = pieces;
+  a.decay = decay; a.ends = ends;
+  const int threads = width >= 256 ? 256 : 64;
+  const dim3 grid((width + threads - 1) / threads, batch * pieces);
+  if (pieces > 1) {
+    hipLaunchKernelGGL(rg_lru_kernel<1>, grid, dim3(threads), 0, (hipStream_t)stream, a);
+    NNIS_LAUNCH_CHECK("rg_lru (first pass)");
+  }
+  hipLaunchKernelGGL(rg_lru_kernel<2>, grid, dim3(threads), 0, (hipStream_t)stream, a);
+  NNIS_LAUNCH_CHECK("rg_lru");
   return 0;
 }

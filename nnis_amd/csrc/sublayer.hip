@@ -336,12 +336,18 @@ constexpr int kRouteMost = 16;  // outputs a lane holds: n <= 64 * kRouteMost
 // one row by one wave; `logits`: the row's n logits (global memory or LDS)
 // group_count > 1: the outputs form that many equal groups of neighbours; a group's mark is its largest corrected
 // score, and only outputs of the group_keep groups with the largest marks (the lower group on a tie) can be chosen.
-// bias: joins the logits before anything else (null: none).  chosen_softmax: outputs are chosen by logit (+ correction)
-// and the weights are the softmax over the chosen logits alone.
+// With group_marks 2 the mark is the sum of the group's two largest.
+// bias: joins the logits before anything else (null: none).  scoring kChosenSoftmax: outputs are chosen by logit (+ correction)
+// and the weights are the softmax over the chosen logits alone; kSigmoid: s = sigmoid(logits), and the weights are the chosen
+// scores over their sum (+ 1e-20), times weight_scale.  shared_gate: the logits have one more behind the n outputs, whose sigmoid
+// is keep[row].
+enum : int { kSoftmax = 0, kChosenSoftmax = 1, kSigmoid = 2 };
 struct RouteRule {
   const float* bias;
   const float* correction;
-  int chosen_softmax, group_count, group_keep;
+  int scoring, group_count, group_keep;
+  float weight_scale;
+  int group_marks, shared_gate;
   int* chosen;     // [rows, top] or null: the chosen outputs, best first
   float* weights;  // [rows, top], with `chosen`: their weights
 };
@@ -361,20 +367,26 @@ __device__ __forceinline__ void route_row_slots(const float* logits, const Route
     choice[i] = s[i];  // (stays where outputs are chosen by logit)
     top_logit = fmaxf(top_logit, s[i]);
   }
-  top_logit = wave_max(top_logit);
-  float sum = 0.0f;
+  float inv = 1.0f;
+  if (rule.scoring == kSigmoid) {
 #pragma unroll
-  for (int i = 0; i < SLOTS; ++i) {
-    s[i] = (i * kWave + lane) < n ? expf(s[i] - top_logit) : 0.0f;
-    sum += s[i];
+    for (int i = 0; i < SLOTS; ++i) s[i] = (i * kWave + lane) < n ? 1.0f / (1.0f + expf(-s[i])) : 0.0f;
+  } else {
+    top_logit = wave_max(top_logit);
+    float sum = 0.0f;
+#pragma unroll
+    for (int i = 0; i < SLOTS; ++i) {
+      s[i] = (i * kWave + lane) < n ? expf(s[i] - top_logit) : 0.0f;
+      sum += s[i];
+    }
+    if (rule.scoring == kSoftmax) inv = 1.0f / wave_sum(sum);
   }
-  const float inv = rule.chosen_softmax ? 1.0f : 1.0f / wave_sum(sum);
   unsigned chosen = 0;
 #pragma unroll
   for (int i = 0; i < SLOTS; ++i) {
     const int e = i * kWave + lane;
     s[i] *= inv;
-    choice[i] = e < n ? (rule.chosen_softmax ? choice[i] : s[i]) + (correction ? correction[e] : 0.0f) : -INFINITY;
+    choice[i] = e < n ? (rule.scoring == kChosenSoftmax ? choice[i] : s[i]) + (correction ? correction[e] : 0.0f) : -INFINITY;
   }
   if (group_count > 1 && group_keep < group_count) {
     // lane g holds group g's mark (up to 64 groups); the kept groups are found one at a time
@@ -387,8 +399,27 @@ __device__ __forceinline__ void route_row_slots(const float* logits, const Route
         const int e = i * kWave + lane;
         if (e < n && e / size == g) best = fmaxf(best, choice[i]);
       }
-      best = wave_max(best);
-      if (lane == g) mark = best;
+      const float largest = wave_max(best);
+      float marks = largest;
+      if (rule.group_marks > 1 && size > 1) {
+        // the second largest: without one holder of the largest (the first lane that has it)
+        const int holder = __ffsll(__ballot(best == largest)) - 1;
+        float second = best;
+        if (lane == holder) {
+          second = -INFINITY;
+          bool passed = false;
+#pragma unroll
+          for (int i = 0; i < SLOTS; ++i) {
+            const int e = i * kWave + lane;
+            if (e < n && e / size == g) {
+              if (!passed && choice[i] == largest) passed = true;
+              else second = fmaxf(second, choice[i]);
+            }
+          }
+        }
+        marks += wave_max(second);
+      }
+      if (lane == g) mark = marks;
     }
     unsigned long long allowed = 0ull;
     for (int round = 0; round < group_keep; ++round) {
@@ -457,7 +488,8 @@ __device__ __forceinline__ void route_row_slots(const float* logits, const Route
       }
     }
   }
-  const float share = rule.chosen_softmax ? 1.0f / wave_sum(weight) : 1.0f;
+  const float share = rule.scoring == kSoftmax ? 1.0f
+                      : (rule.scoring == kSigmoid ? rule.weight_scale / (wave_sum(weight) + 1e-20f) : 1.0f / wave_sum(weight));
 #pragma unroll
   for (int i = 0; i < SLOTS; ++i) {
     const int e = i * kWave + lane;
@@ -468,7 +500,7 @@ __device__ __forceinline__ void route_row_slots(const float* logits, const Route
     rule.weights[(size_t)row * top + lane] = picked_weight * share;
   }
   kept = wave_sum(kept) * share;
-  if (lane == 0) keep[row] = kept;
+  if (lane == 0) keep[row] = rule.shared_gate ? 1.0f / (1.0f + expf(-logits[n])) : kept;
 }
 
 __device__ __forceinline__ void route_row(const float* logits, const RouteRule& rule, int row, int n, int experts, int top,
@@ -481,7 +513,7 @@ __global__ __launch_bounds__(256) void route_top_kernel(const float* __restrict_
                                                         int top, float* __restrict__ gates, float* __restrict__ keep) {
   const int row = blockIdx.x * 4 + threadIdx.x / kWave;
   if (row >= rows) return;
-  route_row(logits + (size_t)row * n, rule, row, n, experts, top, gates, keep, threadIdx.x % kWave);
+  route_row(logits + (size_t)row * (n + rule.shared_gate), rule, row, n, experts, top, gates, keep, threadIdx.x % kWave);
 }
 
 // the dot products of R rows with every output's weights, into `out` [R][n] (LDS or global memory with a row stride
@@ -526,7 +558,7 @@ template <int R>
 __global__ __launch_bounds__(R == 1 ? 1024 : 256) void route_kernel(const void* __restrict__ x, int x_dtype, const float* __restrict__ w,
                                                     RouteRule rule, int rows, int n, int width, int experts, int top,
                                                     float* __restrict__ gates, float* __restrict__ keep) {
-  extern __shared__ __attribute__((aligned(16))) float lds[];  // [R][width] rows, then [R][n] logits
+  extern __shared__ __attribute__((aligned(16))) float lds[];  // [R][width] rows, then [R][n (+ 1)] logits
   float* xs = lds;
   float* lg = lds + (size_t)R * width;
   const int row0 = blockIdx.x * R;
@@ -535,11 +567,12 @@ __global__ __launch_bounds__(R == 1 ? 1024 : 256) void route_kernel(const void* 
     xs[i] = row0 + r < rows ? load_as_f32(x, x_dtype, (size_t)(row0 + r) * width + i % width) : 0.0f;
   }
   __syncthreads();
-  router_dots<R>(xs, w, lg, n, width);
+  const int dots = n + rule.shared_gate;
+  router_dots<R>(xs, w, lg, dots, width);
   __syncthreads();
   const int wave = threadIdx.x / kWave;
   if (wave < R && row0 + wave < rows)
-    route_row(lg + wave * n, rule, row0 + wave, n, experts, top, gates, keep, threadIdx.x % kWave);
+    route_row(lg + wave * dots, rule, row0 + wave, n, experts, top, gates, keep, threadIdx.x % kWave);
 }
 
 // The same behind an RMS norm of the 32-bit stream, in one kernel: x[row] (+ delta[row], summed into x), its norm with
@@ -560,7 +593,7 @@ template <int R>
 __global__ __launch_bounds__(R == 1 ? 1024 : 64 * R) void route_norm_kernel(RouteNormArgs a, const float* __restrict__ w, RouteRule rule, int rows, int n,
                                                                        int width, int experts, int top, float* __restrict__ gates,
                                                                        float* __restrict__ keep) {
-  extern __shared__ __attribute__((aligned(16))) float lds[];  // [R][width] rows, then [R][n] logits
+  extern __shared__ __attribute__((aligned(16))) float lds[];  // [R][width] rows, then [R][n (+ 1)] logits
   __shared__ float scratch[16];
   float* lg = lds + (size_t)R * width;
   const int row0 = blockIdx.x * R;
@@ -615,9 +648,10 @@ __global__ __launch_bounds__(R == 1 ? 1024 : 64 * R) void route_norm_kernel(Rout
     }
   }
   __syncthreads();
-  router_dots<R>(lds, w, lg, n, width);
+  const int dots = n + rule.shared_gate;
+  router_dots<R>(lds, w, lg, dots, width);
   __syncthreads();
-  if (wave < R && row0 + wave < rows) route_row(lg + wave * n, rule, row0 + wave, n, experts, top, gates, keep, lane);
+  if (wave < R && row0 + wave < rows) route_row(lg + wave * dots, rule, row0 + wave, n, experts, top, gates, keep, lane);
 }
 
 // The same for few rows, a row a block, rows of a multiple of 4 channels: nothing waits for the norm's sum.  A wave takes two
@@ -630,9 +664,10 @@ __global__ __launch_bounds__(512) void route_norm_few_kernel(RouteNormArgs a, co
   const float* __restrict__ x = a.x + (size_t)row * width;
   auto gain_at = [&](int c) { return a.gain_dtype == NNIS_F32 ? load4((const float*)a.gain + c) : load4((const bf16_t*)a.gain + c); };
   float inv = 0.0f;
-  for (int e = 2 * wave; e < n; e += 2 * waves) {
+  const int dots = n + rule.shared_gate;
+  for (int e = 2 * wave; e < dots; e += 2 * waves) {
     const float* __restrict__ w0 = w + (size_t)e * width;
-    const float* __restrict__ w1 = w + (size_t)(e + 1 < n ? e + 1 : e) * width;
+    const float* __restrict__ w1 = w + (size_t)(e + 1 < dots ? e + 1 : e) * width;
     float ss = 0.0f, dot0 = 0.0f, dot1 = 0.0f;
 #pragma unroll 8
     for (int c = 4 * lane; c < width; c += 4 * kWave) {
@@ -652,7 +687,7 @@ __global__ __launch_bounds__(512) void route_norm_few_kernel(RouteNormArgs a, co
     inv = 1.0f / sqrtf(ss / (float)width + a.eps);
     if (lane == 0) {
       lg[e] = dot0 * inv;
-      if (e + 1 < n) lg[e + 1] = dot1 * inv;
+      if (e + 1 < dots) lg[e + 1] = dot1 * inv;
     }
   }
   __syncthreads();
@@ -719,8 +754,9 @@ __global__ __launch_bounds__(512) void route_norm_many_kernel(RouteNormArgs a, c
     }
   }
   __syncthreads();
-  for (int o0 = 0; o0 < n; o0 += 16) {
-    const bf16_t* w_row = w + (size_t)(o0 + r < n ? o0 + r : n - 1) * width + 8 * g;
+  const int dots = n + rule.shared_gate;
+  for (int o0 = 0; o0 < dots; o0 += 16) {
+    const bf16_t* w_row = w + (size_t)(o0 + r < dots ? o0 + r : dots - 1) * width + 8 * g;
     const bf16_t* x_row = hs + (size_t)(r % 8) * stride + 8 * g;
     f32x4_t acc = {0.0f, 0.0f, 0.0f, 0.0f};
 #pragma unroll 4
@@ -735,9 +771,11 @@ __global__ __launch_bounds__(512) void route_norm_many_kernel(RouteNormArgs a, c
   if (!live) return;
   float logit = 0.0f;
 #pragma unroll
-  for (int o = 0; o < 8; ++o) logit += lane < n ? partial[o][lane][wave] : 0.0f;
-  if (lane < n) lg[wave][lane] = logit;
-  route_row_slots<1>(lg[wave], rule, row, n, experts, top, gates, keep, lane);  // (a lane reads what it wrote itself)
+  for (int o = 0; o < 8; ++o) logit += lane < dots ? partial[o][lane][wave] : 0.0f;
+  if (lane < dots) lg[wave][lane] = logit;
+  __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+  __builtin_amdgcn_wave_barrier();  // (lane 0 reads the shared expert's; of the outputs a lane reads its own)
+  route_row_slots<1>(lg[wave], rule, row, n, experts, top, gates, keep, lane);
 }
 
 // the logits alone, to global memory [rows, n]
@@ -845,12 +883,12 @@ __global__ void routed_act_bf16x8_kernel(RoutedActArgs a, size_t total8) {
   *(bf16x8_t*)((bf16_t*)a.out + row * a.out_stride + (size_t)at * 8) = o;
 }
 
-// y[row, c] += keep[row] * h[row, c]
+// y[row, c] += keep[row] * h[row, c] (without keep: times one)
 __global__ void rows_axpy_kernel(void* __restrict__ y, int y_dtype, const void* __restrict__ h, int h_dtype,
                                  const float* __restrict__ keep, int width, size_t total) {
   const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= total) return;
-  const float k = keep[i / width];
+  const float k = keep ? keep[i / width] : 1.0f;
   if (k != 0.0f) store_from_f32(y, y_dtype, i, fmaf(k, load_as_f32(h, h_dtype, i), load_as_f32(y, y_dtype, i)));
 }
 
@@ -1231,23 +1269,25 @@ extern "C" int nnis_router_logits(const void* x, int x_dtype, const float* w, fl
 }
 
 extern "C" int nnis_route(const void* x, int x_dtype, const float* w, const float* bias, const float* correction, int rows, int n, int width,
-                          int experts, int top, int chosen_softmax, float* gates, float* keep, int* chosen, float* weights, int group_count,
+                          int experts, int top, int scoring, float weight_scale, int group_marks, int shared_gate, float* gates, float* keep, int* chosen, float* weights, int group_count,
                           int group_keep, void* stream) {
   NNIS_REQUIRE((chosen == nullptr) == (weights == nullptr) && (chosen == nullptr || top <= kWave), "route: up to %d choices are listed", kWave);
   NNIS_REQUIRE(x && w && gates && keep && n > 0 && width > 0, "route: missing operand");
   NNIS_REQUIRE(group_count >= 1 && group_count <= kWave && n % group_count == 0 && group_keep >= 1 && group_keep <= group_count,
                "route: %d outputs in %d groups (up to %d, equal ones) of which %d are kept", n, group_count, kWave, group_keep);
   NNIS_REQUIRE(nnis_dtype_ok(x_dtype), "route: unknown dtype");
-  NNIS_REQUIRE(n <= kWave * kRouteMost && width <= 8192, "route: up to %d outputs of rows of up to 8192 channels, got %d and %d", kWave * kRouteMost,
+  NNIS_REQUIRE(n + (shared_gate ? 1 : 0) <= kWave * kRouteMost && width <= 8192, "route: up to %d outputs of rows of up to 8192 channels, got %d and %d", kWave * kRouteMost,
                n, width);
+  NNIS_REQUIRE(scoring >= kSoftmax && scoring <= kSigmoid && (group_marks == 1 || group_marks == 2), "router: unknown scoring %d or group mark %d", scoring, group_marks);
   NNIS_REQUIRE(experts >= 0 && experts <= n && top > 0 && top <= n, "route: %d experts and the %d largest of %d outputs", experts, top, n);
   if (rows <= 0) return 0;
   // several rows a block where they fit 48 KB of LDS and there are rows enough to fill the chip with such blocks
-  const int together = rows <= 256 ? 1 : ((size_t)4 * (width + n) * 4 <= 49152 ? 4 : ((size_t)2 * (width + n) * 4 <= 49152 ? 2 : 1));
-  const size_t lds = (size_t)together * (width + n) * sizeof(float);
+  const int dots = n + (shared_gate ? 1 : 0);  // logits of a row
+  const int together = rows <= 256 ? 1 : ((size_t)4 * (width + dots) * 4 <= 49152 ? 4 : ((size_t)2 * (width + dots) * 4 <= 49152 ? 2 : 1));
+  const size_t lds = (size_t)together * (width + dots) * sizeof(float);
   const dim3 grid((rows + together - 1) / together);
   hipStream_t s = (hipStream_t)stream;
-  const RouteRule rule = {bias, correction, chosen_softmax ? 1 : 0, group_count, group_keep, chosen, weights};
+  const RouteRule rule = {bias, correction, scoring, group_count, group_keep, weight_scale, group_marks, shared_gate ? 1 : 0, chosen, weights};
   if (together == 4) {
     hipLaunchKernelGGL((route_kernel<4>), grid, dim3(256), lds, s, x, x_dtype, w, rule, rows, n, width, experts, top, gates, keep);
   } else if (together == 2) {
@@ -1265,25 +1305,27 @@ extern "C" int nnis_route(const void* x, int x_dtype, const float* w, const floa
 // 32-bit products too); chosen (null, or [rows, top] for up to 64 choices) and weights: the choices as a list beside the gates
 extern "C" int nnis_route_norm(float* x, const void* delta, int delta_dtype, const void* gain, int gain_dtype, float eps, void* h, int h_dtype,
                                const float* w, const void* w_bf16, const float* bias, const float* correction, int rows, int n, int width,
-                               int experts, int top, int chosen_softmax, float* gates, float* keep, int* chosen, float* weights, int group_count, int group_keep,
+                               int experts, int top, int scoring, float weight_scale, int group_marks, int shared_gate, float* gates, float* keep, int* chosen, float* weights, int group_count, int group_keep,
                                void* stream) {
   NNIS_REQUIRE(x && gain && h && w && gates && keep && n > 0 && width > 0, "route_norm: missing operand");
   NNIS_REQUIRE(group_count >= 1 && group_count <= kWave && n % group_count == 0 && group_keep >= 1 && group_keep <= group_count,
                "route_norm: %d outputs in %d groups (up to %d, equal ones) of which %d are kept", n, group_count, kWave, group_keep);
   NNIS_REQUIRE(nnis_dtype_ok(gain_dtype) && nnis_dtype_ok(h_dtype) && (delta == nullptr || nnis_dtype_ok(delta_dtype)), "route_norm: unknown dtype");
-  NNIS_REQUIRE(n <= kWave * kRouteMost && width <= 8192, "route_norm: up to %d outputs of rows of up to 8192 channels, got %d and %d",
+  NNIS_REQUIRE(n + (shared_gate ? 1 : 0) <= kWave * kRouteMost && width <= 8192, "route_norm: up to %d outputs of rows of up to 8192 channels, got %d and %d",
                kWave * kRouteMost, n, width);
+  NNIS_REQUIRE(scoring >= kSoftmax && scoring <= kSigmoid && (group_marks == 1 || group_marks == 2), "router: unknown scoring %d or group mark %d", scoring, group_marks);
   NNIS_REQUIRE(experts >= 0 && experts <= n && top > 0 && top <= n, "route_norm: %d experts and the %d largest of %d outputs", experts, top, n);
   NNIS_REQUIRE((chosen == nullptr) == (weights == nullptr) && (chosen == nullptr || top <= kWave), "route_norm: up to %d choices are listed", kWave);
   if (rows <= 0) return 0;
-  const int together = rows <= 256 ? 1 : ((size_t)4 * (width + n) * 4 <= 49152 ? 4 : ((size_t)2 * (width + n) * 4 <= 49152 ? 2 : 1));
-  const size_t lds = (size_t)together * (width + n) * sizeof(float);
+  const int dots = n + (shared_gate ? 1 : 0);  // logits of a row
+  const int together = rows <= 256 ? 1 : ((size_t)4 * (width + dots) * 4 <= 49152 ? 4 : ((size_t)2 * (width + dots) * 4 <= 49152 ? 2 : 1));
+  const size_t lds = (size_t)together * (width + dots) * sizeof(float);
   const dim3 grid((rows + together - 1) / together);
   hipStream_t s = (hipStream_t)stream;
-  const RouteRule rule = {bias, correction, chosen_softmax ? 1 : 0, group_count, group_keep, chosen, weights};
+  const RouteRule rule = {bias, correction, scoring, group_count, group_keep, weight_scale, group_marks, shared_gate ? 1 : 0, chosen, weights};
   const RouteNormArgs a = {x, delta, delta_dtype, gain, gain_dtype, eps, h, h_dtype};
   const bool fours = width % 4 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)gain % 16 == 0 && (uintptr_t)h % 16 == 0 && (uintptr_t)w % 16 == 0;
-  if (rows > 256 && fours && w_bf16 && h_dtype == NNIS_BF16 && n <= kWave && width % 32 == 0 && width <= kRouteManyMost &&
+  if (rows > 256 && fours && w_bf16 && h_dtype == NNIS_BF16 && dots <= kWave && width % 32 == 0 && width <= kRouteManyMost &&
       (uintptr_t)w_bf16 % 16 == 0 && (uintptr_t)delta % 16 == 0) {
     const size_t bytes = (size_t)8 * (width + 8) * sizeof(bf16_t);
     static const hipError_t allowed = hipFuncSetAttribute((const void*)route_norm_many_kernel, hipFuncAttributeMaxDynamicSharedMemorySize,
@@ -1295,7 +1337,7 @@ extern "C" int nnis_route_norm(float* x, const void* delta, int delta_dtype, con
     return 0;
   }
   if (rows <= 256 && fours && delta == nullptr) {
-    const int waves = n < 16 ? (n + 1) / 2 : 8;  // (each has outputs of its own, and with them the row's root mean square)
+    const int waves = dots < 16 ? (dots + 1) / 2 : 8;  // (each has outputs of its own, and with them the row's root mean square)
     hipLaunchKernelGGL(route_norm_few_kernel, dim3(rows), dim3(kWave * waves), 0, s, a, w, rule, n, width, experts, top, gates, keep);
     NNIS_LAUNCH_CHECK("route_norm");
     return 0;
@@ -1313,14 +1355,16 @@ extern "C" int nnis_route_norm(float* x, const void* delta, int delta_dtype, con
 }
 
 extern "C" int nnis_route_top(const float* logits, const float* bias, const float* correction, int rows, int n, int experts, int top,
-                              int chosen_softmax, float* gates, float* keep, int group_count, int group_keep, void* stream) {
+                              int scoring, float weight_scale, int group_marks, int shared_gate, float* gates, float* keep, int group_count,
+                              int group_keep, void* stream) {
   NNIS_REQUIRE(logits && gates && keep, "route_top: missing operand");
   NNIS_REQUIRE(group_count >= 1 && group_count <= kWave && n % group_count == 0 && group_keep >= 1 && group_keep <= group_count,
                "route_top: %d outputs in %d groups (up to %d, equal ones) of which %d are kept", n, group_count, kWave, group_keep);
-  NNIS_REQUIRE(n > 0 && n <= kWave * kRouteMost, "route_top: 1 to %d router outputs, got %d", kWave * kRouteMost, n);
+  NNIS_REQUIRE(n > 0 && n + (shared_gate ? 1 : 0) <= kWave * kRouteMost, "route_top: 1 to %d router outputs, got %d", kWave * kRouteMost, n);
+  NNIS_REQUIRE(scoring >= kSoftmax && scoring <= kSigmoid && (group_marks == 1 || group_marks == 2), "router: unknown scoring %d or group mark %d", scoring, group_marks);
   NNIS_REQUIRE(experts >= 0 && experts <= n && top > 0 && top <= n, "route_top: %d experts and the %d largest of %d outputs", experts, top, n);
   if (rows <= 0) return 0;
-  const RouteRule rule = {bias, correction, chosen_softmax ? 1 : 0, group_count, group_keep, nullptr, nullptr};
+  const RouteRule rule = {bias, correction, scoring, group_count, group_keep, weight_scale, group_marks, shared_gate ? 1 : 0, nullptr, nullptr};
   hipLaunchKernelGGL(route_top_kernel, dim3((rows + 3) / 4), dim3(256), 0, (hipStream_t)stream, logits, rule, rows, n, experts, top, gates,
                      keep);
   NNIS_LAUNCH_CHECK("route_top");
@@ -1355,7 +1399,7 @@ extern "C" int nnis_routed_act(const void* z, int z_dtype, int z_stride, const f
 }
 
 extern "C" int nnis_rows_axpy(void* y, int y_dtype, const void* h, int h_dtype, const float* keep, int rows, int width, void* stream) {
-  NNIS_REQUIRE(y && h && keep && width > 0, "rows_axpy: missing operand");
+  NNIS_REQUIRE(y && h && width > 0, "rows_axpy: missing operand");
   NNIS_REQUIRE(nnis_dtype_ok(y_dtype) && nnis_dtype_ok(h_dtype), "rows_axpy: unknown dtype");
   if (rows <= 0) return 0;
   const size_t total = (size_t)rows * width;
@@ -1449,5 +1493,29 @@ extern "C" int nnis_pool_blocks(const void* k_pages, const void* v_pages, int ca
     hipLaunchKernelGGL(pool_blocks_kernel<bf16_t>, dim3(tokens / pool + batch, kv_heads), dim3(256), (size_t)4 * value_dim * sizeof(float), (hipStream_t)stream, a);
   }
   NNIS_LAUNCH_CHECK("pool_blocks");
+  return 0;
+}
+
+// out[t, c] = gelu_tanh(z[t, c]) * table[ids[t], first + c]: a layer's gate on the tokens' own input
+__global__ void token_gate_kernel(const void* __restrict__ z, int z_dtype, const int* __restrict__ ids, const void* __restrict__ table, int table_dtype,
+                                  int columns, int first, void* __restrict__ out, int out_dtype, int dim, size_t total) {
+  for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += (size_t)gridDim.x * blockDim.x) {
+    const size_t t = i / dim, c = i % dim;
+    const float v = load_as_f32(z, z_dtype, i);
+    const float gate = v * sigmoid_f(1.5957691216057308f * fmaf(0.044715f * v * v, v, v));  // (1 + tanh u) / 2 = sigmoid(2 u)
+    store_from_f32(out, out_dtype, i, gate * load_as_f32(table, table_dtype, (size_t)ids[t] * columns + first + c));
+  }
+}
+
+extern "C" int nnis_token_gate(const void* z, int z_dtype, const int* ids, const void* table, int table_dtype, int vocab, int columns, int first,
+                               void* out, int out_dtype, int rows, int dim, void* stream) {
+  NNIS_REQUIRE(z && ids && table && out && dim > 0 && first >= 0 && first + dim <= columns && vocab > 0, "token_gate: bad arguments");
+  NNIS_REQUIRE(nnis_dtype_ok(z_dtype) && nnis_dtype_ok(table_dtype) && nnis_dtype_ok(out_dtype), "token_gate: unknown dtype");
+  if (rows <= 0) return 0;
+  const size_t total = (size_t)rows * dim;
+  const size_t blocks = (total + 255) / 256;
+  hipLaunchKernelGGL(token_gate_kernel, dim3((unsigned)(blocks > 65536 ? 65536 : blocks)), dim3(256), 0, (hipStream_t)stream, z, z_dtype, ids, table,
+                     table_dtype, columns, first, out, out_dtype, dim, total);
+  NNIS_LAUNCH_CHECK("token_gate");
   return 0;
 }

@@ -124,6 +124,7 @@ class StepContext:
     plan_rows: int = 0
     options: dict = field(default_factory=dict)  # launch options by part kind, for tests and tuning: {"causal_attention": {...}}
     lists: Optional[StepLists] = None  # the parts' host-made work lists (``StepLists``)
+    ids: Optional[torch.Tensor] = None  # int32 [tokens]: the step's tokens, for parts that read them beside the stream
     tables: dict = field(default_factory=dict)  # the step's tables, made by the first layer that asks (``step_tables``)
 
     def __post_init__(self):

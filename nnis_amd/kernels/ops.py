@@ -105,7 +105,7 @@ _ATTN_SIGNATURES = {
 
 _RECURRENT_SIGNATURES = {
     "nnis_conv_silu": [_VOID, _INT, _INT, _VOID, _VOID, _INT, _VOID, _VOID, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _VOID, _INT,
-                       _INT, _VOID],
+                       _INT, _VOID, _INT, _INT, _VOID],
     "nnis_selective_scan": [_VOID, _INT, _VOID, _VOID, _VOID, _INT, _INT, _VOID, _VOID, _VOID, _VOID, _VOID, _VOID, _INT, _INT, _INT,
                             _VOID, _INT, _INT, _INT, _VOID, _VOID, _VOID],
     "nnis_gla_scan": [_VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _VOID, _FLT, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT,
@@ -116,19 +116,28 @@ _RECURRENT_SIGNATURES = {
                          _VOID, _VOID],
     "nnis_gla_decays": [_VOID, _VOID, _INT, _INT, _FLT, _VOID],
     "nnis_head_norm_gate": [_VOID, _VOID, _INT, _INT, _VOID, _INT, _VOID, _INT, _INT, _INT, _INT, _FLT, _VOID],
+    "nnis_rg_lru": [_VOID, _VOID, _VOID, _VOID, _VOID, _INT, _INT, _VOID, _INT, _INT, _VOID, _VOID, _VOID, _VOID, _INT, _INT, _INT, _VOID, _INT, _INT,
+                    _INT, _VOID, _VOID, _VOID],
     "nnis_min_gru": [_VOID, _INT, _INT, _VOID, _VOID, _INT, _VOID, _VOID, _VOID, _INT, _INT, _VOID, _INT, _INT, _INT, _VOID, _VOID, _VOID],
 }
 
+_STATE_SPACE_SIGNATURES = {
+    "nnis_state_space": [_VOID, _INT, _INT, _VOID, _INT, _INT, _VOID, _VOID, _VOID, _VOID, _INT, _INT, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT,
+                         _VOID, _INT, _VOID],
+    "nnis_parts_norm": [_VOID, _INT, _VOID, _VOID, _INT, _INT, _INT, _INT, _FLT, _VOID],
+}
+
 _SUBLAYER_SIGNATURES = {
+    "nnis_token_gate": [_VOID, _INT, _VOID, _VOID, _INT, _INT, _INT, _INT, _VOID, _INT, _INT, _INT, _VOID],
     "nnis_cast_rows": [_VOID, _INT, _VOID, _INT, _VOID, _INT, _INT, _VOID],
     "nnis_rms_post_step": [_VOID, _VOID, _INT, _VOID, _INT, _FLT, _FLT, _VOID, _INT, _INT, _INT, _VOID, _VOID, _INT, _VOID],
     "nnis_rms_between": [_VOID, _VOID, _INT, _VOID, _VOID, _INT, _FLT, _VOID, _INT, _INT, _INT, _VOID, _VOID, _INT, _VOID],
-    "nnis_route": [_VOID, _INT, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _VOID, _VOID, _VOID, _VOID, _INT, _INT, _VOID],
-    "nnis_route_norm": [_VOID, _VOID, _INT, _VOID, _INT, _FLT, _VOID, _INT, _VOID, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _VOID,
-                        _VOID, _VOID, _VOID, _INT, _INT, _VOID],
+    "nnis_route": [_VOID, _INT, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _FLT, _INT, _INT, _VOID, _VOID, _VOID, _VOID, _INT, _INT, _VOID],
+    "nnis_route_norm": [_VOID, _VOID, _INT, _VOID, _INT, _FLT, _VOID, _INT, _VOID, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _FLT, _INT, _INT,
+                        _VOID, _VOID, _VOID, _VOID, _INT, _INT, _VOID],
     "nnis_poly_norm": [_VOID, _INT, _VOID, _FLT, _VOID, _INT, _INT, _INT, _VOID],
     "nnis_router_logits": [_VOID, _INT, _VOID, _VOID, _INT, _INT, _INT, _VOID],
-    "nnis_route_top": [_VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _VOID, _VOID, _INT, _INT, _VOID],
+    "nnis_route_top": [_VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _FLT, _INT, _INT, _VOID, _VOID, _INT, _INT, _VOID],
     "nnis_routed_act": [_VOID, _INT, _INT, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _FLT, _VOID],
     "nnis_rows_axpy": [_VOID, _INT, _VOID, _INT, _VOID, _INT, _INT, _VOID],
     "nnis_sigmoid_gate": [_VOID, _INT, _VOID, _INT, _INT, _INT, _INT, _VOID],
@@ -139,11 +148,11 @@ _SUBLAYER_SIGNATURES = {
 }
 
 _EXPERTS_SIGNATURES = {
-    "nnis_experts_up_few": [_VOID, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _FLT, _FLT, _VOID],
+    "nnis_experts_up_few": [_VOID, _VOID, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _FLT, _FLT, _VOID],
     "nnis_experts_down_few": [_VOID, _VOID, _VOID, _VOID, _VOID, _VOID, _INT, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _VOID, _VOID,
                               _INT, _VOID],
     "nnis_experts_lists": [_VOID, _INT, _INT, _INT, _VOID, _VOID, _VOID],
-    "nnis_experts_many": [_INT, _VOID, _VOID, _VOID, _VOID, _VOID, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _INT, _FLT, _FLT, _VOID],
+    "nnis_experts_many": [_INT, _VOID, _VOID, _VOID, _VOID, _VOID, _VOID, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT, _INT, _INT, _FLT, _FLT, _VOID],
     "nnis_experts_combine": [_VOID, _VOID, _VOID, _VOID, _VOID, _INT, _VOID, _VOID, _INT, _INT, _INT, _VOID],
 }
 
@@ -213,6 +222,17 @@ def recurrent():
     if _recurrent is None:
         _recurrent = _bind("recurrent", _RECURRENT_SIGNATURES)
     return _recurrent
+
+
+_state_space = None
+
+
+def state_space_module():
+    """The module of Mamba-2's state spaces."""
+    global _state_space
+    if _state_space is None:
+        _state_space = _bind("state_space", _STATE_SPACE_SIGNATURES)
+    return _state_space
 
 
 _latent = None
@@ -1472,7 +1492,9 @@ def attention(q: torch.Tensor, out: torch.Tensor, view, ctx, heads: int, kv_head
     as ``KeyRuns`` instead of the output (see ``attention_decode_bf16``).
     ``plan``: (runs, waves) of a step of single tokens (``decode_plan``), or
     (waves, columns) of a step of prompts (``prefill_plan``); None: as those
-    functions choose for the step's planned sizes."""
+    functions choose for the step's planned sizes.  ``window``: 0, or n > 0
+    for the last n keys, or n < 0 for the keys of the query's own chunk of -n
+    positions."""
     value_dim = value_dim or head_dim
     fast = attention_on_matrix_cores(q.dtype, view.k_pages.dtype, head_dim, value_dim, softcap, extras)
     size = max(head_dim, value_dim)  # what a wave's registers are sized by
@@ -1706,27 +1728,107 @@ def _step_arrays(ctx, what: str):
 
 
 def conv_silu(x: torch.Tensor, channels: int, weight: torch.Tensor, bias: Optional[torch.Tensor], state: Optional[torch.Tensor],
-              ctx, out: torch.Tensor) -> torch.Tensor:
-    """out[t, c] = silu(bias[c] + sum_j weight[c, j] x[t - (taps - 1) + j, c]) over each sequence's own tokens, the
-    last tap on the token itself.  ``x``: [tokens, >= channels], its first ``channels`` columns are taken.
-    ``state`` (float32 [slots, taps - 1, channels]) holds each sequence's last inputs and is brought up to date."""
-    _dev(x, "x"), _dev(weight, "weight"), _dev(out, "out")
+              ctx, out: torch.Tensor, x_bias: Optional[torch.Tensor] = None, activation: Optional[str] = "silu", ring: bool = False) -> torch.Tensor:
+    """out[t, c] = act(bias[c] + sum_j weight[c, j] (x + x_bias)[t - (taps - 1) + j, c]) over each sequence's own tokens, the
+    last tap on the token itself; ``activation``: "silu" or None.  ``x``: [tokens, >= channels], its first ``channels``
+    columns are taken.  ``state`` (float32 [slots, taps - 1, channels]) holds each sequence's last inputs and is brought up
+    to date; with ``ring`` it is [slots, taps, channels], position p's input in row p % taps."""
+    _dev(weight, "weight"), _dev(out, "out")
     tokens = x.shape[0]
     taps = weight.shape[1]
-    if weight.shape[0] != channels or x.shape[1] < channels or tuple(out.shape) != (tokens, channels):
+    if not x.is_cuda or x.stride(1) != 1 or weight.shape[0] != channels or x.shape[1] < channels or tuple(out.shape) != (tokens, channels):
         raise KernelError(f"conv_silu: x {tuple(x.shape)}, weight {tuple(weight.shape)}, out {tuple(out.shape)} do not fit {channels} channels")
     if bias is not None and (bias.numel() != channels or bias.dtype != weight.dtype):
         raise KernelError("conv_silu: the bias has one entry per channel and the weight's type")
-    if taps > 1:
+    if x_bias is not None:
+        _dev(x_bias, "x_bias")
+        if x_bias.dtype != torch.float32 or x_bias.numel() != channels:
+            raise KernelError("conv_silu: the inputs' bias is float32 with one entry per channel")
+    if activation not in ("silu", None):
+        raise KernelError(f"conv_silu: unknown activation {activation!r}")
+    held = taps if ring else taps - 1
+    if held > 0:
         _dev(state, "state")
-        if state.dtype != torch.float32 or tuple(state.shape[1:]) != (taps - 1, channels):
-            raise KernelError(f"conv_silu: state must be float32 [slots, {taps - 1}, {channels}], got {tuple(state.shape)}")
+        if state.dtype != torch.float32 or tuple(state.shape[1:]) != (held, channels):
+            raise KernelError(f"conv_silu: state must be float32 [slots, {held}, {channels}], got {tuple(state.shape)}")
     _step_arrays(ctx, "conv_silu")
     lib = recurrent()
-    _check(lib, lib.nnis_conv_silu(x.data_ptr(), _code(x), x.stride(0), weight.data_ptr(), _ptr(bias), _code(weight), _ptr(state),
-                                   ctx.tok_slot.data_ptr(), ctx.tok_pos.data_ptr(), ctx.seq_slot.data_ptr(), ctx.seq_start.data_ptr(),
-                                   tokens, ctx.batch, channels, taps, out.data_ptr(), _code(out),
-                                   1 if (ctx.decode and tokens == ctx.batch) else 0, _stream()))
+    _check(lib, lib.nnis_conv_silu(x.data_ptr(), _code(x), x.stride(0) if tokens > 1 else max(x.stride(0), channels), weight.data_ptr(), _ptr(bias),
+                                   _code(weight), _ptr(state), ctx.tok_slot.data_ptr(), ctx.tok_pos.data_ptr(), ctx.seq_slot.data_ptr(),
+                                   ctx.seq_start.data_ptr(), tokens, ctx.batch, channels, taps, out.data_ptr(), _code(out),
+                                   1 if (ctx.decode and tokens == ctx.batch) else 0, _ptr(x_bias), 1 if activation is None else 0,
+                                   1 if ring else 0, _stream()))
+    return out
+
+
+def _columns(t: torch.Tensor, tokens: int, width: int, what: str) -> int:
+    """The row stride of a view [tokens, >= width] with adjacent columns."""
+    if not t.is_cuda or t.dim() != 2 or t.shape[0] != tokens or t.shape[1] < width or t.stride(1) != 1:
+        raise KernelError(f"{what}: rows [{tokens}, {width}] with adjacent columns are needed, got {tuple(t.shape)}")
+    return t.stride(0) if tokens > 1 else max(t.stride(0), width)
+
+
+def state_space(xbc: torch.Tensor, dt: torch.Tensor, z: torch.Tensor, rate: torch.Tensor, dt_bias: torch.Tensor, D: torch.Tensor,
+                state: torch.Tensor, ctx, groups: int, out: torch.Tensor) -> torch.Tensor:
+    """Mamba-2's recurrence over each sequence's tokens, from and into ``state`` (float32 [slots, heads, P, N]): with
+    ``xbc`` [tokens, heads * P + 2 * groups * N] = (x | B | C) and dt = softplus(dt + dt_bias) [tokens, heads],
+    S <- exp(-rate dt) S + dt x B^T;  out = (S C + D x) * silu(z).  ``dt``, ``z``: views whose rows may be further apart."""
+    tokens = xbc.shape[0]
+    for t, what in ((state, "state"), (out, "out"), (rate, "rate"), (dt_bias, "dt_bias"), (D, "D")):
+        _dev(t, what)
+    _, heads, P, N = state.shape
+    if state.dtype != torch.float32 or tuple(out.shape) != (tokens, heads * P):
+        raise KernelError(f"state_space: a float32 state [slots, heads, P, N] and out [tokens, heads * P], got {tuple(state.shape)} and {tuple(out.shape)}")
+    if any(t.dtype != torch.float32 or t.numel() != heads for t in (rate, dt_bias, D)):
+        raise KernelError(f"state_space: rate, dt_bias and D are float32 with one entry for each of {heads} heads")
+    xs, ds, zs = (_columns(xbc, tokens, heads * P + 2 * groups * N, "state_space: xbc"), _columns(dt, tokens, heads, "state_space: dt"),
+                  _columns(z, tokens, heads * P, "state_space: z"))
+    _step_arrays(ctx, "state_space")
+    lib = state_space_module()
+    _check(lib, lib.nnis_state_space(xbc.data_ptr(), _code(xbc), xs, dt.data_ptr(), _code(dt), ds, rate.data_ptr(), dt_bias.data_ptr(), D.data_ptr(),
+                                     z.data_ptr(), _code(z), zs, state.data_ptr(), ctx.seq_slot.data_ptr(), ctx.seq_start.data_ptr(), ctx.batch,
+                                     heads, groups, P, N, out.data_ptr(), _code(out), _stream()))
+    return out
+
+
+def parts_norm(x: torch.Tensor, weight: torch.Tensor, parts: int, eps: float, out: torch.Tensor) -> torch.Tensor:
+    """Each of a row's ``parts`` equal parts over its own root mean square, times ``weight`` (float32, a row's length)."""
+    _dev(x, "x"), _dev(weight, "weight"), _dev(out, "out")
+    rows, width = x.shape
+    if width % parts or out.shape != x.shape or weight.dtype != torch.float32 or weight.numel() != width:
+        raise KernelError(f"parts_norm: x {tuple(x.shape)} in {parts} parts, out {tuple(out.shape)}, a float32 weight of {weight.numel()}")
+    lib = state_space_module()
+    _check(lib, lib.nnis_parts_norm(x.data_ptr(), _code(x), weight.data_ptr(), out.data_ptr(), _code(out), rows, int(parts), width // parts,
+                                    float(eps), _stream()))
+    return out
+
+
+def rg_lru(logits: torch.Tensor, blocks: int, r_bias: torch.Tensor, i_bias: torch.Tensor, rate: torch.Tensor, u: torch.Tensor, y: torch.Tensor,
+           y_bias: Optional[torch.Tensor], state: torch.Tensor, ctx, out: torch.Tensor) -> torch.Tensor:
+    """The real-gated linear recurrent unit's recurrence over each sequence's tokens, from and into ``state`` (float32
+    [slots, width]).  ``logits`` float32 [tokens, blocks * 2 * (width / blocks)]: block by block the logits of r, then of
+    i; log a = -8 sigmoid(r + r_bias) rate;  S <- a S + sqrt(1 - a^2) sigmoid(i + i_bias) u;  out = S * gelu_tanh(y + y_bias)."""
+    tokens, width = out.shape
+    for t, what in ((logits, "logits"), (r_bias, "r_bias"), (i_bias, "i_bias"), (rate, "rate"), (state, "state"), (out, "out")):
+        _dev(t, what)
+    if width % blocks or logits.dtype != torch.float32 or tuple(logits.shape) != (tokens, 2 * width):
+        raise KernelError(f"rg_lru: float32 logits [{tokens}, {2 * width}] in {blocks} blocks, got {tuple(logits.shape)} {logits.dtype}")
+    if state.dtype != torch.float32 or tuple(state.shape[1:]) != (width,):
+        raise KernelError(f"rg_lru: state must be float32 [slots, {width}], got {tuple(state.shape)} {state.dtype}")
+    vectors = [r_bias, i_bias, rate] + ([y_bias] if y_bias is not None else [])
+    if any(t.dtype != torch.float32 or t.numel() != width for t in vectors):
+        raise KernelError(f"rg_lru: biases and rates are float32 with one entry for each of {width} channels")
+    us, ys = _columns(u, tokens, width, "rg_lru: u"), _columns(y, tokens, width, "rg_lru: y")
+    _step_arrays(ctx, "rg_lru")
+    piece, pieces = run_pieces(ctx, width * 8)
+    decay = ends = None
+    if pieces > 1:
+        scratch = torch.empty(2, ctx.batch * pieces * width, dtype=torch.float32, device=u.device)
+        decay, ends = scratch[0], scratch[1]
+    lib = recurrent()
+    _check(lib, lib.nnis_rg_lru(logits.data_ptr(), r_bias.data_ptr(), i_bias.data_ptr(), rate.data_ptr(), u.data_ptr(), _code(u), us, y.data_ptr(),
+                                _code(y), ys, _ptr(y_bias), state.data_ptr(), ctx.seq_slot.data_ptr(), ctx.seq_start.data_ptr(), ctx.batch, width,
+                                width // blocks, out.data_ptr(), _code(out), piece, pieces, _ptr(decay), _ptr(ends), _stream()))
     return out
 
 
@@ -2204,6 +2306,15 @@ def _route_groups(groups, n: int, what: str):
     return count, keep
 
 
+_ROUTE_SCORINGS = {"softmax": 0, "chosen_softmax": 1, "sigmoid": 2}
+
+
+def _route_scoring(scoring: str, weight_scale: float, group_marks: int, shared_gate: bool):
+    if scoring not in _ROUTE_SCORINGS or group_marks not in (1, 2):
+        raise KernelError(f"a router's scores are one of {', '.join(_ROUTE_SCORINGS)}, a group's mark adds up one or two; got {scoring!r}, {group_marks}")
+    return _ROUTE_SCORINGS[scoring], float(weight_scale), int(group_marks), 1 if shared_gate else 0
+
+
 def _check_router_bias(bias: Optional[torch.Tensor], n: int, what: str) -> None:
     if bias is not None:
         _dev(bias, "router bias")
@@ -2212,13 +2323,18 @@ def _check_router_bias(bias: Optional[torch.Tensor], n: int, what: str) -> None:
 
 
 def route_top(logits: torch.Tensor, correction: Optional[torch.Tensor], experts: int, top: int, gates: torch.Tensor,
-              keep: torch.Tensor, groups=None, bias: Optional[torch.Tensor] = None, chosen_softmax: bool = False):
+              keep: torch.Tensor, groups=None, bias: Optional[torch.Tensor] = None, scoring: str = "softmax", weight_scale: float = 1.0,
+              group_marks: int = 1, shared_gate: bool = False):
     """Scores softmax(logits) [rows, n]; the ``top`` largest of score + correction are chosen.  ``gates`` [rows, experts]
     gets the score of every chosen output below ``experts`` and 0 elsewhere; ``keep`` [rows] the summed scores of the
-    chosen outputs from ``experts`` on.  ``bias`` [n] joins the logits first.  ``chosen_softmax``: chosen are the ``top``
-    largest logits (+ correction), and their weights are the softmax over the chosen logits alone.  All float32."""
+    chosen outputs from ``experts`` on.  ``bias`` [n] joins the logits first.  ``scoring="chosen_softmax"``: chosen are the ``top``
+    largest logits (+ correction), and their weights are the softmax over the chosen logits alone; ``"sigmoid"``: scores
+    are sigmoid(logits), and the weights are the chosen scores over their sum, times ``weight_scale``.  ``group_marks``: how many of
+    its largest choices a group's mark adds up (1 or 2).  ``shared_gate``: the logits have one more column behind the n
+    outputs, whose sigmoid goes into ``keep`` instead.  All float32."""
     _dev(logits, "logits"), _dev(gates, "gates"), _dev(keep, "keep")
     rows, n = logits.shape
+    n -= 1 if shared_gate else 0
     if logits.dtype != torch.float32 or gates.dtype != torch.float32 or keep.dtype != torch.float32 \
             or tuple(gates.shape) != (rows, experts) or keep.numel() != rows:
         raise KernelError(f"route_top: float32 logits {tuple(logits.shape)}, gates {tuple(gates.shape)}, keep {tuple(keep.shape)}")
@@ -2226,13 +2342,13 @@ def route_top(logits: torch.Tensor, correction: Optional[torch.Tensor], experts:
         _dev(correction, "correction")
         if correction.dtype != torch.float32 or correction.numel() != n:
             raise KernelError(f"route_top: a float32 correction per output ({n}), got {tuple(correction.shape)} {correction.dtype}")
-    if not (0 < n <= ROUTE_MOST_OUTPUTS and 0 <= experts <= n and 0 < top <= n):
+    if not (0 < n and n + int(shared_gate) <= ROUTE_MOST_OUTPUTS and 0 <= experts <= n and 0 < top <= n):
         raise KernelError(f"route_top: {experts} experts and the {top} largest of {n} outputs (at most {ROUTE_MOST_OUTPUTS})")
     _check_router_bias(bias, n, "route_top")
     group_count, group_keep = _route_groups(groups, n, "route_top")
     lib = sublayer()
-    _check(lib, lib.nnis_route_top(logits.data_ptr(), _ptr(bias), _ptr(correction), rows, n, experts, top, 1 if chosen_softmax else 0,
-                                   gates.data_ptr(), keep.data_ptr(),
+    _check(lib, lib.nnis_route_top(logits.data_ptr(), _ptr(bias), _ptr(correction), rows, n, experts, top,
+                                   *_route_scoring(scoring, weight_scale, group_marks, shared_gate), gates.data_ptr(), keep.data_ptr(),
                                    group_count, group_keep, _stream()))
     return gates, keep
 
@@ -2241,14 +2357,16 @@ ROUTE_FUSED_MOST_CHANNELS = 8192
 
 
 def route(x: torch.Tensor, weight: torch.Tensor, correction: Optional[torch.Tensor], experts: int, top: int, gates: torch.Tensor,
-          keep: torch.Tensor, groups=None, bias: Optional[torch.Tensor] = None, chosen_softmax: bool = False, chosen=None):
+          keep: torch.Tensor, groups=None, bias: Optional[torch.Tensor] = None, scoring: str = "softmax", weight_scale: float = 1.0,
+          group_marks: int = 1, shared_gate: bool = False, chosen=None):
     """``router_logits`` and ``route_top`` in one kernel (rows of up to ``ROUTE_FUSED_MOST_CHANNELS`` channels).
     ``groups``: (count, keep): the outputs form ``count`` equal groups of neighbours, a group's mark is its largest
     corrected score, and only outputs of the ``keep`` groups with the largest marks can be chosen.  ``chosen``: (int32 [rows, top],
-    float32 [rows, top]) that take the choices and their weights as lists, best first."""
+    float32 [rows, top]) that take the choices and their weights as lists, best first.  ``scoring``, ``weight_scale``,
+    ``group_marks``, ``shared_gate`` (then one more row of ``weight``) as ``route_top``."""
     _dev(x, "x"), _dev(weight, "router weight"), _dev(gates, "gates"), _dev(keep, "keep")
     rows, width = x.shape
-    n = weight.shape[0]
+    n = weight.shape[0] - (1 if shared_gate else 0)
     if (x.dim() != 2 or not x.is_contiguous() or weight.dtype != torch.float32 or weight.dim() != 2 or weight.shape[1] != width
             or gates.dtype != torch.float32 or keep.dtype != torch.float32 or tuple(gates.shape) != (rows, experts) or keep.numel() != rows):
         raise KernelError(f"route: x {tuple(x.shape)}, a float32 weight {tuple(weight.shape)}, float32 gates {tuple(gates.shape)} and keep {tuple(keep.shape)}")
@@ -2256,13 +2374,14 @@ def route(x: torch.Tensor, weight: torch.Tensor, correction: Optional[torch.Tens
         _dev(correction, "correction")
         if correction.dtype != torch.float32 or correction.numel() != n:
             raise KernelError(f"route: a float32 correction per output ({n}), got {tuple(correction.shape)} {correction.dtype}")
-    if not (0 < n <= ROUTE_MOST_OUTPUTS and 0 <= experts <= n and 0 < top <= n and width <= ROUTE_FUSED_MOST_CHANNELS):
+    if not (0 < n and n + int(shared_gate) <= ROUTE_MOST_OUTPUTS and 0 <= experts <= n and 0 < top <= n and width <= ROUTE_FUSED_MOST_CHANNELS):
         raise KernelError(f"route: {experts} experts and the {top} largest of {n} outputs (at most {ROUTE_MOST_OUTPUTS}) of rows of {width} channels")
     _check_router_bias(bias, n, "route")
     group_count, group_keep = _route_groups(groups, n, "route")
     lib = sublayer()
     _check(lib, lib.nnis_route(x.data_ptr(), _code(x), weight.data_ptr(), _ptr(bias), _ptr(correction), rows, n, width, experts, top,
-                               1 if chosen_softmax else 0, gates.data_ptr(), keep.data_ptr(), *_chosen_lists(chosen, rows, top, "route"),
+                               *_route_scoring(scoring, weight_scale, group_marks, shared_gate), gates.data_ptr(), keep.data_ptr(),
+                               *_chosen_lists(chosen, rows, top, "route"),
                                group_count, group_keep, _stream()))
     return gates, keep
 
@@ -2283,13 +2402,14 @@ def _chosen_lists(chosen, rows: int, top: int, what: str):
 
 def route_norm(x: torch.Tensor, delta: Optional[torch.Tensor], gain: torch.Tensor, eps: float, h: torch.Tensor, weight: torch.Tensor,
                correction: Optional[torch.Tensor], experts: int, top: int, gates: torch.Tensor, keep: torch.Tensor, groups=None,
-               bias: Optional[torch.Tensor] = None, chosen_softmax: bool = False, chosen=None, weight_bf16: Optional[torch.Tensor] = None):
+               bias: Optional[torch.Tensor] = None, scoring: str = "softmax", weight_scale: float = 1.0, group_marks: int = 1,
+               shared_gate: bool = False, chosen=None, weight_bf16: Optional[torch.Tensor] = None):
     """``route`` behind the RMS norm of the 32-bit stream ``x`` (+ ``delta``, summed into ``x``), in one kernel: ``h`` takes
     the normed rows, the router's logits are 32-bit sums over them.  ``weight_bf16``: the router's weight as it is stored,
     where that is bfloat16: many rows then take their logits on the matrix cores, from the rows as ``h`` rounds them."""
     _dev(x, "x"), _dev(gain, "norm weight"), _dev(h, "h"), _dev(weight, "router weight"), _dev(gates, "gates"), _dev(keep, "keep")
     rows, width = x.shape
-    n = weight.shape[0]
+    n = weight.shape[0] - (1 if shared_gate else 0)
     if (x.dtype != torch.float32 or h.shape != x.shape or gain.numel() != width or weight.dtype != torch.float32 or weight.dim() != 2
             or weight.shape[1] != width or gates.dtype != torch.float32 or keep.dtype != torch.float32
             or tuple(gates.shape) != (rows, experts) or keep.numel() != rows):
@@ -2302,7 +2422,7 @@ def route_norm(x: torch.Tensor, delta: Optional[torch.Tensor], gain: torch.Tenso
         _dev(correction, "correction")
         if correction.dtype != torch.float32 or correction.numel() != n:
             raise KernelError(f"route_norm: a float32 correction per output ({n}), got {tuple(correction.shape)} {correction.dtype}")
-    if not (0 < n <= ROUTE_MOST_OUTPUTS and 0 <= experts <= n and 0 < top <= n and width <= ROUTE_FUSED_MOST_CHANNELS):
+    if not (0 < n and n + int(shared_gate) <= ROUTE_MOST_OUTPUTS and 0 <= experts <= n and 0 < top <= n and width <= ROUTE_FUSED_MOST_CHANNELS):
         raise KernelError(f"route_norm: {experts} experts and the {top} largest of {n} outputs (at most {ROUTE_MOST_OUTPUTS}) of rows of {width} channels")
     _check_router_bias(bias, n, "route_norm")
     if weight_bf16 is not None:
@@ -2313,7 +2433,8 @@ def route_norm(x: torch.Tensor, delta: Optional[torch.Tensor], gain: torch.Tenso
     lib = sublayer()
     _check(lib, lib.nnis_route_norm(x.data_ptr(), _ptr(delta), _code(delta) if delta is not None else 0, gain.data_ptr(), _code(gain), float(eps),
                                     h.data_ptr(), _code(h), weight.data_ptr(), _ptr(weight_bf16), _ptr(bias), _ptr(correction), rows, n, width, experts, top,
-                                    1 if chosen_softmax else 0, gates.data_ptr(), keep.data_ptr(), *_chosen_lists(chosen, rows, top, "route_norm"),
+                                    *_route_scoring(scoring, weight_scale, group_marks, shared_gate), gates.data_ptr(), keep.data_ptr(),
+                                    *_chosen_lists(chosen, rows, top, "route_norm"),
                                     group_count, group_keep, _stream()))
     return h
 
@@ -2349,6 +2470,18 @@ def routed_act(z: torch.Tensor, gates: Optional[torch.Tensor], out: torch.Tensor
     return out
 
 
+def token_gate(z: torch.Tensor, ids: torch.Tensor, table: torch.Tensor, first: int, out: torch.Tensor) -> torch.Tensor:
+    """out[t, c] = gelu_tanh(z[t, c]) * table[ids[t], first + c]; ``ids`` int32, in range (the engine checks a step's)."""
+    _dev(z, "z"), _dev(ids, "ids"), _dev(table, "table"), _dev(out, "out")
+    rows, dim = z.shape
+    if out.shape != z.shape or ids.dtype != torch.int32 or ids.numel() < rows or not 0 <= first <= table.shape[1] - dim:
+        raise KernelError(f"token_gate: z {tuple(z.shape)}, out {tuple(out.shape)}, columns {first}.. of a table {tuple(table.shape)}")
+    lib = sublayer()
+    _check(lib, lib.nnis_token_gate(z.data_ptr(), _code(z), ids.data_ptr(), table.data_ptr(), _code(table), table.shape[0], table.shape[1], int(first),
+                                    out.data_ptr(), _code(out), rows, dim, _stream()))
+    return out
+
+
 def rows_axpy(y: torch.Tensor, h: torch.Tensor, keep: torch.Tensor) -> torch.Tensor:
     """y[row] += keep[row] * h[row]."""
     _dev(y, "y"), _dev(h, "h"), _dev(keep, "keep")
@@ -2356,6 +2489,16 @@ def rows_axpy(y: torch.Tensor, h: torch.Tensor, keep: torch.Tensor) -> torch.Ten
         raise KernelError(f"rows_axpy: y {tuple(y.shape)}, h {tuple(h.shape)}, a float32 factor per row")
     lib = sublayer()
     _check(lib, lib.nnis_rows_axpy(y.data_ptr(), _code(y), h.data_ptr(), _code(h), keep.data_ptr(), y.shape[0], y.shape[1], _stream()))
+    return y
+
+
+def add_rows(y: torch.Tensor, h: torch.Tensor) -> torch.Tensor:
+    """y += h, in place (``y`` the 32-bit stream, say)."""
+    _dev(y, "y"), _dev(h, "h")
+    if y.dim() != 2 or h.shape != y.shape:
+        raise KernelError(f"add_rows: y {tuple(y.shape)}, h {tuple(h.shape)}")
+    lib = sublayer()
+    _check(lib, lib.nnis_rows_axpy(y.data_ptr(), _code(y), h.data_ptr(), _code(h), None, y.shape[0], y.shape[1], _stream()))
     return y
 
 
@@ -2529,18 +2672,28 @@ def _into_stream(residual, gain, scaled, ss, rows: int, width: int, parts: int, 
     return [residual.data_ptr(), gain.data_ptr(), _code(gain), scaled.data_ptr(), ss.data_ptr()]
 
 
-def experts_few(x: torch.Tensor, up, down, regions: ExpertRegions, gates: torch.Tensor, out: Optional[torch.Tensor], into=None) -> int:
+def _check_shared_weights(weights: Optional[torch.Tensor], rows: int, what: str) -> None:
+    if weights is not None:
+        _dev(weights, "shared weights")
+        if weights.dtype != torch.float32 or weights.numel() != rows or not weights.is_contiguous():
+            raise KernelError(f"{what}: a float32 weight of the shared expert for each of {rows} rows, got {tuple(weights.shape)} {weights.dtype}")
+
+
+def experts_few(x: torch.Tensor, up, down, regions: ExpertRegions, gates: torch.Tensor, out: Optional[torch.Tensor], into=None,
+                shared_weights: Optional[torch.Tensor] = None) -> int:
     """out = the weighted sum of the chosen experts' outputs and the shared
     one's, for up to ``EXPERTS_FEW_ROWS`` rows: two kernels that read the
     weights of experts somebody chose (``gates`` [rows, experts], zero where
     not) and no others.  ``into``: (residual, gain, scaled, ss) as
     ``gemm_residual`` takes them, in place of ``out``; returns the parts of ss
-    written."""
+    written.  ``shared_weights`` (float32 [rows]): the shared expert's weight
+    in each row, in place of one."""
     _dev(x, "x"), _dev(gates, "gates")
     rows, width = x.shape
     regions.check(up, down, width)
     if x.dtype != torch.bfloat16 or gates.dtype != torch.float32 or tuple(gates.shape) != (rows, regions.experts) or rows > EXPERTS_FEW_ROWS:
         raise KernelError(f"experts_few: bfloat16 x {tuple(x.shape)} (up to {EXPERTS_FEW_ROWS} rows) and float32 gates {tuple(gates.shape)}")
+    _check_shared_weights(shared_weights, rows, "experts_few")
     parts = (width + 15) // 16
     if into is not None:
         ends = [None] + _into_stream(*into, rows, width, parts, "experts_few")
@@ -2554,7 +2707,7 @@ def experts_few(x: torch.Tensor, up, down, regions: ExpertRegions, gates: torch.
     if work is None:
         raise KernelError("experts_few: the products' workspace would have to be made inside a graph capture")
     lib = experts()
-    _check(lib, lib.nnis_experts_up_few(x.data_ptr(), up.data_ptr(), gates.data_ptr(), hidden.data_ptr(), rows, width, regions.experts,
+    _check(lib, lib.nnis_experts_up_few(x.data_ptr(), up.data_ptr(), gates.data_ptr(), _ptr(shared_weights), hidden.data_ptr(), rows, width, regions.experts,
                                         regions.inner, regions.shared, regions.form, regions.limit, regions.shared_limit, _stream()))
     _check(lib, lib.nnis_experts_down_few(hidden.data_ptr(), down.data_ptr(), gates.data_ptr(), *ends, rows, width, regions.experts,
                                           regions.inner, regions.shared, regions.form, work.data_ptr(), work.data_ptr() + GEMM_WORKSPACE_BYTES,
@@ -2563,7 +2716,7 @@ def experts_few(x: torch.Tensor, up, down, regions: ExpertRegions, gates: torch.
 
 
 def experts_many(x: torch.Tensor, up, down, regions: ExpertRegions, chosen: torch.Tensor, weights: torch.Tensor,
-                 out: Optional[torch.Tensor], into=None) -> int:
+                 out: Optional[torch.Tensor], into=None, shared_weights: Optional[torch.Tensor] = None) -> int:
     """The same for any number of rows: every expert's products run over the
     rows that chose it (``chosen`` int32 and ``weights`` float32 [rows, top]),
     gathered by lists that are made on the device."""
@@ -2574,6 +2727,7 @@ def experts_many(x: torch.Tensor, up, down, regions: ExpertRegions, chosen: torc
     if (x.dtype != torch.bfloat16 or chosen.dtype != torch.int32 or weights.dtype != torch.float32 or chosen.shape[0] != rows
             or weights.shape != chosen.shape or not 0 < top <= regions.experts):
         raise KernelError(f"experts_many: bfloat16 x {tuple(x.shape)}, int32 chosen {tuple(chosen.shape)}, float32 weights {tuple(weights.shape)}")
+    _check_shared_weights(shared_weights, rows, "experts_many")
     if into is not None:
         ends = [None] + _into_stream(*into, rows, width, 1, "experts_many")
     else:
@@ -2588,9 +2742,9 @@ def experts_many(x: torch.Tensor, up, down, regions: ExpertRegions, chosen: torc
     lib = experts()
     sizes = (rows, top, width, regions.experts, regions.inner, regions.shared, regions.form, regions.limit, regions.shared_limit)
     _check(lib, lib.nnis_experts_lists(chosen.data_ptr(), rows, top, regions.experts, counts.data_ptr(), lists.data_ptr(), _stream()))
-    _check(lib, lib.nnis_experts_many(0, x.data_ptr(), None, up.data_ptr(), hidden.data_ptr(), _ptr(hidden_shared), weights.data_ptr(),
+    _check(lib, lib.nnis_experts_many(0, x.data_ptr(), None, up.data_ptr(), hidden.data_ptr(), _ptr(hidden_shared), weights.data_ptr(), None,
                                       counts.data_ptr(), lists.data_ptr(), *sizes, _stream()))
     _check(lib, lib.nnis_experts_many(1, hidden.data_ptr(), _ptr(hidden_shared), down.data_ptr(), pairs.data_ptr(), _ptr(shared),
-                                      weights.data_ptr(), counts.data_ptr(), lists.data_ptr(), *sizes, _stream()))
+                                      weights.data_ptr(), _ptr(shared_weights), counts.data_ptr(), lists.data_ptr(), *sizes, _stream()))
     _check(lib, lib.nnis_experts_combine(pairs.data_ptr(), _ptr(shared), *ends, rows, top, width, _stream()))
     return 1

@@ -128,6 +128,7 @@ class DecoderModel:
         """ids: int32 [tokens] on the device; want_rows: int32 indices of the
         packed tokens whose logits are asked for.  Returns float32
         [len(want_rows), vocab]."""
+        ctx.ids = ids
         if hasattr(self.embedding, "forward_step"):
             x = self.embedding.forward_step(ids, ctx, cache.view("embedding"), rt)
         else:

@@ -19,7 +19,9 @@ a projection of the mixer's input, on the head's output (``head_gate``);
 queries and keys divided, head by head, by their root mean square
 (``unit_heads``), a learned factor per head on the queries behind that
 (``temperature``), and scores that fall with the logarithm of the distance by
-two learned numbers per head (``decay``).
+two learned numbers per head (``decay``); in a window's place, chunks of the
+sequence, counted from its first token, across whose borders nothing is seen
+(``chunk``).
 """
 
 from __future__ import annotations
@@ -52,7 +54,7 @@ class CausalSelfAttention(Mixer):
                  value_dim=None, scale=None, softcap=None, q_bias=None, k_bias=None, v_bias=None, o_bias=None,
                  keep_first=None, distance_bias=None, bias_reach=None, bias_buckets=None, sink=None, values_from_keys=False,
                  head_gate=None, unit_heads=None,
-                 temperature=None, decay=None):
+                 temperature=None, decay=None, chunk=None):
         """``keep_first``: with a ``window``, keys at positions below it stay
         visible.  ``distance_bias``: the name of a table [buckets, heads]; the
         scaled score of a key n positions back gets row ``distance_bucket(n,
@@ -64,7 +66,8 @@ class CausalSelfAttention(Mixer):
         that every head's query and key go through.  ``temperature``: the name
         of a tensor [heads], a factor of the head's scores.  ``decay``: the
         names of two tensors [heads], r1 and r2: the scaled score of a key n
-        positions back loses r1 * ln(1 + r2 * n)."""
+        positions back loses r1 * ln(1 + r2 * n).  ``chunk``: position i sees
+        j <= i if i // chunk == j // chunk."""
         if heads % kv_heads != 0:
             raise InvalidInput(f"{heads} query heads do not divide into {kv_heads} key/value heads")
         self.width, self.heads, self.kv_heads, self.head_dim = int(width), int(heads), int(kv_heads), int(head_dim)
@@ -85,6 +88,9 @@ class CausalSelfAttention(Mixer):
         self.output_bias = None
         self.names = {"q": q, "k": k, "v": v, "o": o}
         self.window = None if not window else int(window)
+        self.chunk = None if not chunk else int(chunk)
+        if self.chunk is not None and (self.window is not None or self.chunk < 0):
+            raise InvalidInput(f"chunks of {chunk} positions stand in a window's place ({window})")
         self.position = None
         if position is not None:
             if positions is None or position not in positions:
@@ -175,7 +181,8 @@ class CausalSelfAttention(Mixer):
         return self.qkv.weight_bytes() + self.out.weight_bytes() + (self.gate.weight_bytes() if self.gate is not None else 0)
 
     def cache_request(self):
-        return KVRequest(self.kv_heads, self.head_dim, self.window, None if self.value_dim == self.head_dim else self.value_dim)
+        # (the last ``chunk`` tokens hold whatever a chunk still shows)
+        return KVRequest(self.kv_heads, self.head_dim, self.window or self.chunk, None if self.value_dim == self.head_dim else self.value_dim)
 
     def check(self, rt):
         ops = rt.ops
@@ -199,9 +206,10 @@ class CausalSelfAttention(Mixer):
         # (runs of the keys, waves of a block) of a step of single tokens with these sizes
         if not self._matrix_cores(rt):
             return None
-        if not self.window:
+        reach = self.window or self.chunk
+        if not reach:
             return rt.ops.decode_plan(batch, self.kv_heads, longest, width=self.heads * self.value_dim)
-        longest = min(longest, self.window + 63)  # (a window of n tokens touches the pages of at most n + 63)
+        longest = min(longest, reach + 63)  # (a window of n tokens touches the pages of at most n + 63)
         runs, waves = rt.ops.decode_plan(batch, self.kv_heads, longest, width=self.heads * self.value_dim)
         # A window's keys in runs of a few pages: two waves a run (16/4 heads of 128 in a window of 1,024, whole steps of eight
         # layers in four runs: batch 1 0.481 ms against 0.493 with four waves, batch 8 0.507 against 0.520).
@@ -228,7 +236,10 @@ class CausalSelfAttention(Mixer):
 
         tables = self.position.rotary() if self.position is not None else None
         writes = not view.read_only
-        if isinstance(x, PendingNorm):
+        if isinstance(x, PendingNorm) and not self._plain and x.can_fuse(self.qkv.weight):
+            # residual sum, norm and the three projections in one kernel; biases and values of another size behind it
+            qkv = x.fused(self.qkv.weight, rt.empty(x.rows, self.qkv.out_features), rt.ops.EPILOGUE_STORE)
+        elif isinstance(x, PendingNorm):
             if (self._plain and x.can_fuse(self.qkv.weight) and tables is not None and tables.rot_dim == self.head_dim
                     and self.head_dim % 32 == 0 and view.k_pages.dtype == torch.bfloat16):
                 # residual sum, norm, the three projections, the rotation and the cache write in one kernel
@@ -238,9 +249,10 @@ class CausalSelfAttention(Mixer):
                             block_table=view.block_table if writes else None, heads=self.heads,
                             kv_heads=self.kv_heads, head_dim=self.head_dim)
                 return x.fused(self.qkv.weight, rt.empty(x.rows, self.heads * self.head_dim), rt.ops.EPILOGUE_ROPE, rope)
-            x = x.materialize()
-        tokens = x.shape[0]
-        qkv = self.qkv(x, rt)
+            qkv = self.qkv(x.materialize(), rt)
+        else:
+            qkv = self.qkv(x, rt)
+        tokens = qkv.shape[0]
         q = rt.empty(tokens, self.heads * self.head_dim)
         rt.ops.rope_kv_write(
             qkv, q,
@@ -299,7 +311,7 @@ class CausalSelfAttention(Mixer):
         if plan is None and fast:
             plan = (self.decode_plan(ctx.batch, ctx.planned_len, rt) if ctx.decode
                     else self.prompt_plan(ctx.batch, ctx.planned_rows, ctx.planned_len, rt))
-        attn = rt.ops.attention(q, attn, view, ctx, self.heads, self.kv_heads, self.head_dim, self.scale, self.window or 0,
+        attn = rt.ops.attention(q, attn, view, ctx, self.heads, self.kv_heads, self.head_dim, self.scale, self.window or -(self.chunk or 0),
                                 keep_runs=into is not None and self.output_bias is None and not (terms and terms.gated), tables=step,
                                 plan=plan, value_dim=self.value_dim, softcap=self.softcap, extras=self.extras, terms=terms)
         if isinstance(attn, rt.ops.KeyRuns) and not (into.can_take(attn, self.out.weight) and attn.fits(self.out.weight.shape[0])):

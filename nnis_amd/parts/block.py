@@ -20,7 +20,7 @@ import torch
 from ..errors import InvalidInput
 from ..weights.random_init import register_init_rule
 from .base import Block, TensorSpec, build_part, register_part
-from .lazy import PendingNorm, PostNormed, PreparedRows, PreparedStreams, ResidualInto, TanhInto
+from .lazy import PendingNorm, PostNormed, PreparedRows, PreparedStreams, ResidualInto, StreamInto, TanhInto
 
 
 def _joined(plans):
@@ -31,9 +31,10 @@ def _joined(plans):
 
 
 class PreNormBlock(Block):
-    """Without a feed-forward (and its norm) the layer is its mixer alone."""
+    """Without a feed-forward (and its norm) the layer is its mixer alone.  ``side``: a last sublayer ("part", a
+    feed-forward) that reads the stream as it is and is normed on its way out ("norm"): x += norm(part(x))."""
 
-    def __init__(self, width, norm1, mixer, norm2=None, feed_forward=None, positions=None):
+    def __init__(self, width, norm1, mixer, norm2=None, feed_forward=None, positions=None, side=None):
         self.width = int(width)
         if (feed_forward is None) != (norm2 is None):
             raise InvalidInput("a feed-forward comes with its norm, or neither")
@@ -41,7 +42,14 @@ class PreNormBlock(Block):
         self.mixer = build_part("mixer", mixer, positions=positions)
         self.norm2 = build_part("norm", norm2) if norm2 is not None else None
         self.feed_forward = build_part("feed_forward", feed_forward) if feed_forward is not None else None
-        self._parts = [part for part in (self.norm1, self.mixer, self.norm2, self.feed_forward) if part is not None]
+        self.side = self.side_norm = self.side_entry = None
+        if side is not None:
+            self.side_entry = build_part("norm", {"kind": "none", "width": self.width})  # how the side reads the stream
+            self.side, self.side_norm = build_part("feed_forward", side["part"]), build_part("norm", side["norm"])
+            if not hasattr(self.side_norm, "post_step"):
+                raise InvalidInput("a sublayer that is normed on its way out needs a norm that brings it into the stream (post_step)")
+        self._parts = [part for part in (self.norm1, self.mixer, self.norm2, self.feed_forward, self.side_entry, self.side, self.side_norm)
+                       if part is not None]
         self.graph_safe = all(getattr(part, "graph_safe", False) for part in self._parts)
 
     def tensors(self):
@@ -84,11 +92,15 @@ class PreNormBlock(Block):
         ``then``, the stream and the output not yet added)."""
         given = normed if getattr(part, "takes_pending_norm", False) else normed.materialize()
         if then is not None and getattr(part, "adds_to_residual", False):
-            out = part.forward(given, *args, into=ResidualInto(normed, then, rt))
+            out = part.forward(given, *args, into=(StreamInto if then is self.side_entry else ResidualInto)(normed, then, rt))
         else:
             out = part.forward(given, *args)
-        if isinstance(out, PendingNorm):
+        if isinstance(out, (PendingNorm, PreparedRows)):
             return out
+        if then is self.side_entry and then is not None:
+            x = normed.residual
+            rt.ops.add_rows(x, out)
+            return PreparedRows(then, x, then.forward(x, rt))
         if then is None:
             return normed.residual, out
         return then.defer(normed.residual, out, rt)
@@ -105,10 +117,21 @@ class PreNormBlock(Block):
         else:
             x, pending = stream
             normed = self.norm1.defer(x, pending, rt)
+        last = following if self.side is None else self.side_entry  # what comes behind the mixer and the feed-forward
         if self.feed_forward is None:
-            return self._run(self.mixer, normed, (ctx, view, rt), following, rt)
-        normed = self._run(self.mixer, normed, (ctx, view, rt), self.norm2, rt)
-        return self._run(self.feed_forward, normed, (ctx, rt), following, rt)
+            out = self._run(self.mixer, normed, (ctx, view, rt), last, rt)
+        else:
+            normed = self._run(self.mixer, normed, (ctx, view, rt), self.norm2, rt)
+            out = self._run(self.feed_forward, normed, (ctx, rt), last, rt)
+        if self.side is None:
+            return out
+        x, y = out.x, self.side.forward(out.h, ctx, rt)
+        if following is not None and PrePostNormBlock._rms_pair(self.side_norm, following) and y.is_contiguous():
+            # the norm on the side's way out, the sum into the stream and the next block's first norm in one kernel
+            h = rt.ops.rms_between(x, y, self.side_norm.weight, following.weight, following.eps, h=rt.empty(x.shape[0], self.width))
+            return PendingNorm.from_rows(following, x, h, rt)
+        self.side_norm.post_step(x, y, rt)
+        return (x, None) if following is None else following.defer(x, None, rt)
 
 
 class HyperConnectionBlock(Block):

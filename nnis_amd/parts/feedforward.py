@@ -112,17 +112,19 @@ class RoutedFeedForward(FeedForward):
     softmax over the chosen logits alone; ``router_bias`` (a name): joins the logits.  ``activation="clamped_swiglu"``:
     down_e(a sigmoid(1.702 a) (u + 1)), a = min(gate_e x, limit), u = up_e x held within plus or minus ``limit`` (None:
     not held).  ``shared`` (``inner``, ``limit``, ``gate``, ``up``, ``down``): one more expert of the same form, with an
-    inner size and a limit of its own, that every token uses with weight one.
+    inner size and a limit of its own, that every token uses with weight one, or with ``weight`` (a name) times
+    sigmoid(w . x), w the row of that tensor.  ``scoring="sigmoid"``: scores are sigmoid(W_r x), and the weights are the
+    chosen scores over their sum (+ 1e-20), times ``weight_scale``.
 
     ``groups`` (count, keep): the outputs, identity outputs included, form ``count`` equal groups of
-    neighbours; a group's mark is its largest corrected score, and only outputs of the ``keep`` groups with the largest
+    neighbours; a group's mark is its largest corrected score (with ``group_marks=2`` the sum of its two largest), and only outputs of the ``keep`` groups with the largest
     marks can be chosen.  The experts' up projections are one product over all experts, gated row by row with the
     scores (zero for the experts not chosen) before one down projection over all of them."""
 
     graph_safe = True
 
     def __init__(self, width, inner, experts, top, router, up, down, identity=0, correction=None, activation="relu_squared", gate=None,
-                 groups=None, scoring="softmax", router_bias=None, limit=None, shared=None):
+                 groups=None, scoring="softmax", router_bias=None, limit=None, shared=None, weight_scale=1.0, group_marks=1):
         """``up``, ``down`` and ``gate``: names with ``{}`` in the expert's place."""
         self.width, self.inner, self.experts, self.top, self.identity = int(width), int(inner), int(experts), int(top), int(identity or 0)
         if min(self.width, self.inner, self.experts, self.top) <= 0 or self.identity < 0 or self.top > self.experts + self.identity:
@@ -130,14 +132,20 @@ class RoutedFeedForward(FeedForward):
         if activation not in ("relu_squared", "silu_gated", "clamped_swiglu") or (activation != "relu_squared") != (gate is not None):
             raise InvalidInput(f"experts are relu_squared, or silu_gated or clamped_swiglu with gate projections; got {activation!r}")
         self.activation, self.limit = activation, 0.0 if limit is None else float(limit)
-        if scoring not in ("softmax", "chosen_softmax"):
-            raise InvalidInput(f"a router weighs by softmax or chosen_softmax; got {scoring!r}")
+        if scoring not in ("softmax", "chosen_softmax", "sigmoid"):
+            raise InvalidInput(f"a router weighs by softmax, chosen_softmax or sigmoid; got {scoring!r}")
+        self.weight_scale, self.group_marks = float(weight_scale), int(group_marks)
+        if (self.weight_scale != 1.0 and scoring != "sigmoid") or self.group_marks not in (1, 2):
+            raise InvalidInput(f"weights are scaled under sigmoid scores and a group's mark adds up one or two; got {weight_scale} and {group_marks}")
         if self.limit < 0.0 or (limit is not None and (activation != "clamped_swiglu" or self.limit == 0.0)):
             raise InvalidInput(f"a positive limit belongs to clamped_swiglu experts; got {limit!r} with {activation!r}")
         self.scoring = scoring
         self.shared = None if shared is None else dict(shared, inner=int(shared["inner"]), limit=float(shared.get("limit") or 0.0))
         if self.shared is not None and (activation == "relu_squared" or self.shared["inner"] <= 0):
             raise InvalidInput("a shared expert has the form of gated experts and a size of its own")
+        self.shared_weight = None if self.shared is None else self.shared.get("weight")
+        if self.shared_weight and self.identity:
+            raise InvalidInput("a router weighs identity outputs or a shared expert for each token, not both")
         self.groups = None
         if groups is not None and int(groups[0]) > 1:
             count, keep = int(groups[0]), int(groups[1])
@@ -158,6 +166,8 @@ class RoutedFeedForward(FeedForward):
             inner = self.shared["inner"]
             out += [TensorSpec(self.shared["gate"], (inner, self.width)), TensorSpec(self.shared["up"], (inner, self.width)),
                     TensorSpec(self.shared["down"], (self.width, inner))]
+            if self.shared_weight:
+                out.append(TensorSpec(self.shared_weight, (1, self.width), init="router"))
         for e in range(self.experts):
             if n["gate"]:
                 out.append(TensorSpec(n["gate"].format(e), (self.inner, self.width)))
@@ -165,14 +175,16 @@ class RoutedFeedForward(FeedForward):
         return out
 
     def check(self, rt):
-        if self.experts + self.identity > rt.ops.ROUTE_MOST_OUTPUTS or self.width > rt.ops.ROUTE_MOST_CHANNELS:
+        if self.experts + self.identity + bool(self.shared_weight) > rt.ops.ROUTE_MOST_OUTPUTS or self.width > rt.ops.ROUTE_MOST_CHANNELS:
             raise Unsupported(f"the router kernels take up to {rt.ops.ROUTE_MOST_OUTPUTS} outputs of rows of up to "
                               f"{rt.ops.ROUTE_MOST_CHANNELS} channels, got {self.experts + self.identity} and {self.width}")
 
     def bind(self, weights, rt):
         n, ops = self.names, rt.ops
-        self.router = weights[n["router"]].float().contiguous()  # its logits are a 32-bit product under either runtime
         stored = weights[n["router"]]
+        if self.shared_weight:  # (the shared expert's logit is one more output of the router's product)
+            stored = torch.cat([stored, weights[self.shared_weight]], dim=0)
+        self.router = stored.float().contiguous()  # its logits are a 32-bit product under either runtime
         self.router_stored = stored.contiguous() if stored.dtype == torch.bfloat16 else None
         self.correction = weights[n["correction"]].float().contiguous() if n["correction"] else None
         self.router_bias = weights[n["router_bias"]].float().contiguous() if n["router_bias"] else None
@@ -226,7 +238,7 @@ class RoutedFeedForward(FeedForward):
 
     def _route(self, x, rt, listed):
         """(normed rows, gates, keep, choices as lists or None): the router's own kernel, with the norm before it where
-        that is still to run."""
+        that is still to run.  ``keep``: the identity outputs' share of each row, or the shared expert's weight."""
         from .lazy import PendingNorm
 
         ops = rt.ops
@@ -234,9 +246,10 @@ class RoutedFeedForward(FeedForward):
         tokens = x.rows if pending else x.shape[0]
         gates, keep = rt.empty(tokens, self.experts, dtype=torch.float32), rt.empty(tokens, dtype=torch.float32)
         chosen = (rt.empty(tokens, self.top, dtype=torch.int32), rt.empty(tokens, self.top, dtype=torch.float32)) if listed else None
-        rule = dict(groups=self.groups, bias=self.router_bias, chosen_softmax=self.scoring == "chosen_softmax")
+        rule = dict(groups=self.groups, bias=self.router_bias, scoring=self.scoring, weight_scale=self.weight_scale,
+                    group_marks=self.group_marks, shared_gate=bool(self.shared_weight))
         if (pending and getattr(x.norm, "fusable_rms", False) and x.x.dtype == torch.float32 and x.x.is_contiguous()
-                and self.width <= ops.ROUTE_FUSED_MOST_CHANNELS):
+                and x.ready is None and self.width <= ops.ROUTE_FUSED_MOST_CHANNELS):
             h = ops.route_norm(x.x, x.delta, x.norm.weight, x.norm.eps, rt.empty(tokens, self.width), self.router, self.correction,
                                self.experts, self.top, gates, keep, chosen=chosen, weight_bf16=self.router_stored, **rule)
             x.residual = x.x
@@ -246,7 +259,7 @@ class RoutedFeedForward(FeedForward):
         if self.width <= ops.ROUTE_FUSED_MOST_CHANNELS:
             ops.route(x, self.router, self.correction, self.experts, self.top, gates, keep, chosen=chosen, **rule)
         else:
-            logits = ops.router_logits(x, self.router, rt.empty(tokens, self.experts + self.identity, dtype=torch.float32))
+            logits = ops.router_logits(x, self.router, rt.empty(tokens, self.router.shape[0], dtype=torch.float32))
             ops.route_top(logits, self.correction, self.experts, self.top, gates, keep, **rule)
         return x, gates, keep, chosen
 
@@ -256,11 +269,12 @@ class RoutedFeedForward(FeedForward):
         tokens = x.rows if hasattr(x, "rows") else x.shape[0]
         many = self.regions is not None and tokens >= self.many_rows
         x, gates, keep, chosen = self._route(x, rt, many)
+        shared_weights = keep if self.shared_weight else None
         if self.regions is not None and (many or tokens <= self.few_rows):
             def run(out, stream=None):
                 if many:
-                    return ops.experts_many(x, self.up.weight, self.down.weight, self.regions, chosen[0], chosen[1], out, stream)
-                return ops.experts_few(x, self.up.weight, self.down.weight, self.regions, gates, out, stream)
+                    return ops.experts_many(x, self.up.weight, self.down.weight, self.regions, chosen[0], chosen[1], out, stream, shared_weights)
+                return ops.experts_few(x, self.up.weight, self.down.weight, self.regions, gates, out, stream, shared_weights)
 
             if into is not None and hasattr(into, "take_by") and into.can_take(x, self.down.weight):
                 return into.take_by(lambda *stream: run(None, stream))  # (the last kernel adds to the stream itself)
@@ -274,7 +288,7 @@ class RoutedFeedForward(FeedForward):
             ops.routed_act(z, gates, hidden, self.activation, self.limit)
         else:
             ops.routed_act(z[:, :2 * inner], gates, hidden[:, :inner], self.activation, self.limit, inner=self.padded)
-            ops.routed_act(z[:, 2 * inner:], None, hidden[:, inner:], self.activation, self.shared["limit"], inner=extra)
+            ops.routed_act(z[:, 2 * inner:], None if shared_weights is None else shared_weights.view(tokens, 1), hidden[:, inner:], self.activation, self.shared["limit"], inner=extra)
         if into is not None and not self.identity and into.can_take(hidden, self.down.weight):
             return into.take(hidden, self.down.weight)
         y = self.down(hidden, rt)
@@ -284,6 +298,42 @@ class RoutedFeedForward(FeedForward):
             rt.ops.rows_axpy(y, x, keep)
         return y
 
+
+class TokenInput(FeedForward):
+    """An input of a token's own, gated by the stream: W_p (gelu_tanh(W_g x) * e), e the columns first .. first + inner - 1
+    of the token's row of a table that the layers share."""
+
+    graph_safe = True
+
+    def __init__(self, width, inner, vocab_size, table, columns, first, gate, proj):
+        self.width, self.inner, self.vocab_size = int(width), int(inner), int(vocab_size)
+        self.columns, self.first = int(columns), int(first)
+        if min(self.width, self.inner) <= 0 or not 0 <= self.first <= self.columns - self.inner:
+            raise InvalidInput(f"a token's input of {inner} columns from {first} on does not fit a table of {columns}")
+        self.names = {"table": table, "gate": gate, "proj": proj}
+        self.table = self.gate = self.proj = None
+
+    def tensors(self):
+        n = self.names
+        return [TensorSpec(n["table"], (self.vocab_size, self.columns), init="token_input"), TensorSpec(n["gate"], (self.inner, self.width)),
+                TensorSpec(n["proj"], (self.width, self.inner))]
+
+    def bind(self, weights, rt):
+        self.table = weights[self.names["table"]].contiguous()
+        self.gate = Projection(weights[self.names["gate"]], rt)
+        self.proj = Projection(weights[self.names["proj"]], rt)
+
+    def weight_bytes(self):
+        return self.gate.weight_bytes() + self.proj.weight_bytes()
+
+    def forward(self, x, ctx, rt):
+        z = self.gate(x, rt, out_dtype=torch.float32)
+        return self.proj(rt.ops.token_gate(z, ctx.ids, self.table, self.first, rt.empty(x.shape[0], self.inner)), rt)
+
+
+# what a random model draws: a token's own input of the size of one
+register_init_rule("token_input", lambda spec, generator, dtype: torch.randn(tuple(spec.shape), generator=generator).to(dtype), replace=True)
+register_part("feed_forward", "token_input", TokenInput)
 
 # what a random model draws: coefficients of a size that matters, router rows that spread the scores
 register_init_rule("poly_coefficients", lambda spec, generator, dtype: (0.5 + 0.25 * torch.randn(tuple(spec.shape), generator=generator)).to(dtype),

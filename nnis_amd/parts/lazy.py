@@ -6,13 +6,15 @@ norm into that projection's kernel (``fused``); any other consumer calls
 ``materialize`` and gets the rows from the norm's own kernel.  Either way
 ``residual`` afterwards holds the stream the block goes on with.
 
-It comes in two states.  *Lazy*: ``x`` and a part's output ``delta`` that is
+It comes in three states.  *Lazy*: ``x`` and a part's output ``delta`` that is
 not added yet; the consumer's kernel takes the sum, the statistics and the
 gain itself (up to ``FUSED_MAX_TOKENS`` rows).  *Prepared*: the projection
 that produced the part's output has already added it to the stream and left
 ``scaled`` = bfloat16(stream * gain) and parts of each row's sum of squares
 (``ResidualInto.take``); the consumer's kernel multiplies ``scaled`` and
 applies 1 / sqrt(mean + eps) to the product, for any number of rows.
+*Ready*: the kernel that wrote the stream last ran the norm too; its rows are
+there.
 """
 
 from __future__ import annotations
@@ -33,6 +35,13 @@ class PendingNorm:
         self.scaled: Optional[torch.Tensor] = None  # prepared state
         self.ss: Optional[torch.Tensor] = None
         self.parts = 0
+        self.ready: Optional[torch.Tensor] = None  # the norm's rows, where whoever wrote the stream last made them
+
+    @classmethod
+    def from_rows(cls, norm, residual: torch.Tensor, rows: torch.Tensor, rt) -> "PendingNorm":
+        pending = cls(norm, residual, None, rt)
+        pending.residual, pending.ready = residual, rows
+        return pending
 
     @classmethod
     def prepared(cls, norm, residual: torch.Tensor, scaled: torch.Tensor, ss: torch.Tensor, parts: int, rt) -> "PendingNorm":
@@ -42,6 +51,8 @@ class PendingNorm:
         return pending
 
     def materialize(self) -> torch.Tensor:
+        if self.ready is not None:
+            return self.ready
         if self.delta is None:
             out = self.norm.forward(self.x, self.rt)
         else:
@@ -52,6 +63,8 @@ class PendingNorm:
     def can_fuse(self, weight) -> bool:
         """True when ``fused`` may be called with this projection weight."""
         ops = self.rt.ops
+        if self.ready is not None:
+            return False
         fits = (
             getattr(self.norm, "fusable_rms", False)
             and self.x.dtype == torch.float32
@@ -86,10 +99,12 @@ class ResidualInto:
         self.rt = rt
 
     def can_take(self, x: torch.Tensor, weight) -> bool:
+        return getattr(self.norm, "fusable_rms", False) and self._fits(x, weight)
+
+    def _fits(self, x: torch.Tensor, weight) -> bool:
         residual = self.source.residual
         return (
-            getattr(self.norm, "fusable_rms", False)
-            and residual is not None
+            residual is not None
             and residual.dtype == torch.float32
             and residual.is_contiguous()
             and self.rt.dtype == torch.bfloat16
@@ -112,6 +127,27 @@ class ResidualInto:
         ss = rt.empty(rt.ops.gemm_residual_parts(rows, width), rows, dtype=torch.float32)
         parts = write(residual, self.norm.weight, scaled, ss)
         return PendingNorm.prepared(self.norm, residual, scaled, ss, parts, rt)
+
+
+class StreamInto(ResidualInto):
+    """``ResidualInto`` where what comes next reads the stream as it is (a
+    norm of kind ``none``): ``take`` returns the stream with its rows in the
+    activation type (``PreparedRows``), which the projection's kernel wrote
+    beside its sum."""
+
+    def can_take(self, x: torch.Tensor, weight) -> bool:
+        return getattr(self.norm, "ones", None) is not None and self._fits(x, weight)
+
+    def take_by(self, write):
+        rt, residual = self.rt, self.source.residual
+        rows, width = residual.shape
+        plain = rt.empty(rows, width)
+        ss = rt.empty(rt.ops.gemm_residual_parts(rows, width), rows, dtype=torch.float32)  # (nobody reads it)
+        write(residual, self.norm.ones, plain, ss)
+        return PreparedRows(self.norm, residual, plain)
+
+    def take(self, x: torch.Tensor, weight):
+        return self.take_by(lambda residual, gain, scaled, ss: self.rt.ops.gemm_residual(x, weight, residual, gain, scaled, ss))
 
 
 class PreparedStreams:

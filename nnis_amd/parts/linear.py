@@ -42,3 +42,13 @@ class Projection:
         if rows == 0:
             return out
         return rt.ops.linear(x, self.weight, out)
+
+    def of(self, x, rt) -> torch.Tensor:
+        """The product with rows, or with a norm that has not run yet (``PendingNorm``), in one kernel where that can be."""
+        from .lazy import PendingNorm
+
+        if not isinstance(x, PendingNorm):
+            return self(x, rt)
+        if x.can_fuse(self.weight):
+            return x.fused(self.weight, rt.empty(x.rows, self.out_features), rt.ops.EPILOGUE_STORE)
+        return self(x.materialize(), rt)

@@ -14,23 +14,23 @@ class RMSNorm(Norm):
     graph_safe = True
     fusable_rms = True  # ``weight`` and ``eps`` are all a projection kernel needs to apply this norm itself
 
-    def __init__(self, width: int, eps: float, weight: str, offset: float = 0.0):
+    def __init__(self, width: int, eps: float, weight: str, offset: float = 0.0, wide: bool = False):
         """``offset``: the gain is offset + weight (a weight stored around zero has an offset of 1); the sum is made
-        once, in 32-bit, when the weights are bound, and such a norm is not taken into a projection's kernel."""
+        once, in 32-bit, when the weights are bound.  ``wide``: a gain without an offset is kept in 32-bit too (so that
+        it meets norms with one in a kernel that takes two)."""
         self.width = int(width)
         self.eps = float(eps)
         self.weight_name = weight
         self.offset = float(offset)
+        self.wide = bool(wide) or bool(self.offset)
         self.weight = None
-        if self.offset:
-            self.fusable_rms = False
 
     def tensors(self):
         return [TensorSpec(self.weight_name, (self.width,), init="small" if self.offset else "gain")]
 
     def bind(self, weights, rt):
         self.weight = weights[self.weight_name].contiguous()
-        if self.offset:
+        if self.wide:
             self.weight = (self.weight.float() + self.offset).contiguous()
 
     def weight_bytes(self):
@@ -70,6 +70,11 @@ class NoNorm(Norm):
 
     def __init__(self, width: int):
         self.width = int(width)
+        self.ones = None
+
+    def bind(self, weights, rt):
+        # the gain of kernels that write a stream's rows times the gain of the norm that comes next
+        self.ones = torch.ones(self.width, dtype=torch.bfloat16, device=rt.device)
 
     def forward(self, x, rt, rows=None):
         if rows is None and x.dtype == rt.dtype:

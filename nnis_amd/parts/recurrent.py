@@ -1,6 +1,7 @@
 """Mixers that carry a state of fixed size from token to token instead of
-keys and values: the selective scan, gated linear attention, retention, the
-gated delta rule and the minGRU.  Their state
+keys and values: the selective scan, Mamba-2, gated linear attention,
+retention, the gated delta rule, the minGRU and the real-gated linear recurrent
+unit.  Their state
 lives in the cache's per-slot regions (``StateRequest``), in 32-bit, zero when
 a sequence starts; a step reads it at each sequence's first row and leaves it
 behind the last, so a prompt gives the same in one step, in portions or token
@@ -355,6 +356,148 @@ class MinGRU(Mixer):
         return self.out(y, rt)
 
 
+class StateSpace(Mixer):
+    """Mamba-2's mixer (state-space duality).  With H heads of P value channels, N states, G groups (head h uses group
+    h // (H / G)):
+
+        [z | x | B | C | dt] = W_in h                     z, x: H P each;  B, C: G N each;  dt: H
+        [x | B | C] <- silu(conv([x | B | C]) + b_conv)   causal, per channel, ``taps`` wide, last tap on the token
+        dt <- softplus(dt + dt_bias)                      one step size a head
+        S <- exp(-exp(A_log) dt) S + dt x B^T,   y = S C + D x       per head, S [P, N]
+        out = W_o (R(y * silu(z)) * w_norm)               R: each of ``norm_parts`` equal parts over its own root mean square
+
+    State per sequence: S, and the convolution's last inputs, position p's in row p % taps."""
+
+    graph_safe = True
+
+    def __init__(self, width, heads, value_dim, states, groups, taps, norm_parts, eps, w_in, conv, conv_bias, dt_bias, a_log, d, norm, w_out):
+        self.width, self.heads, self.value_dim, self.states, self.groups = int(width), int(heads), int(value_dim), int(states), int(groups)
+        self.taps, self.norm_parts, self.eps = int(taps), int(norm_parts), float(eps)
+        self.inner = self.heads * self.value_dim
+        if min(self.width, self.heads, self.value_dim, self.states, self.groups, self.taps, self.norm_parts) <= 0:
+            raise InvalidInput("a state space needs positive sizes")
+        if self.heads % self.groups or self.inner % self.norm_parts:
+            raise InvalidInput(f"{heads} heads of {value_dim} do not divide into {groups} groups and {norm_parts} parts of a norm")
+        self.channels = self.inner + 2 * self.groups * self.states  # what the convolution runs over
+        self.names = dict(w_in=w_in, conv=conv, conv_bias=conv_bias, dt_bias=dt_bias, a_log=a_log, d=d, norm=norm, w_out=w_out)
+
+    def tensors(self):
+        n, H = self.names, self.heads
+        return [TensorSpec(n["w_in"], (self.inner + self.channels + H, self.width)), TensorSpec(n["conv"], (self.channels, self.taps), init="conv_taps"),
+                TensorSpec(n["conv_bias"], (self.channels,), init="small"), TensorSpec(n["dt_bias"], (H,), init="step_bias"),
+                TensorSpec(n["a_log"], (H,), init="head_rates"), TensorSpec(n["d"], (H,), init="gain"),
+                TensorSpec(n["norm"], (self.inner,), init="gain"), TensorSpec(n["w_out"], (self.width, self.inner))]
+
+    def check(self, rt):
+        if self.states > 256 or self.taps > 16:
+            raise Unsupported(f"the state-space kernels take up to 256 states and 16 taps, got {self.states} and {self.taps}")
+
+    def bind(self, weights, rt):
+        n = self.names
+        self.w_in = Projection(weights[n["w_in"]], rt)
+        self.conv = weights[n["conv"]].contiguous()
+        self.conv_bias = weights[n["conv_bias"]].contiguous()
+        self.dt_bias = weights[n["dt_bias"]].float().contiguous()
+        self.rate = torch.exp(weights[n["a_log"]].float()).contiguous()  # 32-bit, made once
+        self.D = weights[n["d"]].float().contiguous()
+        self.norm = weights[n["norm"]].float().contiguous()
+        self.w_out = Projection(weights[n["w_out"]], rt)
+
+    def weight_bytes(self):
+        small = sum(t.numel() * t.element_size() for t in (self.conv, self.conv_bias, self.dt_bias, self.rate, self.D, self.norm))
+        return small + self.w_in.weight_bytes() + self.w_out.weight_bytes()
+
+    def cache_request(self):
+        return (StateRequest((self.heads, self.value_dim, self.states)), StateRequest((self.taps, self.channels)))
+
+    takes_pending_norm = True
+    adds_to_residual = True
+
+    def forward(self, x, ctx, view, rt, into=None):
+        state, conv_state = view
+        if state.read_only:
+            raise Unsupported("a state space cannot read another layer's state")
+        rows = self.w_in.of(x, rt)
+        tokens, inner = rows.shape[0], self.inner
+        z, xbc, dt = rows[:, :inner], rows[:, inner:inner + self.channels], rows[:, inner + self.channels:]
+        xbc = rt.ops.conv_silu(xbc, self.channels, self.conv, self.conv_bias, conv_state.state, ctx, rt.empty(tokens, self.channels), ring=True)
+        y = rt.ops.state_space(xbc, dt, z, self.rate, self.dt_bias, self.D, state.state, ctx, self.groups, rt.empty(tokens, inner, dtype=torch.float32))
+        y = rt.ops.parts_norm(y, self.norm, self.norm_parts, self.eps, rt.empty(tokens, inner))
+        if into is not None and into.can_take(y, self.w_out.weight):
+            return into.take(y, self.w_out.weight)
+        return self.w_out(y, rt)
+
+
+class GatedLinearUnit(Mixer):
+    """Griffin's recurrent block with the real-gated linear recurrent unit.  With C channels in ``blocks`` equal parts:
+
+        y = gelu_tanh(W_y h + b_y),   u = conv(W_x h + b_x) + b_conv       causal, per channel, ``taps`` wide, no activation
+        r = sigmoid(R_b u_b + b_r),   i = sigmoid(I_b u_b + b_i)           in each part b, R_b and I_b square
+        log a = -8 r softplus(rate),  S <- a S + sqrt(1 - a^2) i u         element by element, a = exp(log a)
+        out = W_o (S * y)
+
+    State per sequence: S [C], and the convolution's last inputs (biased), position p's in row p % taps.  Everything
+    behind u is 32-bit under either runtime."""
+
+    graph_safe = True
+
+    def __init__(self, width, channels, blocks, taps, y, y_bias, x, x_bias, conv, conv_bias, r, r_bias, i, i_bias, rate, o):
+        self.width, self.channels, self.blocks, self.taps = int(width), int(channels), int(blocks), int(taps)
+        if min(self.width, self.channels, self.blocks, self.taps) <= 0 or self.channels % self.blocks:
+            raise InvalidInput(f"a gated linear unit of {channels} channels in {blocks} blocks with {taps} taps")
+        self.block = self.channels // self.blocks
+        self.names = dict(y=y, y_bias=y_bias, x=x, x_bias=x_bias, conv=conv, conv_bias=conv_bias, r=r, r_bias=r_bias, i=i, i_bias=i_bias,
+                          rate=rate, o=o)
+
+    def tensors(self):
+        n, C, B, b = self.names, self.channels, self.blocks, self.block
+        return [TensorSpec(n["y"], (C, self.width)), TensorSpec(n["y_bias"], (C,), init="small"),
+                TensorSpec(n["x"], (C, self.width)), TensorSpec(n["x_bias"], (C,), init="small"),
+                TensorSpec(n["conv"], (C, self.taps), init="conv_taps"), TensorSpec(n["conv_bias"], (C,), init="small"),
+                TensorSpec(n["r"], (B, b, b)), TensorSpec(n["r_bias"], (B, b), init="small"),
+                TensorSpec(n["i"], (B, b, b)), TensorSpec(n["i_bias"], (B, b), init="small"),
+                TensorSpec(n["rate"], (C,), init="unit_rate"), TensorSpec(n["o"], (self.width, C))]
+
+    def check(self, rt):
+        if self.taps > 16 or self.block > 12288:
+            raise Unsupported(f"the gated linear unit's kernels take up to 16 taps and blocks of 12288 channels, got {self.taps} and {self.block}")
+
+    def bind(self, weights, rt):
+        n = self.names
+        self.yx = Projection(torch.cat([weights[n["y"]], weights[n["x"]]], dim=0), rt)
+        self.y_bias, self.x_bias = weights[n["y_bias"]].float().contiguous(), weights[n["x_bias"]].float().contiguous()
+        self.conv, self.conv_bias = weights[n["conv"]].contiguous(), weights[n["conv_bias"]].contiguous()
+        self.gates = torch.cat([weights[n["r"]], weights[n["i"]]], dim=1).contiguous()  # [blocks, 2 * block, block]
+        self.r_bias, self.i_bias = (weights[n[key]].float().reshape(-1).contiguous() for key in ("r_bias", "i_bias"))
+        self.rate = torch.nn.functional.softplus(weights[n["rate"]].double()).float().contiguous()  # made once
+        self.out = Projection(weights[n["o"]], rt)
+
+    def weight_bytes(self):
+        small = sum(t.numel() * t.element_size() for t in (self.conv, self.conv_bias, self.y_bias, self.x_bias, self.r_bias, self.i_bias, self.rate))
+        return small + self.gates.numel() * self.gates.element_size() + self.yx.weight_bytes() + self.out.weight_bytes()
+
+    def cache_request(self):
+        return (StateRequest((self.channels,)), StateRequest((self.taps, self.channels)))
+
+    takes_pending_norm = True
+    adds_to_residual = True
+
+    def forward(self, x, ctx, view, rt, into=None):
+        state, conv_state = view
+        if state.read_only:
+            raise Unsupported("a gated linear unit cannot read another layer's state")
+        C, ops = self.channels, rt.ops
+        rows = self.yx.of(x, rt)
+        tokens = rows.shape[0]
+        u = ops.conv_silu(rows[:, C:], C, self.conv, self.conv_bias, conv_state.state, ctx, rt.empty(tokens, C), x_bias=self.x_bias,
+                          activation=None, ring=True)
+        logits = ops.heads_linear(u, self.gates, None, self.blocks, rt.empty(tokens, 2 * C, dtype=torch.float32))
+        y = ops.rg_lru(logits, self.blocks, self.r_bias, self.i_bias, self.rate, u, rows[:, :C], self.y_bias, state.state, ctx, rt.empty(tokens, C))
+        if into is not None and into.can_take(y, self.out.weight):
+            return into.take(y, self.out.weight)
+        return self.out(y, rt)
+
+
 class SideBySide(Mixer):
     """Several mixers that read the same input; each output is divided by its
     root mean square over the model width and multiplied by a weight of its
@@ -467,4 +610,9 @@ register_part("mixer", "gated_linear_attention", GatedLinearAttention)
 register_part("mixer", "retention", Retention)
 register_part("mixer", "gated_delta_rule", GatedDeltaRule)
 register_part("mixer", "min_gru", MinGRU)
+register_init_rule("head_rates", lambda spec, generator, dtype: torch.log(1.0 + 3.0 * torch.rand(tuple(spec.shape), generator=generator)).to(dtype),
+                   replace=True)
+register_init_rule("unit_rate", lambda spec, generator, dtype: (-3.0 + _noise(spec, generator)).to(dtype), replace=True)
+register_part("mixer", "mamba2", StateSpace)
+register_part("mixer", "rg_lru", GatedLinearUnit)
 register_part("mixer", "side_by_side", SideBySide)

@@ -293,7 +293,7 @@ def test_the_router_weighs_over_the_chosen_logits(outputs, top, rows, width):
         return (torch.empty(rows, outputs, device="cuda"), torch.empty(rows, device="cuda"),
                 (torch.empty(rows, top, dtype=torch.int32, device="cuda"), torch.empty(rows, top, device="cuda")))
 
-    rule = dict(bias=bias.cuda(), chosen_softmax=True)
+    rule = dict(bias=bias.cuda(), scoring="chosen_softmax")
     gates, keep, chosen = made()
     ops.route(h.float().cuda(), w.cuda(), None, outputs, top, gates, keep, chosen=chosen, **rule)
     check(gates, chosen)
