@@ -59,6 +59,13 @@ beside a Robopel of windowed attention layers and routed feed-forwards of the
 same width, layers, heads, window and vocabulary, its inner sizes chosen so
 that both have the same number of weights.
 
+``--workload tugovik`` measures the Tugovik design (Mamba-2, attention inside
+chunks, the real-gated linear recurrent unit; experts with sigmoid scores
+chosen among groups beside a gated shared expert; a token's own input in every
+layer) beside a Tonanex of windowed attention layers of the same width, layers,
+heads, window and vocabulary, its experts' inner size chosen so that both have
+the same number of weights.
+
 Peaks used for the fractions are the published MI355X ones: HBM 8 TB/s; dense
 matrix rate 2.5 PFLOP/s for bfloat16, 157.3 TFLOP/s for 32-bit.
 """
@@ -241,7 +248,7 @@ def prefill_run(shape, rng, tokens=2048):
     torch.cuda.empty_cache()
     seconds = sorted(times[3:])[3]  # the median of seven runs of a shape that has come before (and is captured, where it is)
     flops = {"Zifunex": zifunex_step_flops, "Mutedra": mutedra_step_flops, "Robopel": robopel_step_flops,
-             "Mafalorn": mafalorn_step_flops, "Tonanex": tonanex_step_flops}.get(shape.config.get("architecture"), step_flops)(
+             "Mafalorn": mafalorn_step_flops, "Tonanex": tonanex_step_flops, "Tugovik": tugovik_step_flops}.get(shape.config.get("architecture"), step_flops)(
         shape.config, [tokens], 1)
     return {"value": round(tokens / seconds, 1), "tokens": tokens, "ms": round(1000.0 * seconds, 3),
             "frac": round(flops / seconds / FLOP_PEAK[shape.dtype], 5), "first_ms": round(1000.0 * times[0], 3)}
@@ -604,6 +611,76 @@ def tonanex_twin_config(sizes):
             "layers": [{"type": "attention", "mixer": mixer, "mlp": mlps[kind]} for kind in TONANEX_LAYERS]}
 
 
+# Tugovik at two sets of layer sizes: M = Mamba-2 (heads, value channels, states, groups), A = attention inside chunks,
+# R = the gated linear recurrent unit (channels, blocks); experts (experts, chosen, inner size, the shared expert's) in every layer.
+TUGOVIK_SETS = {
+    "w1024": dict(width=1024, attention=(16, 4, 64, 64), chunk=512, space=(32, 64, 128, 4), unit=(1280, 5), moe=(16, 2, 352, 704), side=128),
+    "w2048": dict(width=2048, attention=(16, 4, 128, 128), chunk=1024, space=(64, 64, 128, 8), unit=(2560, 10), moe=(16, 2, 704, 1408), side=128),
+}
+TUGOVIK_LAYERS = "MARMARMA"
+
+
+def tugovik_config(sizes):
+    heads, kv_heads, dim, vdim = sizes["attention"]
+    s_heads, s_vdim, states, groups = sizes["space"]
+    channels, blocks = sizes["unit"]
+    experts, top, expert_ff, shared_ff = sizes["moe"]
+    mlp = {"kind": "moe", "expert": {"ff": expert_ff}, "router": {"experts": experts, "top": top, "scale": 2.5, "groups": {"count": 4, "keep": 2}},
+           "shared": {"ff": shared_ff}}
+    kinds = {
+        "A": {"type": "attention", "mlp": mlp, "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": dim ** -0.5,
+                                                         "mask": {"size": sizes["chunk"]}}},
+        "M": {"type": "mamba2", "mlp": mlp, "mixer": {"heads": s_heads, "vdim": s_vdim, "state": states, "groups": groups, "conv": 4,
+                                                      "norm_groups": groups}},
+        "R": {"type": "rglru", "mlp": mlp, "mixer": {"width": channels, "blocks": blocks, "conv": 4}},
+    }
+    return {"architecture": "Tugovik", "vocab": ZIFUNEX_VOCAB, "width": sizes["width"], "norm": {"eps": 1e-6}, "token_side": {"dim": sizes["side"]},
+            "layers": [kinds[kind] for kind in TUGOVIK_LAYERS]}
+
+
+def _tugovik_mixer_weights(layer, w):
+    m = layer["mixer"]
+    if layer["type"] == "attention":
+        return (m["heads"] + m["kv_heads"]) * (m["dim"] + m["vdim"]) * w
+    if layer["type"] == "mamba2":
+        inner = m["heads"] * m["vdim"]
+        return (3 * inner + 2 * m["groups"] * m["state"] + m["heads"]) * w
+    return 3 * m["width"] * w + 2 * m["width"] * (m["width"] // m["blocks"])
+
+
+def tugovik_step_flops(config, tokens_per_sequence, wanted_rows):
+    """Multiply-adds x2 of one step over whole prompts from empty slots: the projections, a chunk's keys, the recurrences,
+    a token's own input, and of the experts those that a token has chosen, and the shared one."""
+    w = config["width"]
+    total = 0
+    for n in tokens_per_sequence:
+        for layer in config["layers"]:
+            m, mlp = layer["mixer"], layer["mlp"]
+            total += 2 * _tugovik_mixer_weights(layer, w) * n
+            if layer["type"] == "attention":
+                total += 2 * m["heads"] * (m["dim"] + m["vdim"]) * sum(i % m["mask"]["size"] + 1 for i in range(n))
+            elif layer["type"] == "mamba2":
+                total += 2 * 2 * m["heads"] * m["vdim"] * m["state"] * n
+            total += 2 * (3 * w * (mlp["expert"]["ff"] * mlp["router"]["top"] + mlp["shared"]["ff"]) + (mlp["router"]["experts"] + 1) * w) * n
+            total += 2 * 2 * config["token_side"]["dim"] * w * n
+    return total + 2 * wanted_rows * w * config["vocab"]
+
+
+def tugovik_twin_config(sizes):
+    """The closest model the library had: a Tonanex whose layers are windowed attention with experts beside a shared one,
+    the experts' inner size such that both models have as many weights in their layers."""
+    own = tugovik_config(sizes)
+    w, count = sizes["width"], len(own["layers"])
+    experts, _, expert_ff, _ = sizes["moe"]
+    attention = next(layer for layer in own["layers"] if layer["type"] == "attention")
+    more = sum(_tugovik_mixer_weights(layer, w) - _tugovik_mixer_weights(attention, w) + 2 * sizes["side"] * w for layer in own["layers"])
+    inner = (expert_ff + more / (3 * w * experts * count)) // 16 * 16
+    twin = dict(width=w, ff=0, attention=sizes["attention"], window=sizes["chunk"], moe=sizes["moe"][:2] + (int(inner),) + sizes["moe"][3:])
+    config = tonanex_config(twin)
+    config["layers"] = [config["layers"][-1]] * count
+    return config
+
+
 def design_run(args, rng, design, sets, config_of, twin_of, twin="llama"):
     """Each set of sizes: the design's model and its Llama twin, a prompt of 2,048 tokens and decode at batch 1, 8, 64."""
     import torch
@@ -656,7 +733,7 @@ def main() -> int:
     parser.add_argument("--no-other-shapes", action="store_true", help="points of the headline's shape only")
     parser.add_argument("--prompt-min", type=int, default=128, help="shortest prompt of the decode batches")
     parser.add_argument("--prompt-max", type=int, default=2048, help="longest prompt of the decode batches (within the context)")
-    parser.add_argument("--workload", choices=["tinyllama-ragged", "zifunex", "mutedra", "robopel", "mafalorn", "tonanex"], help="run this workload alone")
+    parser.add_argument("--workload", choices=["tinyllama-ragged", "zifunex", "mutedra", "robopel", "mafalorn", "tonanex", "tugovik"], help="run this workload alone")
     args = parser.parse_args()
     if args.gpus != 1:
         print(f"bench.py: this library runs on one GPU; --gpus {args.gpus} is not supported")
@@ -722,6 +799,18 @@ def main() -> int:
             "ms_per_step": head["ms_per_step"], "higher_is_better": True, "dtype": "bf16" if args.dtype == "bfloat16" else "fp32",
             "data": "synthetic: random weights from a seed, uniform-random token ids",
             "config": {"model": "Tonanex, 8 layers of width 2048 (decode at batch 8)", "sets": TONANEX_SETS, "layers": TONANEX_LAYERS,
+                       "vocab": ZIFUNEX_VOCAB, "context": ZIFUNEX_CONTEXT, "prompt_min": args.prompt_min, "prompt_max": args.prompt_max},
+            "models": models, "env": environment()}))
+        return 0
+    if args.workload == "tugovik":
+        models = design_run(args, rng, "tugovik", TUGOVIK_SETS, tugovik_config, tugovik_twin_config, twin="tonanex")
+        head = models["tugovik-w2048"]["decode_b8"]
+        print(json.dumps({
+            "metric": "Tugovik at two sets of layer sizes beside a Tonanex of windowed attention of the same sizes: prefill of 2,048 tokens, decode at batch 1, 8, 64",
+            "value": head["tokens_per_second"], "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
+            "ms_per_step": head["ms_per_step"], "higher_is_better": True, "dtype": "bf16" if args.dtype == "bfloat16" else "fp32",
+            "data": "synthetic: random weights from a seed, uniform-random token ids",
+            "config": {"model": "Tugovik, 8 layers of width 2048 (decode at batch 8)", "sets": TUGOVIK_SETS, "layers": TUGOVIK_LAYERS,
                        "vocab": ZIFUNEX_VOCAB, "context": ZIFUNEX_CONTEXT, "prompt_min": args.prompt_min, "prompt_max": args.prompt_max},
             "models": models, "env": environment()}))
         return 0
