@@ -123,7 +123,9 @@ _RECURRENT_SIGNATURES = {
 
 _STATE_SPACE_SIGNATURES = {
     "nnis_state_space": [_VOID, _INT, _INT, _VOID, _INT, _INT, _VOID, _VOID, _VOID, _VOID, _INT, _INT, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _INT,
-                         _VOID, _INT, _VOID],
+                         _VOID, _INT, _INT, _VOID],
+    "nnis_state_space_step": [_VOID, _INT, _INT, _VOID, _INT, _INT, _VOID, _VOID, _VOID, _VOID, _INT, _INT, _VOID, _VOID, _VOID, _VOID, _VOID, _VOID, _VOID,
+                              _INT, _INT, _INT, _INT, _INT, _INT, _VOID, _INT, _VOID],
     "nnis_parts_norm": [_VOID, _INT, _VOID, _VOID, _INT, _INT, _INT, _INT, _FLT, _VOID],
 }
 
@@ -1769,10 +1771,11 @@ def _columns(t: torch.Tensor, tokens: int, width: int, what: str) -> int:
 
 
 def state_space(xbc: torch.Tensor, dt: torch.Tensor, z: torch.Tensor, rate: torch.Tensor, dt_bias: torch.Tensor, D: torch.Tensor,
-                state: torch.Tensor, ctx, groups: int, out: torch.Tensor) -> torch.Tensor:
+                state: torch.Tensor, ctx, groups: int, out: torch.Tensor, longest: Optional[int] = None) -> torch.Tensor:
     """Mamba-2's recurrence over each sequence's tokens, from and into ``state`` (float32 [slots, heads, P, N]): with
     ``xbc`` [tokens, heads * P + 2 * groups * N] = (x | B | C) and dt = softplus(dt + dt_bias) [tokens, heads],
-    S <- exp(-rate dt) S + dt x B^T;  out = (S C + D x) * silu(z).  ``dt``, ``z``: views whose rows may be further apart."""
+    S <- exp(-rate dt) S + dt x B^T;  out = (S C + D x) * silu(z).  ``dt``, ``z``: views whose rows may be further apart.
+    ``longest``: the most tokens a sequence brings (None: the step's); prompts of 16 and more in bfloat16 run on the matrix cores."""
     tokens = xbc.shape[0]
     for t, what in ((state, "state"), (out, "out"), (rate, "rate"), (dt_bias, "dt_bias"), (D, "D")):
         _dev(t, what)
@@ -1787,7 +1790,35 @@ def state_space(xbc: torch.Tensor, dt: torch.Tensor, z: torch.Tensor, rate: torc
     lib = state_space_module()
     _check(lib, lib.nnis_state_space(xbc.data_ptr(), _code(xbc), xs, dt.data_ptr(), _code(dt), ds, rate.data_ptr(), dt_bias.data_ptr(), D.data_ptr(),
                                      z.data_ptr(), _code(z), zs, state.data_ptr(), ctx.seq_slot.data_ptr(), ctx.seq_start.data_ptr(), ctx.batch,
-                                     heads, groups, P, N, out.data_ptr(), _code(out), _stream()))
+                                     heads, groups, P, N, out.data_ptr(), _code(out), int(ctx.max_new) if longest is None else int(longest), _stream()))
+    return out
+
+
+def state_space_step(rows: torch.Tensor, dt: torch.Tensor, z: torch.Tensor, rate: torch.Tensor, dt_bias: torch.Tensor, D: torch.Tensor,
+                     taps: torch.Tensor, conv_bias: torch.Tensor, ring: torch.Tensor, state: torch.Tensor, ctx, groups: int,
+                     out: torch.Tensor) -> torch.Tensor:
+    """``conv_silu`` (its state a ring) and ``state_space`` in one kernel, for a step of one token a sequence: ``rows`` as the
+    projection leaves them, ``taps`` float32 [taps, channels], ``conv_bias`` float32."""
+    tokens = rows.shape[0]
+    for t, what in ((state, "state"), (out, "out"), (rate, "rate"), (dt_bias, "dt_bias"), (D, "D"), (taps, "taps"), (conv_bias, "conv_bias"), (ring, "ring")):
+        _dev(t, what)
+    _, heads, P, N = state.shape
+    channels = heads * P + 2 * groups * N
+    if state.dtype != torch.float32 or tuple(out.shape) != (tokens, heads * P) or not ctx.decode or tokens != ctx.batch:
+        raise KernelError(f"state_space_step: one token a sequence, a float32 state and out [tokens, {heads * P}]")
+    if any(t.dtype != torch.float32 or t.numel() != heads for t in (rate, dt_bias, D)):
+        raise KernelError(f"state_space_step: rate, dt_bias and D are float32 with one entry for each of {heads} heads")
+    if (taps.dtype != torch.float32 or taps.dim() != 2 or taps.shape[1] != channels or conv_bias.dtype != torch.float32 or conv_bias.numel() != channels
+            or ring.dtype != torch.float32 or tuple(ring.shape[1:]) != tuple(taps.shape)):
+        raise KernelError(f"state_space_step: float32 taps [taps, {channels}], a bias and a ring of that shape a slot, got {tuple(taps.shape)}, {tuple(ring.shape)}")
+    xs, ds, zs = (_columns(rows, tokens, channels, "state_space_step: rows"), _columns(dt, tokens, heads, "state_space_step: dt"),
+                  _columns(z, tokens, heads * P, "state_space_step: z"))
+    _step_arrays(ctx, "state_space_step")
+    lib = state_space_module()
+    _check(lib, lib.nnis_state_space_step(rows.data_ptr(), _code(rows), xs, dt.data_ptr(), _code(dt), ds, rate.data_ptr(), dt_bias.data_ptr(),
+                                          D.data_ptr(), z.data_ptr(), _code(z), zs, taps.data_ptr(), conv_bias.data_ptr(), ring.data_ptr(),
+                                          state.data_ptr(), ctx.seq_slot.data_ptr(), ctx.seq_start.data_ptr(), ctx.tok_pos.data_ptr(), ctx.batch,
+                                          heads, groups, P, N, taps.shape[0], out.data_ptr(), _code(out), _stream()))
     return out
 
 

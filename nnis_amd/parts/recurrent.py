@@ -397,6 +397,7 @@ class StateSpace(Mixer):
         self.w_in = Projection(weights[n["w_in"]], rt)
         self.conv = weights[n["conv"]].contiguous()
         self.conv_bias = weights[n["conv_bias"]].contiguous()
+        self.taps_wide, self.bias_wide = self.conv.float().t().contiguous(), self.conv_bias.float()  # as the step's kernel reads them
         self.dt_bias = weights[n["dt_bias"]].float().contiguous()
         self.rate = torch.exp(weights[n["a_log"]].float()).contiguous()  # 32-bit, made once
         self.D = weights[n["d"]].float().contiguous()
@@ -420,8 +421,13 @@ class StateSpace(Mixer):
         rows = self.w_in.of(x, rt)
         tokens, inner = rows.shape[0], self.inner
         z, xbc, dt = rows[:, :inner], rows[:, inner:inner + self.channels], rows[:, inner + self.channels:]
-        xbc = rt.ops.conv_silu(xbc, self.channels, self.conv, self.conv_bias, conv_state.state, ctx, rt.empty(tokens, self.channels), ring=True)
-        y = rt.ops.state_space(xbc, dt, z, self.rate, self.dt_bias, self.D, state.state, ctx, self.groups, rt.empty(tokens, inner, dtype=torch.float32))
+        gated = rt.empty(tokens, inner)
+        if ctx.decode and tokens == ctx.batch and self.states % 4 == 0:
+            y = rt.ops.state_space_step(xbc, dt, z, self.rate, self.dt_bias, self.D, self.taps_wide, self.bias_wide, conv_state.state, state.state,
+                                        ctx, self.groups, gated)
+        else:
+            xbc = rt.ops.conv_silu(xbc, self.channels, self.conv, self.conv_bias, conv_state.state, ctx, rt.empty(tokens, self.channels), ring=True)
+            y = rt.ops.state_space(xbc, dt, z, self.rate, self.dt_bias, self.D, state.state, ctx, self.groups, gated)
         y = rt.ops.parts_norm(y, self.norm, self.norm_parts, self.eps, rt.empty(tokens, inner))
         if into is not None and into.can_take(y, self.w_out.weight):
             return into.take(y, self.w_out.weight)
