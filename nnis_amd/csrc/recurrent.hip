@@ -2,8 +2,7 @@
 // selective scan (a diagonal recurrence per channel with input-dependent steps), gated linear attention (a
 // matrix state per head with a decay per key channel; with one fixed decay a head and turned queries and keys it
 // is retention), the per-head norm and gate behind it, the minGRU, and the gated delta rule (a matrix state per
-// head whose every token first takes back what the state already holds under its key), and the real-gated linear
-// recurrent unit.
+// head whose every token first takes back what the state already holds under its key).
 //
 // A step's rows are packed: sequence b of the step owns rows seq_start[b] .. seq_start[b + 1] - 1, which
 // continue the sequence in slot seq_slot[b] (negative: padding, nothing is read or written for it).  State
@@ -1201,122 +1200,5 @@ extern "C" int nnis_gated_delta(const void* rows, int dtype, int stride, const f
     default: hipLaunchKernelGGL(gated_delta_kernel<32>, grid, dim3(256), lds, s, a); break;
   }
   NNIS_LAUNCH_CHECK("gated_delta");
-  return 0;
-}
-
-// -----------------------------------------------------------------------------
-// The real-gated linear recurrent unit's recurrence.  Per channel c of row t, with the gates' logits zr and zi:
-//     log a = -8 sigmoid(zr + br) rate,   rate = softplus(lam) ready-made
-//     S <- a S + sqrt(1 - a^2) sigmoid(zi + bi) u,   out = S * gelu_tanh(y + by)
-// over each sequence's rows, from and into state [slots, width] (32-bit).  logits [tokens, blocks, 2, width / blocks]: a
-// block's zr, then its zi.  A thread a channel; a long run is cut into pieces as the minGRU's.
-// -----------------------------------------------------------------------------
-namespace {
-
-struct UnitArgs {
-  const float* logits;
-  const float* r_bias;
-  const float* i_bias;
-  const float* rate;
-  const void* u;  // [tokens, u_stride]
-  int u_dtype, u_stride;
-  const void* y;  // [tokens, y_stride]
-  int y_dtype, y_stride;
-  const float* y_bias;
-  float* state;
-  const int* seq_slot;
-  const int* seq_start;
-  int batch, width, block;  // block: channels of one of the gates' maps
-  void* out;
-  int out_dtype;
-  int piece, pieces;
-  float* decay;  // [batch, pieces, width]: a piece's sum of log a
-  float* ends;   // [batch, pieces, width]: a piece's end state from zero
-};
-
-__device__ __forceinline__ float gelu_tanh_f(float z) {
-  const float t = 0.7978845608028654f * fmaf(0.044715f * z * z, z, z);
-  return z * sigmoid_f(2.0f * t);  // (1 + tanh t) / 2 = sigmoid(2 t)
-}
-
-template <int PASS>
-__global__ __launch_bounds__(256) void rg_lru_kernel(UnitArgs a) {
-  const int c = blockIdx.x * blockDim.x + threadIdx.x;
-  const int b = blockIdx.y / a.pieces, piece = blockIdx.y % a.pieces;
-  const int slot = a.seq_slot[b];
-  if (slot < 0 || c >= a.width) return;
-  const int start = a.seq_start[b], stop = a.seq_start[b + 1];
-  int first = start, last = stop;
-  if (a.pieces > 1) {
-    first = start + piece * a.piece;
-    last = min(stop, first + a.piece);
-    if (first >= stop) return;
-    if (PASS == 1 && last == stop && piece > 0) return;
-  }
-  const float br = a.r_bias[c], bi = a.i_bias[c], by = a.y_bias ? a.y_bias[c] : 0.0f, rate = -8.0f * a.rate[c];
-  const size_t gate_at = (size_t)(c / a.block) * 2 * a.block + c % a.block;
-  float s = 0.0f, logs = 0.0f;
-  const size_t mine = ((size_t)b * a.pieces + piece) * a.width + c;
-  if (a.pieces == 1) {
-    s = a.state[(size_t)slot * a.width + c];
-  } else if (PASS == 1) {
-    if (piece == 0) a.decay[mine] = s = a.state[(size_t)slot * a.width + c];  // (a copy of the state: see the minGRU)
-  } else if (piece == 0) {
-    s = a.decay[mine];
-  } else {
-    s = a.ends[(size_t)b * a.pieces * a.width + c];
-#pragma unroll 8
-    for (int k = 1; k < piece; ++k) {
-      const size_t at = ((size_t)b * a.pieces + k) * a.width + c;
-      s = fmaf(expf(a.decay[at]), s, a.ends[at]);
-    }
-  }
-#pragma unroll 4
-  for (int t = first; t < last; ++t) {
-    const float zr = a.logits[(size_t)t * 2 * a.width + gate_at] + br;
-    const float zi = a.logits[(size_t)t * 2 * a.width + gate_at + a.block] + bi;
-    const float u = load_as_f32(a.u, a.u_dtype, (size_t)t * a.u_stride + c);
-    const float log_a = rate / (1.0f + expf(-zr));
-    const float keep = expf(log_a);
-    s = fmaf(keep, s, sqrtf(-expm1f(2.0f * log_a)) * (u / (1.0f + expf(-zi))));
-    if (PASS == 1) {
-      logs += log_a;
-    } else {
-      const float y = load_as_f32(a.y, a.y_dtype, (size_t)t * a.y_stride + c) + by;
-      store_from_f32(a.out, a.out_dtype, (size_t)t * a.width + c, s * gelu_tanh_f(y));
-    }
-  }
-  if (PASS == 1) {
-    if (piece > 0) a.decay[mine] = logs;
-    a.ends[mine] = s;
-  } else if (last == stop) {
-    a.state[(size_t)slot * a.width + c] = s;
-  }
-}
-
-}  // namespace
-
-extern "C" int nnis_rg_lru(const float* logits, const float* r_bias, const float* i_bias, const float* rate, const void* u, int u_dtype,
-                           int u_stride, const void* y, int y_dtype, int y_stride, const float* y_bias, float* state, const int* seq_slot,
-                           const int* seq_start, int batch, int width, int block, void* out, int out_dtype, int piece, int pieces,
-                           float* decay, float* ends, void* stream) {
-  NNIS_REQUIRE(logits && r_bias && i_bias && rate && u && y && state && seq_slot && seq_start && out, "rg_lru: missing operand");
-  NNIS_REQUIRE(nnis_dtype_ok(u_dtype) && nnis_dtype_ok(y_dtype) && nnis_dtype_ok(out_dtype), "rg_lru: unknown dtype");
-  NNIS_REQUIRE(width > 0 && block > 0 && width % block == 0 && u_stride >= width && y_stride >= width, "rg_lru: bad sizes (%d channels in blocks of %d)", width, block);
-  NNIS_REQUIRE(pieces >= 1 && (pieces == 1 || (piece > 0 && decay && ends)) && (long long)batch * pieces <= 65535, "rg_lru: bad pieces");
-  if (batch <= 0) return 0;
-  UnitArgs a;
-  a.logits = logits; a.r_bias = r_bias; a.i_bias = i_bias; a.rate = rate; a.u = u; a.u_dtype = u_dtype; a.u_stride = u_stride;
-  a.y = y; a.y_dtype = y_dtype; a.y_stride = y_stride; a.y_bias = y_bias; a.state = state; a.seq_slot = seq_slot; a.seq_start = seq_start;
-  a.batch = batch; a.width = width; a.block = block; a.out = out; a.out_dtype = out_dtype; a.piece = piece; a.pieces = pieces;
-  a.decay = decay; a.ends = ends;
-  const int threads = width >= 256 ? 256 : 64;
-  const dim3 grid((width + threads - 1) / threads, batch * pieces);
-  if (pieces > 1) {
-    hipLaunchKernelGGL(rg_lru_kernel<1>, grid, dim3(threads), 0, (hipStream_t)stream, a);
-    NNIS_LAUNCH_CHECK("rg_lru (first pass)");
-  }
-  hipLaunchKernelGGL(rg_lru_kernel<2>, grid, dim3(threads), 0, (hipStream_t)stream, a);
-  NNIS_LAUNCH_CHECK("rg_lru");
   return 0;
 }

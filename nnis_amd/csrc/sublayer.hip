@@ -1495,29 +1495,3 @@ extern "C" int nnis_pool_blocks(const void* k_pages, const void* v_pages, int ca
   NNIS_LAUNCH_CHECK("pool_blocks");
   return 0;
 }
-
-// out[t, c] = gelu_tanh(z[t, c]) * table[ids[t], first + c]: a layer's gate on the tokens' own input (0 for an id outside the table)
-__global__ void token_gate_kernel(const void* __restrict__ z, int z_dtype, const int* __restrict__ ids, const void* __restrict__ table, int table_dtype,
-                                  int vocab, int columns, int first, void* __restrict__ out, int out_dtype, int dim, size_t total) {
-  for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += (size_t)gridDim.x * blockDim.x) {
-    const size_t t = i / dim, c = i % dim;
-    const float v = load_as_f32(z, z_dtype, i);
-    const float gate = v * sigmoid_f(1.5957691216057308f * fmaf(0.044715f * v * v, v, v));  // (1 + tanh u) / 2 = sigmoid(2 u)
-    const int id = ids[t];
-    const bool inside = id >= 0 && id < vocab;  // (padding rows carry -1: nothing is read outside the table)
-    store_from_f32(out, out_dtype, i, inside ? gate * load_as_f32(table, table_dtype, (size_t)id * columns + first + c) : 0.0f);
-  }
-}
-
-extern "C" int nnis_token_gate(const void* z, int z_dtype, const int* ids, const void* table, int table_dtype, int vocab, int columns, int first,
-                               void* out, int out_dtype, int rows, int dim, void* stream) {
-  NNIS_REQUIRE(z && ids && table && out && dim > 0 && first >= 0 && first + dim <= columns && vocab > 0, "token_gate: bad arguments");
-  NNIS_REQUIRE(nnis_dtype_ok(z_dtype) && nnis_dtype_ok(table_dtype) && nnis_dtype_ok(out_dtype), "token_gate: unknown dtype");
-  if (rows <= 0) return 0;
-  const size_t total = (size_t)rows * dim;
-  const size_t blocks = (total + 255) / 256;
-  hipLaunchKernelGGL(token_gate_kernel, dim3((unsigned)(blocks > 65536 ? 65536 : blocks)), dim3(256), 0, (hipStream_t)stream, z, z_dtype, ids, table,
-                     table_dtype, vocab, columns, first, out, out_dtype, dim, total);
-  NNIS_LAUNCH_CHECK("token_gate");
-  return 0;
-}

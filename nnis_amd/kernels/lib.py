@@ -159,14 +159,18 @@ def _attention_recipe(rest: str) -> ModuleRecipe:
 register_module("core", ["elementwise.hip", "residual.hip", "gemm.hip", "gemm_mfma.hip", "gemm_fused.hip", "sampling.hip"],
                 headers=["common.h", "epilogue.h", "product.h", "nnis_noalloc.h"], source_flags={"gemm_mfma.hip": _VECTOR_SUMS})
 register_module_family("attn_hd", _attention_recipe)
-# the mixers that carry a state of fixed size (convolution, selective scan, gated linear attention and retention, minGRU, gated delta rule, real-gated linear recurrent unit)
+# the mixers that carry a state of fixed size (convolution, selective scan, gated linear attention and retention, minGRU, gated delta rule)
 register_module("recurrent", ["recurrent.hip"], headers=["common.h"])
+# the real-gated linear recurrent unit
+register_module("gated_unit", ["gated_unit.hip"], headers=["common.h"], source_flags={"gated_unit.hip": _VECTOR_SUMS})
 # Mamba-2's state spaces
 register_module("state_space", ["state_space.hip"], headers=["common.h"], source_flags={"state_space.hip": _VECTOR_SUMS})
 # attention over a cached latent: what lies between its projections (norms of the latents, rotation, cache write, gates)
 register_module("latent", ["latent.hip"], headers=["common.h"])
 # what lies between the projections of sublayers that norm their outputs, gate or pool their heads, or route their tokens
 register_module("sublayer", ["sublayer.hip"], headers=["common.h"])
+# a token's own input to a layer
+register_module("token_side", ["token_side.hip"], headers=["common.h"], source_flags={"token_side.hip": _VECTOR_SUMS})
 # the products of a routed feed-forward over the experts that the router chose
 register_module("experts", ["experts.hip"], headers=["common.h", "product.h"], source_flags={"experts.hip": _VECTOR_SUMS})
 # plain host references of the kernels' operations, for the tests (no device code: the host compiler builds them)
@@ -342,7 +346,7 @@ def load_module(module: str, build_if_missing: bool = True) -> ctypes.CDLL:
 
 
 def all_prebuilt_modules() -> List[str]:
-    return ["core", "reference", "recurrent", "state_space", "latent", "sublayer", "experts"] + [f"attn_hd{d}" for d in PREBUILT_HEAD_DIMS] + list(PREBUILT_WIDE_VALUES)
+    return ["core", "reference", "recurrent", "state_space", "gated_unit", "token_side", "latent", "sublayer", "experts"] + [f"attn_hd{d}" for d in PREBUILT_HEAD_DIMS] + list(PREBUILT_WIDE_VALUES)
 
 
 def build_all(force: bool = True, jobs: int = 4) -> List[str]:

@@ -116,9 +116,15 @@ _RECURRENT_SIGNATURES = {
                          _VOID, _VOID],
     "nnis_gla_decays": [_VOID, _VOID, _INT, _INT, _FLT, _VOID],
     "nnis_head_norm_gate": [_VOID, _VOID, _INT, _INT, _VOID, _INT, _VOID, _INT, _INT, _INT, _INT, _FLT, _VOID],
+    "nnis_min_gru": [_VOID, _INT, _INT, _VOID, _VOID, _INT, _VOID, _VOID, _VOID, _INT, _INT, _VOID, _INT, _INT, _INT, _VOID, _VOID, _VOID],
+}
+
+_GATED_UNIT_SIGNATURES = {
     "nnis_rg_lru": [_VOID, _VOID, _VOID, _VOID, _VOID, _INT, _INT, _VOID, _INT, _INT, _VOID, _VOID, _VOID, _VOID, _INT, _INT, _INT, _VOID, _INT, _INT,
                     _INT, _VOID, _VOID, _VOID],
-    "nnis_min_gru": [_VOID, _INT, _INT, _VOID, _VOID, _INT, _VOID, _VOID, _VOID, _INT, _INT, _VOID, _INT, _INT, _INT, _VOID, _VOID, _VOID],
+    "nnis_rg_lru_chunks": [_VOID, _VOID, _VOID, _VOID, _VOID, _INT, _VOID, _INT, _VOID, _VOID, _VOID, _VOID, _INT, _INT, _INT, _VOID, _VOID],
+    "nnis_rg_lru_step": [_VOID, _VOID, _VOID, _VOID, _VOID, _INT, _VOID, _INT, _VOID, _VOID, _VOID, _VOID, _VOID, _VOID, _VOID, _VOID, _VOID, _INT, _INT,
+                         _INT, _INT, _VOID, _VOID],
 }
 
 _STATE_SPACE_SIGNATURES = {
@@ -129,8 +135,12 @@ _STATE_SPACE_SIGNATURES = {
     "nnis_parts_norm": [_VOID, _INT, _VOID, _VOID, _INT, _INT, _INT, _INT, _FLT, _VOID],
 }
 
-_SUBLAYER_SIGNATURES = {
+_TOKEN_SIDE_SIGNATURES = {
     "nnis_token_gate": [_VOID, _INT, _VOID, _VOID, _INT, _INT, _INT, _INT, _VOID, _INT, _INT, _INT, _VOID],
+    "nnis_token_side": [_VOID, _VOID, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _VOID, _VOID, _VOID, _VOID, _FLT, _INT, _INT, _VOID],
+}
+
+_SUBLAYER_SIGNATURES = {
     "nnis_cast_rows": [_VOID, _INT, _VOID, _INT, _VOID, _INT, _INT, _VOID],
     "nnis_rms_post_step": [_VOID, _VOID, _INT, _VOID, _INT, _FLT, _FLT, _VOID, _INT, _INT, _INT, _VOID, _VOID, _INT, _VOID],
     "nnis_rms_between": [_VOID, _VOID, _INT, _VOID, _VOID, _INT, _FLT, _VOID, _INT, _INT, _INT, _VOID, _VOID, _INT, _VOID],
@@ -235,6 +245,28 @@ def state_space_module():
     if _state_space is None:
         _state_space = _bind("state_space", _STATE_SPACE_SIGNATURES)
     return _state_space
+
+
+_gated_unit = None
+
+
+def gated_unit():
+    """The module of the real-gated linear recurrent unit."""
+    global _gated_unit
+    if _gated_unit is None:
+        _gated_unit = _bind("gated_unit", _GATED_UNIT_SIGNATURES)
+    return _gated_unit
+
+
+_token_side = None
+
+
+def token_side_module():
+    """The module of a token's own input to a layer."""
+    global _token_side
+    if _token_side is None:
+        _token_side = _bind("token_side", _TOKEN_SIDE_SIGNATURES)
+    return _token_side
 
 
 _latent = None
@@ -1856,10 +1888,71 @@ def rg_lru(logits: torch.Tensor, blocks: int, r_bias: torch.Tensor, i_bias: torc
     if pieces > 1:
         scratch = torch.empty(2, ctx.batch * pieces * width, dtype=torch.float32, device=u.device)
         decay, ends = scratch[0], scratch[1]
-    lib = recurrent()
+    lib = gated_unit()
     _check(lib, lib.nnis_rg_lru(logits.data_ptr(), r_bias.data_ptr(), i_bias.data_ptr(), rate.data_ptr(), u.data_ptr(), _code(u), us, y.data_ptr(),
                                 _code(y), ys, _ptr(y_bias), state.data_ptr(), ctx.seq_slot.data_ptr(), ctx.seq_start.data_ptr(), ctx.batch, width,
                                 width // blocks, out.data_ptr(), _code(out), piece, pieces, _ptr(decay), _ptr(ends), _stream()))
+    return out
+
+
+RG_LRU_MOST_BLOCK = 512  # channels of a part that the matrix-core kernels take (a multiple of 8)
+
+
+def rg_lru_on_matrix_cores(dtype, channels: int, block: int) -> bool:
+    """Whether ``rg_lru_chunks`` and ``rg_lru_step`` take these rows."""
+    return dtype == torch.bfloat16 and block % 8 == 0 and block <= RG_LRU_MOST_BLOCK
+
+
+def _check_unit(what, maps, r_bias, i_bias, rate, y_bias, state, out, ctx):
+    tokens, width = out.shape
+    vectors = (r_bias, i_bias, rate, y_bias)
+    for t in (maps, state, out, *vectors):
+        _dev(t, what)
+    if maps.dtype != torch.bfloat16 or maps.dim() != 3 or maps.shape[1] != 2 * maps.shape[2] or maps.shape[0] * maps.shape[2] != width:
+        raise KernelError(f"{what}: bfloat16 maps [parts, 2 * block, block] of {width} channels, got {tuple(maps.shape)} {maps.dtype}")
+    if state.dtype != torch.float32 or tuple(state.shape[1:]) != (width,) or out.dtype != torch.bfloat16:
+        raise KernelError(f"{what}: a float32 state [slots, {width}] and bfloat16 rows out, got {tuple(state.shape)} {state.dtype}, {out.dtype}")
+    if any(t.dtype != torch.float32 or t.numel() != width for t in vectors):
+        raise KernelError(f"{what}: biases and rates are float32 with one entry for each of {width} channels")
+    _step_arrays(ctx, what)
+
+
+def rg_lru_chunks(maps: torch.Tensor, r_bias: torch.Tensor, i_bias: torch.Tensor, rate: torch.Tensor, u: torch.Tensor, y: torch.Tensor,
+                  y_bias: torch.Tensor, state: torch.Tensor, ctx, out: torch.Tensor) -> torch.Tensor:
+    """``rg_lru`` with the gates' maps in it, 128 tokens at a time on the matrix cores: ``maps`` bfloat16 [parts, 2 * block,
+    block] (a part's rows of r, then of i), ``u`` (behind the convolution) and ``y`` bfloat16 rows."""
+    tokens, width = out.shape
+    _check_unit("rg_lru_chunks", maps, r_bias, i_bias, rate, y_bias, state, out, ctx)
+    us, ys = _columns(u, tokens, width, "rg_lru_chunks: u"), _columns(y, tokens, width, "rg_lru_chunks: y")
+    if u.dtype != torch.bfloat16 or y.dtype != torch.bfloat16:
+        raise KernelError("rg_lru_chunks: u and y are bfloat16 rows")
+    lib = gated_unit()
+    _check(lib, lib.nnis_rg_lru_chunks(maps.data_ptr(), r_bias.data_ptr(), i_bias.data_ptr(), rate.data_ptr(), u.data_ptr(), us, y.data_ptr(), ys,
+                                       y_bias.data_ptr(), state.data_ptr(), ctx.seq_slot.data_ptr(), ctx.seq_start.data_ptr(), ctx.batch, width,
+                                       maps.shape[2], out.data_ptr(), _stream()))
+    return out
+
+
+def rg_lru_step(maps: torch.Tensor, r_bias: torch.Tensor, i_bias: torch.Tensor, rate: torch.Tensor, x: torch.Tensor, y: torch.Tensor,
+                y_bias: torch.Tensor, x_bias: torch.Tensor, taps: torch.Tensor, conv_bias: torch.Tensor, ring: torch.Tensor, state: torch.Tensor,
+                ctx, out: torch.Tensor) -> torch.Tensor:
+    """``conv_silu`` (no activation, its state a ring), the gates' maps and ``rg_lru`` in one kernel, for a step of one token
+    a sequence: ``x`` and ``y`` as the projection leaves them (bfloat16), ``taps`` float32 [taps, width]."""
+    tokens, width = out.shape
+    _check_unit("rg_lru_step", maps, r_bias, i_bias, rate, y_bias, state, out, ctx)
+    for t in (x_bias, taps, conv_bias, ring):
+        _dev(t, "rg_lru_step")
+    xs, ys = _columns(x, tokens, width, "rg_lru_step: x"), _columns(y, tokens, width, "rg_lru_step: y")
+    if x.dtype != torch.bfloat16 or y.dtype != torch.bfloat16 or not ctx.decode or tokens != ctx.batch:
+        raise KernelError("rg_lru_step: x and y are bfloat16 rows, one token a sequence")
+    if (any(t.dtype != torch.float32 for t in (x_bias, taps, conv_bias, ring)) or taps.dim() != 2 or taps.shape[1] != width or x_bias.numel() != width
+            or conv_bias.numel() != width or tuple(ring.shape[1:]) != tuple(taps.shape)):
+        raise KernelError(f"rg_lru_step: float32 taps [taps, {width}], biases and a ring of the taps' shape a slot, got {tuple(taps.shape)}, {tuple(ring.shape)}")
+    lib = gated_unit()
+    _check(lib, lib.nnis_rg_lru_step(maps.data_ptr(), r_bias.data_ptr(), i_bias.data_ptr(), rate.data_ptr(), x.data_ptr(), xs, y.data_ptr(), ys,
+                                     y_bias.data_ptr(), x_bias.data_ptr(), taps.data_ptr(), conv_bias.data_ptr(), ring.data_ptr(), state.data_ptr(),
+                                     ctx.seq_slot.data_ptr(), ctx.seq_start.data_ptr(), ctx.tok_pos.data_ptr(), ctx.batch, width, maps.shape[2],
+                                     taps.shape[0], out.data_ptr(), _stream()))
     return out
 
 
@@ -2507,10 +2600,48 @@ def token_gate(z: torch.Tensor, ids: torch.Tensor, table: torch.Tensor, first: i
     rows, dim = z.shape
     if out.shape != z.shape or ids.dtype != torch.int32 or ids.numel() < rows or not 0 <= first <= table.shape[1] - dim:
         raise KernelError(f"token_gate: z {tuple(z.shape)}, out {tuple(out.shape)}, columns {first}.. of a table {tuple(table.shape)}")
-    lib = sublayer()
+    lib = token_side_module()
     _check(lib, lib.nnis_token_gate(z.data_ptr(), _code(z), ids.data_ptr(), table.data_ptr(), _code(table), table.shape[0], table.shape[1], int(first),
                                     out.data_ptr(), _code(out), rows, dim, _stream()))
     return out
+
+
+TOKEN_SIDE_MOST_CHANNELS, TOKEN_SIDE_MOST_INPUT = 4096, 256
+
+
+def token_side_takes(rows: torch.Tensor, gate, proj, table: torch.Tensor) -> bool:
+    """Whether ``token_side`` takes these rows and weights."""
+    return (isinstance(gate, PackedWeight) and isinstance(proj, PackedWeight) and rows.dtype == torch.bfloat16 and table.dtype == torch.bfloat16
+            and gate.shape[1] % 16 == 0 and gate.shape[1] <= TOKEN_SIDE_MOST_CHANNELS and gate.shape[0] % 8 == 0
+            and gate.shape[0] <= TOKEN_SIDE_MOST_INPUT and rows.data_ptr() % 16 == 0)
+
+
+def token_side(rows: torch.Tensor, gate, proj, ids: torch.Tensor, table: torch.Tensor, first: int, x: torch.Tensor, w_out: torch.Tensor,
+               eps: float, w_in: Optional[torch.Tensor] = None, h: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+    """A token's own input in one kernel: y = proj @ (gelu_tanh(gate @ rows) * table[ids, first:]), x += y / sqrt(mean(y^2) +
+    eps) * w_out in place in the 32-bit stream, and h = x / sqrt(mean(x^2) + eps) * w_in (``h`` and ``w_in`` together, or
+    neither).  ``gate`` [dim, width] and ``proj`` [width, dim] packed, the norms' weights float32, ``rows`` the stream's
+    rows in bfloat16."""
+    for t, what in ((rows, "rows"), (ids, "ids"), (table, "table"), (x, "x"), (w_out, "norm weight")):
+        _dev(t, what)
+    _packed(gate, "token_side"), _packed(proj, "token_side")
+    m, width = rows.shape
+    dim = gate.shape[0]
+    if (not token_side_takes(rows, gate, proj, table) or tuple(gate.shape) != (dim, width) or tuple(proj.shape) != (width, dim)
+            or ids.dtype != torch.int32 or ids.numel() < m or x.dtype != torch.float32 or x.shape != rows.shape or w_out.dtype != torch.float32
+            or w_out.numel() != width or not 0 <= first <= table.shape[1] - dim):
+        raise KernelError(f"token_side: rows {tuple(rows.shape)}, weights {tuple(gate.shape)} and {tuple(proj.shape)}, stream {tuple(x.shape)}, "
+                          f"columns {first}.. of a table {tuple(table.shape)}")
+    if (h is None) != (w_in is None):
+        raise KernelError("token_side: the rows out come with the next norm's weight")
+    if h is not None:
+        _dev(h, "h"), _dev(w_in, "next norm weight")
+        if h.dtype != torch.bfloat16 or h.shape != rows.shape or w_in.dtype != torch.float32 or w_in.numel() != width:
+            raise KernelError(f"token_side: bfloat16 rows out {tuple(rows.shape)} and a float32 weight, got {tuple(h.shape)} {h.dtype}")
+    lib = token_side_module()
+    _check(lib, lib.nnis_token_side(rows.data_ptr(), gate.data_ptr(), proj.data_ptr(), ids.data_ptr(), table.data_ptr(), table.shape[0], table.shape[1],
+                                    int(first), dim, x.data_ptr(), w_out.data_ptr(), _ptr(w_in), _ptr(h), float(eps), m, width, _stream()))
+    return h
 
 
 def rows_axpy(y: torch.Tensor, h: torch.Tensor, keep: torch.Tensor) -> torch.Tensor:

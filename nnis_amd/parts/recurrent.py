@@ -473,6 +473,7 @@ class GatedLinearUnit(Mixer):
         self.yx = Projection(torch.cat([weights[n["y"]], weights[n["x"]]], dim=0), rt)
         self.y_bias, self.x_bias = weights[n["y_bias"]].float().contiguous(), weights[n["x_bias"]].float().contiguous()
         self.conv, self.conv_bias = weights[n["conv"]].contiguous(), weights[n["conv_bias"]].contiguous()
+        self.taps_wide, self.bias_wide = self.conv.float().t().contiguous(), self.conv_bias.float()  # as the step's kernel reads them
         self.gates = torch.cat([weights[n["r"]], weights[n["i"]]], dim=1).contiguous()  # [blocks, 2 * block, block]
         self.r_bias, self.i_bias = (weights[n[key]].float().reshape(-1).contiguous() for key in ("r_bias", "i_bias"))
         self.rate = torch.nn.functional.softplus(weights[n["rate"]].double()).float().contiguous()  # made once
@@ -495,10 +496,19 @@ class GatedLinearUnit(Mixer):
         C, ops = self.channels, rt.ops
         rows = self.yx.of(x, rt)
         tokens = rows.shape[0]
+        fast = ops.rg_lru_on_matrix_cores(rows.dtype, C, self.block) and self.gates.dtype == torch.bfloat16
+        if fast and ctx.decode and tokens == ctx.batch:
+            y = ops.rg_lru_step(self.gates, self.r_bias, self.i_bias, self.rate, rows[:, C:], rows[:, :C], self.y_bias, self.x_bias, self.taps_wide,
+                                self.bias_wide, conv_state.state, state.state, ctx, rt.empty(tokens, C))
+            return into.take(y, self.out.weight) if into is not None and into.can_take(y, self.out.weight) else self.out(y, rt)
         u = ops.conv_silu(rows[:, C:], C, self.conv, self.conv_bias, conv_state.state, ctx, rt.empty(tokens, C), x_bias=self.x_bias,
                           activation=None, ring=True)
-        logits = ops.heads_linear(u, self.gates, None, self.blocks, rt.empty(tokens, 2 * C, dtype=torch.float32))
-        y = ops.rg_lru(logits, self.blocks, self.r_bias, self.i_bias, self.rate, u, rows[:, :C], self.y_bias, state.state, ctx, rt.empty(tokens, C))
+        y = rt.empty(tokens, C)
+        if fast:
+            ops.rg_lru_chunks(self.gates, self.r_bias, self.i_bias, self.rate, u, rows[:, :C], self.y_bias, state.state, ctx, y)
+        else:
+            logits = ops.heads_linear(u, self.gates, None, self.blocks, rt.empty(tokens, 2 * C, dtype=torch.float32))
+            ops.rg_lru(logits, self.blocks, self.r_bias, self.i_bias, self.rate, u, rows[:, :C], self.y_bias, state.state, ctx, y)
         if into is not None and into.can_take(y, self.out.weight):
             return into.take(y, self.out.weight)
         return self.out(y, rt)
