@@ -135,6 +135,91 @@ __global__ __launch_bounds__(256) void conv_silu_kernel(ConvArgs a) {
   }
 }
 
+// The same for bfloat16 rows whose channels come in eights: a thread takes eight channels over a strip of rows, 16 bytes an access, the
+// strip's own inputs all asked for at once.
+typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
+typedef __attribute__((ext_vector_type(4))) float f32x4;
+
+template <int TAPS>
+__global__ __launch_bounds__(64) void conv_rows8_kernel(ConvArgs a) {
+  const int c = 8 * (blockIdx.x * blockDim.x + threadIdx.x);
+  if (c >= a.channels) return;
+  const int begin = blockIdx.y * kConvStrip, end = min(a.tokens, begin + kConvStrip);
+  const bf16_t* x = (const bf16_t*)a.x + c;
+  bf16x8 fresh[kConvStrip];
+#pragma unroll
+  for (int i = 0; i < kConvStrip; ++i) fresh[i] = *(const bf16x8*)(x + (size_t)min(begin + i, end - 1) * a.x_stride);
+  float w[TAPS][8], bias[8], x_bias[8];
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) w[j][e] = (float)((const bf16_t*)a.weight)[(size_t)(c + e) * TAPS + j];
+    bias[e] = a.bias ? (float)((const bf16_t*)a.bias)[c + e] : 0.0f;
+    x_bias[e] = a.x_bias ? a.x_bias[c + e] : 0.0f;
+  }
+  float held[TAPS][8];  // held[j]: the input TAPS - 1 - j tokens back
+  int before = -2;
+#pragma unroll
+  for (int i = 0; i < kConvStrip; ++i) {
+    const int token = begin + i;
+    if (token >= end) break;
+    const int slot = a.tok_slot[token];
+    bf16_t* y = (bf16_t*)a.y + (size_t)token * a.channels + c;
+    if (slot < 0) {
+      bf16x8 none;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) none[e] = (__bf16)0.0f;
+      *(bf16x8*)y = none;
+      before = -2;
+      continue;
+    }
+    if (slot == before) {
+#pragma unroll
+      for (int j = 0; j + 1 < TAPS; ++j)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) held[j][e] = held[j + 1][e];
+    } else {
+      const int pos = a.tok_pos[token];
+      bool in_step = true;
+      int behind = 0;
+#pragma unroll
+      for (int back = 1; back < TAPS; ++back) {
+        float(&into)[8] = held[TAPS - 1 - back];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) into[e] = 0.0f;  // zeros before the start
+        if (back > pos) continue;
+        in_step = in_step && token - back >= 0 && a.tok_slot[token - back] == slot;
+        if (in_step) {
+          const bf16x8 v = *(const bf16x8*)(x + (size_t)(token - back) * a.x_stride);
+#pragma unroll
+          for (int e = 0; e < 8; ++e) into[e] = (float)v[e] + x_bias[e];
+        } else {
+          ++behind;
+          const float* row = a.ring ? a.state + ((size_t)slot * TAPS + (pos - back) % TAPS) * a.channels + c
+                                    : a.state + ((size_t)slot * (TAPS - 1) + (TAPS - 1 - behind)) * a.channels + c;
+          const f32x4 lo = *(const f32x4*)row, hi = *(const f32x4*)(row + 4);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            into[e] = lo[e];
+            into[4 + e] = hi[e];
+          }
+        }
+      }
+      before = slot;
+    }
+    bf16x8 out;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      held[TAPS - 1][e] = (float)fresh[i][e] + x_bias[e];
+      float acc = bias[e];
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) acc = fmaf(w[j][e], held[j][e], acc);
+      out[e] = (__bf16)conv_act(a, acc);
+    }
+    *(bf16x8*)y = out;
+  }
+}
+
 // A step of single tokens: output and state in one kernel, a thread a (sequence, channel).  The state's rows
 // before a sequence's start are zeros (a slot starts so, and they are only ever moved down).
 __global__ __launch_bounds__(256) void conv_single_kernel(ConvArgs a) {
@@ -641,7 +726,13 @@ extern "C" int nnis_conv_silu(const void* x, int x_dtype, int x_stride, const vo
     NNIS_LAUNCH_CHECK("conv_single");
     return 0;
   }
-  hipLaunchKernelGGL(conv_silu_kernel, dim3((channels + width - 1) / width, (tokens + kConvStrip - 1) / kConvStrip), dim3(width), 0,
+  const bool eights = x_dtype == NNIS_BF16 && y_dtype == NNIS_BF16 && weight_dtype == NNIS_BF16 && channels % 8 == 0 && x_stride % 8 == 0 &&
+                      (uintptr_t)x % 16 == 0 && (uintptr_t)y % 16 == 0 && (uintptr_t)state % 16 == 0;
+  const dim3 grid8((channels / 8 + 63) / 64, (tokens + kConvStrip - 1) / kConvStrip);
+  if (eights && taps == 4) hipLaunchKernelGGL(conv_rows8_kernel<4>, grid8, dim3(64), 0, (hipStream_t)stream, a);
+  else if (eights && taps == 3) hipLaunchKernelGGL(conv_rows8_kernel<3>, grid8, dim3(64), 0, (hipStream_t)stream, a);
+  else if (eights && taps == 2) hipLaunchKernelGGL(conv_rows8_kernel<2>, grid8, dim3(64), 0, (hipStream_t)stream, a);
+  else hipLaunchKernelGGL(conv_silu_kernel, dim3((channels + width - 1) / width, (tokens + kConvStrip - 1) / kConvStrip), dim3(width), 0,
                      (hipStream_t)stream, a);
   NNIS_LAUNCH_CHECK("conv_silu");
   if (taps > 1 || ring) {

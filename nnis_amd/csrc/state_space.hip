@@ -221,8 +221,11 @@ __global__ __launch_bounds__(256) void state_space_chunks_kernel(SpaceArgs a, in
   };
 
   // what a chunk brings, asked for while the chunk before is worked on
+  // (loads end in the order they were asked for: a number asked for inside a chunk would be waited for behind all of these)
   bf16x8 b_in[kItems][4], c_in[NK], x_in;
+  bf16x4 own_in, z_in;
   float dt_in = 0.0f;
+  const bool z_fours = a.z_stride % 4 == 0;
   auto ask = [&](int t0) {
     auto row = [&](int t) { return (size_t)min(t0 + t, end - 1) * a.xbc_stride; };  // (beyond the end: the last again, its weight is zero)
 #pragma unroll
@@ -237,6 +240,14 @@ __global__ __launch_bounds__(256) void state_space_chunks_kernel(SpaceArgs a, in
       c_in[k] = 32 * k + 8 * g < N ? *(const bf16x8*)(rows + row(16 * wave + r) + c_at + 32 * k + 8 * g) : zero8();
     if (tid < 2 * kSpan) x_in = *(const bf16x8*)(rows + row(tid / 2) + x_at + 8 * (tid % 2));
     dt_in = load_as_f32(a.dt, a.dt_dtype, (size_t)min(t0 + lane, end - 1) * a.dt_stride + head);
+    own_in = *(const bf16x4*)(rows + row(16 * wave + r) + x_at + 4 * g);
+    const bf16_t* zp = (const bf16_t*)a.z + (size_t)min(t0 + 16 * wave + r, end - 1) * a.z_stride + x_at + 4 * g;
+    if (z_fours) {
+      z_in = *(const bf16x4*)zp;
+    } else {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) z_in[e] = zp[e];
+    }
   };
   ask(begin);
   keep_state();
@@ -278,25 +289,12 @@ __global__ __launch_bounds__(256) void state_space_chunks_kernel(SpaceArgs a, in
 #pragma unroll
     for (int k = 0; k < NK; ++k) c[k] = c_in[k];
     const float my_sum = __shfl(sum, 16 * wave + r, kWave);  // of this lane's token
+    const bf16x4 own = own_in, zv = z_in;
     __syncthreads();
     if (t0 + kSpan < end) ask(t0 + kSpan);
     const int t = 16 * wave + r;
     const bool live = t < count;
     const size_t out_row = (size_t)min(t0 + t, end - 1);
-    // what the output needs beside the sums
-    float z[4];
-    bf16x4 x_own = *(const bf16x4*)(rows + out_row * a.xbc_stride + x_at + 4 * g);
-    {
-      const bf16_t* zp = (const bf16_t*)a.z + out_row * a.z_stride + x_at + 4 * g;
-      if (a.z_stride % 4 == 0) {
-        const bf16x4 four = *(const bf16x4*)zp;
-#pragma unroll
-        for (int e = 0; e < 4; ++e) z[e] = (float)four[e];
-      } else {
-#pragma unroll
-        for (int e = 0; e < 4; ++e) z[e] = (float)zp[e];
-      }
-    }
     f32x4 y = {0.0f, 0.0f, 0.0f, 0.0f};
 #pragma unroll
     for (int k = 0; k < NK; ++k) {
@@ -327,7 +325,10 @@ __global__ __launch_bounds__(256) void state_space_chunks_kernel(SpaceArgs a, in
     if (live) {
       float v[4];
 #pragma unroll
-      for (int e = 0; e < 4; ++e) v[e] = fmaf(D, (float)x_own[e], y[e]) * (z[e] * sigmoid_f(z[e]));
+      for (int e = 0; e < 4; ++e) {
+        const float z = (float)zv[e];
+        v[e] = fmaf(D, (float)own[e], y[e]) * (z * sigmoid_f(z));
+      }
       const size_t at = out_row * inner + x_at + 4 * g;
       if (a.out_dtype == NNIS_F32) {
         *(f32x4*)((float*)a.out + at) = (f32x4){v[0], v[1], v[2], v[3]};

@@ -657,7 +657,8 @@ __global__ __launch_bounds__(R == 1 ? 1024 : 64 * R) void route_norm_kernel(Rout
 // The same for few rows, a row a block, rows of a multiple of 4 channels: nothing waits for the norm's sum.  A wave takes two
 // outputs at a time and makes, from one round of loads, the row's sum of squares and both sums x gain w; a logit is such a sum
 // over the root mean square.  The row's share of `h` that a wave writes is its own slice of the channels.
-__global__ __launch_bounds__(512) void route_norm_few_kernel(RouteNormArgs a, const float* __restrict__ w, RouteRule rule, int n, int width,
+template <int MOST>
+__global__ __launch_bounds__(MOST) void route_norm_few_kernel(RouteNormArgs a, const float* __restrict__ w, RouteRule rule, int n, int width,
                                                              int experts, int top, float* __restrict__ gates, float* __restrict__ keep) {
   __shared__ float lg[kWave * kRouteMost];
   const int row = blockIdx.x, wave = threadIdx.x / kWave, lane = threadIdx.x % kWave, waves = blockDim.x / kWave;
@@ -715,7 +716,7 @@ __global__ __launch_bounds__(512) void route_norm_many_kernel(RouteNormArgs a, c
   typedef __attribute__((ext_vector_type(4))) float f32x4_t;
   extern __shared__ __attribute__((aligned(16))) float lds[];  // [8][width + 8] bfloat16
   __shared__ __attribute__((aligned(16))) float partial[8][kWave][8];  // [wave][output][row]
-  __shared__ float lg[8][kWave];
+  __shared__ float lg[8][kWave + 1];
   bf16_t* hs = (bf16_t*)lds;
   const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave, r = lane % 16, g = lane / 16;
   const int row = blockIdx.x * 8 + wave, stride = width + 8;
@@ -753,10 +754,22 @@ __global__ __launch_bounds__(512) void route_norm_many_kernel(RouteNormArgs a, c
       if (live) store4((bf16_t*)a.h + base + c, v[i]);
     }
   }
+  // (the shared expert's logit is one more than the products' steps of 16 outputs: a wave takes its row's from its registers)
+  float shared_logit = 0.0f;
+  if (rule.shared_gate) {
+#pragma unroll
+    for (int i = 0; i < kRouteManyKeep; ++i) {
+      const int c = 4 * (lane + i * kWave);
+      if (c < width) {
+        const float4 m = load4(w + (size_t)n * width + c);
+        shared_logit = fmaf(v[i].x, m.x, fmaf(v[i].y, m.y, fmaf(v[i].z, m.z, fmaf(v[i].w, m.w, shared_logit))));
+      }
+    }
+    shared_logit = wave_sum(shared_logit);
+  }
   __syncthreads();
-  const int dots = n + rule.shared_gate;
-  for (int o0 = 0; o0 < dots; o0 += 16) {
-    const bf16_t* w_row = w + (size_t)(o0 + r < dots ? o0 + r : dots - 1) * width + 8 * g;
+  for (int o0 = 0; o0 < n; o0 += 16) {
+    const bf16_t* w_row = w + (size_t)(o0 + r < n ? o0 + r : n - 1) * width + 8 * g;
     const bf16_t* x_row = hs + (size_t)(r % 8) * stride + 8 * g;
     f32x4_t acc = {0.0f, 0.0f, 0.0f, 0.0f};
 #pragma unroll 4
@@ -771,10 +784,9 @@ __global__ __launch_bounds__(512) void route_norm_many_kernel(RouteNormArgs a, c
   if (!live) return;
   float logit = 0.0f;
 #pragma unroll
-  for (int o = 0; o < 8; ++o) logit += lane < dots ? partial[o][lane][wave] : 0.0f;
-  if (lane < dots) lg[wave][lane] = logit;
-  __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-  __builtin_amdgcn_wave_barrier();  // (lane 0 reads the shared expert's; of the outputs a lane reads its own)
+  for (int o = 0; o < 8; ++o) logit += lane < n ? partial[o][lane][wave] : 0.0f;
+  if (lane < n) lg[wave][lane] = logit;
+  if (rule.shared_gate && lane == 0) lg[wave][n] = shared_logit;  // (a lane reads what it wrote itself)
   route_row_slots<1>(lg[wave], rule, row, n, experts, top, gates, keep, lane);
 }
 
@@ -1325,7 +1337,7 @@ extern "C" int nnis_route_norm(float* x, const void* delta, int delta_dtype, con
   const RouteRule rule = {bias, correction, scoring, group_count, group_keep, weight_scale, group_marks, shared_gate ? 1 : 0, chosen, weights};
   const RouteNormArgs a = {x, delta, delta_dtype, gain, gain_dtype, eps, h, h_dtype};
   const bool fours = width % 4 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)gain % 16 == 0 && (uintptr_t)h % 16 == 0 && (uintptr_t)w % 16 == 0;
-  if (rows > 256 && fours && w_bf16 && h_dtype == NNIS_BF16 && dots <= kWave && width % 32 == 0 && width <= kRouteManyMost &&
+  if (rows > 256 && fours && w_bf16 && h_dtype == NNIS_BF16 && n <= kWave && width % 32 == 0 && width <= kRouteManyMost &&
       (uintptr_t)w_bf16 % 16 == 0 && (uintptr_t)delta % 16 == 0) {
     const size_t bytes = (size_t)8 * (width + 8) * sizeof(bf16_t);
     static const hipError_t allowed = hipFuncSetAttribute((const void*)route_norm_many_kernel, hipFuncAttributeMaxDynamicSharedMemorySize,
@@ -1337,8 +1349,12 @@ extern "C" int nnis_route_norm(float* x, const void* delta, int delta_dtype, con
     return 0;
   }
   if (rows <= 256 && fours && delta == nullptr) {
-    const int waves = dots < 16 ? (dots + 1) / 2 : 8;  // (each has outputs of its own, and with them the row's root mean square)
-    hipLaunchKernelGGL(route_norm_few_kernel, dim3(rows), dim3(kWave * waves), 0, s, a, w, rule, n, width, experts, top, gates, keep);
+    // (each has outputs of its own, and with them the row's root mean square; up to twelve pairs of outputs in one round)
+    const int pairs = (dots + 1) / 2, waves = pairs <= 12 ? pairs : 8;
+    if (waves <= 8)
+      hipLaunchKernelGGL(route_norm_few_kernel<512>, dim3(rows), dim3(kWave * waves), 0, s, a, w, rule, n, width, experts, top, gates, keep);
+    else
+      hipLaunchKernelGGL(route_norm_few_kernel<768>, dim3(rows), dim3(kWave * waves), 0, s, a, w, rule, n, width, experts, top, gates, keep);
     NNIS_LAUNCH_CHECK("route_norm");
     return 0;
   }

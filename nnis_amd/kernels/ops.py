@@ -137,7 +137,7 @@ _STATE_SPACE_SIGNATURES = {
 
 _TOKEN_SIDE_SIGNATURES = {
     "nnis_token_gate": [_VOID, _INT, _VOID, _VOID, _INT, _INT, _INT, _INT, _VOID, _INT, _INT, _INT, _VOID],
-    "nnis_token_side": [_VOID, _VOID, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _VOID, _VOID, _VOID, _VOID, _FLT, _INT, _INT, _VOID],
+    "nnis_token_gate_rows": [_VOID, _VOID, _VOID, _VOID, _INT, _INT, _INT, _INT, _VOID, _INT, _INT, _VOID],
 }
 
 _SUBLAYER_SIGNATURES = {
@@ -2606,42 +2606,19 @@ def token_gate(z: torch.Tensor, ids: torch.Tensor, table: torch.Tensor, first: i
     return out
 
 
-TOKEN_SIDE_MOST_CHANNELS, TOKEN_SIDE_MOST_INPUT = 4096, 256
-
-
-def token_side_takes(rows: torch.Tensor, gate, proj, table: torch.Tensor) -> bool:
-    """Whether ``token_side`` takes these rows and weights."""
-    return (isinstance(gate, PackedWeight) and isinstance(proj, PackedWeight) and rows.dtype == torch.bfloat16 and table.dtype == torch.bfloat16
-            and gate.shape[1] % 16 == 0 and gate.shape[1] <= TOKEN_SIDE_MOST_CHANNELS and gate.shape[0] % 8 == 0
-            and gate.shape[0] <= TOKEN_SIDE_MOST_INPUT and rows.data_ptr() % 16 == 0)
-
-
-def token_side(rows: torch.Tensor, gate, proj, ids: torch.Tensor, table: torch.Tensor, first: int, x: torch.Tensor, w_out: torch.Tensor,
-               eps: float, w_in: Optional[torch.Tensor] = None, h: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
-    """A token's own input in one kernel: y = proj @ (gelu_tanh(gate @ rows) * table[ids, first:]), x += y / sqrt(mean(y^2) +
-    eps) * w_out in place in the 32-bit stream, and h = x / sqrt(mean(x^2) + eps) * w_in (``h`` and ``w_in`` together, or
-    neither).  ``gate`` [dim, width] and ``proj`` [width, dim] packed, the norms' weights float32, ``rows`` the stream's
-    rows in bfloat16."""
-    for t, what in ((rows, "rows"), (ids, "ids"), (table, "table"), (x, "x"), (w_out, "norm weight")):
-        _dev(t, what)
-    _packed(gate, "token_side"), _packed(proj, "token_side")
+def token_gate_rows(rows: torch.Tensor, gate, ids: torch.Tensor, table: torch.Tensor, first: int, out: torch.Tensor) -> torch.Tensor:
+    """out = gelu_tanh(gate @ rows) * table[ids, first:] in one kernel: bfloat16 rows, ``gate`` [dim, width] packed."""
+    _dev(rows, "rows"), _dev(ids, "ids"), _dev(table, "table"), _dev(out, "out")
+    _packed(gate, "token_gate_rows")
     m, width = rows.shape
     dim = gate.shape[0]
-    if (not token_side_takes(rows, gate, proj, table) or tuple(gate.shape) != (dim, width) or tuple(proj.shape) != (width, dim)
-            or ids.dtype != torch.int32 or ids.numel() < m or x.dtype != torch.float32 or x.shape != rows.shape or w_out.dtype != torch.float32
-            or w_out.numel() != width or not 0 <= first <= table.shape[1] - dim):
-        raise KernelError(f"token_side: rows {tuple(rows.shape)}, weights {tuple(gate.shape)} and {tuple(proj.shape)}, stream {tuple(x.shape)}, "
-                          f"columns {first}.. of a table {tuple(table.shape)}")
-    if (h is None) != (w_in is None):
-        raise KernelError("token_side: the rows out come with the next norm's weight")
-    if h is not None:
-        _dev(h, "h"), _dev(w_in, "next norm weight")
-        if h.dtype != torch.bfloat16 or h.shape != rows.shape or w_in.dtype != torch.float32 or w_in.numel() != width:
-            raise KernelError(f"token_side: bfloat16 rows out {tuple(rows.shape)} and a float32 weight, got {tuple(h.shape)} {h.dtype}")
+    if (rows.dtype != torch.bfloat16 or table.dtype != torch.bfloat16 or out.dtype != torch.bfloat16 or tuple(out.shape) != (m, dim) or gate.shape[1] != width
+            or ids.dtype != torch.int32 or ids.numel() < m or not 0 <= first <= table.shape[1] - dim):
+        raise KernelError(f"token_gate_rows: rows {tuple(rows.shape)}, weight {tuple(gate.shape)}, out {tuple(out.shape)}, columns {first}.. of {tuple(table.shape)}")
     lib = token_side_module()
-    _check(lib, lib.nnis_token_side(rows.data_ptr(), gate.data_ptr(), proj.data_ptr(), ids.data_ptr(), table.data_ptr(), table.shape[0], table.shape[1],
-                                    int(first), dim, x.data_ptr(), w_out.data_ptr(), _ptr(w_in), _ptr(h), float(eps), m, width, _stream()))
-    return h
+    _check(lib, lib.nnis_token_gate_rows(rows.data_ptr(), gate.data_ptr(), ids.data_ptr(), table.data_ptr(), table.shape[0], table.shape[1], int(first),
+                                        dim, out.data_ptr(), m, width, _stream()))
+    return out
 
 
 def rows_axpy(y: torch.Tensor, h: torch.Tensor, keep: torch.Tensor) -> torch.Tensor:

@@ -125,15 +125,7 @@ class PreNormBlock(Block):
             out = self._run(self.feed_forward, normed, (ctx, rt), last, rt)
         if self.side is None:
             return out
-        x = out.x
-        next_rms = following if getattr(following, "fusable_rms", False) else None
-        if hasattr(self.side, "into_stream") and getattr(self.side_norm, "fusable_rms", False):
-            h = self.side.into_stream(out.h, x, self.side_norm, next_rms, ctx, rt)
-            if h is not False:
-                if next_rms is not None:
-                    return PendingNorm.from_rows(following, x, h, rt)
-                return (x, None) if following is None else following.defer(x, None, rt)
-        y = self.side.forward(out.h, ctx, rt)
+        x, y = out.x, self.side.forward(out.h, ctx, rt)
         if following is not None and PrePostNormBlock._rms_pair(self.side_norm, following) and y.is_contiguous():
             # the norm on the side's way out, the sum into the stream and the next block's first norm in one kernel
             h = rt.ops.rms_between(x, y, self.side_norm.weight, following.weight, following.eps, h=rt.empty(x.shape[0], self.width))

@@ -326,19 +326,9 @@ class TokenInput(FeedForward):
     def weight_bytes(self):
         return self.gate.weight_bytes() + self.proj.weight_bytes()
 
-    def into_stream(self, rows, x, norm, following, ctx, rt):
-        """The part with its norm on the way out (``norm``), the sum into the stream ``x`` and the norm that comes next
-        (``following`` or None), in one kernel.  Returns that norm's rows (None without it), or False where the kernel
-        does not take these types and sizes."""
-        wide = [n.weight.dtype == torch.float32 for n in (norm, following) if n is not None]
-        if (rt.dtype != torch.bfloat16 or not all(wide) or (following is not None and following.eps != norm.eps)
-                or not rt.ops.token_side_takes(rows, self.gate.weight, self.proj.weight, self.table)):
-            return False
-        h = rt.empty(rows.shape[0], self.width) if following is not None else None
-        return rt.ops.token_side(rows, self.gate.weight, self.proj.weight, ctx.ids, self.table, self.first, x, norm.weight, norm.eps,
-                                 following.weight if following is not None else None, h)
-
     def forward(self, x, ctx, rt):
+        if isinstance(self.gate.weight, rt.ops.PackedWeight) and x.dtype == self.table.dtype == torch.bfloat16:
+            return self.proj(rt.ops.token_gate_rows(x, self.gate.weight, ctx.ids, self.table, self.first, rt.empty(x.shape[0], self.inner)), rt)
         z = self.gate(x, rt, out_dtype=torch.float32)
         return self.proj(rt.ops.token_gate(z, ctx.ids, self.table, self.first, rt.empty(x.shape[0], self.inner)), rt)
 
