@@ -189,9 +189,10 @@ __global__ __launch_bounds__(64 * kWaves) void rg_lru_chunks_kernel(MapArgs m, i
   bf16x4 own_in, y_in;
   auto ask = [&](int t0) {
     const size_t t = min(t0 + 16 * wave + r, end - 1);
-    const bf16_t* row = u_rows + t * a.u_stride + (size_t)part * K + 8 * g;
+    const bf16_t* row = u_rows + t * a.u_stride + (size_t)part * K;
+    // (beyond the part: its last channels again, the maps are zero there; no load stands behind a branch)
 #pragma unroll
-    for (int k = 0; k < KB; ++k) u_in[k] = 32 * k + 8 * g < K ? *(const bf16x8*)(row + 32 * k) : zero8();
+    for (int k = 0; k < KB; ++k) u_in[k] = *(const bf16x8*)(row + min(32 * k + 8 * g, K - 8));
     own_in = *(const bf16x4*)(u_rows + t * a.u_stride + c0);
     y_in = *(const bf16x4*)(y_rows + t * a.y_stride + c0);
   };

@@ -21,6 +21,14 @@ constexpr float kLog2e = 1.4426950408889634f;
 __device__ __forceinline__ float exp2_fast(float x) { return __builtin_amdgcn_exp2f(x); }
 __device__ __forceinline__ float sigmoid_f(float z) { return __builtin_amdgcn_rcpf(1.0f + exp2_fast(-z * kLog2e)); }
 __device__ __forceinline__ float softplus_f(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
+// the same by the hardware's 2^x and log2: e^z itself where it is small (1 + e^z would round it away: three terms of the logarithm's
+// series, a relative error below 2e-6)
+__device__ __forceinline__ float softplus_fast(float z) {
+  const float t = exp2_fast(z * kLog2e);
+  const float small = t * (1.0f - t * (0.5f - t * (1.0f / 3.0f)));
+  const float mid = __builtin_amdgcn_logf(1.0f + t) * 0.6931471805599453f;
+  return z > 20.0f ? z : (t < 0.02f ? small : mid);
+}
 
 struct SpaceArgs {
   const void* xbc;  // [tokens, xbc_stride]
@@ -172,7 +180,17 @@ __device__ __forceinline__ void split_two(const float (&v)[8], bf16x8& hi, bf16x
 
 __device__ __forceinline__ f32x4 mfma(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
 
-template <int NK>
+// x from the lane `OFFSET` places before in its row of 16 lanes, 0 where there is none
+template <int OFFSET>
+__device__ __forceinline__ float from_before(float x) {
+  return __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, x), 0x110 + OFFSET, 0xF, 0xF, false));
+}
+__device__ __forceinline__ float lane_value(float x, int lane) { return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, x), lane)); }
+
+// ZFOURS: z's rows lie on 8-byte boundaries.  Every load of a chunk is asked for unconditionally and kept as it arrives: a load behind a
+// branch, or one that is converted at once, makes the compiler wait for all that were asked for before it.  (States beyond N repeat
+// the last ones; C is zero there, so nothing of them reaches an output, and they are not stored.)
+template <int NK, bool ZFOURS>
 __global__ __launch_bounds__(256) void state_space_chunks_kernel(SpaceArgs a, int slabs, int items) {
   extern __shared__ __attribute__((aligned(16))) char chunk_lds[];
   ChunkLds<NK>& lds = *(ChunkLds<NK>*)chunk_lds;
@@ -202,12 +220,12 @@ __global__ __launch_bounds__(256) void state_space_chunks_kernel(SpaceArgs a, in
 #pragma unroll
   for (int i = 0; i < kTiles; ++i) {
     const int n = 16 * (wave + 4 * i) + 4 * g;
-    S[i] = n < N && wave + 4 * i < 2 * NK ? *(const f32x4*)(state + n) : (f32x4){0.0f, 0.0f, 0.0f, 0.0f};
+    S[i] = *(const f32x4*)(state + min(n, N - 4));
   }
   auto keep_state = [&]() {  // the state as the next chunk's products read it
 #pragma unroll
     for (int i = 0; i < kTiles; ++i) {
-      if (wave + 4 * i >= 2 * NK) continue;
+      if (NK == 1 && wave >= 2) continue;
       bf16x4 hi, lo;
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
@@ -224,8 +242,7 @@ __global__ __launch_bounds__(256) void state_space_chunks_kernel(SpaceArgs a, in
   // (loads end in the order they were asked for: a number asked for inside a chunk would be waited for behind all of these)
   bf16x8 b_in[kItems][4], c_in[NK], x_in;
   bf16x4 own_in, z_in;
-  float dt_in = 0.0f;
-  const bool z_fours = a.z_stride % 4 == 0;
+  bf16_t z_one[4], dt_in;
   auto ask = [&](int t0) {
     auto row = [&](int t) { return (size_t)min(t0 + t, end - 1) * a.xbc_stride; };  // (beyond the end: the last again, its weight is zero)
 #pragma unroll
@@ -233,20 +250,19 @@ __global__ __launch_bounds__(256) void state_space_chunks_kernel(SpaceArgs a, in
       const int it = tid + 256 * i, quad = it % 16, piece = it / 16;
 #pragma unroll
       for (int j = 0; j < 4; ++j)
-        b_in[i][j] = piece < 4 * NK && 8 * piece < N ? *(const bf16x8*)(rows + row(4 * quad + j) + b_at + 8 * piece) : zero8();
+        b_in[i][j] = *(const bf16x8*)(rows + row(4 * quad + j) + b_at + min(8 * piece, N - 8));
     }
 #pragma unroll
-    for (int k = 0; k < NK; ++k)
-      c_in[k] = 32 * k + 8 * g < N ? *(const bf16x8*)(rows + row(16 * wave + r) + c_at + 32 * k + 8 * g) : zero8();
-    if (tid < 2 * kSpan) x_in = *(const bf16x8*)(rows + row(tid / 2) + x_at + 8 * (tid % 2));
-    dt_in = load_as_f32(a.dt, a.dt_dtype, (size_t)min(t0 + lane, end - 1) * a.dt_stride + head);
+    for (int k = 0; k < NK; ++k) c_in[k] = *(const bf16x8*)(rows + row(16 * wave + r) + c_at + min(32 * k + 8 * g, N - 8));
+    x_in = *(const bf16x8*)(rows + row(tid / 2 % kSpan) + x_at + 8 * (tid % 2));
+    dt_in = ((const bf16_t*)a.dt)[(size_t)min(t0 + lane, end - 1) * a.dt_stride + head];
     own_in = *(const bf16x4*)(rows + row(16 * wave + r) + x_at + 4 * g);
     const bf16_t* zp = (const bf16_t*)a.z + (size_t)min(t0 + 16 * wave + r, end - 1) * a.z_stride + x_at + 4 * g;
-    if (z_fours) {
+    if constexpr (ZFOURS) {
       z_in = *(const bf16x4*)zp;
     } else {
 #pragma unroll
-      for (int e = 0; e < 4; ++e) z_in[e] = zp[e];
+      for (int e = 0; e < 4; ++e) z_one[e] = zp[e];
     }
   };
   ask(begin);
@@ -272,14 +288,17 @@ __global__ __launch_bounds__(256) void state_space_chunks_kernel(SpaceArgs a, in
       for (int e = 0; e < 8; ++e) lds.xt[8 * (tid % 2) + e][tid / 2] = x_in[e];
     }
     // lane l: token l's step and the sums of the decays' logarithms (every wave for itself)
-    const float dt = lane < count ? softplus_f(dt_in + dt_bias) : 0.0f;
+    const float dt = lane < count ? softplus_fast((float)dt_in + dt_bias) : 0.0f;
     float sum = -rate * dt;
-#pragma unroll
-    for (int offset = 1; offset < kWave; offset <<= 1) {
-      const float other = __shfl_up(sum, offset, kWave);
-      if (lane >= offset) sum += other;
+    sum += from_before<1>(sum);
+    sum += from_before<2>(sum);
+    sum += from_before<4>(sum);
+    sum += from_before<8>(sum);
+    {  // (rows of 16 lanes are summed up; the rows before a lane's own)
+      const float row0 = lane_value(sum, 15), row1 = row0 + lane_value(sum, 31), row2 = row1 + lane_value(sum, 47);
+      sum += g == 0 ? 0.0f : (g == 1 ? row0 : (g == 2 ? row1 : row2));
     }
-    const float total = __shfl(sum, kWave - 1, kWave);
+    const float total = lane_value(sum, kWave - 1);
     if (wave == 0) {
       lds.sum[lane] = sum;
       lds.dt[lane] = dt;
@@ -287,10 +306,13 @@ __global__ __launch_bounds__(256) void state_space_chunks_kernel(SpaceArgs a, in
     }
     bf16x8 c[NK];
 #pragma unroll
-    for (int k = 0; k < NK; ++k) c[k] = c_in[k];
-    const float my_sum = __shfl(sum, 16 * wave + r, kWave);  // of this lane's token
-    const bf16x4 own = own_in, zv = z_in;
+    for (int k = 0; k < NK; ++k) c[k] = 32 * k + 8 * g < N ? c_in[k] : zero8();
+    const bf16x4 own = own_in;
+    bf16x4 zv;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) zv[e] = ZFOURS ? z_in[e] : z_one[e];
     __syncthreads();
+    const float my_sum = lds.sum[16 * wave + r];  // of this lane's token
     if (t0 + kSpan < end) ask(t0 + kSpan);
     const int t = 16 * wave + r;
     const bool live = t < count;
@@ -355,7 +377,7 @@ __global__ __launch_bounds__(256) void state_space_chunks_kernel(SpaceArgs a, in
       split_two(v, hi, lo);
 #pragma unroll
       for (int i = 0; i < kTiles; ++i) {
-        if (wave + 4 * i >= 2 * NK) continue;
+        if (NK == 1 && wave >= 2) continue;
         const bf16x8 bv = *(const bf16x8*)&lds.bt[16 * (wave + 4 * i) + r][32 * block + 8 * g];
         S[i] = mfma(bv, hi, S[i]);
         S[i] = mfma(bv, lo, S[i]);
@@ -551,25 +573,32 @@ extern "C" int nnis_state_space(const void* xbc, int xbc_dtype, int xbc_stride, 
   a.seq_slot = seq_slot; a.seq_start = seq_start; a.heads = heads; a.groups = groups; a.P = P; a.N = N; a.out = out; a.out_dtype = out_dtype;
   hipStream_t s = (hipStream_t)stream;
   // `longest` tokens or more a sequence, bfloat16 rows on 16-byte boundaries: the matrix cores
-  if (longest >= 16 && xbc_dtype == NNIS_BF16 && z_dtype == NNIS_BF16 && P % kSlab == 0 && N % 8 == 0 && xbc_stride % 8 == 0 &&
-      (uintptr_t)xbc % 16 == 0 && (uintptr_t)out % 16 == 0 && (uintptr_t)state % 16 == 0 && (z_stride % 4 != 0 || (uintptr_t)z % 8 == 0)) {
+  if (longest >= 16 && xbc_dtype == NNIS_BF16 && z_dtype == NNIS_BF16 && dt_dtype == NNIS_BF16 && P % kSlab == 0 && N % 8 == 0 && xbc_stride % 8 == 0 &&
+      (uintptr_t)xbc % 16 == 0 && (uintptr_t)out % 16 == 0 && (uintptr_t)state % 16 == 0) {
+    const bool fours = z_stride % 4 == 0 && (uintptr_t)z % 8 == 0;
     const int slabs = P / kSlab;
     const long long items = (long long)slabs * heads * batch;
     NNIS_REQUIRE(items <= 0x7ffffff0, "state_space: %d sequences exceed the grid limit", batch);
     const dim3 grid((unsigned)((items + 7) / 8 * 8));
     // (beyond 64 KB of LDS a kernel has to be told once; a refusal shows as the launch's failure)
-#define NNIS_CHUNKS(NK_)                                                                                                       \
+#define NNIS_CHUNKS_OF(NK_, FOURS_)                                                                                            \
   do {                                                                                                                         \
-    static const hipError_t allowed = hipFuncSetAttribute((const void*)state_space_chunks_kernel<NK_>,                         \
+    static const hipError_t allowed = hipFuncSetAttribute((const void*)state_space_chunks_kernel<NK_, FOURS_>,                 \
                                                           hipFuncAttributeMaxDynamicSharedMemorySize, (int)sizeof(ChunkLds<NK_>)); \
     (void)allowed;                                                                                                             \
-    hipLaunchKernelGGL(state_space_chunks_kernel<NK_>, grid, dim3(256), sizeof(ChunkLds<NK_>), s, a, slabs, (int)items);        \
+    hipLaunchKernelGGL((state_space_chunks_kernel<NK_, FOURS_>), grid, dim3(256), sizeof(ChunkLds<NK_>), s, a, slabs, (int)items); \
+  } while (0)
+#define NNIS_CHUNKS(NK_)                   \
+  do {                                     \
+    if (fours) NNIS_CHUNKS_OF(NK_, true);  \
+    else NNIS_CHUNKS_OF(NK_, false);       \
   } while (0)
     if (N <= 32) NNIS_CHUNKS(1);
     else if (N <= 64) NNIS_CHUNKS(2);
     else if (N <= 128) NNIS_CHUNKS(4);
     else NNIS_CHUNKS(8);
 #undef NNIS_CHUNKS
+#undef NNIS_CHUNKS_OF
     NNIS_LAUNCH_CHECK("state_space_chunks");
     return 0;
   }

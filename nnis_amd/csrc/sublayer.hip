@@ -389,58 +389,77 @@ __device__ __forceinline__ void route_row_slots(const float* logits, const Route
     choice[i] = e < n ? (rule.scoring == kChosenSoftmax ? choice[i] : s[i]) + (correction ? correction[e] : 0.0f) : -INFINITY;
   }
   if (group_count > 1 && group_keep < group_count) {
-    // lane g holds group g's mark (up to 64 groups); the kept groups are found one at a time
     const int size = n / group_count;
-    float mark = -INFINITY;
-    for (int g = 0; g < group_count; ++g) {
-      float best = -INFINITY;
+    if (SLOTS == 1 && (size & (size - 1)) == 0) {
+      // a group's outputs are neighbouring lanes: every lane gets its own group's two largest, and a group is kept if fewer than
+      // group_keep others have a larger mark (or the same one and a lower number)
+      float first = choice[0], second = -INFINITY;
+      for (int offset = 1; offset < size; offset <<= 1) {
+        const float o1 = __shfl_xor(first, offset, kWave), o2 = __shfl_xor(second, offset, kWave);
+        second = fmaxf(fminf(first, o1), fmaxf(second, o2));
+        first = fmaxf(first, o1);
+      }
+      const float mark = rule.group_marks > 1 && size > 1 ? first + second : first;
+      const int own = lane / size;
+      int ahead = 0;
+      for (int g = 0; g < group_count; ++g) {
+        const float other = __shfl(mark, g * size, kWave);
+        ahead += other > mark || (other == mark && g < own) ? 1 : 0;
+      }
+      if (lane < n && ahead >= group_keep) choice[0] = -INFINITY;
+    } else {
+      // lane g holds group g's mark (up to 64 groups); the kept groups are found one at a time
+      float mark = -INFINITY;
+      for (int g = 0; g < group_count; ++g) {
+        float best = -INFINITY;
+#pragma unroll
+        for (int i = 0; i < SLOTS; ++i) {
+          const int e = i * kWave + lane;
+          if (e < n && e / size == g) best = fmaxf(best, choice[i]);
+        }
+        const float largest = wave_max(best);
+        float marks = largest;
+        if (rule.group_marks > 1 && size > 1) {
+          // the second largest: without one holder of the largest (the first lane that has it)
+          const int holder = __ffsll(__ballot(best == largest)) - 1;
+          float second = best;
+          if (lane == holder) {
+            second = -INFINITY;
+            bool passed = false;
+#pragma unroll
+            for (int i = 0; i < SLOTS; ++i) {
+              const int e = i * kWave + lane;
+              if (e < n && e / size == g) {
+                if (!passed && choice[i] == largest) passed = true;
+                else second = fmaxf(second, choice[i]);
+              }
+            }
+          }
+          marks += wave_max(second);
+        }
+        if (lane == g) mark = marks;
+      }
+      unsigned long long allowed = 0ull;
+      for (int round = 0; round < group_keep; ++round) {
+        float best = lane < group_count && !(allowed >> lane & 1ull) ? mark : -INFINITY;
+        int best_g = lane < group_count && !(allowed >> lane & 1ull) ? lane : 0x7fffffff;
+#pragma unroll
+        for (int offset = kWave / 2; offset > 0; offset >>= 1) {
+          const float other = __shfl_xor(best, offset, kWave);
+          const int other_g = __shfl_xor(best_g, offset, kWave);
+          if (other_g != 0x7fffffff && (best_g == 0x7fffffff || other > best || (other == best && other_g < best_g))) {
+            best = other;
+            best_g = other_g;
+          }
+        }
+        if (best_g == 0x7fffffff) break;
+        allowed |= 1ull << best_g;
+      }
 #pragma unroll
       for (int i = 0; i < SLOTS; ++i) {
         const int e = i * kWave + lane;
-        if (e < n && e / size == g) best = fmaxf(best, choice[i]);
+        if (e < n && !(allowed >> (e / size) & 1ull)) choice[i] = -INFINITY;
       }
-      const float largest = wave_max(best);
-      float marks = largest;
-      if (rule.group_marks > 1 && size > 1) {
-        // the second largest: without one holder of the largest (the first lane that has it)
-        const int holder = __ffsll(__ballot(best == largest)) - 1;
-        float second = best;
-        if (lane == holder) {
-          second = -INFINITY;
-          bool passed = false;
-#pragma unroll
-          for (int i = 0; i < SLOTS; ++i) {
-            const int e = i * kWave + lane;
-            if (e < n && e / size == g) {
-              if (!passed && choice[i] == largest) passed = true;
-              else second = fmaxf(second, choice[i]);
-            }
-          }
-        }
-        marks += wave_max(second);
-      }
-      if (lane == g) mark = marks;
-    }
-    unsigned long long allowed = 0ull;
-    for (int round = 0; round < group_keep; ++round) {
-      float best = lane < group_count && !(allowed >> lane & 1ull) ? mark : -INFINITY;
-      int best_g = lane < group_count && !(allowed >> lane & 1ull) ? lane : 0x7fffffff;
-#pragma unroll
-      for (int offset = kWave / 2; offset > 0; offset >>= 1) {
-        const float other = __shfl_xor(best, offset, kWave);
-        const int other_g = __shfl_xor(best_g, offset, kWave);
-        if (other_g != 0x7fffffff && (best_g == 0x7fffffff || other > best || (other == best && other_g < best_g))) {
-          best = other;
-          best_g = other_g;
-        }
-      }
-      if (best_g == 0x7fffffff) break;
-      allowed |= 1ull << best_g;
-    }
-#pragma unroll
-    for (int i = 0; i < SLOTS; ++i) {
-      const int e = i * kWave + lane;
-      if (e < n && !(allowed >> (e / size) & 1ull)) choice[i] = -INFINITY;
     }
   }
   float kept = 0.0f;
@@ -657,38 +676,50 @@ __global__ __launch_bounds__(R == 1 ? 1024 : 64 * R) void route_norm_kernel(Rout
 // The same for few rows, a row a block, rows of a multiple of 4 channels: nothing waits for the norm's sum.  A wave takes two
 // outputs at a time and makes, from one round of loads, the row's sum of squares and both sums x gain w; a logit is such a sum
 // over the root mean square.  The row's share of `h` that a wave writes is its own slice of the channels.
-template <int MOST>
-__global__ __launch_bounds__(MOST) void route_norm_few_kernel(RouteNormArgs a, const float* __restrict__ w, RouteRule rule, int n, int width,
+__global__ __launch_bounds__(512) void route_norm_few_kernel(RouteNormArgs a, const float* __restrict__ w, RouteRule rule, int n, int width,
                                                              int experts, int top, float* __restrict__ gates, float* __restrict__ keep) {
-  __shared__ float lg[kWave * kRouteMost];
+  __shared__ float lg[kWave * kRouteMost];  // the outputs' logits, the shared expert's behind them
   const int row = blockIdx.x, wave = threadIdx.x / kWave, lane = threadIdx.x % kWave, waves = blockDim.x / kWave;
   const float* __restrict__ x = a.x + (size_t)row * width;
   auto gain_at = [&](int c) { return a.gain_dtype == NNIS_F32 ? load4((const float*)a.gain + c) : load4((const bf16_t*)a.gain + c); };
   float inv = 0.0f;
-  const int dots = n + rule.shared_gate;
-  for (int e = 2 * wave; e < dots; e += 2 * waves) {
+  for (int e = 2 * wave; e < n; e += 2 * waves) {
+    const bool third = rule.shared_gate && e == 0;  // (the shared expert's logit, one more than the pairs)
     const float* __restrict__ w0 = w + (size_t)e * width;
-    const float* __restrict__ w1 = w + (size_t)(e + 1 < dots ? e + 1 : e) * width;
-    float ss = 0.0f, dot0 = 0.0f, dot1 = 0.0f;
-#pragma unroll 8
-    for (int c = 4 * lane; c < width; c += 4 * kWave) {
+    const float* __restrict__ w1 = w + (size_t)(e + 1 < n ? e + 1 : e) * width;
+    const float* __restrict__ w2 = w + (size_t)(third ? n : e) * width;
+    float ss = 0.0f, dot0 = 0.0f, dot1 = 0.0f, dot2 = 0.0f;
+    auto take = [&](int c, bool with_third) {
       const float4 v = *(const float4*)(x + c), m = *(const float4*)(w0 + c), o = *(const float4*)(w1 + c);
       const float4 g = gain_at(c);
       ss = fmaf(v.x, v.x, fmaf(v.y, v.y, fmaf(v.z, v.z, fmaf(v.w, v.w, ss))));
       const float4 y = make_float4(v.x * g.x, v.y * g.y, v.z * g.z, v.w * g.w);
       dot0 = fmaf(y.x, m.x, fmaf(y.y, m.y, fmaf(y.z, m.z, fmaf(y.w, m.w, dot0))));
       dot1 = fmaf(y.x, o.x, fmaf(y.y, o.y, fmaf(y.z, o.z, fmaf(y.w, o.w, dot1))));
+      if (with_third) {
+        const float4 t = *(const float4*)(w2 + c);
+        dot2 = fmaf(y.x, t.x, fmaf(y.y, t.y, fmaf(y.z, t.z, fmaf(y.w, t.w, dot2))));
+      }
+    };
+    if (third) {
+#pragma unroll 8
+      for (int c = 4 * lane; c < width; c += 4 * kWave) take(c, true);
+    } else {
+#pragma unroll 8
+      for (int c = 4 * lane; c < width; c += 4 * kWave) take(c, false);
     }
 #pragma unroll
     for (int offset = kWave / 2; offset > 0; offset >>= 1) {
       ss += __shfl_xor(ss, offset, kWave);
       dot0 += __shfl_xor(dot0, offset, kWave);
       dot1 += __shfl_xor(dot1, offset, kWave);
+      dot2 += __shfl_xor(dot2, offset, kWave);
     }
     inv = 1.0f / sqrtf(ss / (float)width + a.eps);
     if (lane == 0) {
       lg[e] = dot0 * inv;
-      if (e + 1 < dots) lg[e + 1] = dot1 * inv;
+      if (e + 1 < n) lg[e + 1] = dot1 * inv;
+      if (third) lg[n] = dot2 * inv;
     }
   }
   __syncthreads();
@@ -1349,12 +1380,8 @@ extern "C" int nnis_route_norm(float* x, const void* delta, int delta_dtype, con
     return 0;
   }
   if (rows <= 256 && fours && delta == nullptr) {
-    // (each has outputs of its own, and with them the row's root mean square; up to twelve pairs of outputs in one round)
-    const int pairs = (dots + 1) / 2, waves = pairs <= 12 ? pairs : 8;
-    if (waves <= 8)
-      hipLaunchKernelGGL(route_norm_few_kernel<512>, dim3(rows), dim3(kWave * waves), 0, s, a, w, rule, n, width, experts, top, gates, keep);
-    else
-      hipLaunchKernelGGL(route_norm_few_kernel<768>, dim3(rows), dim3(kWave * waves), 0, s, a, w, rule, n, width, experts, top, gates, keep);
+    const int waves = n < 16 ? (n + 1) / 2 : 8;  // (each has outputs of its own, and with them the row's root mean square)
+    hipLaunchKernelGGL(route_norm_few_kernel, dim3(rows), dim3(kWave * waves), 0, s, a, w, rule, n, width, experts, top, gates, keep);
     NNIS_LAUNCH_CHECK("route_norm");
     return 0;
   }
