@@ -173,7 +173,7 @@ def choose(h, w, router):
         pick = torch.where(open_.repeat_interleave(size, dim=1), s, torch.full_like(s, -1.0))
     chosen = torch.topk(pick, router["top"], dim=-1).indices
     weights = torch.gather(s, 1, chosen)
-    return chosen, weights / (weights.sum(-1, keepdim=True) + 1e-20) * router["scale"]
+    return chosen, weights / (weights.sum(-1, keepdim=True) + 1e-20) * router.get("scale", 1.0)
 
 
 def routed_feed_forward(h, w, mlp, rnd=identity):
