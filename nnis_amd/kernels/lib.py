@@ -64,7 +64,9 @@ PREBUILT_WIDE_VALUES = ("attn_hd7v5c", "attn_hd32v16c", "attn_hd16v48c", "attn_h
                         # latents as the one key/value head without any extras, in a window or not: the tests' sizes and the measurements'
                         "attn_hd48v40", "attn_hd64v48", "attn_hd32v24", "attn_hd20v16", "attn_hd160v128", "attn_hd256v192",
                         # scores that fall with the logarithm of the distance and gated heads: the tests' sizes and the measurements'
-                        "attn_hd32v16lg", "attn_hd16v48lg", "attn_hd24v40lg", "attn_hd16lg", "attn_hd32v16clgx", "attn_hd64lg", "attn_hd128lg")
+                        "attn_hd32v16lg", "attn_hd16v48lg", "attn_hd24v40lg", "attn_hd16lg", "attn_hd32v16clgx", "attn_hd64lg", "attn_hd128lg",
+                        # values of another size without any options: the tests' sizes
+                        "attn_hd32v16", "attn_hd16v48")
 
 _loaded: Dict[str, ctypes.CDLL] = {}
 _lock = threading.Lock()

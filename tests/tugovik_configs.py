@@ -60,4 +60,4 @@ TUG_C = tugovik(512, 128, [
     layer(rglru(64, 4), moe(9, 3, 40, (3, 1), 1.75, shared=72)), layer(mamba2(2, 32, 64, 2, 3, 4)),
     layer(attention(4, 1, 16, 16, scale=0.25), moe(4, 2, 16, (4, 3), 0.9))], loop=(0, 3, 3), side=8)
 
-TUGOVIK_CONFIGS = {"A": (TUG_A, 61), "B": (TUG_B, 62), "C": (TUG_C, 63)}
+TUGOVIK_CONFIGS = {"A": (TUG_A, 61), "B": (TUG_B, 62), "C": (TUG_C, 79)}
